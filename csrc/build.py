@@ -10,6 +10,8 @@ There is no JIT op_builder (the reference's `op_builder/*` is a per-op JIT; see 
 every extension is compiled once with hipcc / g++ and loaded with torch.ops.load_library.
 Incremental: an object is rebuilt only if its source or any header under csrc/include changed.
 
+Serving entry points of a checkout without built libraries compile a subset (``build(units=...)``).
+
 Usage: python csrc/build.py [-j N] [--force] [--only hip|cpu]
 """
 import argparse
@@ -69,7 +71,9 @@ def _compile(kind, src, obj, flags, force):
     return obj, True
 
 
-def build(jobs=None, force=False, only=None, verbose=True):
+def build(jobs=None, force=False, only=None, verbose=True, units=None, hip_out=None):
+    """``units``: only these kernels/*.hip (names without suffix), linked into ``hip_out`` -- a library with
+    what one workload needs, for a first run in a checkout that has nothing built."""
     inc, lib, abi = _torch_paths()
     py_inc = sysconfig.get_paths()["include"]
     os.makedirs(BUILD_DIR, exist_ok=True)
@@ -78,21 +82,24 @@ def build(jobs=None, force=False, only=None, verbose=True):
     common += ["-I" + p for p in inc]
     hip_flags = common + [f"--offload-arch={ARCH}", "-D__HIP_PLATFORM_AMD__=1", "-DUSE_ROCM=1",
                           "-fno-gpu-rdc", "-munsafe-fp-atomics", "-Wno-unused-result",
+                          # no packed-FP32 instructions: some of their forms give wrong results on this chip
+                          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
                           "-Wno-return-type", "-ffp-contract=fast"]
     # -fno-math-errno: std::sqrt in the optimizer loops may not set errno, else GCC keeps them scalar
     cpu_flags = common + ["-fopenmp", "-fno-math-errno", "-Wall", "-Wno-unused-function", "-Wno-sign-compare"]
     targets = []
     if only in (None, "hip"):
-        hip_srcs = sorted(f for f in os.listdir(os.path.join(CSRC, "kernels")) if f.endswith(".hip"))
+        hip_srcs = sorted(f for f in os.listdir(os.path.join(CSRC, "kernels"))
+                          if f.endswith(".hip") and (units is None or f[:-4] in units))
         targets.append(("hip", [os.path.join(CSRC, "kernels", f) for f in hip_srcs],
-                        os.path.join(OUT_DIR, "_sxe_hip.so"), hip_flags,
+                        hip_out or os.path.join(OUT_DIR, "_sxe_hip.so"), hip_flags,
                         ["-lc10", "-lc10_hip", "-ltorch", "-ltorch_cpu", "-ltorch_hip", "-lamdhip64"]))
     if only in (None, "cpu"):
         cpu_srcs = sorted(f for f in os.listdir(os.path.join(CSRC, "cpu")) if f.endswith(".cpp"))
         targets.append(("cpu", [os.path.join(CSRC, "cpu", f) for f in cpu_srcs],
                         os.path.join(OUT_DIR, "_sxe_cpu.so"), cpu_flags,
                         ["-lc10", "-ltorch", "-ltorch_cpu", "-fopenmp", "-lpthread"]))
-    jobs = jobs or min(8, os.cpu_count() or 4)
+    jobs = jobs or min(8, os.cpu_count() or 4, int(os.environ.get("MAX_JOBS") or 8))
     results = {}
     with cf.ThreadPoolExecutor(jobs) as ex:
         futs = {}

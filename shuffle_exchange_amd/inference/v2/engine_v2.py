@@ -102,11 +102,17 @@ class InferenceEngineV2:
         dev = self._model.device
         bs = self._config.kv_block_size
         nblocks = self._config.num_kv_blocks or self._size_cache(dev, bs)
-        self._kv = BlockedKVCache(self._model.num_layers, nblocks, bs, self._model.nkv, self._model.head_dim,
-                                  dtype=self._model.dtype, device=dev)
+        self._kv = BlockedKVCache(self._model.num_layers, nblocks, bs, dtype=self._model.dtype, device=dev,
+                                  **self._cache_geometry())
         max_blocks_seq = math.ceil(sm.max_context / bs)
         self._state = DSStateManager(self._kv, sm.max_tracked_sequences, max_blocks_seq)
         self._decode_graphs = None
+
+    def _cache_geometry(self):
+        m = self._model
+        if getattr(m, "kv_shapes", None) is not None:  # layers with sizes of their own
+            return {"layer_shapes": m.kv_shapes}
+        return {"n_kv_heads": m.nkv, "head_dim": m.head_dim}
 
     def _size_cache(self, dev, bs):
         m = self._model
@@ -121,7 +127,7 @@ class InferenceEngineV2:
                 budget = mc.size
             else:
                 budget = max(0, free - mc.size)
-        return BlockedKVCache.blocks_for_budget(budget, m.num_layers, bs, m.nkv, m.head_dim, m.dtype)
+        return BlockedKVCache.blocks_for_budget(budget, m.num_layers, bs, dtype=m.dtype, **self._cache_geometry())
 
     # ------------------------------------------------------------------------------------ API
     @property
@@ -136,15 +142,18 @@ class InferenceEngineV2:
     def model(self):
         return self._model
 
-    def put(self, batch_uids, batch_tokens, do_checks=True):
+    def put(self, batch_uids, batch_tokens, do_checks=True, want=None):
         """Run one forward over the new tokens of every listed sequence; returns [n_seqs, vocab]
-        fp32 logits of each sequence's last new token."""
+        fp32 logits of each sequence's last new token -- or, with ``want`` (per sequence, places among
+        its new tokens, possibly none), the logits of those places in order [n_wanted, vocab]."""
         tokens = [t if torch.is_tensor(t) else torch.tensor(t) for t in batch_tokens]
         tokens = [t.reshape(-1).cpu() for t in tokens]
         if do_checks:
             r = self.can_schedule(batch_uids, [t.numel() for t in tokens])
             if r != SchedulingResult.Success:
                 raise SchedulingError(r)
+        if want is not None and any(not 0 <= int(j) < t.numel() for t, w in zip(tokens, want) for j in w):
+            raise ValueError("want: places outside the new tokens")
         seqs = []
         for uid, t in zip(batch_uids, tokens):
             s = self._state.get_or_create_sequence(uid)
@@ -154,8 +163,11 @@ class InferenceEngineV2:
         runner = self._decode_runner()
         if runner is not None and runner.eligible(seqs, [t.numel() for t in tokens]):
             logits = runner.run(seqs, tokens)
+            if want is not None:  # one new token each: all rows but those of sequences that want none
+                rows = [i for i, w in enumerate(want) for _ in w]
+                logits = logits if rows == list(range(len(seqs))) else logits[rows]
         else:
-            batch = RaggedBatch(seqs, tokens, self._kv.block_size, self._model.device)
+            batch = RaggedBatch(seqs, tokens, self._kv.block_size, self._model.device, want)
             logits = self._model.forward(batch, self._kv)
         for s in seqs:
             s.post_forward()

@@ -4,16 +4,19 @@
   modules in place (no weight copy);
 * ``RaggedDecoder`` (hf_decoder.py): Hugging Face checkpoints of the FastGen families -- Llama-2/3,
   Mistral, Mixtral, Qwen2, Qwen2-MoE, Phi, Phi-3, Falcon, OPT -- converted once into the packed
-  layout of the gfx950 kernels.
+  layout of the gfx950 kernels;
+* ``RaggedLayeredDecoder`` (layered_decoder.py): designs whose config lists every layer with sizes of its
+  own (Tobinex).
 """
 from .hf_decoder import RaggedDecoder, load_hf_decoder, spec_from_hf_config  # noqa: F401
+from .layered_decoder import RaggedLayeredDecoder, load_layered_decoder  # noqa: F401
 from .llama import RaggedLlama  # noqa: F401
 
 
 def ragged_model_for(model, weight_quant=None, tp_group=None, tp_size=1, pins=None):
     """Pick the ragged implementation for a model object (``weight_quant='fp8'``: row-scaled e4m3
     projection / LM-head weights for the decode GEMMs; ``tp_group``: tensor-parallel sharding)."""
-    if isinstance(model, (RaggedDecoder, RaggedLlama)):
+    if isinstance(model, (RaggedDecoder, RaggedLayeredDecoder, RaggedLlama)):
         if getattr(model, "tp", 1) != tp_size:
             raise ValueError(f"model was sharded for tp={getattr(model, 'tp', 1)}, engine tp_size={tp_size}: "
                              "build it with the same tensor_parallel config (build_hf_engine does)")

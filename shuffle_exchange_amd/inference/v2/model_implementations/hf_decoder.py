@@ -652,10 +652,15 @@ class RaggedDecoder:
 def load_hf_decoder(model_or_path, dtype=torch.bfloat16, device=None, weight_quant=None, tp_group=None, tp_size=1):
     """A transformers model instance or a local checkpoint directory (config.json + safetensors /
     pytorch_model*.bin, loaded without executing pickled code) -> RaggedDecoder (this rank's
-    tensor-parallel shard when ``tp_size > 1``)."""
+    tensor-parallel shard when ``tp_size > 1``). A directory whose config names one of
+    ``layered_decoder.ARCHITECTURES`` gives a RaggedLayeredDecoder."""
     if isinstance(model_or_path, (str, os.PathLike)):
         with open(os.path.join(model_or_path, "config.json")) as f:
             cfg = json.load(f)
+        from .layered_decoder import is_layered_config, load_layered_decoder
+        if is_layered_config(cfg):
+            return load_layered_decoder(model_or_path, dtype=dtype, device=device, weight_quant=weight_quant,
+                                        tp_size=tp_size)
         sd = _load_state_dict(model_or_path)
     else:
         cfg = model_or_path.config.to_dict()

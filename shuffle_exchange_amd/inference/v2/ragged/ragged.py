@@ -51,20 +51,45 @@ class BlockedAllocator:
 
 
 class BlockedKVCache:
-    def __init__(self, num_layers, num_blocks, block_size, n_kv_heads, head_dim, dtype=torch.bfloat16, device=None):
+    """One block id addresses the same block in every layer. Uniform models: one allocation [layers,
+    blocks, 2, nkv, bs, D]. ``layer_shapes`` (one (kv heads, k row, v row) per layer): an allocation
+    per layer whose blocks hold that layer's k [nkv, bs, k row] then v [nkv, bs, v row]."""
+
+    def __init__(self, num_layers, num_blocks, block_size, n_kv_heads=0, head_dim=0, dtype=torch.bfloat16, device=None,
+                 layer_shapes=None):
         self.num_layers, self.num_blocks, self.block_size = num_layers, num_blocks, block_size
         self.n_kv_heads, self.head_dim = n_kv_heads, head_dim
-        self.cache = torch.zeros(num_layers, num_blocks, 2, n_kv_heads, block_size, head_dim, dtype=dtype,
-                                 device=device)
+        self.layer_shapes = layer_shapes
+        if layer_shapes is None:
+            self.cache = torch.zeros(num_layers, num_blocks, 2, n_kv_heads, block_size, head_dim, dtype=dtype,
+                                     device=device)
+        else:
+            assert len(layer_shapes) == num_layers, "one cache shape per layer"
+            self.cache = None
+            self._kv = []
+            for nkv, dk, dv in layer_shapes:
+                buf = torch.zeros(num_blocks, nkv * block_size * (dk + dv), dtype=dtype, device=device)
+                n = nkv * block_size * dk
+                self._kv.append((buf[:, :n].unflatten(1, (nkv, block_size, dk)),
+                                 buf[:, n:].unflatten(1, (nkv, block_size, dv))))
         self.allocator = BlockedAllocator(num_blocks)
 
     @staticmethod
-    def blocks_for_budget(budget_bytes, num_layers, block_size, n_kv_heads, head_dim, dtype=torch.bfloat16):
-        per_block = num_layers * 2 * n_kv_heads * block_size * head_dim * torch.tensor([], dtype=dtype).element_size()
+    def blocks_for_budget(budget_bytes, num_layers, block_size, n_kv_heads=0, head_dim=0, dtype=torch.bfloat16,
+                          layer_shapes=None):
+        rows = (num_layers * 2 * n_kv_heads * head_dim if layer_shapes is None
+                else sum(nkv * (dk + dv) for nkv, dk, dv in layer_shapes))
+        per_block = rows * block_size * torch.tensor([], dtype=dtype).element_size()
         return max(1, int(budget_bytes // per_block))
 
     def layer(self, i):
         return self.cache[i]
+
+    def layer_kv(self, i):
+        """(k, v) views [blocks, nkv, bs, row] of layer ``i``."""
+        if self.layer_shapes is None:
+            return self.cache[i][:, 0], self.cache[i][:, 1]
+        return self._kv[i]
 
     def reserve(self, n):
         return self.allocator.allocate(n)
@@ -145,22 +170,27 @@ class RaggedBatch:
     """Device metadata of one forward over a ragged set of sequences (all int tensors on device).
 
     input_ids [T]; positions [T] (absolute); slots [T] (cache slot of every new token);
-    q_start / q_len / kv_len [S] int32; block_table [S, max_blocks] int32; last_idx [S] int64.
-    Host copies of the small per-sequence ints are kept for scheduling decisions.
+    q_start / q_len / kv_len [S] int32; block_table [S, max_blocks] int32; last_idx int64: the rows whose
+    logits are returned -- every sequence's last new token [S], or with ``want`` (per sequence, places
+    among its new tokens) those places in order. Host copies of the small per-sequence ints are kept
+    for scheduling decisions.
     """
 
-    def __init__(self, seqs, tokens, block_size, device):
+    def __init__(self, seqs, tokens, block_size, device, want=None):
         S = len(seqs)
         lens = [int(t.numel()) for t in tokens]
         T = sum(lens)
+        if want is None:
+            want = [(n - 1,) for n in lens]
+        n_want = sum(len(x) for x in want)
         maxb = max(1, max(len(s.blocks) for s in seqs))
-        i64 = torch.empty(3 * T + S, dtype=torch.int64, pin_memory=torch.cuda.is_available() and device.type == "cuda")
+        i64 = torch.empty(3 * T + n_want, dtype=torch.int64, pin_memory=torch.cuda.is_available() and device.type == "cuda")
         i32 = torch.zeros(3 * S + S * maxb, dtype=torch.int32,
                           pin_memory=torch.cuda.is_available() and device.type == "cuda")
         ids, pos, slots, last = i64[:T], i64[T:2 * T], i64[2 * T:3 * T], i64[3 * T:]
         qs, ql, kl = i32[:S], i32[S:2 * S], i32[2 * S:3 * S]
         bt = i32[3 * S:].view(S, maxb)
-        t = 0
+        t, nw = 0, 0
         self.host_q_len, self.host_kv_len, self.host_seen = [], [], []
         for i, (s, tk) in enumerate(zip(seqs, tokens)):
             n = lens[i]
@@ -171,7 +201,9 @@ class RaggedBatch:
             slots[t:t + n] = blk[p // block_size] * block_size + p % block_size
             qs[i], ql[i], kl[i] = t, n, s.seen_tokens + n
             bt[i, :len(s.blocks)] = torch.tensor(s.blocks, dtype=torch.int32)
-            last[i] = t + n - 1
+            for j in want[i]:
+                last[nw] = t + int(j)
+                nw += 1
             self.host_q_len.append(n)
             self.host_kv_len.append(s.seen_tokens + n)
             self.host_seen.append(s.seen_tokens)

@@ -100,7 +100,7 @@ def restore_entries(tensors, meta, device):
 # ------------------------------------------------------------------------------------------------
 def serialize_engine(engine, save_path):
     """Write ``engine``'s model (this rank's shard) under ``save_path`` (every TP rank calls this)."""
-    from .model_implementations import RaggedDecoder, RaggedLlama
+    from .model_implementations import RaggedDecoder, RaggedLayeredDecoder, RaggedLlama
     os.makedirs(save_path, exist_ok=True)
     m = engine._model
     cfg = engine._config
@@ -108,13 +108,13 @@ def serialize_engine(engine, save_path):
               "kv_block_size": cfg.kv_block_size, "weight_quant": getattr(m, "weight_quant", None)
               or getattr(m, "_weight_quant", None)}
     rank = int(getattr(m, "tp_rank", 0))
-    if isinstance(m, RaggedDecoder):
+    if isinstance(m, (RaggedDecoder, RaggedLayeredDecoder)):
         named = {k: v for k, v in m.w.items() if k != "layers"}
         for i, L in enumerate(m.w["layers"]):
             named.update({f"layers.{i}.{k}": v for k, v in L.items()})
-        desc = dict(common, implementation="RaggedDecoder", spec=_jsonable(dataclasses.asdict(m.spec)),
+        desc = dict(common, implementation=type(m).__name__, spec=_jsonable(dataclasses.asdict(m.spec)),
                     n_layers=len(m.w["layers"]))
-        rank_meta = {"nq": m.nq, "nkv": m.nkv}
+        rank_meta = {"nq": m.nq, "nkv": m.nkv} if isinstance(m, RaggedDecoder) else {}
     elif isinstance(m, RaggedLlama):
         named = dict(m.model.state_dict())
         desc = dict(common, implementation="RaggedLlama", model_class=type(m.model).__name__,
@@ -137,8 +137,9 @@ def build_engine_from_ds_checkpoint(path, engine_config=None, debug_level=None):
     with (``tensor_parallel.tp_size`` is taken from the checkpoint)."""
     from ... import comm as dist
     from .engine_v2 import InferenceEngineV2, RaggedInferenceEngineConfig, _tp_group
-    from .model_implementations import RaggedDecoder, RaggedLlama
+    from .model_implementations import RaggedDecoder, RaggedLayeredDecoder, RaggedLlama
     from .model_implementations.hf_decoder import DecoderSpec, _rope_cache
+    from .model_implementations.layered_decoder import LayeredSpec
     with open(os.path.join(path, "ds_model_config.json")) as f:
         desc = json.load(f)
     if desc.get("format") != FORMAT:
@@ -154,9 +155,8 @@ def build_engine_from_ds_checkpoint(path, engine_config=None, debug_level=None):
     device = torch.device("cuda", torch.cuda.current_device()) if torch.cuda.is_available() else torch.device("cpu")
     dtype = getattr(torch, desc["dtype"])
     named = restore_entries(tensors, rmeta["entries"], device)
-    if desc["implementation"] == "RaggedDecoder":
+    if desc["implementation"] in ("RaggedDecoder", "RaggedLayeredDecoder"):
         sd = _unjson(desc["spec"])
-        spec = DecoderSpec(**{k: (tuple(v) if isinstance(v, list) else v) for k, v in sd.items()})
         w = {"layers": [dict() for _ in range(int(desc["n_layers"]))]}
         for k, v in named.items():
             if k.startswith("layers."):
@@ -164,6 +164,10 @@ def build_engine_from_ds_checkpoint(path, engine_config=None, debug_level=None):
                 w["layers"][int(i)][key] = v
             else:
                 w[k] = v
+    if desc["implementation"] == "RaggedLayeredDecoder":
+        m = RaggedLayeredDecoder.restore(LayeredSpec.from_dict(sd), w, dtype, device, desc.get("weight_quant"))
+    elif desc["implementation"] == "RaggedDecoder":
+        spec = DecoderSpec(**{k: (tuple(v) if isinstance(v, list) else v) for k, v in sd.items()})
         m = RaggedDecoder.__new__(RaggedDecoder)
         m.spec, m.tp, m.tp_group, m.tp_rank = spec, tp, group, rank
         m.nq, m.nkv = int(rmeta["nq"]), int(rmeta["nkv"])

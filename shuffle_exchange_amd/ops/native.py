@@ -68,6 +68,28 @@ def require_cpu():
     return torch.ops.sxe_cpu
 
 
+SERVING_UNITS = ("act", "mix_attn", "residual_norm", "skinny_gemm")
+
+
+def ensure_serving_library():
+    """For command-line serving: use the full HIP library when it is built, else compile the kernels of the
+    layered decoders (SERVING_UNITS) into a library of their own, once per checkout (the build is
+    incremental: it is brought up to date when a source changed)."""
+    global HIP_LIB
+    if _state["hip"] is not None or os.path.exists(HIP_LIB):
+        return
+    import importlib.util
+    import sys
+    root = os.path.dirname(os.path.dirname(_HERE))
+    spec = importlib.util.spec_from_file_location("sxe_build", os.path.join(root, "csrc", "build.py"))
+    b = importlib.util.module_from_spec(spec)
+    spec.loader.exec_module(b)
+    out = os.path.join(_HERE, "_sxe_hip_serving.so")
+    print("compiling the serving kernels", file=sys.stderr, flush=True)
+    b.build(only="hip", units=SERVING_UNITS, hip_out=out, verbose=False)
+    HIP_LIB = out
+
+
 def use_hip(t):
     """Dispatch predicate for a tensor argument: GPU tensors go to the HIP kernels (and fail
     loudly if those are missing); CPU tensors use the PyTorch reference path."""

@@ -20,6 +20,7 @@ def main():
              "-I" + os.path.join(ROOT, "csrc", "include"), "-I" + sysconfig.get_paths()["include"]]
     flags += ["-I" + p for p in inc]
     flags += [f"--offload-arch={build.ARCH}", "-D__HIP_PLATFORM_AMD__=1", "-DUSE_ROCM=1", "-fno-gpu-rdc",
+              "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
               "-munsafe-fp-atomics", "-Wno-unused-result", "-Wno-return-type", "-ffp-contract=fast",
               "--offload-device-only", "-Rpass-analysis=kernel-resource-usage"]
     r = subprocess.run(["hipcc"] + flags + ["-c", src, "-o", "/tmp/_kres.o"], capture_output=True, text=True)
