@@ -15,6 +15,8 @@
 // Caches are [blocks, nkv, bs, D] views (k and v separately, block stride free).
 #include "sxe_common.h"
 #include <torch/library.h>
+#include <climits>
+#include <set>
 
 namespace sxe {
 namespace ma {
@@ -144,6 +146,694 @@ __global__ __launch_bounds__(kGenThreads) void mix_attn_generic_kernel(Args a, i
   }
 }
 
+// ---- matrix-core building blocks (bf16, head rows D = 64 / 128 / 256) ------------------------------
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef short i16x4 __attribute__((ext_vector_type(4)));
+typedef short i16x8 __attribute__((ext_vector_type(8)));
+typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+__device__ __forceinline__ bf16x8 frag(const unsigned short* p) {
+  return __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(p));
+}
+__device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float lg2(float x) { return __builtin_amdgcn_logf(x); }
+
+// swizzle of the 16-byte chunks of row `row` of a [rows][D bf16] LDS image (transposed reads conflict-free)
+template <int D>
+__device__ __forceinline__ int chunk_xor(int row) {
+  constexpr int CH = D / 8;
+  return (((row & 3) << 2) | ((row >> 2) & 3)) & (CH >= 16 ? 15 : CH - 1);
+}
+// lane group g's 4-row block of a 16-row tile in transposed reads (see paged_attn.hip)
+__device__ __forceinline__ int kperm(int g) { return ((g & 1) << 3) | ((g & 2) << 1); }
+
+// V^T operand of a 16x16x32 product: lane (g, i) holds column 16 dt + i of rows r0 + kperm(g) + 0..3 and
+// of the same rows 16 further down
+template <int D>
+__device__ __forceinline__ bf16x8 v_frag(const char* img, int r0, int dt, int lane) {
+  const int g = lane >> 4, i = lane & 15, p4 = i & 3;
+  const int ra = r0 + kperm(g) + (i >> 2);  // r0 a multiple of 16: the row 16 further down has the same swizzle
+  const int at = ra * 2 * D + ((16 * ((p4 >> 1) ^ chunk_xor<D>(ra)) + 8 * (p4 & 1)) ^ (32 * dt));
+  const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+      (__attribute__((address_space(3))) i16x4*)(const_cast<char*>(img) + at));
+  const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+      (__attribute__((address_space(3))) i16x4*)(const_cast<char*>(img) + at + 32 * D));
+  return __builtin_bit_cast(bf16x8, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+}
+
+// bf16 head and remainder of a weight: p = hi + lo to ~2^-17, so the head mix sees 32-bit-grade weights
+struct HiLo {
+  unsigned short hi, lo;
+};
+__device__ __forceinline__ HiLo hi_lo(float p) {
+  HiLo r;
+  r.hi = f32_to_bf16(p);
+  r.lo = f32_to_bf16(p - bf16_to_f32(r.hi));
+  return r;
+}
+// a value the compiler cannot see through: what is computed from it stays inside the loop
+__device__ __forceinline__ int opaque(int v) {
+  asm volatile("" : "+v"(v));
+  return v;
+}
+__device__ __forceinline__ unsigned pack2(float a, float b) {
+  typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
+  const bf16x2 v = {(__bf16)a, (__bf16)b};
+  return __builtin_bit_cast(unsigned, v);
+}
+
+// ---- token form: scores of one token through memory ------------------------------------------------
+// Two launches for tokens that come alone (decode, short continuations, any head count): the first
+// computes biased scores of one kv head's query heads over a split of the token's visible keys, writes
+// them (log2 domain, fp32) and each split's (max, sum); the second turns the scores of ALL heads into
+// weights, mixes them for one kv head's query heads and multiplies that head's values. A split's output
+// is already normalised, so splits just add up.
+struct TokArgs {
+  float* scores;  // [rows, nq, nv]
+  float* ml;      // [splits, rows, nq, 2]
+  float* part;    // [splits, rows, nq, dv] (splits > 1)
+  int nv, splits, keys_per_split;
+  int nt, tok0, max_len;  // rows = S * nt: tokens tok0 .. tok0 + nt - 1 of sequences with q_len <= max_len
+};
+
+template <int D>
+struct TokGeo {
+  static constexpr int NT = D >= 256 ? 2 : 4;
+  static constexpr int KC = 16 * NT, KS = D / 32, DT = D / 16;
+  static constexpr int VIMG = KC * 2 * D;
+};
+constexpr int kTokWaves = 4, kMaxHeads = 256;
+
+struct TokRow {
+  int seq, pos;
+  int64_t t;
+  bool ok;
+};
+__device__ __forceinline__ TokRow tok_row(const Args& a, const TokArgs& k, int row) {
+  TokRow r;
+  r.seq = row / k.nt;
+  const int tok = k.tok0 + row - r.seq * k.nt, ql = a.q_len[r.seq];
+  r.ok = tok < ql && ql <= k.max_len;
+  r.pos = a.kv_len[r.seq] - ql + tok;
+  r.t = a.q_start[r.seq] + tok;
+  return r;
+}
+
+template <int D>
+__global__ __launch_bounds__(256) void mix_scores_kernel(Args a, TokArgs k) {
+  using P = TokGeo<D>;
+  constexpr int NT = P::NT, KC = P::KC, KS = P::KS;
+  __shared__ float red[kTokWaves][16][2];
+  const int row = blockIdx.x / a.nkv, c = blockIdx.x - row * a.nkv, split = blockIdx.y;
+  const TokRow r = tok_row(a, k, row);
+  if (!r.ok) return;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, i = lane & 15, G = a.nq / a.nkv;
+  const Vis vis = visible(r.pos, a.window, a.keep_first);
+  const int cb = split * k.keys_per_split, ce = min(vis.n, cb + k.keys_per_split);
+  const int* bt = a.block_table + (int64_t)r.seq * a.max_blocks;
+  const unsigned short* kc = static_cast<const unsigned short*>(a.kc);
+  const int rows = gridDim.x / a.nkv;
+  const float sc2 = a.scale * kLog2e;
+  for (int h0 = 0; h0 < G; h0 += 16) {
+    const bool hok = h0 + i < G;
+    const int h = c * G + (hok ? h0 + i : 0);
+    bf16x8 qb[KS];
+    const unsigned short* qp = static_cast<const unsigned short*>(a.q) + (r.t * a.nq + h) * D + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) qb[ks] = frag(qp + 32 * ks);
+    const float r1 = a.r1 != nullptr ? a.r1[h] : 0.f, r2 = a.r1 != nullptr ? a.r2[h] : 0.f;
+    float m = -INFINITY, l = 0.f;
+    float* srow = k.scores + ((int64_t)row * a.nq + h) * k.nv;
+    for (int kb = cb + wave * KC; kb < ce; kb += kTokWaves * KC) {
+      bf16x8 kr[NT][KS];
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        const int key = vis_key(vis, min(kb + 16 * t + i, ce - 1));
+        const unsigned short* kp = kc + bt[key / a.bs] * a.k_block + ((int64_t)c * a.bs + key % a.bs) * D + 8 * g;
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) kr[t][ks] = frag(kp + 32 * ks);
+      }
+      f32x4 s[NT];
+      float mx = -INFINITY;
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) s[t] = mfma16(kr[t][ks], qb[ks], s[t]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int ci = kb + 16 * t + 4 * g + e;
+          const float d = (float)(r.pos - vis_key(vis, ci));
+          s[t][e] = ci < ce ? s[t][e] * sc2 - r1 * lg2(1.f + r2 * d) : -INFINITY;
+          mx = fmaxf(mx, s[t][e]);
+        }
+        const int ci = kb + 16 * t + 4 * g;  // < nv: nv is a multiple of 64 and ci of 4
+        if (hok && ci < ce) *reinterpret_cast<f32x4*>(srow + ci) = s[t];
+      }
+      const float mn = fmaxf(m, mx);
+      if (mn != -INFINITY) {
+        l *= ex2(m - mn);
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) l += ex2(s[t][e] - mn);
+        m = mn;
+      }
+    }
+#pragma unroll
+    for (int o = 16; o < 64; o <<= 1) {
+      const float m2 = __shfl_xor(m, o, 64), l2 = __shfl_xor(l, o, 64), mn = fmaxf(m, m2);
+      l = mn == -INFINITY ? 0.f : l * ex2(m - mn) + l2 * ex2(m2 - mn);
+      m = mn;
+    }
+    __syncthreads();
+    if (g == 0) {
+      red[wave][i][0] = m;
+      red[wave][i][1] = l;
+    }
+    __syncthreads();
+    if (threadIdx.x < 16 && h0 + (int)threadIdx.x < G) {
+      float M = -INFINITY, L = 0.f;
+#pragma unroll
+      for (int w = 0; w < kTokWaves; ++w) M = fmaxf(M, red[w][threadIdx.x][0]);
+      if (M != -INFINITY)
+#pragma unroll
+        for (int w = 0; w < kTokWaves; ++w) L += red[w][threadIdx.x][1] * ex2(red[w][threadIdx.x][0] - M);
+      float* o = k.ml + (((int64_t)split * rows + row) * a.nq + c * G + h0 + threadIdx.x) * 2;
+      o[0] = M;
+      o[1] = L;
+    }
+  }
+}
+
+template <int D>
+__global__ __launch_bounds__(256) void mix_values_kernel(Args a, TokArgs k) {
+  using P = TokGeo<D>;
+  constexpr int NT = P::NT, KC = P::KC, DT = P::DT;
+  extern __shared__ __attribute__((aligned(16))) char smem[];  // V images, then the wave-merge buffer
+  __shared__ int64_t voff[kTokWaves][KC];
+  __shared__ float lse[kMaxHeads];
+  __shared__ __attribute__((aligned(16))) unsigned short tl[16][kMaxHeads + 8];
+  const int row = blockIdx.x / a.nkv, c = blockIdx.x - row * a.nkv, split = blockIdx.y;
+  const TokRow r = tok_row(a, k, row);
+  if (!r.ok) return;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, i = lane & 15, G = a.nq / a.nkv;
+  const Vis vis = visible(r.pos, a.window, a.keep_first);
+  const int cb = split * k.keys_per_split, ce = min(vis.n, cb + k.keys_per_split);
+  const int* bt = a.block_table + (int64_t)r.seq * a.max_blocks;
+  const int rows = gridDim.x / a.nkv, HP = (a.nq + 31) / 32 * 32;
+  char* vimg = smem + wave * P::VIMG;
+  float* mrg = reinterpret_cast<float*>(smem);  // [kTokWaves][16][D] after the key loop
+  const unsigned short* vc = static_cast<const unsigned short*>(a.vc);
+  for (int h = threadIdx.x; h < a.nq; h += 256) {  // log-sum-exp of every head's row, sink included
+    const float sk = a.sink != nullptr ? a.sink[h] * kLog2e : -INFINITY;
+    float M = sk;
+    for (int s = 0; s < k.splits; ++s) M = fmaxf(M, k.ml[(((int64_t)s * rows + row) * a.nq + h) * 2]);
+    float L = a.sink != nullptr ? ex2(sk - M) : 0.f;
+    for (int s = 0; s < k.splits; ++s) {
+      const float* ml = k.ml + (((int64_t)s * rows + row) * a.nq + h) * 2;
+      if (ml[0] != -INFINITY) L += ml[1] * ex2(ml[0] - M);
+    }
+    lse[h] = M + lg2(L);
+  }
+  for (int h0 = 0; h0 < G; h0 += 16) {
+    __syncthreads();  // the previous pass is done with `tl` and the merge buffer
+    for (int e = threadIdx.x; e < 16 * HP; e += 256) {
+      const int n = e / HP, gg = e - n * HP;
+      float v = 0.f;
+      if (h0 + n < G && gg < a.nq)
+        v = a.talk != nullptr ? a.talk[(int64_t)(c * G + h0 + n) * a.nq + gg] : (gg == c * G + h0 + n ? 1.f : 0.f);
+      tl[n][gg] = f32_to_bf16(v);
+    }
+    __syncthreads();
+    f32x4 o[DT];
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) o[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int kb = cb + wave * KC; kb < ce; kb += kTokWaves * KC) {
+      if (lane < KC) {
+        const int key = vis_key(vis, min(kb + lane, ce - 1));
+        voff[wave][lane] = bt[key / a.bs] * a.v_block + ((int64_t)c * a.bs + key % a.bs) * D;
+      }
+      __builtin_amdgcn_s_waitcnt(0xc07f);  // lgkmcnt(0)
+      __builtin_amdgcn_wave_barrier();
+      {
+        constexpr int CH = D / 8, RPK = 64 / CH;
+#pragma unroll
+        for (int n = 0; n < KC / RPK; ++n) {
+          const int rw = RPK * n + lane / CH, ch = (lane % CH) ^ chunk_xor<D>(rw);
+          __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(vc + voff[wave][rw] + ch * 8),
+                                           (__attribute__((address_space(3))) void*)(vimg + n * 1024), 16, 0, 0);
+        }
+      }
+      // W^T = P^T T^T: rows = keys (lane i <-> key kperm(i >> 2) + (i & 3)), columns = this group's heads
+      f32x4 w[NT];
+#pragma unroll
+      for (int t = 0; t < NT; ++t) w[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int kk = 0; kk < HP; kk += 32) {
+        const bf16x8 tb = *reinterpret_cast<const bf16x8*>(&tl[i][kk + 8 * g]);
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+          const int ci = kb + 16 * t + kperm(i >> 2) + (i & 3);
+          i16x8 hi, lo;
+          float sv[8];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            const int h = kk + 8 * g + j;
+            sv[j] = ci < ce && h < a.nq ? k.scores[((int64_t)row * a.nq + h) * k.nv + ci] - lse[h] : -INFINITY;
+          }
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            const HiLo p = hi_lo(ex2(sv[j]));
+            hi[j] = (short)p.hi;
+            lo[j] = (short)p.lo;
+          }
+          w[t] = mfma16(__builtin_bit_cast(bf16x8, hi), tb, w[t]);
+          w[t] = mfma16(__builtin_bit_cast(bf16x8, lo), tb, w[t]);
+        }
+      }
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's V image has landed
+      __builtin_amdgcn_wave_barrier();
+#pragma unroll
+      for (int pp = 0; pp < NT / 2; ++pp) {
+        bf16x8 pb;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          pb[e] = (__bf16)w[2 * pp][e];
+          pb[4 + e] = (__bf16)w[2 * pp + 1][e];
+        }
+#pragma unroll
+        for (int dt = 0; dt < DT; ++dt) o[dt] = mfma16(v_frag<D>(vimg, 32 * pp, dt, lane), pb, o[dt]);
+      }
+      __builtin_amdgcn_s_waitcnt(0xc07f);  // the V image is read before the next chunk overwrites it
+      __builtin_amdgcn_wave_barrier();
+    }
+    __syncthreads();  // every wave is done with its V image (the merge buffer aliases it)
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) *reinterpret_cast<f32x4*>(mrg + (wave * 16 + i) * D + 16 * dt + 4 * g) = o[dt];
+    __syncthreads();
+    const int nh = min(16, G - h0);
+    for (int e = threadIdx.x; e < nh * a.dv; e += 256) {
+      const int n = e / a.dv, d = e - n * a.dv, h = c * G + h0 + n;
+      float v = 0.f;
+#pragma unroll
+      for (int w = 0; w < kTokWaves; ++w) v += mrg[(w * 16 + n) * D + d];
+      const int64_t col = (int64_t)h * a.dv + d;
+      if (k.splits == 1) {
+        if (a.gate != nullptr)
+          v /= 1.f + __expf(-bf16_to_f32(static_cast<const unsigned short*>(a.gate)[r.t * a.gate_ld + col]));
+        static_cast<unsigned short*>(a.out)[r.t * a.nq * a.dv + col] = f32_to_bf16(v);
+      } else {
+        k.part[((int64_t)split * rows + row) * a.nq * a.dv + col] = v;
+      }
+    }
+  }
+}
+
+// out = (sum over splits) * sigmoid(gate)
+__global__ __launch_bounds__(256) void mix_reduce_kernel(Args a, TokArgs k) {
+  const int row = blockIdx.x, rows = gridDim.x;
+  const TokRow r = tok_row(a, k, row);
+  if (!r.ok) return;
+  const int n = a.nq * a.dv;
+  for (int col = blockIdx.y * 256 + threadIdx.x; col < n; col += gridDim.y * 256) {
+    float v = 0.f;
+    for (int s0 = 0; s0 < k.splits; s0 += 8) {  // eight loads in flight, then their sum
+      float p[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) p[u] = k.part[((int64_t)min(s0 + u, k.splits - 1) * rows + row) * n + col];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) v += s0 + u < k.splits ? p[u] : 0.f;
+    }
+    if (a.gate != nullptr)
+      v /= 1.f + __expf(-bf16_to_f32(static_cast<const unsigned short*>(a.gate)[r.t * a.gate_ld + col]));
+    static_cast<unsigned short*>(a.out)[r.t * n + col] = f32_to_bf16(v);
+  }
+}
+
+// ---- tile form: 16 consecutive tokens of a sequence, all heads -------------------------------------
+// Prompts and long continuations. First launch: log-sum-exp of every (token, head) row, one wave per (16
+// tokens, kv head). Second launch: one 8-wave workgroup per 16 tokens; wave w owns HPW query heads.
+// Per 32-key tile: (a) every wave computes its heads' weights 2^(s - lse) (S^T = K Q^T, K fragments
+// straight from the cache, shared by the heads of a kv head) and puts their bf16 head and remainder
+// into LDS; (b) the waves mix: W = P T^T as matrix products over the head axis, 4 (token, 16-key)
+// tiles a wave, W to LDS in the order of the value product's operand; (c) every wave multiplies its
+// heads' W with its kv head's V (row image in LDS, transposed reads). The value product of a tile and the
+// weights of the next one lie between the same two barriers, so two barriers a tile suffice.
+// The distance bias takes 47 values per (head, tile) -- one logarithm per lane, handed round by
+// ds_bpermute -- instead of one per score.
+struct TileArgs {
+  float* lse;            // [T, nq]
+  unsigned short* talk;  // [2][64][8] bf16: lane l's operand of the mix, T[16 n + (l & 15)][8 (l >> 4) .. + 7]
+  int min_len, tiles;  // sequences with q_len >= min_len; 16-token tiles per sequence
+};
+constexpr int kTileWaves = 8, kTileKeys = 32, kTileHeads = 32;
+
+struct TileIdx {
+  int seq, p0, ntok;  // sequence, first position, tokens in the tile
+  int64_t t0;
+  bool ok;
+};
+__device__ __forceinline__ TileIdx tile_idx(const Args& a, const TileArgs& k, int id) {
+  TileIdx x;
+  x.seq = id / k.tiles;
+  const int tok = (id - x.seq * k.tiles) * 16, ql = x.seq < a.S ? a.q_len[x.seq] : 0;
+  x.ok = tok < ql && ql >= k.min_len;
+  if (!x.ok) return x;
+  x.p0 = a.kv_len[x.seq] - ql + tok;
+  x.ntok = min(16, ql - tok);
+  x.t0 = a.q_start[x.seq] + tok;
+  return x;
+}
+
+// 32-key tiles of a token tile: [0, kt) cover the kept keys in front of the window, then [wt, end)
+struct KeyTiles {
+  int kt, wt, n;
+};
+__device__ __forceinline__ KeyTiles key_tiles(const Args& a, const TileIdx& x) {
+  KeyTiles k;
+  const int lo = a.window > 0 ? max(0, x.p0 + 1 - a.window) : 0;
+  k.wt = lo / kTileKeys;
+  k.kt = min(k.wt, (a.keep_first + kTileKeys - 1) / kTileKeys);
+  k.n = k.kt + (x.p0 + x.ntok - 1) / kTileKeys + 1 - k.wt;
+  return k;
+}
+__device__ __forceinline__ int key0(const KeyTiles& k, int n) { return (n < k.kt ? n : k.wt + n - k.kt) * kTileKeys; }
+
+// whether some (token, key) pair of the tile is hidden
+__device__ __forceinline__ bool needs_mask(const Args& a, const TileIdx& x, int k0) {
+  const int k1 = k0 + kTileKeys - 1;
+  if (k1 > x.p0) return true;
+  return a.window > 0 && x.p0 + 15 - k0 >= a.window && k1 >= a.keep_first;
+}
+__device__ __forceinline__ bool sees(const Args& a, int pos, int key) {
+  return key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
+}
+
+template <int D>
+__global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int total) {
+  constexpr int KS = D / 32, HB = 4;  // heads per round
+  if (blockIdx.x == 0)  // the next launch's operand of the head mix (no mix: the identity)
+    for (int e = threadIdx.x; e < 1024; e += 256) {
+      const int h = 16 * (e >> 9) + ((e >> 3) & 15), gg = 8 * ((e >> 7) & 3) + (e & 7);
+      float f = h == gg ? 1.f : 0.f;
+      if (a.talk != nullptr) f = h < a.nq && gg < a.nq ? a.talk[h * a.nq + gg] : 0.f;
+      k.talk[e] = f32_to_bf16(f);
+    }
+  const int unit = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (unit >= total) return;
+  const int c = unit % a.nkv;
+  const TileIdx x = tile_idx(a, k, unit / a.nkv);
+  if (!x.ok) return;
+  const int lane = threadIdx.x & 63, g = lane >> 4, i = lane & 15, G = a.nq / a.nkv;
+  const KeyTiles kt = key_tiles(a, x);
+  const int* bt = a.block_table + (int64_t)x.seq * a.max_blocks;
+  const unsigned short *kc = static_cast<const unsigned short*>(a.kc), *q = static_cast<const unsigned short*>(a.q);
+  const int tok = min(i, x.ntok - 1);
+  const float sc2 = a.scale * kLog2e;
+  const int bidx = 4 * (4 * g - i + 15);
+  for (int h0 = 0; h0 < G; h0 += HB) {
+    bf16x8 qb[HB][KS];
+    float m[HB], l[HB], r1[HB], r2[HB];
+#pragma unroll
+    for (int hh = 0; hh < HB; ++hh) {
+      const int h = c * G + min(h0 + hh, G - 1);
+      const unsigned short* qp = q + ((x.t0 + tok) * a.nq + h) * D + 8 * g;
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) qb[hh][ks] = frag(qp + 32 * ks);
+      m[hh] = -INFINITY;
+      l[hh] = 0.f;
+      r1[hh] = a.r1 != nullptr ? a.r1[h] : 0.f;
+      r2[hh] = a.r1 != nullptr ? a.r2[h] : 0.f;
+    }
+    for (int n = 0; n < kt.n; ++n) {
+      const int k0 = key0(kt, n);
+      const bool msk = needs_mask(a, x, k0);
+      const unsigned short* kp = kc + bt[k0 / a.bs] * a.k_block + ((int64_t)c * a.bs + k0 % a.bs + i) * D + 8 * g;
+      bf16x8 kr[2][KS];
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) kr[t][ks] = frag(kp + 16 * t * D + 32 * ks);
+      const float dl = (float)max(0, x.p0 - k0 + 15 - lane);  // the distance whose bias this lane computes
+#pragma unroll
+      for (int hh = 0; hh < HB; ++hh) {
+        if (h0 + hh >= G) break;
+        f32x4 s[2];
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+          s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int ks = 0; ks < KS; ++ks) s[t] = mfma16(kr[t][ks], qb[hh][ks], s[t]);
+        }
+        const int tb = __builtin_bit_cast(int, r1[hh] * lg2(1.f + r2[hh] * dl));
+        float mx = -INFINITY;
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            s[t][e] = s[t][e] * sc2 - __builtin_bit_cast(float, __builtin_amdgcn_ds_bpermute(bidx + 4 * (16 * t + e), tb));
+            if (msk && !sees(a, x.p0 + i, k0 + 16 * t + 4 * g + e)) s[t][e] = -INFINITY;
+            mx = fmaxf(mx, s[t][e]);
+          }
+        const float mn = fmaxf(m[hh], mx), mr = mn == -INFINITY ? 0.f : mn;
+        float ls = 0.f;
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) ls += ex2(s[t][e] - mr);
+        l[hh] = l[hh] * ex2(m[hh] - mr) + ls;
+        m[hh] = mn;
+      }
+    }
+#pragma unroll
+    for (int hh = 0; hh < HB; ++hh) {
+      if (h0 + hh >= G) break;
+      float M = m[hh], L = l[hh];
+#pragma unroll
+      for (int o = 16; o < 64; o <<= 1) {
+        const float m2 = __shfl_xor(M, o, 64), l2 = __shfl_xor(L, o, 64), mn = fmaxf(M, m2);
+        L = mn == -INFINITY ? 0.f : L * ex2(M - mn) + l2 * ex2(m2 - mn);
+        M = mn;
+      }
+      const int h = c * G + h0 + hh;
+      if (a.sink != nullptr) {
+        const float sk = a.sink[h] * kLog2e, mn = fmaxf(M, sk);
+        L = L * ex2(M - mn) + ex2(sk - mn);
+        M = mn;
+      }
+      if (g == 0 && i < x.ntok) k.lse[(x.t0 + i) * a.nq + h] = M + lg2(L);
+    }
+  }
+}
+
+// ONE_KV: every wave's HPW heads exist and belong to one kv head (nq / nkv a multiple of HPW)
+template <int D, int HPW, bool ONE_KV>
+__global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, TileArgs k, int total) {
+  constexpr int KS = D / 32, DT = D / 16, PB = 16 * kTileKeys * kTileHeads * 2, VIMG = kTileKeys * 2 * D;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  char *phi = smem, *plo = smem + PB, *wbuf = smem + 2 * PB;
+  // consecutive tiles of a sequence share most of their window: keep them on one XCD's L2
+  const int per = (total + 7) / 8, id = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+  if (id >= total) return;
+  const TileIdx x = tile_idx(a, k, id);
+  if (!x.ok) return;
+  const int lane_ = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), G = a.nq / a.nkv;
+  const int g = lane_ >> 4, i = lane_ & 15;
+  char* vimg = smem + 3 * PB + wave * VIMG;
+  const KeyTiles kt = key_tiles(a, x);
+  const int* bt = a.block_table + (int64_t)x.seq * a.max_blocks;
+  const unsigned short *kc = static_cast<const unsigned short*>(a.kc), *vc = static_cast<const unsigned short*>(a.vc);
+  const int hw = wave * HPW;  // first head of this wave
+  const int nh = min(HPW, a.nq - hw);
+  const int tok = min(i, x.ntok - 1);
+  const float sc2 = a.scale * kLog2e;
+  // heads past nq are never written by a wave: their weights stay zero
+  for (int e = threadIdx.x; e < 2 * PB / 16; e += kTileWaves * 64) reinterpret_cast<u32x4*>(smem)[e] = u32x4{0u, 0u, 0u, 0u};
+  bf16x8 qb[HPW][KS];
+  float lse[HPW];
+  f32x4 o[HPW][DT];
+#pragma unroll
+  for (int hh = 0; hh < HPW; ++hh) {
+    const int h = min(hw + hh, a.nq - 1);
+    const unsigned short* qp = static_cast<const unsigned short*>(a.q) + ((x.t0 + tok) * a.nq + h) * D + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) qb[hh][ks] = frag(qp + 32 * ks);
+    lse[hh] = k.lse[(x.t0 + tok) * a.nq + h];
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) o[hh][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  const int nmix = a.nq > 16 ? 2 : 1;
+  __syncthreads();
+
+  auto stage_v = [&](int lane, int c, int k0) {
+    constexpr int CH = D / 8, RPK = 64 / CH;
+    const unsigned short* vp = vc + bt[k0 / a.bs] * a.v_block + ((int64_t)c * a.bs + k0 % a.bs) * D;
+#pragma unroll
+    for (int n = 0; n < kTileKeys / RPK; ++n) {
+      const int rw = RPK * n + lane / CH, ch = (lane % CH) ^ chunk_xor<D>(rw);
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(vp + rw * D + ch * 8),
+                                       (__attribute__((address_space(3))) void*)(vimg + n * 1024), 16, 0, 0);
+    }
+  };
+
+  for (int n = 0; n < kt.n; ++n) {
+    const int k0 = key0(kt, n);
+    // LDS and cache addresses are recomputed from the lane in every phase: kept across the loop they
+    // would not fit the registers beside the accumulators and the queries
+    if (nh > 0) {
+      const int lane = opaque(lane_), g = lane >> 4, i = lane & 15;
+      const bool msk = needs_mask(a, x, k0);
+      __builtin_amdgcn_s_waitcnt(0xc07f);  // the previous tile's V reads are done
+      stage_v(lane, hw / G, k0);
+      const float dl = (float)max(0, x.p0 - k0 + 15 - lane);
+      int tbl[HPW];
+#pragma unroll
+      for (int hh = 0; hh < HPW; ++hh) {
+        const int h = min(hw + hh, a.nq - 1);
+        tbl[hh] = a.r1 != nullptr ? __builtin_bit_cast(int, a.r1[h] * lg2(1.f + a.r2[h] * dl)) : 0;
+      }
+      const unsigned short* kp = kc + bt[k0 / a.bs] * a.k_block + ((int64_t)k0 % a.bs + i) * D + 8 * g;
+#pragma unroll 1
+      for (int t = 0; t < 2; ++t) {
+        bf16x8 kr[KS];
+        unsigned ph[4][HPW == 4 ? 2 : 1], pl[4][HPW == 4 ? 2 : 1];  // bf16 pairs of neighbouring heads
+        const int bx = 4 * (4 * g - i + 15) + 64 * t;
+        auto load_k = [&](int c) {
+          const unsigned short* p = kp + ((int64_t)c * a.bs + 16 * t) * D;
+#pragma unroll
+          for (int ks = 0; ks < KS; ++ks) kr[ks] = frag(p + 32 * ks);
+        };
+        if constexpr (ONE_KV) load_k(hw / G);
+#pragma unroll
+        for (int hp = 0; hp < (HPW + 1) / 2; ++hp) {
+          float v[2][4];
+#pragma unroll
+          for (int u = 0; u < (HPW == 1 ? 1 : 2); ++u) {
+            const int hh = 2 * hp + u;
+            if constexpr (!ONE_KV) {
+              const int h = min(hw + hh, a.nq - 1);
+              if (hh == 0 || h / G != (h - 1) / G) load_k(h / G);
+            }
+            f32x4 sc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int ks = 0; ks < KS; ++ks) sc = mfma16(kr[ks], qb[hh][ks], sc);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              v[u][e] = sc[e] * sc2 - __builtin_bit_cast(float, __builtin_amdgcn_ds_bpermute(bx + 4 * e, tbl[hh])) - lse[hh];
+              if (msk && !sees(a, x.p0 + i, k0 + 16 * t + 4 * g + e)) v[u][e] = -INFINITY;
+            }
+            if (!ONE_KV && hh >= nh)
+#pragma unroll
+              for (int e = 0; e < 4; ++e) v[u][e] = -INFINITY;
+          }
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const float p0 = ex2(v[0][e]), p1 = HPW == 1 ? 0.f : ex2(v[1][e]);
+            const unsigned h2 = pack2(p0, p1);
+            ph[e][hp] = h2;
+            pl[e][hp] = pack2(p0 - __uint_as_float(h2 << 16), p1 - __uint_as_float(h2 & 0xffff0000u));
+          }
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int key = 16 * t + 4 * g + e, b = 2 * hw;
+          const int at = (i * kTileKeys + (key ^ (i & 3))) * (2 * kTileHeads) + 16 * ((b >> 4) ^ ((i >> 2) & 3)) + (b & 15);
+          if constexpr (HPW == 4) {
+            *reinterpret_cast<uint2*>(phi + at) = uint2{ph[e][0], ph[e][1]};
+            *reinterpret_cast<uint2*>(plo + at) = uint2{pl[e][0], pl[e][1]};
+          } else if constexpr (HPW == 2) {
+            *reinterpret_cast<unsigned*>(phi + at) = ph[e][0];
+            *reinterpret_cast<unsigned*>(plo + at) = pl[e][0];
+          } else {
+            *reinterpret_cast<unsigned short*>(phi + at) = (unsigned short)ph[e][0];
+            *reinterpret_cast<unsigned short*>(plo + at) = (unsigned short)pl[e][0];
+          }
+        }
+      }
+    }
+    bf16x8 tb[2];
+#pragma unroll
+    for (int nn = 0; nn < 2; ++nn) tb[nn] = frag(k.talk + (nn * 64 + lane_) * 8);
+    __syncthreads();
+    // ---- mix: this wave's tokens 2 wave, 2 wave + 1, both 16-key halves ------------------------------
+    const int lm = opaque(lane_);
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int g = lm >> 4, i = lm & 15;
+      const int q = 2 * wave + (u >> 1), t = u & 1, key = 16 * t + i;
+      const int at = (q * kTileKeys + (key ^ (q & 3))) * (2 * kTileHeads) + 16 * (g ^ ((q >> 2) & 3));
+      const bf16x8 hi = *reinterpret_cast<const bf16x8*>(phi + at), lo = *reinterpret_cast<const bf16x8*>(plo + at);
+#pragma unroll
+      for (int nn = 0; nn < 2; ++nn) {
+        if (nn >= nmix) break;
+        f32x4 w = {0.f, 0.f, 0.f, 0.f};
+        w = mfma16(hi, tb[nn], w);
+        w = mfma16(lo, tb[nn], w);
+        // lane: head h, keys 16 t + 4 g .. + 3 of token q -> chunk of the lane group that reads those rows of V
+        const int h = 16 * nn + i, ch = ((g & 1) << 1) | (g >> 1);
+        const int wt = (h * 16 + (q ^ (h & 3))) * (2 * kTileKeys) + 16 * (ch ^ ((h >> 2) & 3)) + 8 * t;
+        *reinterpret_cast<u16x4*>(wbuf + wt) = u16x4{f32_to_bf16(w[0]), f32_to_bf16(w[1]), f32_to_bf16(w[2]), f32_to_bf16(w[3])};
+      }
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // V image
+    __syncthreads();
+    // ---- O^T += V^T W^T ------------------------------------------------------------------------------
+    if (nh > 0) {
+      const int lane = opaque(lane_), g = lane >> 4, i = lane & 15;
+      bf16x8 wf[HPW];
+#pragma unroll
+      for (int hh = 0; hh < HPW; ++hh) {
+        const int h = hw + hh;  // < 32: eight waves of at most four heads
+        wf[hh] = *reinterpret_cast<const bf16x8*>(wbuf + (h * 16 + (i ^ (h & 3))) * (2 * kTileKeys) + 16 * (g ^ ((h >> 2) & 3)));
+      }
+      if constexpr (ONE_KV) {
+#pragma unroll
+        for (int dt = 0; dt < DT; ++dt) {
+          const bf16x8 vf = v_frag<D>(vimg, 0, dt, lane);
+#pragma unroll
+          for (int hh = 0; hh < HPW; ++hh) o[hh][dt] = mfma16(vf, wf[hh], o[hh][dt]);
+        }
+      } else {
+#pragma unroll
+        for (int hh = 0; hh < HPW; ++hh) {  // the wave's heads span several kv heads: stage each V in turn
+          if (hh >= nh) break;
+          const int h = hw + hh;
+          if (hh > 0 && h / G != (h - 1) / G) {
+            __builtin_amdgcn_s_waitcnt(0xc07f);
+            stage_v(lane, h / G, k0);
+            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+            __builtin_amdgcn_wave_barrier();
+          }
+#pragma unroll
+          for (int dt = 0; dt < DT; ++dt) o[hh][dt] = mfma16(v_frag<D>(vimg, 0, dt, lane), wf[hh], o[hh][dt]);
+        }
+      }
+    }
+  }
+  if (i >= x.ntok) return;
+  const int64_t t = x.t0 + i;
+  unsigned short* out = static_cast<unsigned short*>(a.out) + t * a.nq * a.dv;
+  const unsigned short* gate = a.gate != nullptr ? static_cast<const unsigned short*>(a.gate) + t * a.gate_ld : nullptr;
+#pragma unroll
+  for (int hh = 0; hh < HPW; ++hh) {
+    if (hh >= nh) break;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int d = 16 * dt + 4 * g + e;
+        if (d >= a.dv) continue;
+        const int64_t col = (int64_t)(hw + hh) * a.dv + d;
+        float v = o[hh][dt][e];
+        if (gate != nullptr) v /= 1.f + __expf(-bf16_to_f32(gate[col]));
+        out[col] = f32_to_bf16(v);
+      }
+  }
+}
+
 }  // namespace ma
 
 namespace {
@@ -155,16 +845,98 @@ const float* head_vec(const c10::optional<at::Tensor>& t, int64_t n, const char*
   return t->data_ptr<float>();
 }
 
+// dynamic LDS above 64 KiB must be opted into, once per kernel
+template <typename F>
+void allow_lds(F* kern, size_t bytes) {
+  static std::set<const void*> done;
+  const void* f = reinterpret_cast<const void*>(kern);
+  if (done.insert(f).second)
+    SXE_HIP_CHECK(hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes));
+}
+
+template <int D>
+void launch_tokens_d(const ma::Args& a, const ma::TokArgs& k, int rows) {
+  const dim3 grid(rows * a.nkv, k.splits);
+  constexpr int merge = ma::kTokWaves * 16 * D * 4, img = ma::kTokWaves * ma::TokGeo<D>::VIMG;
+  constexpr size_t lds = img > merge ? img : merge;
+  hipLaunchKernelGGL(ma::mix_scores_kernel<D>, grid, dim3(256), 0, cur_stream(), a, k);
+  allow_lds(ma::mix_values_kernel<D>, lds);
+  hipLaunchKernelGGL(ma::mix_values_kernel<D>, grid, dim3(256), lds, cur_stream(), a, k);
+  if (k.splits > 1) {
+    const int cols = a.nq * a.dv;
+    hipLaunchKernelGGL(ma::mix_reduce_kernel, dim3(rows, std::min(64, (cols + 255) / 256)), dim3(256), 0, cur_stream(), a, k);
+  }
+  SXE_LAUNCH_CHECK();
+}
+
+void launch_tokens(const ma::Args& a, const at::Tensor& q, int nv, int splits, int tok0, int nt, int max_len) {
+  ma::TokArgs k{};
+  const int rows = a.S * nt;
+  int kps = (nv + std::max(1, splits) - 1) / std::max(1, splits);
+  kps = (kps + 63) / 64 * 64;
+  k.nv = nv;
+  k.keys_per_split = kps;
+  k.splits = (nv + kps - 1) / kps;
+  k.nt = nt;
+  k.tok0 = tok0;
+  k.max_len = max_len;
+  const auto f32 = q.options().dtype(at::kFloat);
+  auto scores = at::empty({(int64_t)rows * a.nq * nv}, f32), ml = at::empty({(int64_t)k.splits * rows * a.nq * 2}, f32);
+  at::Tensor part;
+  if (k.splits > 1) part = at::empty({(int64_t)k.splits * rows * a.nq * a.dv}, f32);
+  k.scores = scores.data_ptr<float>();
+  k.ml = ml.data_ptr<float>();
+  k.part = k.splits > 1 ? part.data_ptr<float>() : nullptr;
+  if (a.Dk == 64) launch_tokens_d<64>(a, k, rows);
+  else if (a.Dk == 128) launch_tokens_d<128>(a, k, rows);
+  else launch_tokens_d<256>(a, k, rows);
+}
+
+template <int D, int HPW>
+void launch_tile_kernel(const ma::Args& a, const ma::TileArgs& k, int total) {
+  constexpr size_t lds = 3 * 16 * ma::kTileKeys * ma::kTileHeads * 2 + ma::kTileWaves * ma::kTileKeys * 2 * D;
+  auto go = [&](auto kern) {
+    allow_lds(kern, lds);
+    hipLaunchKernelGGL(kern, dim3((total + 7) / 8 * 8), dim3(ma::kTileWaves * 64), lds, cur_stream(), a, k, total);
+  };
+  if (a.nq / a.nkv % HPW == 0) go(ma::mix_tile_kernel<D, HPW, true>);
+  else go(ma::mix_tile_kernel<D, HPW, false>);
+}
+
+void launch_tiles(const ma::Args& a, const at::Tensor& q, int min_len, int max_q_len) {
+  ma::TileArgs k{};
+  auto lse = at::empty({(int64_t)a.T * a.nq}, q.options().dtype(at::kFloat)), talk = at::empty({1024}, q.options());
+  k.lse = lse.data_ptr<float>();
+  k.talk = static_cast<unsigned short*>(talk.data_ptr());
+  k.min_len = min_len;
+  k.tiles = (max_q_len + 15) / 16;
+  const int total = a.S * k.tiles, units = total * a.nkv;
+  if (a.Dk == 64) hipLaunchKernelGGL(ma::mix_lse_kernel<64>, dim3((units + 3) / 4), dim3(256), 0, cur_stream(), a, k, units);
+  else hipLaunchKernelGGL(ma::mix_lse_kernel<128>, dim3((units + 3) / 4), dim3(256), 0, cur_stream(), a, k, units);
+  const int hpw = a.nq <= 8 ? 1 : a.nq <= 16 ? 2 : 4;
+#define SXE_MIX_TILE(D)                                     \
+  do {                                                      \
+    if (hpw == 1) launch_tile_kernel<D, 1>(a, k, total);     \
+    else if (hpw == 2) launch_tile_kernel<D, 2>(a, k, total); \
+    else launch_tile_kernel<D, 4>(a, k, total);              \
+  } while (0)
+  if (a.Dk == 64) SXE_MIX_TILE(64);
+  else SXE_MIX_TILE(128);
+#undef SXE_MIX_TILE
+  SXE_LAUNCH_CHECK();
+}
+
 }  // namespace
 
 // q [T, nq, Dk], kc / vc [blocks, nkv, bs, Dk / Dv] -> out [T, nq * dv]; see the top of the file.
-// max_q_len bounds every q_len; force_generic picks the any-size kernel (fp32 always uses it).
+// min_q_len / max_q_len bound every q_len. form: 0 = by shape, 1 = any-size kernel (fp32 always), 2 = token
+// form, 3 = tile form. splits: KV splits of the token form.
 at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& block_table,
                          const at::Tensor& q_start, const at::Tensor& q_len, const at::Tensor& kv_len,
-                         int64_t max_q_len, int64_t max_kv_len, int64_t dk, int64_t dv, double scale, int64_t window,
+                         int64_t min_q_len, int64_t max_q_len, int64_t max_kv_len, int64_t splits, int64_t dk, int64_t dv, double scale, int64_t window,
                          int64_t keep_first, const c10::optional<at::Tensor>& r1, const c10::optional<at::Tensor>& r2,
                          const c10::optional<at::Tensor>& sink, const c10::optional<at::Tensor>& talk,
-                         const c10::optional<at::Tensor>& gate, bool force_generic) {
+                         const c10::optional<at::Tensor>& gate, int64_t form) {
   SXE_CHECK_CUDA(q);
   SXE_CHECK(q.dim() == 3 && q.is_contiguous(), "mix_attention: q [T, nq, Dk] contiguous");
   const int64_t T = q.size(0), nq = q.size(1), nkv = kc.size(1), S = block_table.size(0);
@@ -220,6 +992,27 @@ at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Te
   }
   a.out = out.data_ptr();
   c10::DeviceGuard g(q.device());
+  const int64_t D = kc.size(3);
+  const bool mfma = q.scalar_type() == at::kBFloat16 && D == vc.size(3) && (D == 64 || D == 128 || D == 256) &&
+                    nq <= ma::kMaxHeads && kc.stride(0) % 8 == 0 && vc.stride(0) % 8 == 0 &&
+                    reinterpret_cast<uintptr_t>(a.kc) % 16 == 0 && reinterpret_cast<uintptr_t>(a.vc) % 16 == 0;
+  const bool tile_ok = mfma && nq <= ma::kTileHeads && D <= 128 && a.bs % ma::kTileKeys == 0;
+  SXE_CHECK(form != 2 || mfma, "mix_attention: token form needs bf16 rows of 64, 128 or 256");
+  SXE_CHECK(form != 3 || tile_ok, "mix_attention: tile form needs bf16 rows of 64 or 128, <= 32 heads, blocks of 32 n");
+  if (mfma && form != 1) {
+    constexpr int64_t kTileMin = 8;  // shorter runs of new tokens go token by token
+    const int64_t tile_min = form == 2 || !tile_ok ? INT_MAX : form == 3 ? 1 : kTileMin;
+    if (max_q_len >= tile_min) launch_tiles(a, q, (int)tile_min, (int)max_q_len);
+    if (min_q_len < tile_min) {
+      // the scores of one launch stay within 256 MiB: long runs of tokens take several
+      const int64_t nv = (std::min<int64_t>(max_kv_len, a.window > 0 ? a.window + a.keep_first : max_kv_len) + 63) / 64 * 64;
+      const int64_t run = std::min(max_q_len, tile_min - 1);
+      const int64_t per = std::max<int64_t>(1, (int64_t(1) << 28) / (S * nq * nv * 4));
+      for (int64_t t0 = 0; t0 < run; t0 += per)
+        launch_tokens(a, q, (int)nv, (int)splits, (int)t0, (int)std::min(per, run - t0), (int)std::min<int64_t>(tile_min - 1, INT_MAX));
+    }
+    return out;
+  }
   const size_t lds = sizeof(float) * (nq * (dk + dv) + 2 * nq * ma::kGenKeys + 2 * nq);
   SXE_CHECK(lds <= 160 * 1024, "mix_attention: heads x sizes exceed the LDS of one compute unit");
   SXE_DISPATCH_DT(dtype_of(q), D, {
@@ -240,7 +1033,7 @@ at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Te
 
 TORCH_LIBRARY_FRAGMENT(sxe, m) {
   m.def("mix_attention(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor q_start, Tensor q_len, Tensor kv_len, "
-        "int max_q_len, int max_kv_len, int dk, int dv, float scale, int window, int keep_first, Tensor? r1, Tensor? r2, "
-        "Tensor? sink, Tensor? talk, Tensor? gate, bool force_generic=False) -> Tensor");
+        "int min_q_len, int max_q_len, int max_kv_len, int splits, int dk, int dv, float scale, int window, int keep_first, Tensor? r1, Tensor? r2, "
+        "Tensor? sink, Tensor? talk, Tensor? gate, int form=0) -> Tensor");
 }
 TORCH_LIBRARY_IMPL(sxe, CUDA, m) { m.impl("mix_attention", &sxe::mix_attention); }

@@ -8,7 +8,9 @@ from typing import Optional
 import torch
 
 from . import native
+from .paged_attention import choose_splits
 
+FORMS = {"auto": 0, "generic": 1, "token": 2, "tile": 3}
 MFMA_ROWS = (64, 128, 256)  # cache row lengths of the matrix-core kernels
 
 
@@ -31,14 +33,18 @@ class MixParams:
     talk: Optional[torch.Tensor] = None   # [nq, nq]
 
 
-def mix_attention(q, kc, vc, batch, dk, dv, scale, params, window=None, keep_first=0, gate=None, force_generic=False):
+def mix_attention(q, kc, vc, batch, dk, dv, scale, params, window=None, keep_first=0, gate=None, form="auto"):
     """q [T, nq, D] against the paged k / v caches [blocks, nkv, bs, D] of ``batch`` (RaggedBatch fields)
-    -> [T, nq * dv]. ``gate`` [T, nq * dv]: the output is multiplied by its sigmoid."""
+    -> [T, nq * dv]. ``gate`` [T, nq * dv]: the output is multiplied by its sigmoid. ``form``: which HIP
+    kernels ("auto": by shape; "generic" any size, one token per workgroup; "token" scores through
+    memory; "tile" 16 tokens x all heads)."""
     if native.use_hip(q):
+        visible = batch.max_kv_len if not window else min(batch.max_kv_len, window + keep_first)
+        splits = choose_splits(batch.num_seqs, kc.shape[1], visible, min_keys=64)
         return torch.ops.sxe.mix_attention(q, kc, vc, batch.block_table, batch.q_start, batch.q_len, batch.kv_len,
-                                           max(batch.host_q_len), int(batch.max_kv_len), int(dk), int(dv), float(scale),
-                                           int(window or 0), int(keep_first), params.r1, params.r2, params.sink,
-                                           params.talk, gate, bool(force_generic))
+                                           min(batch.host_q_len), max(batch.host_q_len), int(batch.max_kv_len), splits,
+                                           int(dk), int(dv), float(scale), int(window or 0), int(keep_first), params.r1,
+                                           params.r2, params.sink, params.talk, gate, FORMS[form])
     return mix_attention_reference(q, kc, vc, batch, dk, dv, scale, params, window, keep_first, gate)
 
 
