@@ -31,6 +31,7 @@ struct Args {
   int max_blocks;
   const int *q_start, *q_len, *kv_len;
   int S, T, nq, nkv, dk, dv, Dk, Dv, bs;  // dk / dv real sizes, Dk / Dv row lengths of the caches
+  int bs_shift;                           // log2(bs) (matrix-core forms)
   float scale;
   int window, keep_first;      // window 0: every key <= i
   const float *r1, *r2, *sink;  // [nq] or null (r1, r2 together)
@@ -184,26 +185,38 @@ __device__ __forceinline__ bf16x8 v_frag(const char* img, int r0, int dt, int la
   return __builtin_bit_cast(bf16x8, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
 }
 
-// bf16 head and remainder of a weight: p = hi + lo to ~2^-17, so the head mix sees 32-bit-grade weights
-struct HiLo {
-  unsigned short hi, lo;
-};
-__device__ __forceinline__ HiLo hi_lo(float p) {
-  HiLo r;
-  r.hi = f32_to_bf16(p);
-  r.lo = f32_to_bf16(p - bf16_to_f32(r.hi));
-  return r;
-}
 // a value the compiler cannot see through: what is computed from it stays inside the loop
 __device__ __forceinline__ int opaque(int v) {
   asm volatile("" : "+v"(v));
   return v;
 }
+// two bf16 in a word. Weights p enter the head mix as p = hi + lo, lo = bf16(p - hi), which is p to ~2^-17.
 __device__ __forceinline__ unsigned pack2(float a, float b) {
   typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
   const bf16x2 v = {(__bf16)a, (__bf16)b};
   return __builtin_bit_cast(unsigned, v);
 }
+
+// LDS byte address of a pointer into shared memory (wave-uniform, for m0)
+__device__ __forceinline__ unsigned lds_at(const char* p) {
+  return __builtin_amdgcn_readfirstlane((unsigned)(uintptr_t)(const __attribute__((address_space(3))) char*)p);
+}
+// the same with a base per lane
+__device__ __forceinline__ void dma16(unsigned lds, const void* src) {
+  asm volatile("s_mov_b32 m0, %0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(lds), "v"(src) : "memory");
+}
+__device__ __forceinline__ const unsigned short* uniform_ptr(const unsigned short* p) {
+  const uint64_t v = (uint64_t)p;
+  const unsigned lo = __builtin_amdgcn_readfirstlane((unsigned)v), hi = __builtin_amdgcn_readfirstlane((unsigned)(v >> 32));
+  return reinterpret_cast<const unsigned short*>(((uint64_t)hi << 32) | lo);
+}
+// 16 bytes per lane from base + off straight to LDS at lds + 16 lane. Inline asm: the compiler's wait-count
+// pass would put a full wait before every later LDS read that might alias it.
+__device__ __forceinline__ void dma16(unsigned lds, const void* base, unsigned off) {
+  asm volatile("s_mov_b32 m0, %0\n\tglobal_load_lds_dwordx4 %1, %2" ::"s"(lds), "v"(off), "s"(base) : "memory");
+}
+// LDS traffic of this wave done, then the workgroup barrier; loads from memory stay in flight across it
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
 // ---- token form: scores of one token through memory ------------------------------------------------
 // Two launches for tokens that come alone (decode, short continuations, any head count): the first
@@ -242,12 +255,18 @@ __device__ __forceinline__ TokRow tok_row(const Args& a, const TokArgs& k, int r
   return r;
 }
 
+// the kv heads of one row on one XCD: they share its scores through that L2
+__device__ __forceinline__ int tok_block() {
+  const int n = gridDim.x, b = blockIdx.x;
+  return n % 8 == 0 ? (b & 7) * (n / 8) + (b >> 3) : b;
+}
+
 template <int D>
 __global__ __launch_bounds__(256) void mix_scores_kernel(Args a, TokArgs k) {
   using P = TokGeo<D>;
   constexpr int NT = P::NT, KC = P::KC, KS = P::KS;
   __shared__ float red[kTokWaves][16][2];
-  const int row = blockIdx.x / a.nkv, c = blockIdx.x - row * a.nkv, split = blockIdx.y;
+  const int blk = tok_block(), row = blk / a.nkv, c = blk - row * a.nkv, split = blockIdx.y;
   const TokRow r = tok_row(a, k, row);
   if (!r.ok) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, i = lane & 15, G = a.nq / a.nkv;
@@ -272,7 +291,8 @@ __global__ __launch_bounds__(256) void mix_scores_kernel(Args a, TokArgs k) {
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
         const int key = vis_key(vis, min(kb + 16 * t + i, ce - 1));
-        const unsigned short* kp = kc + bt[key / a.bs] * a.k_block + ((int64_t)c * a.bs + key % a.bs) * D + 8 * g;
+        const unsigned short* kp =
+            kc + bt[key >> a.bs_shift] * a.k_block + ((c << a.bs_shift) + (key & (a.bs - 1))) * D + 8 * g;
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) kr[t][ks] = frag(kp + 32 * ks);
       }
@@ -330,14 +350,14 @@ __global__ __launch_bounds__(256) void mix_scores_kernel(Args a, TokArgs k) {
 }
 
 template <int D>
-__global__ __launch_bounds__(256) void mix_values_kernel(Args a, TokArgs k) {
+__global__ __launch_bounds__(256, 2) void mix_values_kernel(Args a, TokArgs k) {
   using P = TokGeo<D>;
   constexpr int NT = P::NT, KC = P::KC, DT = P::DT;
   extern __shared__ __attribute__((aligned(16))) char smem[];  // V images, then the wave-merge buffer
   __shared__ int64_t voff[kTokWaves][KC];
-  __shared__ float lse[kMaxHeads];
+  __shared__ __attribute__((aligned(16))) float lse[kMaxHeads];
   __shared__ __attribute__((aligned(16))) unsigned short tl[16][kMaxHeads + 8];
-  const int row = blockIdx.x / a.nkv, c = blockIdx.x - row * a.nkv, split = blockIdx.y;
+  const int blk = tok_block(), row = blk / a.nkv, c = blk - row * a.nkv, split = blockIdx.y;
   const TokRow r = tok_row(a, k, row);
   if (!r.ok) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, i = lane & 15, G = a.nq / a.nkv;
@@ -348,19 +368,62 @@ __global__ __launch_bounds__(256) void mix_values_kernel(Args a, TokArgs k) {
   char* vimg = smem + wave * P::VIMG;
   float* mrg = reinterpret_cast<float*>(smem);  // [kTokWaves][16][D] after the key loop
   const unsigned short* vc = static_cast<const unsigned short*>(a.vc);
-  for (int h = threadIdx.x; h < a.nq; h += 256) {  // log-sum-exp of every head's row, sink included
-    const float sk = a.sink != nullptr ? a.sink[h] * kLog2e : -INFINITY;
-    float M = sk;
-    for (int s = 0; s < k.splits; ++s) M = fmaxf(M, k.ml[(((int64_t)s * rows + row) * a.nq + h) * 2]);
-    float L = a.sink != nullptr ? ex2(sk - M) : 0.f;
-    for (int s = 0; s < k.splits; ++s) {
-      const float* ml = k.ml + (((int64_t)s * rows + row) * a.nq + h) * 2;
-      if (ml[0] != -INFINITY) L += ml[1] * ex2(ml[0] - M);
+  const float* srow = k.scores + (int64_t)row * a.nq * k.nv;
+  const int kb0 = cb + wave * KC;
+  float raw[NT][8];
+  // scores of heads 0 .. 31 for the chunk at kb (lane i <-> key kperm(i >> 2) + (i & 3), heads 8 g .. + 7)
+  auto load_scores = [&](int kb) {
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int ci = kb + 16 * t + kperm(i >> 2) + (i & 3);
+        raw[t][j] = srow[(int64_t)min(8 * g + j, a.nq - 1) * k.nv + min(ci, k.nv - 1)];
+      }
+  };
+  auto stage_v = [&](int kb) {
+    if (lane < KC) {
+      const int key = vis_key(vis, min(kb + lane, ce - 1));
+      voff[wave][lane] = bt[key >> a.bs_shift] * a.v_block + ((c << a.bs_shift) + (key & (a.bs - 1))) * D;
     }
-    lse[h] = M + lg2(L);
-  }
+    __builtin_amdgcn_s_waitcnt(0xc07f);  // lgkmcnt(0)
+    __builtin_amdgcn_wave_barrier();
+    constexpr int CH = D / 8, RPK = 64 / CH;
+    const unsigned dst = lds_at(vimg);
+#pragma unroll
+    for (int n = 0; n < KC / RPK; ++n) {
+      const int rw = RPK * n + lane / CH, ch = (lane % CH) ^ chunk_xor<D>(rw);
+      dma16(dst + n * 1024, vc + voff[wave][rw] + ch * 8);
+    }
+  };
+  auto lse_of_rows = [&]() {  // log-sum-exp of every head's row, sink included
+    const float2* ml = reinterpret_cast<const float2*>(k.ml);
+    for (int h = threadIdx.x; h < a.nq; h += 256) {
+      float M = a.sink != nullptr ? a.sink[h] * kLog2e : -INFINITY, L = a.sink != nullptr ? 1.f : 0.f;
+      for (int s0 = 0; s0 < k.splits; s0 += 8) {
+        float2 v[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) v[u] = ml[((int64_t)min(s0 + u, k.splits - 1) * rows + row) * a.nq + h];
+        float mn = M;
+#pragma unroll
+        for (int u = 0; u < 8; ++u) mn = s0 + u < k.splits ? fmaxf(mn, v[u].x) : mn;
+        L = M == -INFINITY ? 0.f : L * ex2(M - mn);
+#pragma unroll
+        for (int u = 0; u < 8; ++u) L += s0 + u < k.splits && v[u].x != -INFINITY ? v[u].y * ex2(v[u].x - mn) : 0.f;
+        M = mn;
+      }
+      lse[h] = M + lg2(L);
+    }
+    for (int h = a.nq + threadIdx.x; h < HP; h += 256) lse[h] = INFINITY;  // heads past nq: weight 0
+  };
   for (int h0 = 0; h0 < G; h0 += 16) {
-    __syncthreads();  // the previous pass is done with `tl` and the merge buffer
+    const bool some = kb0 < ce;
+    if (h0 > 0) __syncthreads();  // the previous pass is done with `tl` and the merge buffer
+    if (some) {
+      load_scores(kb0);
+      stage_v(kb0);
+    }
+    if (h0 == 0) lse_of_rows();
     for (int e = threadIdx.x; e < 16 * HP; e += 256) {
       const int n = e / HP, gg = e - n * HP;
       float v = 0.f;
@@ -372,63 +435,53 @@ __global__ __launch_bounds__(256) void mix_values_kernel(Args a, TokArgs k) {
     f32x4 o[DT];
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) o[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int kb = cb + wave * KC; kb < ce; kb += kTokWaves * KC) {
-      if (lane < KC) {
-        const int key = vis_key(vis, min(kb + lane, ce - 1));
-        voff[wave][lane] = bt[key / a.bs] * a.v_block + ((int64_t)c * a.bs + key % a.bs) * D;
-      }
-      __builtin_amdgcn_s_waitcnt(0xc07f);  // lgkmcnt(0)
-      __builtin_amdgcn_wave_barrier();
-      {
-        constexpr int CH = D / 8, RPK = 64 / CH;
-#pragma unroll
-        for (int n = 0; n < KC / RPK; ++n) {
-          const int rw = RPK * n + lane / CH, ch = (lane % CH) ^ chunk_xor<D>(rw);
-          __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(vc + voff[wave][rw] + ch * 8),
-                                           (__attribute__((address_space(3))) void*)(vimg + n * 1024), 16, 0, 0);
-        }
-      }
-      // W^T = P^T T^T: rows = keys (lane i <-> key kperm(i >> 2) + (i & 3)), columns = this group's heads
+    for (int kb = kb0; kb < ce; kb += kTokWaves * KC) {
+      const int kn = kb + kTokWaves * KC;
+      // W^T = P^T T^T: rows = keys, columns = this group's heads
       f32x4 w[NT];
 #pragma unroll
       for (int t = 0; t < NT; ++t) w[t] = f32x4{0.f, 0.f, 0.f, 0.f};
       for (int kk = 0; kk < HP; kk += 32) {
         const bf16x8 tb = *reinterpret_cast<const bf16x8*>(&tl[i][kk + 8 * g]);
+        const f32x4 la = *reinterpret_cast<const f32x4*>(&lse[kk + 8 * g]), lb = *reinterpret_cast<const f32x4*>(&lse[kk + 8 * g + 4]);
 #pragma unroll
         for (int t = 0; t < NT; ++t) {
           const int ci = kb + 16 * t + kperm(i >> 2) + (i & 3);
-          i16x8 hi, lo;
-          float sv[8];
+          u32x4 hi, lo;
+          float p[8];
+          if (kk > 0)
 #pragma unroll
-          for (int j = 0; j < 8; ++j) {
-            const int h = kk + 8 * g + j;
-            sv[j] = ci < ce && h < a.nq ? k.scores[((int64_t)row * a.nq + h) * k.nv + ci] - lse[h] : -INFINITY;
-          }
+            for (int j = 0; j < 8; ++j)
+              raw[t][j] = srow[(int64_t)min(kk + 8 * g + j, a.nq - 1) * k.nv + min(ci, k.nv - 1)];
 #pragma unroll
-          for (int j = 0; j < 8; ++j) {
-            const HiLo p = hi_lo(ex2(sv[j]));
-            hi[j] = (short)p.hi;
-            lo[j] = (short)p.lo;
+          for (int j = 0; j < 8; ++j) p[j] = ci < ce ? ex2(raw[t][j] - (j < 4 ? la[j & 3] : lb[j & 3])) : 0.f;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            hi[j] = pack2(p[2 * j], p[2 * j + 1]);
+            lo[j] = pack2(p[2 * j] - __uint_as_float(hi[j] << 16), p[2 * j + 1] - __uint_as_float(hi[j] & 0xffff0000u));
           }
           w[t] = mfma16(__builtin_bit_cast(bf16x8, hi), tb, w[t]);
           w[t] = mfma16(__builtin_bit_cast(bf16x8, lo), tb, w[t]);
         }
       }
-      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's V image has landed
+      if (kn < ce) {  // the next chunk's scores are in flight while this one's values are multiplied
+        load_scores(kn);
+        asm volatile("s_waitcnt vmcnt(%0)" ::"n"(8 * NT) : "memory");  // this wave's V image has landed
+      } else {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      }
       __builtin_amdgcn_wave_barrier();
 #pragma unroll
       for (int pp = 0; pp < NT / 2; ++pp) {
-        bf16x8 pb;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          pb[e] = (__bf16)w[2 * pp][e];
-          pb[4 + e] = (__bf16)w[2 * pp + 1][e];
-        }
+        const bf16x8 pb = __builtin_bit_cast(bf16x8, u32x4{pack2(w[2 * pp][0], w[2 * pp][1]), pack2(w[2 * pp][2], w[2 * pp][3]),
+                                                           pack2(w[2 * pp + 1][0], w[2 * pp + 1][1]),
+                                                           pack2(w[2 * pp + 1][2], w[2 * pp + 1][3])});
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) o[dt] = mfma16(v_frag<D>(vimg, 32 * pp, dt, lane), pb, o[dt]);
       }
       __builtin_amdgcn_s_waitcnt(0xc07f);  // the V image is read before the next chunk overwrites it
       __builtin_amdgcn_wave_barrier();
+      if (kn < ce) stage_v(kn);
     }
     __syncthreads();  // every wave is done with its V image (the merge buffer aliases it)
 #pragma unroll
@@ -542,7 +595,7 @@ __global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int to
       if (a.talk != nullptr) f = h < a.nq && gg < a.nq ? a.talk[h * a.nq + gg] : 0.f;
       k.talk[e] = f32_to_bf16(f);
     }
-  const int unit = blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int unit = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   if (unit >= total) return;
   const int c = unit % a.nkv;
   const TileIdx x = tile_idx(a, k, unit / a.nkv);
@@ -565,53 +618,68 @@ __global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int to
       for (int ks = 0; ks < KS; ++ks) qb[hh][ks] = frag(qp + 32 * ks);
       m[hh] = -INFINITY;
       l[hh] = 0.f;
-      r1[hh] = a.r1 != nullptr ? a.r1[h] : 0.f;
+      r1[hh] = a.r1 != nullptr ? a.r1[h] * (-1.f / sc2) : 0.f;  // bias in units of the raw product
       r2[hh] = a.r1 != nullptr ? a.r2[h] : 0.f;
     }
-    for (int n = 0; n < kt.n; ++n) {
-      const int k0 = key0(kt, n);
-      const bool msk = needs_mask(a, x, k0);
-      const unsigned short* kp = kc + bt[k0 / a.bs] * a.k_block + ((int64_t)c * a.bs + k0 % a.bs + i) * D + 8 * g;
-      bf16x8 kr[2][KS];
+    bf16x8 kr[2][KS];
+    auto load_k = [&](int k0) {
+      const unsigned short* base =
+          uniform_ptr(kc + bt[k0 >> a.bs_shift] * a.k_block + ((c << a.bs_shift) + (k0 & (a.bs - 1))) * D);
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int ks = 0; ks < KS; ++ks) kr[t][ks] = frag(kp + 16 * t * D + 32 * ks);
+        for (int ks = 0; ks < KS; ++ks) kr[t][ks] = frag(base + (unsigned)(i * D + 8 * g + 16 * t * D + 32 * ks));
+    };
+    load_k(key0(kt, 0));
+    for (int n = 0; n < kt.n; ++n) {
+      const int k0 = key0(kt, n);
+      const bool msk = needs_mask(a, x, k0);
       const float dl = (float)max(0, x.p0 - k0 + 15 - lane);  // the distance whose bias this lane computes
+      f32x4 s[HB][2];
 #pragma unroll
       for (int hh = 0; hh < HB; ++hh) {
-        if (h0 + hh >= G) break;
-        f32x4 s[2];
+        const int tb = __builtin_bit_cast(int, r1[hh] * lg2(1.f + r2[hh] * dl));
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
-          s[t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-          for (int ks = 0; ks < KS; ++ks) s[t] = mfma16(kr[t][ks], qb[hh][ks], s[t]);
+          for (int e = 0; e < 4; ++e)
+            s[hh][t][e] = __builtin_bit_cast(float, __builtin_amdgcn_ds_bpermute(bidx + 4 * (16 * t + e), tb));
+#pragma unroll
+          for (int ks = 0; ks < KS; ++ks) s[hh][t] = mfma16(kr[t][ks], qb[hh][ks], s[hh][t]);
         }
-        const int tb = __builtin_bit_cast(int, r1[hh] * lg2(1.f + r2[hh] * dl));
-        float mx = -INFINITY;
+      }
+      load_k(key0(kt, min(n + 1, kt.n - 1)));
+      if (msk) {
 #pragma unroll
         for (int t = 0; t < 2; ++t)
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
-            s[t][e] = s[t][e] * sc2 - __builtin_bit_cast(float, __builtin_amdgcn_ds_bpermute(bidx + 4 * (16 * t + e), tb));
-            if (msk && !sees(a, x.p0 + i, k0 + 16 * t + 4 * g + e)) s[t][e] = -INFINITY;
-            mx = fmaxf(mx, s[t][e]);
+            const bool vis = sees(a, x.p0 + i, k0 + 16 * t + 4 * g + e);
+#pragma unroll
+            for (int hh = 0; hh < HB; ++hh) s[hh][t][e] = vis ? s[hh][t][e] : -INFINITY;
           }
-        const float mn = fmaxf(m[hh], mx), mr = mn == -INFINITY ? 0.f : mn;
-        float ls = 0.f;
+      }
+#pragma unroll
+      for (int hh = 0; hh < HB; ++hh) {  // max and sum of raw products + bias (scale > 0: the order is the scores')
+        float mx = m[hh];
 #pragma unroll
         for (int t = 0; t < 2; ++t)
 #pragma unroll
-          for (int e = 0; e < 4; ++e) ls += ex2(s[t][e] - mr);
-        l[hh] = l[hh] * ex2(m[hh] - mr) + ls;
-        m[hh] = mn;
+          for (int e = 0; e < 4; ++e) mx = fmaxf(mx, s[hh][t][e]);
+        const float mr = mx == -INFINITY ? 0.f : mx * sc2;
+        float ls = l[hh] * ex2(m[hh] * sc2 - mr);
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) ls += ex2(s[hh][t][e] * sc2 - mr);
+        l[hh] = ls;
+        m[hh] = mx;
       }
     }
 #pragma unroll
     for (int hh = 0; hh < HB; ++hh) {
       if (h0 + hh >= G) break;
-      float M = m[hh], L = l[hh];
+      float M = m[hh] * sc2, L = l[hh];
 #pragma unroll
       for (int o = 16; o < 64; o <<= 1) {
         const float m2 = __shfl_xor(M, o, 64), l2 = __shfl_xor(L, o, 64), mn = fmaxf(M, m2);
@@ -633,6 +701,7 @@ __global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int to
 template <int D, int HPW, bool ONE_KV>
 __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, TileArgs k, int total) {
   constexpr int KS = D / 32, DT = D / 16, PB = 16 * kTileKeys * kTileHeads * 2, VIMG = kTileKeys * 2 * D;
+  constexpr int NP = (HPW + 1) / 2;  // bf16 pairs of heads
   extern __shared__ __attribute__((aligned(16))) char smem[];
   char *phi = smem, *plo = smem + PB, *wbuf = smem + 2 * PB;
   // consecutive tiles of a sequence share most of their window: keep them on one XCD's L2
@@ -649,11 +718,12 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
   const int hw = wave * HPW;  // first head of this wave
   const int nh = min(HPW, a.nq - hw);
   const int tok = min(i, x.ntok - 1);
-  const float sc2 = a.scale * kLog2e;
+  const float sc2 = a.scale * kLog2e, nsc = -1.f / sc2;
   // heads past nq are never written by a wave: their weights stay zero
   for (int e = threadIdx.x; e < 2 * PB / 16; e += kTileWaves * 64) reinterpret_cast<u32x4*>(smem)[e] = u32x4{0u, 0u, 0u, 0u};
-  bf16x8 qb[HPW][KS];
+  bf16x8 qb[HPW][KS], tb[2];
   float lse[HPW];
+  int kvh[HPW];
   f32x4 o[HPW][DT];
 #pragma unroll
   for (int hh = 0; hh < HPW; ++hh) {
@@ -662,125 +732,136 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) qb[hh][ks] = frag(qp + 32 * ks);
     lse[hh] = k.lse[(x.t0 + tok) * a.nq + h];
+    kvh[hh] = __builtin_amdgcn_readfirstlane(h / G);
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) o[hh][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
+#pragma unroll
+  for (int nn = 0; nn < 2; ++nn) tb[nn] = frag(k.talk + (nn * 64 + lane_) * 8);
   const int nmix = a.nq > 16 ? 2 : 1;
-  __syncthreads();
+  bf16x8 kr[KS];
 
+  // K fragments of half t (16 keys) of the tile at key k0, kv head c
+  auto load_k = [&](int lane, int c, int k0, int t) {
+    const unsigned short* base =
+        uniform_ptr(kc + bt[k0 >> a.bs_shift] * a.k_block + ((c << a.bs_shift) + (k0 & (a.bs - 1)) + 16 * t) * D);
+    const unsigned off = (lane & 15) * D + 8 * (lane >> 4);
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) kr[ks] = frag(base + off + 32 * ks);
+  };
+  // V rows of the tile at key k0, kv head c -> this wave's image
   auto stage_v = [&](int lane, int c, int k0) {
     constexpr int CH = D / 8, RPK = 64 / CH;
-    const unsigned short* vp = vc + bt[k0 / a.bs] * a.v_block + ((int64_t)c * a.bs + k0 % a.bs) * D;
+    const unsigned short* base =
+        uniform_ptr(vc + bt[k0 >> a.bs_shift] * a.v_block + ((c << a.bs_shift) + (k0 & (a.bs - 1))) * D);
+    const unsigned dst = lds_at(vimg);
 #pragma unroll
     for (int n = 0; n < kTileKeys / RPK; ++n) {
       const int rw = RPK * n + lane / CH, ch = (lane % CH) ^ chunk_xor<D>(rw);
-      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(vp + rw * D + ch * 8),
-                                       (__attribute__((address_space(3))) void*)(vimg + n * 1024), 16, 0, 0);
+      dma16(dst + n * 1024, base, (rw * D + ch * 8) * 2);
+    }
+  };
+  // the weights of this wave's heads over one tile, to LDS; K of the tile's first half is in kr
+  auto weights = [&](int n) {
+    const int lane = opaque(lane_), g = lane >> 4, i = lane & 15;
+    const int k0 = key0(kt, n), k1 = key0(kt, min(n + 1, kt.n - 1));
+    const bool msk = needs_mask(a, x, k0);
+    const float dl = (float)max(0, x.p0 - k0 + 15 - lane);  // the distance whose bias this lane computes
+    int tbl[HPW];
+#pragma unroll
+    for (int hh = 0; hh < HPW; ++hh) {
+      const int h = min(hw + hh, a.nq - 1);
+      tbl[hh] = a.r1 != nullptr ? __builtin_bit_cast(int, a.r1[h] * nsc * lg2(1.f + a.r2[h] * dl)) : 0;
+    }
+    const int bx = 4 * (4 * g - i + 15), at0 = i * (kTileKeys * 2 * kTileHeads) + 16 * (((2 * hw) >> 4) ^ ((i >> 2) & 3)) + ((2 * hw) & 15);
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      f32x4 sc[HPW];  // starts from the bias (in units of the raw product), then + q . k
+#pragma unroll
+      for (int hh = 0; hh < HPW; ++hh)
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          sc[hh][e] = __builtin_bit_cast(float, __builtin_amdgcn_ds_bpermute(bx + 4 * (16 * t + e), tbl[hh]));
+#pragma unroll
+      for (int hh = 0; hh < HPW; ++hh) {
+        if constexpr (!ONE_KV)
+          if (hh > 0 && kvh[hh] != kvh[hh - 1]) load_k(lane, kvh[hh], k0, t);
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) sc[hh] = mfma16(kr[ks], qb[hh][ks], sc[hh]);
+      }
+      if (t == 0) {
+        stage_v(lane, kvh[0], k0);
+        load_k(lane, kvh[0], k0, 1);
+      } else {
+        load_k(lane, kvh[0], k1, 0);  // the next tile's first half, in flight across mix and value product
+      }
+      if (msk) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const bool vis = sees(a, x.p0 + i, k0 + 16 * t + 4 * g + e);
+#pragma unroll
+          for (int hh = 0; hh < HPW; ++hh) sc[hh][e] = vis ? sc[hh][e] : -INFINITY;
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        unsigned ph[NP], pl[NP];
+#pragma unroll
+        for (int hp = 0; hp < NP; ++hp) {
+          const float p0 = ex2(sc[2 * hp][e] * sc2 - lse[2 * hp]);
+          float p1 = 0.f;
+          if constexpr (HPW > 1) p1 = ex2(sc[2 * hp + 1][e] * sc2 - lse[2 * hp + 1]);
+          if constexpr (!ONE_KV && HPW > 1) p1 = 2 * hp + 1 < nh ? p1 : 0.f;
+          ph[hp] = pack2(p0, p1);
+          pl[hp] = pack2(p0 - __uint_as_float(ph[hp] << 16), p1 - __uint_as_float(ph[hp] & 0xffff0000u));
+          if constexpr (!ONE_KV)
+            if (2 * hp >= nh) ph[hp] = pl[hp] = 0u;
+        }
+        const int at = at0 + ((16 * t + 4 * g + (e ^ (i & 3))) * (2 * kTileHeads));
+        if constexpr (HPW == 4) {
+          *reinterpret_cast<uint2*>(phi + at) = uint2{ph[0], ph[1]};
+          *reinterpret_cast<uint2*>(plo + at) = uint2{pl[0], pl[1]};
+        } else if constexpr (HPW == 2) {
+          *reinterpret_cast<unsigned*>(phi + at) = ph[0];
+          *reinterpret_cast<unsigned*>(plo + at) = pl[0];
+        } else {
+          *reinterpret_cast<unsigned short*>(phi + at) = (unsigned short)ph[0];
+          *reinterpret_cast<unsigned short*>(plo + at) = (unsigned short)pl[0];
+        }
+      }
     }
   };
 
+  if (nh > 0) load_k(lane_, kvh[0], key0(kt, 0), 0);
+  lds_barrier();  // the zeroed weights
+  if (nh > 0) weights(0);
   for (int n = 0; n < kt.n; ++n) {
-    const int k0 = key0(kt, n);
-    // LDS and cache addresses are recomputed from the lane in every phase: kept across the loop they
-    // would not fit the registers beside the accumulators and the queries
-    if (nh > 0) {
-      const int lane = opaque(lane_), g = lane >> 4, i = lane & 15;
-      const bool msk = needs_mask(a, x, k0);
-      __builtin_amdgcn_s_waitcnt(0xc07f);  // the previous tile's V reads are done
-      stage_v(lane, hw / G, k0);
-      const float dl = (float)max(0, x.p0 - k0 + 15 - lane);
-      int tbl[HPW];
-#pragma unroll
-      for (int hh = 0; hh < HPW; ++hh) {
-        const int h = min(hw + hh, a.nq - 1);
-        tbl[hh] = a.r1 != nullptr ? __builtin_bit_cast(int, a.r1[h] * lg2(1.f + a.r2[h] * dl)) : 0;
-      }
-      const unsigned short* kp = kc + bt[k0 / a.bs] * a.k_block + ((int64_t)k0 % a.bs + i) * D + 8 * g;
-#pragma unroll 1
-      for (int t = 0; t < 2; ++t) {
-        bf16x8 kr[KS];
-        unsigned ph[4][HPW == 4 ? 2 : 1], pl[4][HPW == 4 ? 2 : 1];  // bf16 pairs of neighbouring heads
-        const int bx = 4 * (4 * g - i + 15) + 64 * t;
-        auto load_k = [&](int c) {
-          const unsigned short* p = kp + ((int64_t)c * a.bs + 16 * t) * D;
-#pragma unroll
-          for (int ks = 0; ks < KS; ++ks) kr[ks] = frag(p + 32 * ks);
-        };
-        if constexpr (ONE_KV) load_k(hw / G);
-#pragma unroll
-        for (int hp = 0; hp < (HPW + 1) / 2; ++hp) {
-          float v[2][4];
-#pragma unroll
-          for (int u = 0; u < (HPW == 1 ? 1 : 2); ++u) {
-            const int hh = 2 * hp + u;
-            if constexpr (!ONE_KV) {
-              const int h = min(hw + hh, a.nq - 1);
-              if (hh == 0 || h / G != (h - 1) / G) load_k(h / G);
-            }
-            f32x4 sc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int ks = 0; ks < KS; ++ks) sc = mfma16(kr[ks], qb[hh][ks], sc);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-              v[u][e] = sc[e] * sc2 - __builtin_bit_cast(float, __builtin_amdgcn_ds_bpermute(bx + 4 * e, tbl[hh])) - lse[hh];
-              if (msk && !sees(a, x.p0 + i, k0 + 16 * t + 4 * g + e)) v[u][e] = -INFINITY;
-            }
-            if (!ONE_KV && hh >= nh)
-#pragma unroll
-              for (int e = 0; e < 4; ++e) v[u][e] = -INFINITY;
-          }
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            const float p0 = ex2(v[0][e]), p1 = HPW == 1 ? 0.f : ex2(v[1][e]);
-            const unsigned h2 = pack2(p0, p1);
-            ph[e][hp] = h2;
-            pl[e][hp] = pack2(p0 - __uint_as_float(h2 << 16), p1 - __uint_as_float(h2 & 0xffff0000u));
-          }
-        }
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const int key = 16 * t + 4 * g + e, b = 2 * hw;
-          const int at = (i * kTileKeys + (key ^ (i & 3))) * (2 * kTileHeads) + 16 * ((b >> 4) ^ ((i >> 2) & 3)) + (b & 15);
-          if constexpr (HPW == 4) {
-            *reinterpret_cast<uint2*>(phi + at) = uint2{ph[e][0], ph[e][1]};
-            *reinterpret_cast<uint2*>(plo + at) = uint2{pl[e][0], pl[e][1]};
-          } else if constexpr (HPW == 2) {
-            *reinterpret_cast<unsigned*>(phi + at) = ph[e][0];
-            *reinterpret_cast<unsigned*>(plo + at) = pl[e][0];
-          } else {
-            *reinterpret_cast<unsigned short*>(phi + at) = (unsigned short)ph[e][0];
-            *reinterpret_cast<unsigned short*>(plo + at) = (unsigned short)pl[e][0];
-          }
-        }
-      }
-    }
-    bf16x8 tb[2];
-#pragma unroll
-    for (int nn = 0; nn < 2; ++nn) tb[nn] = frag(k.talk + (nn * 64 + lane_) * 8);
-    __syncthreads();
+    lds_barrier();
     // ---- mix: this wave's tokens 2 wave, 2 wave + 1, both 16-key halves ------------------------------
-    const int lm = opaque(lane_);
+    {
+      const int lane = opaque(lane_), g = lane >> 4, i = lane & 15;
+      // lane: head h = i (+ 16), keys 16 t + 4 g .. + 3 of token q -> chunk of the lane group that reads those rows of V
+      const int ch = ((g & 1) << 1) | (g >> 1), wt0 = i * (16 * 2 * kTileKeys) + 16 * (ch ^ ((i >> 2) & 3));
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int g = lm >> 4, i = lm & 15;
-      const int q = 2 * wave + (u >> 1), t = u & 1, key = 16 * t + i;
-      const int at = (q * kTileKeys + (key ^ (q & 3))) * (2 * kTileHeads) + 16 * (g ^ ((q >> 2) & 3));
-      const bf16x8 hi = *reinterpret_cast<const bf16x8*>(phi + at), lo = *reinterpret_cast<const bf16x8*>(plo + at);
+      for (int u = 0; u < 4; ++u) {
+        const int q = 2 * wave + (u >> 1), t = u & 1;
+        const int at = (q * kTileKeys + 16 * t + (i ^ (q & 3))) * (2 * kTileHeads) + 16 * (g ^ ((q >> 2) & 3));
+        const bf16x8 hi = *reinterpret_cast<const bf16x8*>(phi + at), lo = *reinterpret_cast<const bf16x8*>(plo + at);
 #pragma unroll
-      for (int nn = 0; nn < 2; ++nn) {
-        if (nn >= nmix) break;
-        f32x4 w = {0.f, 0.f, 0.f, 0.f};
-        w = mfma16(hi, tb[nn], w);
-        w = mfma16(lo, tb[nn], w);
-        // lane: head h, keys 16 t + 4 g .. + 3 of token q -> chunk of the lane group that reads those rows of V
-        const int h = 16 * nn + i, ch = ((g & 1) << 1) | (g >> 1);
-        const int wt = (h * 16 + (q ^ (h & 3))) * (2 * kTileKeys) + 16 * (ch ^ ((h >> 2) & 3)) + 8 * t;
-        *reinterpret_cast<u16x4*>(wbuf + wt) = u16x4{f32_to_bf16(w[0]), f32_to_bf16(w[1]), f32_to_bf16(w[2]), f32_to_bf16(w[3])};
+        for (int nn = 0; nn < 2; ++nn) {
+          if (nn >= nmix) break;
+          f32x4 w = {0.f, 0.f, 0.f, 0.f};
+          w = mfma16(hi, tb[nn], w);
+          w = mfma16(lo, tb[nn], w);
+          const int wt = wt0 + nn * (16 * 16 * 2 * kTileKeys) + (q ^ (i & 3)) * (2 * kTileKeys) + 8 * t;
+          *reinterpret_cast<uint2*>(wbuf + wt) = uint2{pack2(w[0], w[1]), pack2(w[2], w[3])};
+        }
       }
     }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // V image
-    __syncthreads();
-    // ---- O^T += V^T W^T ------------------------------------------------------------------------------
+    // the V image: older than the K fragments in flight for the next tile
+    asm volatile("s_waitcnt vmcnt(%0)" ::"n"(KS) : "memory");
+    lds_barrier();
+    // ---- O^T += V^T W^T, then the next tile's weights ------------------------------------------------
     if (nh > 0) {
       const int lane = opaque(lane_), g = lane >> 4, i = lane & 15;
       bf16x8 wf[HPW];
@@ -800,19 +881,20 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
 #pragma unroll
         for (int hh = 0; hh < HPW; ++hh) {  // the wave's heads span several kv heads: stage each V in turn
           if (hh >= nh) break;
-          const int h = hw + hh;
-          if (hh > 0 && h / G != (h - 1) / G) {
-            __builtin_amdgcn_s_waitcnt(0xc07f);
-            stage_v(lane, h / G, k0);
+          if (hh > 0 && kvh[hh] != kvh[hh - 1]) {
+            __builtin_amdgcn_s_waitcnt(0xc07f);  // the image has been read
+            stage_v(lane, kvh[hh], key0(kt, n));
             asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-            __builtin_amdgcn_wave_barrier();
           }
 #pragma unroll
           for (int dt = 0; dt < DT; ++dt) o[hh][dt] = mfma16(v_frag<D>(vimg, 0, dt, lane), wf[hh], o[hh][dt]);
         }
       }
+      __builtin_amdgcn_s_waitcnt(0xc07f);  // V and W reads are done before the image is refilled
+      if (n + 1 < kt.n) weights(n + 1);
     }
   }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
   if (i >= x.ntok) return;
   const int64_t t = x.t0 + i;
   unsigned short* out = static_cast<unsigned short*>(a.out) + t * a.nq * a.dv;
@@ -975,6 +1057,7 @@ at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Te
   a.Dk = kc.size(3);
   a.Dv = vc.size(3);
   a.bs = kc.size(2);
+  while ((1 << a.bs_shift) < a.bs) ++a.bs_shift;
   a.scale = (float)scale;
   a.window = (int)std::max<int64_t>(0, window);
   a.keep_first = (int)std::max<int64_t>(0, keep_first);
@@ -994,10 +1077,11 @@ at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Te
   c10::DeviceGuard g(q.device());
   const int64_t D = kc.size(3);
   const bool mfma = q.scalar_type() == at::kBFloat16 && D == vc.size(3) && (D == 64 || D == 128 || D == 256) &&
-                    nq <= ma::kMaxHeads && kc.stride(0) % 8 == 0 && vc.stride(0) % 8 == 0 &&
+                    nq <= ma::kMaxHeads && (1 << a.bs_shift) == a.bs && scale > 0 &&
+                    kc.stride(0) % 8 == 0 && vc.stride(0) % 8 == 0 &&
                     reinterpret_cast<uintptr_t>(a.kc) % 16 == 0 && reinterpret_cast<uintptr_t>(a.vc) % 16 == 0;
   const bool tile_ok = mfma && nq <= ma::kTileHeads && D <= 128 && a.bs % ma::kTileKeys == 0;
-  SXE_CHECK(form != 2 || mfma, "mix_attention: token form needs bf16 rows of 64, 128 or 256");
+  SXE_CHECK(form != 2 || mfma, "mix_attention: token form needs bf16 rows of 64, 128 or 256, a scale > 0 and a power-of-two block size");
   SXE_CHECK(form != 3 || tile_ok, "mix_attention: tile form needs bf16 rows of 64 or 128, <= 32 heads, blocks of 32 n");
   if (mfma && form != 1) {
     constexpr int64_t kTileMin = 8;  // shorter runs of new tokens go token by token

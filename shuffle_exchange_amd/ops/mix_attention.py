@@ -40,7 +40,7 @@ def mix_attention(q, kc, vc, batch, dk, dv, scale, params, window=None, keep_fir
     memory; "tile" 16 tokens x all heads)."""
     if native.use_hip(q):
         visible = batch.max_kv_len if not window else min(batch.max_kv_len, window + keep_first)
-        splits = choose_splits(batch.num_seqs, kc.shape[1], visible, min_keys=64)
+        splits = choose_splits(batch.num_seqs, kc.shape[1], visible)
         return torch.ops.sxe.mix_attention(q, kc, vc, batch.block_table, batch.q_start, batch.q_len, batch.kv_len,
                                            min(batch.host_q_len), max(batch.host_q_len), int(batch.max_kv_len), splits,
                                            int(dk), int(dv), float(scale), int(window or 0), int(keep_first), params.r1,
