@@ -549,15 +549,20 @@ struct TileIdx {
   int64_t t0;
   bool ok;
 };
+// wave-uniform values that the compiler would otherwise keep in vector registers
+__device__ __forceinline__ int uni(int v) { return __builtin_amdgcn_readfirstlane(v); }
+__device__ __forceinline__ float uni(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_readfirstlane(__builtin_bit_cast(int, v)));
+}
 __device__ __forceinline__ TileIdx tile_idx(const Args& a, const TileArgs& k, int id) {
   TileIdx x;
-  x.seq = id / k.tiles;
-  const int tok = (id - x.seq * k.tiles) * 16, ql = x.seq < a.S ? a.q_len[x.seq] : 0;
+  x.seq = uni(id / k.tiles);
+  const int tok = (id - x.seq * k.tiles) * 16, ql = x.seq < a.S ? uni(a.q_len[x.seq]) : 0;
   x.ok = tok < ql && ql >= k.min_len;
   if (!x.ok) return x;
-  x.p0 = a.kv_len[x.seq] - ql + tok;
+  x.p0 = uni(a.kv_len[x.seq]) - ql + tok;
   x.ntok = min(16, ql - tok);
-  x.t0 = a.q_start[x.seq] + tok;
+  x.t0 = uni(a.q_start[x.seq]) + tok;
   return x;
 }
 
@@ -595,9 +600,9 @@ __global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int to
       if (a.talk != nullptr) f = h < a.nq && gg < a.nq ? a.talk[h * a.nq + gg] : 0.f;
       k.talk[e] = f32_to_bf16(f);
     }
-  const int unit = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int unit = blockIdx.x * 4 + uni((int)threadIdx.x >> 6);
   if (unit >= total) return;
-  const int c = unit % a.nkv;
+  const int c = uni(unit % a.nkv);
   const TileIdx x = tile_idx(a, k, unit / a.nkv);
   if (!x.ok) return;
   const int lane = threadIdx.x & 63, g = lane >> 4, i = lane & 15, G = a.nq / a.nkv;
@@ -701,7 +706,8 @@ __global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int to
 template <int D, int HPW, bool ONE_KV>
 __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, TileArgs k, int total) {
   constexpr int KS = D / 32, DT = D / 16, PB = 16 * kTileKeys * kTileHeads * 2, VIMG = kTileKeys * 2 * D;
-  constexpr int NP = (HPW + 1) / 2;  // bf16 pairs of heads
+  constexpr int NP = (HPW + 1) / 2;       // bf16 pairs of heads
+  constexpr int NMIX = HPW == 4 ? 2 : 1;  // 16-head tiles of the mix
   extern __shared__ __attribute__((aligned(16))) char smem[];
   char *phi = smem, *plo = smem + PB, *wbuf = smem + 2 * PB;
   // consecutive tiles of a sequence share most of their window: keep them on one XCD's L2
@@ -709,7 +715,7 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
   if (id >= total) return;
   const TileIdx x = tile_idx(a, k, id);
   if (!x.ok) return;
-  const int lane_ = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), G = a.nq / a.nkv;
+  const int lane_ = threadIdx.x & 63, wave = uni((int)threadIdx.x >> 6), G = uni(a.nq / a.nkv);
   const int g = lane_ >> 4, i = lane_ & 15;
   char* vimg = smem + 3 * PB + wave * VIMG;
   const KeyTiles kt = key_tiles(a, x);
@@ -721,8 +727,8 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
   const float sc2 = a.scale * kLog2e, nsc = -1.f / sc2;
   // heads past nq are never written by a wave: their weights stay zero
   for (int e = threadIdx.x; e < 2 * PB / 16; e += kTileWaves * 64) reinterpret_cast<u32x4*>(smem)[e] = u32x4{0u, 0u, 0u, 0u};
-  bf16x8 qb[HPW][KS], tb[2];
-  float lse[HPW];
+  bf16x8 qb[HPW][KS];
+  float lse[HPW], r1[HPW], r2[HPW];
   int kvh[HPW];
   f32x4 o[HPW][DT];
 #pragma unroll
@@ -732,48 +738,52 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) qb[hh][ks] = frag(qp + 32 * ks);
     lse[hh] = k.lse[(x.t0 + tok) * a.nq + h];
-    kvh[hh] = __builtin_amdgcn_readfirstlane(h / G);
+    kvh[hh] = uni(h / G);
+    r1[hh] = a.r1 != nullptr ? uni(a.r1[h]) * nsc : 0.f;  // bias in units of the raw product
+    r2[hh] = a.r1 != nullptr ? uni(a.r2[h]) : 0.f;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) o[hh][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
-#pragma unroll
-  for (int nn = 0; nn < 2; ++nn) tb[nn] = frag(k.talk + (nn * 64 + lane_) * 8);
-  const int nmix = a.nq > 16 ? 2 : 1;
   bf16x8 kr[KS];
 
-  // K fragments of half t (16 keys) of the tile at key k0, kv head c
-  auto load_k = [&](int lane, int c, int k0, int t) {
+  // block ids of 64 tiles, one a lane (a load per tile would wait behind the image in flight)
+  int blocks = 0;
+  auto fetch_blocks = [&](int n) { blocks = bt[key0(kt, min(n + lane_, kt.n - 1)) >> a.bs_shift]; };
+  auto row_of = [&](int n, int c) {  // element offset / D inside its block of the tile's first key, kv head c
+    return (c << a.bs_shift) + (key0(kt, n) & (a.bs - 1));
+  };
+  // K fragments of half t (16 keys) of tile n, kv head c
+  auto load_k = [&](int lane, int c, int n, int t) {
     const unsigned short* base =
-        uniform_ptr(kc + bt[k0 >> a.bs_shift] * a.k_block + ((c << a.bs_shift) + (k0 & (a.bs - 1)) + 16 * t) * D);
+        kc + (int64_t)__builtin_amdgcn_readlane(blocks, n & 63) * a.k_block + (row_of(n, c) + 16 * t) * D;
     const unsigned off = (lane & 15) * D + 8 * (lane >> 4);
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) kr[ks] = frag(base + off + 32 * ks);
   };
-  // V rows of the tile at key k0, kv head c -> this wave's image
-  auto stage_v = [&](int lane, int c, int k0) {
+  // V rows of tile n, kv head c -> this wave's image
+  auto stage_v = [&](int lane, int c, int n) {
     constexpr int CH = D / 8, RPK = 64 / CH;
-    const unsigned short* base =
-        uniform_ptr(vc + bt[k0 >> a.bs_shift] * a.v_block + ((c << a.bs_shift) + (k0 & (a.bs - 1))) * D);
-    const unsigned dst = lds_at(vimg);
+    const unsigned short* base = vc + (int64_t)__builtin_amdgcn_readlane(blocks, n & 63) * a.v_block + row_of(n, c) * D;
+    const unsigned dst = lds_at(vimg), off = (lane / CH) * 2 * D + 16 * ((lane % CH) ^ chunk_xor<D>(lane / CH));
 #pragma unroll
-    for (int n = 0; n < kTileKeys / RPK; ++n) {
-      const int rw = RPK * n + lane / CH, ch = (lane % CH) ^ chunk_xor<D>(rw);
-      dma16(dst + n * 1024, base, (rw * D + ch * 8) * 2);
-    }
+    for (int j = 0; j < kTileKeys / RPK; ++j)  // the swizzles of lane / CH and of RPK j are disjoint bits
+      dma16(dst + j * 1024, base + j * 512, off ^ (16 * chunk_xor<D>(RPK * j)));
   };
   // the weights of this wave's heads over one tile, to LDS; K of the tile's first half is in kr
   auto weights = [&](int n) {
     const int lane = opaque(lane_), g = lane >> 4, i = lane & 15;
-    const int k0 = key0(kt, n), k1 = key0(kt, min(n + 1, kt.n - 1));
+    const int k0 = key0(kt, n);
     const bool msk = needs_mask(a, x, k0);
+    __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0): K of the first half
+    stage_v(lane, kvh[0], n);
     const float dl = (float)max(0, x.p0 - k0 + 15 - lane);  // the distance whose bias this lane computes
     int tbl[HPW];
 #pragma unroll
-    for (int hh = 0; hh < HPW; ++hh) {
-      const int h = min(hw + hh, a.nq - 1);
-      tbl[hh] = a.r1 != nullptr ? __builtin_bit_cast(int, a.r1[h] * nsc * lg2(1.f + a.r2[h] * dl)) : 0;
-    }
-    const int bx = 4 * (4 * g - i + 15), at0 = i * (kTileKeys * 2 * kTileHeads) + 16 * (((2 * hw) >> 4) ^ ((i >> 2) & 3)) + ((2 * hw) & 15);
+    for (int hh = 0; hh < HPW; ++hh) tbl[hh] = __builtin_bit_cast(int, r1[hh] * lg2(1.f + r2[hh] * dl));
+    const int bx = 4 * (4 * g - i + 15);
+    // row (token i, key 16 t + 4 g + (e ^ i & 3)), chunk of this wave's heads
+    const int at0 = i * (kTileKeys * 2 * kTileHeads) + (4 * g + (i & 3)) * (2 * kTileHeads) +
+                    16 * (((2 * hw) >> 4) ^ ((i >> 2) & 3)) + ((2 * hw) & 15);
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
       f32x4 sc[HPW];  // starts from the bias (in units of the raw product), then + q . k
@@ -785,15 +795,15 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
 #pragma unroll
       for (int hh = 0; hh < HPW; ++hh) {
         if constexpr (!ONE_KV)
-          if (hh > 0 && kvh[hh] != kvh[hh - 1]) load_k(lane, kvh[hh], k0, t);
+          if (hh > 0 && kvh[hh] != kvh[hh - 1]) load_k(lane, kvh[hh], n, t);
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) sc[hh] = mfma16(kr[ks], qb[hh][ks], sc[hh]);
       }
       if (t == 0) {
-        stage_v(lane, kvh[0], k0);
-        load_k(lane, kvh[0], k0, 1);
-      } else {
-        load_k(lane, kvh[0], k1, 0);  // the next tile's first half, in flight across mix and value product
+        load_k(lane, kvh[0], n, 1);
+      } else {  // the next tile's first half, in flight across mix and value product
+        if (((n + 1) & 63) == 0) fetch_blocks(n + 1);
+        load_k(lane, kvh[0], min(n + 1, kt.n - 1), 0);
       }
       if (msk) {
 #pragma unroll
@@ -817,25 +827,31 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
           if constexpr (!ONE_KV)
             if (2 * hp >= nh) ph[hp] = pl[hp] = 0u;
         }
-        const int at = at0 + ((16 * t + 4 * g + (e ^ (i & 3))) * (2 * kTileHeads));
+        char* at = phi + (at0 ^ (e * 2 * kTileHeads)) + t * (16 * 2 * kTileHeads);
         if constexpr (HPW == 4) {
-          *reinterpret_cast<uint2*>(phi + at) = uint2{ph[0], ph[1]};
-          *reinterpret_cast<uint2*>(plo + at) = uint2{pl[0], pl[1]};
+          *reinterpret_cast<uint2*>(at) = uint2{ph[0], ph[1]};
+          *reinterpret_cast<uint2*>(at + PB) = uint2{pl[0], pl[1]};
         } else if constexpr (HPW == 2) {
-          *reinterpret_cast<unsigned*>(phi + at) = ph[0];
-          *reinterpret_cast<unsigned*>(plo + at) = pl[0];
+          *reinterpret_cast<unsigned*>(at) = ph[0];
+          *reinterpret_cast<unsigned*>(at + PB) = pl[0];
         } else {
-          *reinterpret_cast<unsigned short*>(phi + at) = (unsigned short)ph[0];
-          *reinterpret_cast<unsigned short*>(plo + at) = (unsigned short)pl[0];
+          *reinterpret_cast<unsigned short*>(at) = (unsigned short)ph[0];
+          *reinterpret_cast<unsigned short*>(at + PB) = (unsigned short)pl[0];
         }
       }
     }
   };
 
-  if (nh > 0) load_k(lane_, kvh[0], key0(kt, 0), 0);
+  if (nh > 0) {
+    fetch_blocks(0);
+    load_k(lane_, kvh[0], 0, 0);
+  }
   lds_barrier();  // the zeroed weights
   if (nh > 0) weights(0);
   for (int n = 0; n < kt.n; ++n) {
+    bf16x8 tb[NMIX];  // read again for every tile: registers that the weights need
+#pragma unroll
+    for (int nn = 0; nn < NMIX; ++nn) tb[nn] = frag(k.talk + (nn * 64 + opaque(lane_)) * 8);
     lds_barrier();
     // ---- mix: this wave's tokens 2 wave, 2 wave + 1, both 16-key halves ------------------------------
     {
@@ -845,11 +861,11 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
 #pragma unroll
       for (int u = 0; u < 4; ++u) {
         const int q = 2 * wave + (u >> 1), t = u & 1;
-        const int at = (q * kTileKeys + 16 * t + (i ^ (q & 3))) * (2 * kTileHeads) + 16 * (g ^ ((q >> 2) & 3));
+        const int at = ((i * (2 * kTileHeads) + 16 * g) ^ ((q & 3) * (2 * kTileHeads) + 16 * ((q >> 2) & 3))) +
+                       (q * kTileKeys + 16 * t) * (2 * kTileHeads);
         const bf16x8 hi = *reinterpret_cast<const bf16x8*>(phi + at), lo = *reinterpret_cast<const bf16x8*>(plo + at);
 #pragma unroll
-        for (int nn = 0; nn < 2; ++nn) {
-          if (nn >= nmix) break;
+        for (int nn = 0; nn < NMIX; ++nn) {
           f32x4 w = {0.f, 0.f, 0.f, 0.f};
           w = mfma16(hi, tb[nn], w);
           w = mfma16(lo, tb[nn], w);
@@ -883,7 +899,7 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
           if (hh >= nh) break;
           if (hh > 0 && kvh[hh] != kvh[hh - 1]) {
             __builtin_amdgcn_s_waitcnt(0xc07f);  // the image has been read
-            stage_v(lane, kvh[hh], key0(kt, n));
+            stage_v(lane, kvh[hh], n);
             asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
           }
 #pragma unroll
