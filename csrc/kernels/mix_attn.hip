@@ -229,7 +229,7 @@ struct TokArgs {
   float* ml;      // [splits, rows, nq, 2]
   float* part;    // [splits, rows, nq, dv] (splits > 1)
   int nv, splits, keys_per_split;
-  int nt, tok0, max_len;  // rows = S * nt: tokens tok0 .. tok0 + nt - 1 of sequences with q_len <= max_len
+  int nt, tok0, min_len, max_len;  // rows = S * nt: tokens tok0 .. + nt - 1 of sequences of min_len .. max_len new ones
 };
 
 template <int D>
@@ -249,7 +249,7 @@ __device__ __forceinline__ TokRow tok_row(const Args& a, const TokArgs& k, int r
   TokRow r;
   r.seq = row / k.nt;
   const int tok = k.tok0 + row - r.seq * k.nt, ql = a.q_len[r.seq];
-  r.ok = tok < ql && ql <= k.max_len;
+  r.ok = tok < ql && ql >= k.min_len && ql <= k.max_len;
   r.pos = a.kv_len[r.seq] - ql + tok;
   r.t = a.q_start[r.seq] + tok;
   return r;
@@ -540,7 +540,9 @@ __global__ __launch_bounds__(256) void mix_reduce_kernel(Args a, TokArgs k) {
 struct TileArgs {
   float* lse;            // [T, nq]
   unsigned short* talk;  // [2][64][8] bf16: lane l's operand of the mix, T[16 n + (l & 15)][8 (l >> 4) .. + 7]
-  int min_len, tiles;  // sequences with q_len >= min_len; 16-token tiles per sequence
+  float* part;           // [splits, S * max_len, nq * dv] (splits > 1)
+  int min_len, max_len, tiles, splits;  // sequences with q_len >= min_len; 16-token tiles per sequence
+  int vec;               // gate and output rows allow 8-byte accesses
 };
 constexpr int kTileWaves = 8, kTileKeys = 32, kTileHeads = 32;
 
@@ -605,7 +607,7 @@ __global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int to
   const int c = uni(unit % a.nkv);
   const TileIdx x = tile_idx(a, k, unit / a.nkv);
   if (!x.ok) return;
-  const int lane = threadIdx.x & 63, g = lane >> 4, i = lane & 15, G = a.nq / a.nkv;
+  const int lane = threadIdx.x & 63, g = lane >> 4, i = lane & 15, G = uni(a.nq / a.nkv);
   const KeyTiles kt = key_tiles(a, x);
   const int* bt = a.block_table + (int64_t)x.seq * a.max_blocks;
   const unsigned short *kc = static_cast<const unsigned short*>(a.kc), *q = static_cast<const unsigned short*>(a.q);
@@ -623,19 +625,21 @@ __global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int to
       for (int ks = 0; ks < KS; ++ks) qb[hh][ks] = frag(qp + 32 * ks);
       m[hh] = -INFINITY;
       l[hh] = 0.f;
-      r1[hh] = a.r1 != nullptr ? a.r1[h] * (-1.f / sc2) : 0.f;  // bias in units of the raw product
-      r2[hh] = a.r1 != nullptr ? a.r2[h] : 0.f;
+      r1[hh] = a.r1 != nullptr ? uni(a.r1[h]) * (-1.f / sc2) : 0.f;  // bias in units of the raw product
+      r2[hh] = a.r1 != nullptr ? uni(a.r2[h]) : 0.f;
     }
     bf16x8 kr[2][KS];
-    auto load_k = [&](int k0) {
-      const unsigned short* base =
-          uniform_ptr(kc + bt[k0 >> a.bs_shift] * a.k_block + ((c << a.bs_shift) + (k0 & (a.bs - 1))) * D);
+    int blocks = 0;  // block ids of 64 tiles, one a lane
+    auto load_k = [&](int n) {
+      if ((n & 63) == 0) blocks = bt[key0(kt, min(n + lane, kt.n - 1)) >> a.bs_shift];
+      const unsigned short* base = kc + (int64_t)__builtin_amdgcn_readlane(blocks, n & 63) * a.k_block +
+                                   ((c << a.bs_shift) + (key0(kt, n) & (a.bs - 1))) * D;
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) kr[t][ks] = frag(base + (unsigned)(i * D + 8 * g + 16 * t * D + 32 * ks));
     };
-    load_k(key0(kt, 0));
+    load_k(0);
     for (int n = 0; n < kt.n; ++n) {
       const int k0 = key0(kt, n);
       const bool msk = needs_mask(a, x, k0);
@@ -653,7 +657,7 @@ __global__ __launch_bounds__(256) void mix_lse_kernel(Args a, TileArgs k, int to
           for (int ks = 0; ks < KS; ++ks) s[hh][t] = mfma16(kr[t][ks], qb[hh][ks], s[hh][t]);
         }
       }
-      load_k(key0(kt, min(n + 1, kt.n - 1)));
+      if (n + 1 < kt.n) load_k(n + 1);
       if (msk) {
 #pragma unroll
         for (int t = 0; t < 2; ++t)
@@ -842,13 +846,15 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
     }
   };
 
-  if (nh > 0) {
-    fetch_blocks(0);
-    load_k(lane_, kvh[0], 0, 0);
+  // a small batch splits the key tiles over workgroups: weights are normalised, so the splits' outputs add up
+  const int nb = kt.n * blockIdx.y / k.splits, ne = kt.n * (blockIdx.y + 1) / k.splits;
+  if (nh > 0 && nb < ne) {
+    fetch_blocks(nb & ~63);
+    load_k(lane_, kvh[0], nb, 0);
   }
   lds_barrier();  // the zeroed weights
-  if (nh > 0) weights(0);
-  for (int n = 0; n < kt.n; ++n) {
+  if (nh > 0 && nb < ne) weights(nb);
+  for (int n = nb; n < ne; ++n) {
     bf16x8 tb[NMIX];  // read again for every tile: registers that the weights need
 #pragma unroll
     for (int nn = 0; nn < NMIX; ++nn) tb[nn] = frag(k.talk + (nn * 64 + opaque(lane_)) * 8);
@@ -907,28 +913,56 @@ __global__ __launch_bounds__(kTileWaves * 64, 2) void mix_tile_kernel(Args a, Ti
         }
       }
       __builtin_amdgcn_s_waitcnt(0xc07f);  // V and W reads are done before the image is refilled
-      if (n + 1 < kt.n) weights(n + 1);
+      if (n + 1 < ne) weights(n + 1);
     }
   }
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
   if (i >= x.ntok) return;
-  const int64_t t = x.t0 + i;
-  unsigned short* out = static_cast<unsigned short*>(a.out) + t * a.nq * a.dv;
-  const unsigned short* gate = a.gate != nullptr ? static_cast<const unsigned short*>(a.gate) + t * a.gate_ld : nullptr;
+  const int64_t t = x.t0 + i, cols = (int64_t)a.nq * a.dv;
+  float* part = nullptr;
+  if (k.splits > 1)
+    part = k.part + ((int64_t)blockIdx.y * a.S * k.max_len + (int64_t)x.seq * k.max_len + (x.t0 + i - a.q_start[x.seq])) * cols;
+  unsigned short* out = static_cast<unsigned short*>(a.out) + t * cols;
+  const unsigned short* gate =
+      a.gate != nullptr && part == nullptr ? static_cast<const unsigned short*>(a.gate) + t * a.gate_ld : nullptr;
 #pragma unroll
   for (int hh = 0; hh < HPW; ++hh) {
     if (hh >= nh) break;
+    const int64_t col0 = (int64_t)(hw + hh) * a.dv + 4 * g;
+    u16x4 gv[DT];
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt)
+    for (int dt = 0; dt < DT; ++dt) {  // a head's gate values are all in flight before the first is used
+      const int d = 16 * dt + 4 * g;
+      gv[dt] = u16x4{0, 0, 0, 0};
+      if (gate == nullptr || d >= a.dv) continue;
+      if (k.vec) {
+        gv[dt] = *reinterpret_cast<const u16x4*>(gate + col0 + 16 * dt);
+      } else {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int d = 16 * dt + 4 * g + e;
-        if (d >= a.dv) continue;
-        const int64_t col = (int64_t)(hw + hh) * a.dv + d;
-        float v = o[hh][dt][e];
-        if (gate != nullptr) v /= 1.f + __expf(-bf16_to_f32(gate[col]));
-        out[col] = f32_to_bf16(v);
+        for (int e = 0; e < 4; ++e)
+          if (d + e < a.dv) gv[dt][e] = gate[col0 + 16 * dt + e];
       }
+    }
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      const int d = 16 * dt + 4 * g;
+      if (d >= a.dv) continue;
+      f32x4 v = o[hh][dt];
+      if (gate != nullptr)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] *= __builtin_amdgcn_rcpf(1.f + __expf(-bf16_to_f32(gv[dt][e])));
+      if (k.vec) {
+        if (part != nullptr) *reinterpret_cast<f32x4*>(part + col0 + 16 * dt) = v;
+        else *reinterpret_cast<uint2*>(out + col0 + 16 * dt) = uint2{pack2(v[0], v[1]), pack2(v[2], v[3])};
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          if (d + e >= a.dv) continue;
+          if (part != nullptr) part[col0 + 16 * dt + e] = v[e];
+          else out[col0 + 16 * dt + e] = f32_to_bf16(v[e]);
+        }
+      }
+    }
   }
 }
 
@@ -995,20 +1029,29 @@ void launch_tile_kernel(const ma::Args& a, const ma::TileArgs& k, int total) {
   constexpr size_t lds = 3 * 16 * ma::kTileKeys * ma::kTileHeads * 2 + ma::kTileWaves * ma::kTileKeys * 2 * D;
   auto go = [&](auto kern) {
     allow_lds(kern, lds);
-    hipLaunchKernelGGL(kern, dim3((total + 7) / 8 * 8), dim3(ma::kTileWaves * 64), lds, cur_stream(), a, k, total);
+    hipLaunchKernelGGL(kern, dim3((total + 7) / 8 * 8, k.splits), dim3(ma::kTileWaves * 64), lds, cur_stream(), a, k, total);
   };
   if (a.nq / a.nkv % HPW == 0) go(ma::mix_tile_kernel<D, HPW, true>);
   else go(ma::mix_tile_kernel<D, HPW, false>);
 }
 
-void launch_tiles(const ma::Args& a, const at::Tensor& q, int min_len, int max_q_len) {
+void launch_tiles(const ma::Args& a, const at::Tensor& q, int min_len, int max_q_len, int max_keys) {
   ma::TileArgs k{};
   auto lse = at::empty({(int64_t)a.T * a.nq}, q.options().dtype(at::kFloat)), talk = at::empty({1024}, q.options());
   k.lse = lse.data_ptr<float>();
   k.talk = static_cast<unsigned short*>(talk.data_ptr());
   k.min_len = min_len;
+  k.max_len = max_q_len;
   k.tiles = (max_q_len + 15) / 16;
   const int total = a.S * k.tiles, units = total * a.nkv;
+  k.vec = a.dv % 4 == 0 && a.gate_ld % 4 == 0 && reinterpret_cast<uintptr_t>(a.gate) % 8 == 0;
+  // one workgroup per compute unit: fewer tiles than units split their keys (while a split keeps 8 tiles of 32)
+  k.splits = std::max(1, std::min(std::min(4, kNumCUs / total), max_keys / (8 * ma::kTileKeys)));
+  at::Tensor part;
+  if (k.splits > 1) {
+    part = at::empty({(int64_t)k.splits * a.S * max_q_len * a.nq * a.dv}, q.options().dtype(at::kFloat));
+    k.part = part.data_ptr<float>();
+  }
   if (a.Dk == 64) hipLaunchKernelGGL(ma::mix_lse_kernel<64>, dim3((units + 3) / 4), dim3(256), 0, cur_stream(), a, k, units);
   else hipLaunchKernelGGL(ma::mix_lse_kernel<128>, dim3((units + 3) / 4), dim3(256), 0, cur_stream(), a, k, units);
   const int hpw = a.nq <= 8 ? 1 : a.nq <= 16 ? 2 : 4;
@@ -1021,6 +1064,16 @@ void launch_tiles(const ma::Args& a, const at::Tensor& q, int min_len, int max_q
   if (a.Dk == 64) SXE_MIX_TILE(64);
   else SXE_MIX_TILE(128);
 #undef SXE_MIX_TILE
+  if (k.splits > 1) {
+    ma::TokArgs r{};
+    r.part = k.part;
+    r.splits = k.splits;
+    r.nt = max_q_len;
+    r.min_len = min_len;
+    r.max_len = INT_MAX;
+    const int rows = a.S * max_q_len;
+    hipLaunchKernelGGL(ma::mix_reduce_kernel, dim3(rows, std::min(16, (a.nq * a.dv + 255) / 256)), dim3(256), 0, cur_stream(), a, r);
+  }
   SXE_LAUNCH_CHECK();
 }
 
@@ -1102,10 +1155,11 @@ at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Te
   if (mfma && form != 1) {
     constexpr int64_t kTileMin = 8;  // shorter runs of new tokens go token by token
     const int64_t tile_min = form == 2 || !tile_ok ? INT_MAX : form == 3 ? 1 : kTileMin;
-    if (max_q_len >= tile_min) launch_tiles(a, q, (int)tile_min, (int)max_q_len);
+    const int64_t keys = std::min<int64_t>(max_kv_len, a.window > 0 ? a.window + a.keep_first : max_kv_len);
+    if (max_q_len >= tile_min) launch_tiles(a, q, (int)tile_min, (int)max_q_len, (int)keys);
     if (min_q_len < tile_min) {
       // the scores of one launch stay within 256 MiB: long runs of tokens take several
-      const int64_t nv = (std::min<int64_t>(max_kv_len, a.window > 0 ? a.window + a.keep_first : max_kv_len) + 63) / 64 * 64;
+      const int64_t nv = (keys + 63) / 64 * 64;
       const int64_t run = std::min(max_q_len, tile_min - 1);
       const int64_t per = std::max<int64_t>(1, (int64_t(1) << 28) / (S * nq * nv * 4));
       for (int64_t t0 = 0; t0 < run; t0 += per)
