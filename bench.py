@@ -27,6 +27,9 @@ architecture (no network access for checkpoints/datasets).
                       sequence per SP group (strong scaling); activation checkpointing by HBM budget
                       (auto_ac_policy: none when the activations fit -- from 2 GPUs --, else the
                       MLP-only policy that keeps the attention outputs, else full layers)
+``--serve`` measures serving instead (one GPU, random weights): prefill and decode tokens/s of the layered
+decoder and of Llama at equal layer sizes.
+
 Every JSON line carries the full ZeRO/SP/EP configuration, the measured per-step communication
 volume per collective (``comm_measured``: calls and bytes per rank per step, from the comm facade's
 counters) and an analytic model of it (``comm_model``), so a scaling curve can be checked against the
@@ -235,9 +238,16 @@ def main():
     ap.add_argument("--offload-ratio", type=float, default=None,
                     help="offload configs: Twin-Flow offload_optimizer.ratio (share of the optimizer on the "
                          "host; default 1.0 = the whole optimizer, the reference's ZeRO-Infinity setting)")
+    ap.add_argument("--serve", nargs="?", const="all", default=None, metavar="SIZE[,SIZE]",
+                    help="instead of training: prefill / decode throughput of the Tobinex decoder beside Llama at "
+                         "equal layer sizes (shuffle_exchange_amd/inference/v2/serve_bench.py), one JSON line each")
     ap.add_argument("--device", default="cuda", choices=["cuda", "cpu"],
                     help="cpu = plumbing dry-run over gloo (tests only; invalid for the metric)")
     args = ap.parse_args()
+    if args.serve is not None:
+        from shuffle_exchange_amd.inference.v2 import serve_bench
+        serve_bench.run(sizes=None if args.serve == "all" else args.serve.split(","))
+        return
     c = CONFIGS[args.config]
     on_gpu = args.device == "cuda"
     seq = args.seq or int(os.environ.get("SXE_BENCH_SEQ", c["seq"]))

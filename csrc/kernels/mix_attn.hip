@@ -987,21 +987,23 @@ void allow_lds(F* kern, size_t bytes) {
 }
 
 template <int D>
-void launch_tokens_d(const ma::Args& a, const ma::TokArgs& k, int rows) {
+void launch_tokens_d(const ma::Args& a, const ma::TokArgs& k, int rows, bool keep_part) {
   const dim3 grid(rows * a.nkv, k.splits);
   constexpr int merge = ma::kTokWaves * 16 * D * 4, img = ma::kTokWaves * ma::TokGeo<D>::VIMG;
   constexpr size_t lds = img > merge ? img : merge;
   hipLaunchKernelGGL(ma::mix_scores_kernel<D>, grid, dim3(256), 0, cur_stream(), a, k);
   allow_lds(ma::mix_values_kernel<D>, lds);
   hipLaunchKernelGGL(ma::mix_values_kernel<D>, grid, dim3(256), lds, cur_stream(), a, k);
-  if (k.splits > 1) {
+  if (k.splits > 1 && !keep_part) {
     const int cols = a.nq * a.dv;
     hipLaunchKernelGGL(ma::mix_reduce_kernel, dim3(rows, std::min(64, (cols + 255) / 256)), dim3(256), 0, cur_stream(), a, k);
   }
   SXE_LAUNCH_CHECK();
 }
 
-void launch_tokens(const ma::Args& a, const at::Tensor& q, int nv, int splits, int tok0, int nt, int max_len) {
+// keep_part: with several splits leave their outputs unsummed and return them [splits, rows, nq dv]
+at::Tensor launch_tokens(const ma::Args& a, const at::Tensor& q, int nv, int splits, int tok0, int nt, int max_len,
+                         bool keep_part = false) {
   ma::TokArgs k{};
   const int rows = a.S * nt;
   int kps = (nv + std::max(1, splits) - 1) / std::max(1, splits);
@@ -1015,13 +1017,14 @@ void launch_tokens(const ma::Args& a, const at::Tensor& q, int nv, int splits, i
   const auto f32 = q.options().dtype(at::kFloat);
   auto scores = at::empty({(int64_t)rows * a.nq * nv}, f32), ml = at::empty({(int64_t)k.splits * rows * a.nq * 2}, f32);
   at::Tensor part;
-  if (k.splits > 1) part = at::empty({(int64_t)k.splits * rows * a.nq * a.dv}, f32);
+  if (k.splits > 1) part = at::empty({k.splits, rows, (int64_t)a.nq * a.dv}, f32);
   k.scores = scores.data_ptr<float>();
   k.ml = ml.data_ptr<float>();
   k.part = k.splits > 1 ? part.data_ptr<float>() : nullptr;
-  if (a.Dk == 64) launch_tokens_d<64>(a, k, rows);
-  else if (a.Dk == 128) launch_tokens_d<128>(a, k, rows);
-  else launch_tokens_d<256>(a, k, rows);
+  if (a.Dk == 64) launch_tokens_d<64>(a, k, rows, keep_part);
+  else if (a.Dk == 128) launch_tokens_d<128>(a, k, rows, keep_part);
+  else launch_tokens_d<256>(a, k, rows, keep_part);
+  return part;
 }
 
 template <int D, int HPW>
@@ -1081,13 +1084,13 @@ void launch_tiles(const ma::Args& a, const at::Tensor& q, int min_len, int max_q
 
 // q [T, nq, Dk], kc / vc [blocks, nkv, bs, Dk / Dv] -> out [T, nq * dv]; see the top of the file.
 // min_q_len / max_q_len bound every q_len. form: 0 = by shape, 1 = any-size kernel (fp32 always), 2 = token
-// form, 3 = tile form. splits: KV splits of the token form.
-at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& block_table,
+// form, 3 = tile form. splits: KV splits of the token form. part: see mix_attention_parts.
+static at::Tensor mix_attention_impl(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& block_table,
                          const at::Tensor& q_start, const at::Tensor& q_len, const at::Tensor& kv_len,
                          int64_t min_q_len, int64_t max_q_len, int64_t max_kv_len, int64_t splits, int64_t dk, int64_t dv, double scale, int64_t window,
                          int64_t keep_first, const c10::optional<at::Tensor>& r1, const c10::optional<at::Tensor>& r2,
                          const c10::optional<at::Tensor>& sink, const c10::optional<at::Tensor>& talk,
-                         const c10::optional<at::Tensor>& gate, int64_t form) {
+                         const c10::optional<at::Tensor>& gate, int64_t form, at::Tensor* part) {
   SXE_CHECK_CUDA(q);
   SXE_CHECK(q.dim() == 3 && q.is_contiguous(), "mix_attention: q [T, nq, Dk] contiguous");
   const int64_t T = q.size(0), nq = q.size(1), nkv = kc.size(1), S = block_table.size(0);
@@ -1152,6 +1155,12 @@ at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Te
   const bool tile_ok = mfma && nq <= ma::kTileHeads && D <= 128 && a.bs % ma::kTileKeys == 0;
   SXE_CHECK(form != 2 || mfma, "mix_attention: token form needs bf16 rows of 64, 128 or 256, a scale > 0 and a power-of-two block size");
   SXE_CHECK(form != 3 || tile_ok, "mix_attention: tile form needs bf16 rows of 64 or 128, <= 32 heads, blocks of 32 n");
+  if (part != nullptr) {
+    SXE_CHECK(mfma && max_q_len == 1 && T == S, "mix_attention_parts: one token per sequence on the matrix-core form");
+    const int64_t keys = std::min<int64_t>(max_kv_len, a.window > 0 ? a.window + a.keep_first : max_kv_len);
+    *part = launch_tokens(a, q, (int)((keys + 63) / 64 * 64), (int)splits, 0, 1, INT_MAX, true);
+    return out;
+  }
   if (mfma && form != 1) {
     constexpr int64_t kTileMin = 8;  // shorter runs of new tokens go token by token
     const int64_t tile_min = form == 2 || !tile_ok ? INT_MAX : form == 3 ? 1 : kTileMin;
@@ -1183,11 +1192,44 @@ at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Te
   return out;
 }
 
+at::Tensor mix_attention(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& block_table,
+                         const at::Tensor& q_start, const at::Tensor& q_len, const at::Tensor& kv_len, int64_t min_q_len,
+                         int64_t max_q_len, int64_t max_kv_len, int64_t splits, int64_t dk, int64_t dv, double scale,
+                         int64_t window, int64_t keep_first, const c10::optional<at::Tensor>& r1,
+                         const c10::optional<at::Tensor>& r2, const c10::optional<at::Tensor>& sink,
+                         const c10::optional<at::Tensor>& talk, const c10::optional<at::Tensor>& gate, int64_t form) {
+  return mix_attention_impl(q, kc, vc, block_table, q_start, q_len, kv_len, min_q_len, max_q_len, max_kv_len, splits, dk, dv,
+                            scale, window, keep_first, r1, r2, sink, talk, gate, form, nullptr);
+}
+
+// Decode (one token per sequence, rows in token order): [out, part]. One split: out as mix_attention's and an
+// empty part. Several: out unwritten and part fp32 [splits, T, nq dv], whose sum over the splits (times the
+// sigmoid of the gate) is the output -- for a consumer that adds them itself (skinny_gemm_gatesum).
+std::vector<at::Tensor> mix_attention_parts(const at::Tensor& q, const at::Tensor& kc, const at::Tensor& vc,
+                                            const at::Tensor& block_table, const at::Tensor& q_start,
+                                            const at::Tensor& q_len, const at::Tensor& kv_len, int64_t max_kv_len,
+                                            int64_t splits, int64_t dk, int64_t dv, double scale, int64_t window,
+                                            int64_t keep_first, const c10::optional<at::Tensor>& r1,
+                                            const c10::optional<at::Tensor>& r2, const c10::optional<at::Tensor>& sink,
+                                            const c10::optional<at::Tensor>& talk, const c10::optional<at::Tensor>& gate) {
+  at::Tensor part;
+  auto out = mix_attention_impl(q, kc, vc, block_table, q_start, q_len, kv_len, 1, 1, max_kv_len, splits, dk, dv, scale,
+                                window, keep_first, r1, r2, sink, talk, gate, 0, &part);
+  if (!part.defined()) part = at::empty({0}, q.options().dtype(at::kFloat));
+  return {out, part};
+}
+
 }  // namespace sxe
 
 TORCH_LIBRARY_FRAGMENT(sxe, m) {
   m.def("mix_attention(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor q_start, Tensor q_len, Tensor kv_len, "
         "int min_q_len, int max_q_len, int max_kv_len, int splits, int dk, int dv, float scale, int window, int keep_first, Tensor? r1, Tensor? r2, "
         "Tensor? sink, Tensor? talk, Tensor? gate, int form=0) -> Tensor");
+  m.def("mix_attention_parts(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor q_start, Tensor q_len, "
+        "Tensor kv_len, int max_kv_len, int splits, int dk, int dv, float scale, int window, int keep_first, Tensor? r1, "
+        "Tensor? r2, Tensor? sink, Tensor? talk, Tensor? gate) -> Tensor[]");
 }
-TORCH_LIBRARY_IMPL(sxe, CUDA, m) { m.impl("mix_attention", &sxe::mix_attention); }
+TORCH_LIBRARY_IMPL(sxe, CUDA, m) {
+  m.impl("mix_attention", &sxe::mix_attention);
+  m.impl("mix_attention_parts", &sxe::mix_attention_parts);
+}

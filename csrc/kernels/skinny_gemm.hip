@@ -55,7 +55,7 @@ __device__ __forceinline__ void load_x(Frag& f, const unsigned short* __restrict
   }
 }
 
-enum : int { PRO_NONE = 0, PRO_RMS = 1, PRO_SWIGLU = 2, PRO_MERGE = 3 };
+enum : int { PRO_NONE = 0, PRO_RMS = 1, PRO_SWIGLU = 2, PRO_MERGE = 3, PRO_ADDNORM = 4, PRO_GATESUM = 5 };
 constexpr int kProMaxM = 4;
 
 struct ProArgs {
@@ -78,6 +78,19 @@ struct ProArgs {
   unsigned short* rcache;
   int rnq, rnkv, rbs;
   int nt;  // non-temporal weight loads (SXE_SKINNY_NT)
+  // ADDNORM: norm AFTER a scaled residual sum over a 32-bit residual stream, v = alpha r + x, input =
+  // rms(v) (offset + gw). r is given either as it is (rw == nullptr) or as an earlier such sum still to be
+  // normalised: r = res32 rrinv[m] (offset + rw). hout32 = v and rinv_out = 1 / rms(v) are written by
+  // workgroup 0, so the next consumer gets r in that form and nobody writes the normalised stream.
+  const float* res32;
+  const float* rrinv;
+  const unsigned short* rw;
+  float* hout32;
+  float* rinv_out;
+  float alpha, offset;
+  // GATESUM: input = sigmoid(gate) * sum over `splits` of po [splits, M, K] (fp32)
+  const unsigned short* gate;
+  int64_t gate_ld;
 };
 
 // output column of lane `col` in tile `tile` (identity unless the RoPE epilogue pairs columns)
@@ -168,6 +181,44 @@ __device__ __forceinline__ void build_merge(int M, int K, int klo, int khi, cons
   __syncthreads();
 }
 
+// PRO_GATESUM: act[m][c] = sigmoid(gate[m][c]) * sum_s po[s][m][c], every load of a group of 8 splits in flight
+// before the first use
+template <int NT>
+__device__ __forceinline__ void build_gatesum(int M, int K, const ProArgs& p, unsigned short* act) {
+  constexpr int U = 8;
+  const int per = K / 8, n = M * per;
+  for (int idx = threadIdx.x; idx < n; idx += NT) {
+    const int m = idx / per, c = (idx - m * per) * 8;
+    float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    u16x8 gv = {0, 0, 0, 0, 0, 0, 0, 0};
+    if (p.gate != nullptr) gv = *reinterpret_cast<const u16x8*>(p.gate + m * p.gate_ld + c);
+    for (int s0 = 0; s0 < p.splits; s0 += U) {
+      f32x4 o0[U], o1[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const float* src = p.po + ((int64_t)min(s0 + u, p.splits - 1) * M + m) * K + c;
+        o0[u] = *reinterpret_cast<const f32x4*>(src);
+        o1[u] = *reinterpret_cast<const f32x4*>(src + 4);
+      }
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+        if (s0 + u < p.splits) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            acc[j] += o0[u][j];
+            acc[4 + j] += o1[u][j];
+          }
+        }
+    }
+    if (p.gate != nullptr) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) acc[j] /= 1.f + __expf(-bf16_to_f32(gv[j]));
+    }
+    store8<DT::BF16>(act + (int64_t)m * K + c, acc);
+  }
+  __syncthreads();
+}
+
 // Only columns [klo, khi) of the input are built (a split-K part needs no more), except under
 // PRO_RMS, whose row norm needs the whole row.
 template <int MODE, int NT>
@@ -177,19 +228,25 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
     build_merge<NT>(M, K, klo, khi, p, act);
     return;
   }
-  if constexpr (MODE == PRO_RMS) {
+  if constexpr (MODE == PRO_GATESUM) {
+    build_gatesum<NT>(M, K, p, act);
+    return;
+  }
+  constexpr bool NORM = MODE == PRO_RMS || MODE == PRO_ADDNORM;
+  if constexpr (NORM) {
     klo = 0;
     khi = K;
   }
   // U chunks of 8 per thread per round, every load of a round issued before the first use: a loop
   // that consumes each chunk before loading the next is a chain of dependent L2 round trips (it made
   // the fused down projection 9 us slower than the separate SwiGLU launch)
-  constexpr int U = 4;
+  constexpr int U = MODE == PRO_ADDNORM ? 2 : 4;
   __shared__ float red[NT / 64][kProMaxM];
   const int per = (khi - klo) / 8, n = M * per;
   float ss[kProMaxM] = {0.f, 0.f, 0.f, 0.f};
   for (int base = 0; base < n; base += U * NT) {
     u16x8 a[U], b[U], gw[U];
+    f32x4 r0[U], r1[U];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
       const int idx = base + u * NT + threadIdx.x;
@@ -201,7 +258,12 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
         b[u] = *reinterpret_cast<const u16x8*>(xr + K);
       } else {
         gw[u] = *reinterpret_cast<const u16x8*>(p.gw + (ok ? c : 0));
-        if (p.res != nullptr) b[u] = *reinterpret_cast<const u16x8*>(p.res + (int64_t)(ok ? m : 0) * ldx + (ok ? c : 0));
+        if constexpr (MODE == PRO_ADDNORM) {
+          const float* rp = p.res32 + (int64_t)(ok ? m : 0) * K + (ok ? c : 0);
+          r0[u] = *reinterpret_cast<const f32x4*>(rp);
+          r1[u] = *reinterpret_cast<const f32x4*>(rp + 4);
+          if (p.rw != nullptr) b[u] = *reinterpret_cast<const u16x8*>(p.rw + (ok ? c : 0));
+        } else if (p.res != nullptr) b[u] = *reinterpret_cast<const u16x8*>(p.res + (int64_t)(ok ? m : 0) * ldx + (ok ? c : 0));
       }
     }
 #pragma unroll
@@ -220,7 +282,19 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
         float v[8];
 #pragma unroll
         for (int j = 0; j < 8; ++j) v[j] = bf16_to_f32(a[u][j]);
-        if (p.res != nullptr) {
+        if constexpr (MODE == PRO_ADDNORM) {
+          const float ri = p.rw != nullptr ? p.rrinv[m] : 1.f;
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            float r = (j < 4 ? r0[u][j & 3] : r1[u][j & 3]) * ri;
+            if (p.rw != nullptr) r *= p.offset + bf16_to_f32(b[u][j]);
+            v[j] += p.alpha * r;
+          }
+          if (blockIdx.x == 0) {
+            *reinterpret_cast<f32x4*>(p.hout32 + (int64_t)m * K + c) = f32x4{v[0], v[1], v[2], v[3]};
+            *reinterpret_cast<f32x4*>(p.hout32 + (int64_t)m * K + c + 4) = f32x4{v[4], v[5], v[6], v[7]};
+          }
+        } else if (p.res != nullptr) {
 #pragma unroll
           for (int j = 0; j < 8; ++j) v[j] = bf16_to_f32(f32_to_bf16(v[j] + bf16_to_f32(b[u][j])));
           if (p.hout != nullptr && blockIdx.x == 0) store8<DT::BF16>(p.hout + (int64_t)m * K + c, v);
@@ -229,7 +303,7 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
           q += v[j] * v[j];
-          o[j] = v[j] * bf16_to_f32(gw[u][j]);
+          o[j] = v[j] * (MODE == PRO_ADDNORM ? p.offset + bf16_to_f32(gw[u][j]) : bf16_to_f32(gw[u][j]));
         }
 #pragma unroll
         for (int mm = 0; mm < kProMaxM; ++mm)
@@ -238,7 +312,7 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
       store8<DT::BF16>(act + (int64_t)m * K + c, o);
     }
   }
-  if constexpr (MODE == PRO_RMS) {
+  if constexpr (NORM) {
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 #pragma unroll
     for (int mm = 0; mm < kProMaxM; ++mm) {
@@ -251,6 +325,8 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
 #pragma unroll
       for (int w = 0; w < NT / 64; ++w) t += red[w][threadIdx.x];
       rinv[threadIdx.x] = rsqrtf(t / (float)K + p.eps);
+      if constexpr (MODE == PRO_ADDNORM)
+        if (blockIdx.x == 0 && (int)threadIdx.x < M) p.rinv_out[threadIdx.x] = rinv[threadIdx.x];
     }
   }
   __syncthreads();
@@ -327,7 +403,7 @@ __global__ __launch_bounds__(NW * 64) void skinny_gemm_kernel(const unsigned sho
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int m = 4 * g + r;
-        const float sc = MODE == PRO_RMS ? rinv[m < kProMaxM ? m : 0] : 1.f;
+        const float sc = MODE == PRO_RMS || MODE == PRO_ADDNORM ? rinv[m < kProMaxM ? m : 0] : 1.f;
         if (m < M) y[(int64_t)m * ldy + n] = f32_to_bf16(t[r] * sc + b);
       }
     }
@@ -771,6 +847,105 @@ at::Tensor skinny_gemm_merge(const at::Tensor& part_o, const at::Tensor& part_ml
   return y;
 }
 
+// Common tail of the bf16-weight prologue launches below: y [M, N] = input(pro) . w^T
+static at::Tensor skinny_launch(int mode, const unsigned short* xp, int64_t ldx, int M, const at::Tensor& w, sg::ProArgs pro) {
+  const int N = w.size(0), K = w.size(1);
+  SXE_CHECK(w.is_cuda() && w.scalar_type() == at::kBFloat16 && w.dim() == 2 && w.is_contiguous() &&
+                reinterpret_cast<uintptr_t>(w.data_ptr()) % 16 == 0 && K % 8 == 0,
+            "skinny gemm: w bf16 [N, K], 16-B rows");
+  SXE_CHECK(M >= 1 && M <= sg::kProMaxM, "skinny gemm: 1 <= M <= 4");
+  const size_t lds = (size_t)M * K * 2;
+  SXE_CHECK(lds <= 144 * 1024, "skinny gemm: M x K input exceeds the LDS budget");
+  auto y = at::empty({M, N}, w.options());
+  if (N == 0) return y;
+  const int ss_total = (K + sg::kSS - 1) / sg::kSS, tiles = (N + 15) / 16;
+  int nw = 4, spw = 1;
+  sg::plan(tiles, ss_total, nw, spw);
+  pro.nt = sg::nt_loads();
+  static bool attr[2][2] = {};
+  auto go = [&](auto kern, int ni) {
+    bool& done = attr[mode == sg::PRO_ADDNORM][ni];
+    if (!done) {
+      SXE_HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, 144 * 1024));
+      done = true;
+    }
+    hipLaunchKernelGGL(kern, dim3(tiles), dim3(nw * 64), lds, cur_stream(), xp, ldx,
+                       reinterpret_cast<const unsigned short*>(w.data_ptr()), w.stride(0), (const unsigned short*)nullptr,
+                       reinterpret_cast<unsigned short*>(y.data_ptr()), y.stride(0), M, N, K, spw, pro);
+  };
+  if (mode == sg::PRO_ADDNORM) {
+    if (nw == 4) go(sg::skinny_gemm_kernel<4, sg::PRO_ADDNORM, false>, 0);
+    else go(sg::skinny_gemm_kernel<8, sg::PRO_ADDNORM, false>, 1);
+  } else {
+    if (nw == 4) go(sg::skinny_gemm_kernel<4, sg::PRO_GATESUM, false>, 0);
+    else go(sg::skinny_gemm_kernel<8, sg::PRO_GATESUM, false>, 1);
+  }
+  SXE_LAUNCH_CHECK();
+  return y;
+}
+
+// Decode, norm after the residual sum (PRO_ADDNORM): v = alpha r + y, out = (rms(v) (offset + gw)) . w^T.
+// r: res fp32 [M, K], or with (res_rinv [M], res_w [K]) res * res_rinv * (offset + res_w).
+// Returns [out [M, N], v fp32 [M, K], 1 / rms(v) fp32 [M]] -- r of the next call.
+std::vector<at::Tensor> skinny_gemm_addnorm(const at::Tensor& y, const at::Tensor& res, const c10::optional<at::Tensor>& res_rinv,
+                                            const c10::optional<at::Tensor>& res_w, const at::Tensor& gw, double alpha,
+                                            double eps, double offset, const at::Tensor& w) {
+  SXE_CHECK_CUDA(y);
+  SXE_CHECK(y.scalar_type() == at::kBFloat16 && y.dim() == 2 && y.is_contiguous(), "skinny_gemm_addnorm: y bf16 [M, K]");
+  const int M = y.size(0), K = y.size(1);
+  SXE_CHECK(w.dim() == 2 && w.size(1) == K, "skinny_gemm_addnorm: w [N, K]");
+  SXE_CHECK(res.is_cuda() && res.scalar_type() == at::kFloat && res.is_contiguous() && res.sizes() == y.sizes(),
+            "skinny_gemm_addnorm: res fp32 like y");
+  SXE_CHECK(gw.is_cuda() && gw.scalar_type() == at::kBFloat16 && gw.is_contiguous() && gw.numel() == K, "skinny_gemm_addnorm: gw [K]");
+  const bool lazy = res_w.has_value() && res_w->defined();
+  SXE_CHECK(lazy == (res_rinv.has_value() && res_rinv->defined()), "skinny_gemm_addnorm: res_rinv and res_w together");
+  sg::ProArgs pro{};
+  for (const void* q : {(const void*)y.data_ptr(), (const void*)res.data_ptr(), (const void*)gw.data_ptr(),
+                        lazy ? (const void*)res_w->data_ptr() : nullptr})
+    SXE_CHECK(reinterpret_cast<uintptr_t>(q) % 16 == 0, "skinny_gemm_addnorm: 16-byte aligned operands");
+  if (lazy) {
+    SXE_CHECK(res_w->is_cuda() && res_w->scalar_type() == at::kBFloat16 && res_w->is_contiguous() && res_w->numel() == K &&
+                  res_rinv->is_cuda() && res_rinv->scalar_type() == at::kFloat && res_rinv->is_contiguous() && res_rinv->numel() == M,
+              "skinny_gemm_addnorm: res_rinv fp32 [M], res_w bf16 [K]");
+    pro.rrinv = res_rinv->data_ptr<float>();
+    pro.rw = reinterpret_cast<const unsigned short*>(res_w->data_ptr());
+  }
+  c10::DeviceGuard gd(y.device());
+  auto h = at::empty({M, K}, res.options()), rinv = at::empty({M}, res.options());
+  pro.gw = reinterpret_cast<const unsigned short*>(gw.data_ptr());
+  pro.eps = (float)eps;
+  pro.res32 = res.data_ptr<float>();
+  pro.hout32 = h.data_ptr<float>();
+  pro.rinv_out = rinv.data_ptr<float>();
+  pro.alpha = (float)alpha;
+  pro.offset = (float)offset;
+  auto out = skinny_launch(sg::PRO_ADDNORM, reinterpret_cast<const unsigned short*>(y.data_ptr()), y.stride(0), M, w, pro);
+  return {out, h, rinv};
+}
+
+// Decode output projection of split attention whose splits add up (PRO_GATESUM): part fp32 [splits, M, K],
+// gate bf16 [M, K] (row stride free) or None -> (sigmoid(gate) * sum_s part) . w^T
+at::Tensor skinny_gemm_gatesum(const at::Tensor& part, const c10::optional<at::Tensor>& gate, const at::Tensor& w) {
+  SXE_CHECK_CUDA(part);
+  SXE_CHECK(part.scalar_type() == at::kFloat && part.dim() == 3 && part.is_contiguous() && part.size(0) >= 1,
+            "skinny_gemm_gatesum: part fp32 [splits, M, K]");
+  const int M = part.size(1), K = part.size(2);
+  SXE_CHECK(w.dim() == 2 && w.size(1) == K && reinterpret_cast<uintptr_t>(part.data_ptr()) % 16 == 0, "skinny_gemm_gatesum: w [N, K]");
+  sg::ProArgs pro{};
+  pro.po = part.data_ptr<float>();
+  pro.splits = part.size(0);
+  if (gate.has_value() && gate->defined()) {
+    SXE_CHECK(gate->is_cuda() && gate->scalar_type() == at::kBFloat16 && gate->dim() == 2 && gate->size(0) == M &&
+                  gate->size(1) == K && gate->stride(1) == 1 && gate->stride(0) % 8 == 0 &&
+                  reinterpret_cast<uintptr_t>(gate->data_ptr()) % 16 == 0,
+              "skinny_gemm_gatesum: gate bf16 [M, K], 16-B rows");
+    pro.gate = reinterpret_cast<const unsigned short*>(gate->data_ptr());
+    pro.gate_ld = gate->stride(0);
+  }
+  c10::DeviceGuard gd(part.device());
+  return skinny_launch(sg::PRO_GATESUM, nullptr, K, M, w, pro);
+}
+
 }  // namespace sxe
 
 TORCH_LIBRARY_FRAGMENT(sxe, m) {
@@ -778,6 +953,9 @@ TORCH_LIBRARY_FRAGMENT(sxe, m) {
   m.def("skinny_gemm_fp8w(Tensor x, Tensor wq, Tensor wscale, Tensor? bias) -> Tensor");
   m.def("skinny_gemm_pro(Tensor x, Tensor? res, Tensor? gw, float eps, Tensor w, Tensor? wscale, Tensor? bias, "
         "int mode) -> Tensor[]");
+  m.def("skinny_gemm_addnorm(Tensor y, Tensor res, Tensor? res_rinv, Tensor? res_w, Tensor gw, float alpha, float eps, "
+        "float offset, Tensor w) -> Tensor[]");
+  m.def("skinny_gemm_gatesum(Tensor part, Tensor? gate, Tensor w) -> Tensor");
   m.def("skinny_gemm_merge(Tensor part_o, Tensor part_ml, Tensor w, Tensor? wscale, Tensor? bias) -> Tensor");
   m.def("skinny_gemm_pro_rope(Tensor x, Tensor? res, Tensor gw, float eps, Tensor w, Tensor? wscale, Tensor cos, "
         "Tensor sin, Tensor pos, Tensor slots, Tensor(a!) cache, int nq, int nkv) -> Tensor[]");
@@ -786,6 +964,8 @@ TORCH_LIBRARY_IMPL(sxe, CUDA, m) {
   m.impl("skinny_gemm", &sxe::skinny_gemm);
   m.impl("skinny_gemm_fp8w", &sxe::skinny_gemm_fp8w);
   m.impl("skinny_gemm_pro", &sxe::skinny_gemm_pro);
+  m.impl("skinny_gemm_addnorm", &sxe::skinny_gemm_addnorm);
+  m.impl("skinny_gemm_gatesum", &sxe::skinny_gemm_gatesum);
   m.impl("skinny_gemm_merge", &sxe::skinny_gemm_merge);
   m.impl("skinny_gemm_pro_rope", &sxe::skinny_gemm_pro_rope);
 }

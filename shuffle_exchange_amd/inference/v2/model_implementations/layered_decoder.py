@@ -24,8 +24,8 @@ from typing import List, Optional
 import torch
 
 from ....ops.activation import gated_act
-from ....ops.linear import linear
-from ....ops.mix_attention import MixParams, cache_row, mix_attention
+from ....ops.linear import fused_addnorm_linear, fused_gatesum_linear, fused_swiglu_linear, linear
+from ....ops.mix_attention import MixParams, cache_row, mix_attention, mix_attention_parts
 from ....ops.residual_norm import embed_scale, qkv_norm_append, residual_rms_norm
 
 FF_MULTIPLE = 16
@@ -184,26 +184,69 @@ class RaggedLayeredDecoder:
             sd.update({f"layers.{i}.{k}": v for k, v in L.items() if torch.is_tensor(v)})
         return sd
 
-    def _attn(self, xb, L, li, batch, kv_cache):
+    # decode (<= 2 tokens): the norm after the residual sum runs as the prologue of the next projection, the
+    # gated sum of the attention's KV splits as the output projection's, SwiGLU as the down projection's
+    FUSE_MAX_T = 2  # at 4 rows every workgroup rebuilding them costs more than the launches saved
+
+    def _fusable(self, T):
+        return (T <= self.FUSE_MAX_T and self._device.type == "cuda" and self._dtype == torch.bfloat16
+                and os.environ.get("SXE_DECODE_FUSE", "1") == "1")
+
+    def _attn(self, proj, L, li, batch, kv_cache):
+        """``proj`` [T, q | k | v | gate] -> the mixer's output [T, width]."""
         a = self.spec.layers[li].mixer
         nq, nkv, dk, dv = a.heads, a.kv_heads, a.dim, a.vdim
-        proj = linear(xb, L["qkvg"])
         kc, vc = kv_cache.layer_kv(li)
         q = qkv_norm_append(proj, L["q_norm"], L["k_norm"], kc, vc, batch.slots, nq, nkv, dk, dv, self.spec.eps)
-        o = mix_attention(q, kc, vc, batch, dk, dv, a.scale, self._mix[li], a.window, a.keep_first,
-                          gate=proj[:, nq * dk + nkv * (dk + dv):])
+        gate = proj[:, nq * dk + nkv * (dk + dv):]
+        args = (q, kc, vc, batch, dk, dv, a.scale, self._mix[li], a.window, a.keep_first, gate)
+        parts = mix_attention_parts(*args) if self._fusable(proj.shape[0]) else None
+        if parts is None:
+            return linear(mix_attention(*args), L["o"])
+        o, part = parts
+        y = fused_gatesum_linear(part, gate, L["o"]) if part is not None else None
+        if y is not None:
+            return y
+        if part is not None:
+            o = (part.sum(0) * torch.sigmoid(gate.float())).to(proj.dtype)
         return linear(o, L["o"])
+
+    def _norm_linear(self, pending, x, xb, weight):
+        """The projection of the layer input: ``linear(xb, weight)`` when no norm is pending, else the
+        pending ``(y, norm weight)`` -- x <- norm(alpha x + y) -- and the projection, in one launch where the
+        fused kernel covers it. Returns (projection, x, xb); x may come back as the fused kernel's state."""
+        if pending is None:
+            return linear(xb, weight), x, xb
+        s = self.spec
+        if self._fusable(pending[0].shape[0]):
+            r = fused_addnorm_linear(pending[0], x, pending[1], s.alpha, s.eps, s.norm_offset, weight)
+            if r is not None:
+                return r[0], r[1], None
+        x, xb = residual_rms_norm(self._stream(x), pending[0], pending[1], s.alpha, s.eps, s.norm_offset)
+        return linear(xb, weight), x, xb
+
+    def _stream(self, x):
+        """The fp32 residual stream itself (a fused state holds the sum in front of its norm)."""
+        if isinstance(x, tuple):
+            return residual_rms_norm(x[0], None, x[2], 1.0, self.spec.eps, self.spec.norm_offset)[0]
+        return x
 
     @torch.no_grad()
     def forward(self, batch, kv_cache):
         s, W = self.spec, self.w
         x, xb = embed_scale(W["embed"], batch.input_ids, s.embed_scale)
+        pending = None  # the last sublayer's (output, norm weight), not yet added to x
         for li, L in enumerate(W["layers"]):
-            y = self._attn(xb, L, li, batch, kv_cache)
-            x, xb = residual_rms_norm(x, y, L["norm1"], s.alpha, s.eps, s.norm_offset)
+            proj, x, xb = self._norm_linear(pending, x, xb, L["qkvg"])
+            pending = (self._attn(proj, L, li, batch, kv_cache), L["norm1"])
             if "gu" in L:
-                y = linear(gated_act(linear(xb, L["gu"]), s.layers[li].act), L["down"])
-                x, xb = residual_rms_norm(x, y, L["norm2"], s.alpha, s.eps, s.norm_offset)
+                gu, x, xb = self._norm_linear(pending, x, xb, L["gu"])
+                y = fused_swiglu_linear(gu, L["down"]) if self._fusable(gu.shape[0]) and s.layers[li].act == "silu" else None
+                if y is None:
+                    y = linear(gated_act(gu, s.layers[li].act), L["down"])
+                pending = (y, L["norm2"])
+        if pending is not None:
+            x, _ = residual_rms_norm(self._stream(x), pending[0], pending[1], s.alpha, s.eps, s.norm_offset)
         _, h = residual_rms_norm(x, None, W["final"], 1.0, s.eps, s.norm_offset, index=batch.last_idx, need_x=False)
         return linear(h, W["embed"]).float()
 

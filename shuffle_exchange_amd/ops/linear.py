@@ -136,6 +136,31 @@ def fused_merge_linear(part_o, part_ml, weight, bias=None):
     return torch.ops.sxe.skinny_gemm_merge(part_o, part_ml, w, sc, bias)
 
 
+def fused_addnorm_linear(y, res, norm_weight, alpha, eps, offset, weight):
+    """Decode (<= 4 rows), norm after a scaled 32-bit residual sum, in ONE launch (skinny_gemm.hip
+    PRO_ADDNORM): v = alpha r + y, returns ``(linear(rms(v) (offset + norm_weight), weight), state)``. ``res`` is
+    either r itself (fp32 tensor) or the ``state`` (v, 1 / rms(v), norm_weight) of an earlier call, whose
+    normalised sum is r. None when not covered."""
+    wk = _pro_weight(weight)
+    if (wk is None or wk[1] is not None or not _pro_ok(y) or not y.is_contiguous() or y.shape[1] != wk[0].shape[1]
+            or y.shape[1] % 8 or norm_weight.dtype != torch.bfloat16 or norm_weight.data_ptr() % 16
+            or y.numel() * 2 > 144 * 1024):
+        return None
+    h, rinv, rw = res if isinstance(res, tuple) else (res, None, None)
+    out, v, ri = torch.ops.sxe.skinny_gemm_addnorm(y, h, rinv, rw, norm_weight, float(alpha), float(eps), float(offset), wk[0])
+    return out, (v, ri, norm_weight)
+
+
+def fused_gatesum_linear(part, gate, weight):
+    """Decode (<= 4 rows): ``linear(sigmoid(gate) * part.sum(0), weight)`` in ONE launch (skinny_gemm.hip
+    PRO_GATESUM); part fp32 [splits, M, K]. None when not covered."""
+    wk = _pro_weight(weight)
+    if (wk is None or wk[1] is not None or part.shape[1] > 4 or part.shape[2] % 8 or gate.stride(0) % 8
+            or gate.data_ptr() % 16 or part.shape[1] * part.shape[2] * 2 > 144 * 1024):
+        return None
+    return torch.ops.sxe.skinny_gemm_gatesum(part, gate, wk[0])
+
+
 # Hand-written weight-gradient GEMM (csrc/kernels/gemm_wgrad.hip: k-major operands read through LDS
 # with ds_read_b64_tr_b16, fp32 accumulate in the epilogue): no transposed copies of dY / X at all.
 # Measured on MI355X at 8192 tokens (tools/wgrad_exp.py, profiles/wgrad_kernel.log): 28672x4096

@@ -39,13 +39,32 @@ def mix_attention(q, kc, vc, batch, dk, dv, scale, params, window=None, keep_fir
     kernels ("auto": by shape; "generic" any size, one token per workgroup; "token" scores through
     memory; "tile" 16 tokens x all heads)."""
     if native.use_hip(q):
-        visible = batch.max_kv_len if not window else min(batch.max_kv_len, window + keep_first)
-        splits = choose_splits(batch.num_seqs, kc.shape[1], visible)
+        splits = _splits(kc, batch, window, keep_first)
         return torch.ops.sxe.mix_attention(q, kc, vc, batch.block_table, batch.q_start, batch.q_len, batch.kv_len,
                                            min(batch.host_q_len), max(batch.host_q_len), int(batch.max_kv_len), splits,
                                            int(dk), int(dv), float(scale), int(window or 0), int(keep_first), params.r1,
                                            params.r2, params.sink, params.talk, gate, FORMS[form])
     return mix_attention_reference(q, kc, vc, batch, dk, dv, scale, params, window, keep_first, gate)
+
+
+def _splits(kc, batch, window, keep_first):
+    return choose_splits(batch.num_seqs, kc.shape[1],
+                         batch.max_kv_len if not window else min(batch.max_kv_len, window + keep_first))
+
+
+def mix_attention_parts(q, kc, vc, batch, dk, dv, scale, params, window=None, keep_first=0, gate=None):
+    """Decode (HIP, bf16, one new token per sequence): ``(out, None)`` when the keys fit one split, else
+    ``(None, part)`` with part fp32 [splits, T, nq * dv] for ``ops.linear.fused_gatesum_linear``, which
+    adds the splits and applies the gate. None where the kernels do not cover the shape."""
+    bs, D = kc.shape[2], kc.shape[3]
+    if (q.dtype != torch.bfloat16 or D not in MFMA_ROWS or vc.shape[3] != D or bs & (bs - 1) or scale <= 0
+            or q.shape[1] > 256 or max(batch.host_q_len) != 1 or q.shape[0] != batch.num_seqs):
+        return None
+    out, part = torch.ops.sxe.mix_attention_parts(q, kc, vc, batch.block_table, batch.q_start, batch.q_len, batch.kv_len,
+                                                  int(batch.max_kv_len), _splits(kc, batch, window, keep_first), int(dk),
+                                                  int(dv), float(scale), int(window or 0), int(keep_first), params.r1,
+                                                  params.r2, params.sink, params.talk, gate)
+    return (out, None) if part.numel() == 0 else (None, part)
 
 
 def mix_attention_reference(q, kc, vc, batch, dk, dv, scale, params, window=None, keep_first=0, gate=None):

@@ -175,6 +175,14 @@ def test_many_splits_and_long_context():
         check(c.run(0.09, window, keep), c.oracle(0.09, window, keep), torch.bfloat16)
 
 
+@gpu
+def test_tile_form_key_splits_and_many_tiles():
+    for lens, H, G, D in (([(0, 700)], 32, 8, 64), ([(1400, 90), (0, 20)], 16, 4, 128), ([(0, 2300)], 4, 2, 64)):
+        c = Case(lens, H, G, D, D, torch.bfloat16, "cuda", bs=64)
+        for window, keep in ((None, 0), (600, 50)):
+            check(c.run(0.1, window, keep, "tile"), c.oracle(0.1, window, keep), torch.bfloat16)
+
+
 # ------------------------------------------------------------------------------------- row ops
 def _row_case(W, dtype, device):
     g = torch.Generator().manual_seed(W)
@@ -252,3 +260,31 @@ def test_append_cpu(shape):
 @pytest.mark.parametrize("shape", [(6, 2, 20, 12), (8, 8, 64, 64), (32, 8, 128, 128), (3, 1, 40, 72), (5, 5, 33, 7)])
 def test_append_gpu(shape, dtype):
     _check_append(*shape, dtype, "cuda")
+
+
+# --------------------------------------------------------------------------- fused decode projections
+@gpu
+@pytest.mark.parametrize("M", [1, 3, 4])
+@pytest.mark.parametrize("K,N", [(64, 48), (256, 1000), (4096, 4096), (1048, 40)])
+def test_fused_addnorm_and_gatesum(M, K, N):
+    from shuffle_exchange_amd.ops.linear import fused_addnorm_linear, fused_gatesum_linear
+    g = torch.Generator().manual_seed(K + M)
+    bf = (lambda *s, std=1.0: (torch.randn(*s, generator=g) * std).to(torch.bfloat16).cuda())
+    w1, w2 = bf(N, K, std=K ** -0.5), bf(N, K, std=K ** -0.5)
+    y1, y2, n1, n2 = bf(M, K), bf(M, K), bf(K, std=0.3), bf(K, std=0.3)
+    x = torch.randn(M, K, generator=g).cuda()
+    o1, st = fused_addnorm_linear(y1, x, n1, 2.0, 1e-3, 1.0, w1)
+    o2, st2 = fused_addnorm_linear(y2, st, n2, 2.0, 1e-3, 1.0, w2)
+    d = (lambda t: t.double().cpu())
+    r1 = O.norm_around_zero(2.0 * d(x) + d(y1), d(n1), 1e-3)
+    r2 = O.norm_around_zero(2.0 * r1 + d(y2), d(n2), 1e-3)
+    for o, r, w in ((o1, r1, w1), (o2, r2, w2)):
+        torch.testing.assert_close(d(o), r @ d(w).T, rtol=2e-2, atol=3e-2)
+    torch.testing.assert_close(d(st2[0]), 2.0 * r1 + d(y2), rtol=1e-5, atol=1e-5)
+    stream = residual_rms_norm(st2[0], None, n2, 1.0, 1e-3, 1.0)[0]
+    torch.testing.assert_close(d(stream), r2, rtol=1e-5, atol=1e-5)
+    torch.testing.assert_close(d(stream), d(st2[0]) * d(st2[1])[:, None] * (1 + d(n2)), rtol=1e-5, atol=1e-5)
+    for splits in (1, 3, 11):
+        part, gate = torch.randn(splits, M, K, generator=g).cuda(), bf(M, K + 8)[:, 8:]
+        ref = (d(part).sum(0) * torch.sigmoid(d(gate))) @ d(w1).T
+        torch.testing.assert_close(d(fused_gatesum_linear(part, gate, w1)), ref, rtol=2e-2, atol=0.02 * splits ** 0.5 + 0.02)
