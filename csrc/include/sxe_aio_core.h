@@ -140,17 +140,19 @@ class Engine {
  private:
   void run(Task& t) {
     int64_t done = 0;
+    bool direct = true;  // this task may still be refused by direct I/O
     while (done < t.nbytes) {
       ssize_t r = t.write ? ::pwrite(t.file->fd, t.buf + done, t.nbytes - done, t.offset + done)
                           : ::pread(t.file->fd, t.buf + done, t.nbytes - done, t.offset + done);
       if (r < 0 && errno == EINTR) continue;
-      if (r < 0 && errno == EINVAL) {
-        // O_DIRECT refused for this piece (filesystem without direct I/O): fall back to buffered
+      if (r < 0 && (errno == EINVAL || errno == EFAULT) && direct) {
+        // O_DIRECT refused for this piece (EINVAL: filesystem without direct I/O; EFAULT: driver-mapped pinned
+        // pages that the block layer cannot take): fall back to buffered, once per task -- another
+        // worker may have cleared the flag while this call was under way
+        direct = false;
         const int fl = ::fcntl(t.file->fd, F_GETFL);
-        if (fl & O_DIRECT) {
-          ::fcntl(t.file->fd, F_SETFL, fl & ~O_DIRECT);
-          continue;
-        }
+        if (fl & O_DIRECT) ::fcntl(t.file->fd, F_SETFL, fl & ~O_DIRECT);
+        continue;
       }
       if (r <= 0) {
         const std::string why = (r == 0 ? std::string("unexpected end of file") : std::string(std::strerror(errno)));

@@ -40,7 +40,7 @@ __device__ __forceinline__ void store4(typename dt_traits<T>::storage* p, f32x4 
   }
 }
 
-template <DT T>
+template <DT T, bool VEC>
 __global__ __launch_bounds__(kThreads) void embed_scale_kernel(const typename dt_traits<T>::storage* __restrict table,
                                                                const int64_t* __restrict ids, int rows, int W,
                                                                float scale, float* __restrict x,
@@ -49,6 +49,15 @@ __global__ __launch_bounds__(kThreads) void embed_scale_kernel(const typename dt
   const int64_t id = ids[t];
   const bool ok = id >= 0 && id < rows;
   const auto* src = table + (ok ? id : 0) * W;
+  if constexpr (VEC) {
+    for (int c = threadIdx.x * 4; c < W; c += kThreads * 4) {
+      f32x4 v = load4<T>(src + c) * scale;
+      if (!ok) v = f32x4{0.f, 0.f, 0.f, 0.f};
+      *reinterpret_cast<f32x4*>(x + t * W + c) = v;
+      if (xb != nullptr) store4<T>(xb + t * W + c, v);
+    }
+    return;
+  }
   for (int c = threadIdx.x; c < W; c += kThreads) {
     const float v = ok ? to_f32<T>(src[c]) * scale : 0.f;
     x[t * W + c] = v;
@@ -227,11 +236,16 @@ std::vector<at::Tensor> embed_scale(const at::Tensor& table, const at::Tensor& i
   auto xb = dt == DT::F32 ? x : at::empty({T, W}, table.options());
   if (T == 0 || W == 0) return {x, xb};
   c10::DeviceGuard g(table.device());
+  const bool vec = W % 4 == 0 && rn::aligned(table.data_ptr(), 16);
   SXE_DISPATCH_DT(dt, D, {
     using S = dt_traits<D>::storage;
-    hipLaunchKernelGGL(rn::embed_scale_kernel<D>, dim3(T), dim3(rn::kThreads), 0, cur_stream(),
-                       static_cast<const S*>(table.data_ptr()), ids.data_ptr<int64_t>(), (int)table.size(0), (int)W,
-                       (float)scale, x.data_ptr<float>(), D == DT::F32 ? nullptr : static_cast<S*>(xb.data_ptr()));
+    auto go = [&](auto kern) {
+      hipLaunchKernelGGL(kern, dim3(T), dim3(rn::kThreads), 0, cur_stream(), static_cast<const S*>(table.data_ptr()),
+                         ids.data_ptr<int64_t>(), (int)table.size(0), (int)W, (float)scale, x.data_ptr<float>(),
+                         D == DT::F32 ? nullptr : static_cast<S*>(xb.data_ptr()));
+    };
+    if (vec) go(rn::embed_scale_kernel<D, true>);
+    else go(rn::embed_scale_kernel<D, false>);
   });
   SXE_LAUNCH_CHECK();
   return {x, xb};
