@@ -6,6 +6,11 @@
 //    weight). x, x' and every intermediate are fp32, y is the sublayer's output in the compute
 //    dtype; the 16-bit copy of x' the next projection reads is written in the same pass. Rows may be
 //    picked by index (the last-token rows before the LM head);
+//  * sandwich_norm: a sublayer with a norm on both sides and the next one's input in one pass,
+//    x' = x + rms(y) * wp [+ add], h = rms(x') * wn (plain weights); y may be the sum of several rows
+//    (expert outputs, one row per (token, expert));
+//  * embed_norm: x = rms(table[id]) * w and h = rms(x) * wn;
+//  * gated_rms_norm: rms(x) * w * sigmoid(gate) over whole rows;
 //  * qkv_norm_append: RMS norm over a token's WHOLE query projection and whole key projection (all
 //    heads at once, plain weights), the normalised q to [T, nq, Dq] and k, v to their paged cache
 //    slots, head rows zero-padded to the cache's row length.
@@ -117,6 +122,156 @@ __global__ __launch_bounds__(kThreads) void residual_rms_norm_kernel(
   }
 }
 
+struct SandwichArgs {
+  const float* x;        // [T, W] or nullptr (zero: embed_norm)
+  const void* y;         // [T, W], rows picked by ids (table) or summed over slots
+  const void *wp, *wn;   // norm weights after y and for h
+  const float* add;      // [T, W] or nullptr
+  const int* slots;      // [T, k] or nullptr
+  const int64_t* ids;    // rows of y, or nullptr
+  const int64_t* index;  // which rows to produce, or nullptr
+  float* xo;             // nullptr: not wanted
+  void* h;
+  int W, k, rows;        // rows: of y, for ids
+  float eps;
+};
+
+// C as in residual_rms_norm_kernel; C == 0 recomputes the sums in every pass
+template <DT T, int C>
+__global__ __launch_bounds__(kThreads) void sandwich_norm_kernel(SandwichArgs a) {
+  using S = typename dt_traits<T>::storage;
+  __shared__ float red[kThreads / 64];
+  const int W = a.W;
+  const int64_t o = blockIdx.x, r = a.index != nullptr ? a.index[o] : o;
+  const float* xr = a.x != nullptr ? a.x + r * W : nullptr;
+  const float* ar = a.add != nullptr ? a.add + r * W : nullptr;
+  int64_t y0 = r;
+  bool ok = true;
+  if (a.ids != nullptr) {
+    y0 = a.ids[r];
+    ok = y0 >= 0 && y0 < a.rows;
+    if (!ok) y0 = 0;
+  }
+  const S* yb = static_cast<const S*>(a.y);
+  const S *wp = static_cast<const S*>(a.wp), *wn = static_cast<const S*>(a.wn);
+  S* hr = static_cast<S*>(a.h) + o * W;
+  float ss = 0.f;
+  if constexpr (C > 0) {
+    f32x4 v[C];
+#pragma unroll
+    for (int i = 0; i < C; ++i) v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int k = a.slots != nullptr ? a.k : 1;
+    for (int j = 0; j < k; ++j) {
+      const S* yr = yb + (a.slots != nullptr ? (int64_t)a.slots[r * a.k + j] : y0) * W;
+#pragma unroll
+      for (int i = 0; i < C; ++i) {
+        const int c = (i * kThreads + threadIdx.x) * 4;
+        if (c < W && ok) v[i] += load4<T>(yr + c);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < C; ++i) ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
+    ss = block_sum<kThreads / 64>(ss, red);
+    const float rp = 1.f / sqrtf(ss / (float)W + a.eps);
+    ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < C; ++i) {
+      const int c = (i * kThreads + threadIdx.x) * 4;
+      if (c >= W) continue;
+      const f32x4 g = load4<T>(wp + c);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[i][j] = v[i][j] * rp * g[j];
+      if (xr != nullptr) v[i] += *reinterpret_cast<const f32x4*>(xr + c);
+      if (ar != nullptr) v[i] += *reinterpret_cast<const f32x4*>(ar + c);
+      if (a.xo != nullptr) *reinterpret_cast<f32x4*>(a.xo + o * W + c) = v[i];
+      ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
+    }
+    ss = block_sum<kThreads / 64>(ss, red);
+    const float rn = 1.f / sqrtf(ss / (float)W + a.eps);
+#pragma unroll
+    for (int i = 0; i < C; ++i) {
+      const int c = (i * kThreads + threadIdx.x) * 4;
+      if (c >= W) continue;
+      const f32x4 g = load4<T>(wn + c);
+      f32x4 h;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) h[j] = v[i][j] * rn * g[j];
+      store4<T>(hr + c, h);
+    }
+  } else {
+    auto ysum = [&](int c) {
+      if (a.slots == nullptr) return ok ? to_f32<T>(yb[y0 * W + c]) : 0.f;
+      float t = 0.f;
+      for (int j = 0; j < a.k; ++j) t += to_f32<T>(yb[(int64_t)a.slots[r * a.k + j] * W + c]);
+      return t;
+    };
+    for (int c = threadIdx.x; c < W; c += kThreads) {
+      const float t = ysum(c);
+      ss += t * t;
+    }
+    ss = block_sum<kThreads / 64>(ss, red);
+    const float rp = 1.f / sqrtf(ss / (float)W + a.eps);
+    auto sum = [&](int c) {
+      return ysum(c) * rp * to_f32<T>(wp[c]) + (xr != nullptr ? xr[c] : 0.f) + (ar != nullptr ? ar[c] : 0.f);
+    };
+    ss = 0.f;
+    for (int c = threadIdx.x; c < W; c += kThreads) {
+      const float t = sum(c);
+      ss += t * t;
+    }
+    ss = block_sum<kThreads / 64>(ss, red);
+    const float rn = 1.f / sqrtf(ss / (float)W + a.eps);
+    for (int c = threadIdx.x; c < W; c += kThreads) {
+      const float t = sum(c);
+      if (a.xo != nullptr) a.xo[o * W + c] = t;
+      hr[c] = from_f32<T>(t * rn * to_f32<T>(wn[c]));
+    }
+  }
+}
+
+// C as above, for the columns of x
+template <DT T, int C>
+__global__ __launch_bounds__(kThreads) void gated_rms_norm_kernel(const typename dt_traits<T>::storage* __restrict x,
+                                                                  const typename dt_traits<T>::storage* __restrict w,
+                                                                  const typename dt_traits<T>::storage* __restrict gate,
+                                                                  int64_t ldg, int W, float eps,
+                                                                  typename dt_traits<T>::storage* __restrict out) {
+  __shared__ float red[kThreads / 64];
+  const int64_t t = blockIdx.x;
+  const auto *xr = x + t * W, *gr = gate + t * ldg;
+  float ss = 0.f;
+  if constexpr (C > 0) {
+    f32x4 v[C];
+#pragma unroll
+    for (int i = 0; i < C; ++i) {
+      const int c = (i * kThreads + threadIdx.x) * 4;
+      v[i] = c < W ? load4<T>(xr + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+      ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
+    }
+    ss = block_sum<kThreads / 64>(ss, red);
+    const float rs = 1.f / sqrtf(ss / (float)W + eps);
+#pragma unroll
+    for (int i = 0; i < C; ++i) {
+      const int c = (i * kThreads + threadIdx.x) * 4;
+      if (c >= W) continue;
+      const f32x4 g = load4<T>(gr + c), q = load4<T>(w + c);
+      f32x4 h;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) h[j] = v[i][j] * rs * q[j] / (1.f + __expf(-g[j]));
+      store4<T>(out + t * W + c, h);
+    }
+  } else {
+    for (int c = threadIdx.x; c < W; c += kThreads) {
+      const float v = to_f32<T>(xr[c]);
+      ss += v * v;
+    }
+    ss = block_sum<kThreads / 64>(ss, red);
+    const float rs = 1.f / sqrtf(ss / (float)W + eps);
+    for (int c = threadIdx.x; c < W; c += kThreads)
+      out[t * W + c] = from_f32<T>(to_f32<T>(xr[c]) * rs * to_f32<T>(w[c]) / (1.f + __expf(-to_f32<T>(gr[c]))));
+  }
+}
+
 struct AppendArgs {
   const void* proj;  // [T, ld]: q | k | v (| anything) columns
   int64_t ld;
@@ -223,7 +378,120 @@ __global__ __launch_bounds__(kThreads) void qkv_norm_append_kernel(AppendArgs a)
 
 inline bool aligned(const void* p, size_t n) { return reinterpret_cast<uintptr_t>(p) % n == 0; }
 
+// chunks of 4 x kThreads columns held in registers, 0 for the scalar form
+inline int row_chunks(int64_t W, bool vec) {
+  const int64_t n = (W + 1023) / 1024;
+  return !vec || n > 16 ? 0 : n <= 1 ? 1 : n <= 2 ? 2 : n <= 4 ? 4 : n <= 8 ? 8 : 16;
+}
+
+template <DT D>
+void launch_sandwich(const SandwichArgs& a, int64_t rows, bool vec) {
+  auto go = [&](auto kern) { hipLaunchKernelGGL(kern, dim3(rows), dim3(kThreads), 0, cur_stream(), a); };
+  switch (row_chunks(a.W, vec)) {
+    case 1: go(sandwich_norm_kernel<D, 1>); break;
+    case 2: go(sandwich_norm_kernel<D, 2>); break;
+    case 4: go(sandwich_norm_kernel<D, 4>); break;
+    case 8: go(sandwich_norm_kernel<D, 8>); break;
+    case 16: go(sandwich_norm_kernel<D, 16>); break;
+    default: go(sandwich_norm_kernel<D, 0>); break;
+  }
+}
+
 }  // namespace rn
+
+// table [V, W], ids int64 [T], w and wn [W] like the table -> [x = rms(table[id]) w fp32, h = rms(x) wn]
+std::vector<at::Tensor> embed_norm(const at::Tensor& table, const at::Tensor& ids, const at::Tensor& w, const at::Tensor& wn,
+                                   double eps) {
+  SXE_CHECK_CUDA(table);
+  SXE_CHECK(table.dim() == 2 && table.is_contiguous(), "embed_norm: table [V, W] contiguous");
+  SXE_CHECK(ids.scalar_type() == at::kLong && ids.is_contiguous() && ids.is_cuda(), "embed_norm: ids int64 [T]");
+  const int64_t T = ids.numel(), W = table.size(1);
+  for (const auto* p : {&w, &wn})
+    SXE_CHECK(p->is_cuda() && p->is_contiguous() && p->numel() == W && p->scalar_type() == table.scalar_type(),
+              "embed_norm: norm weights [W] in the table's dtype");
+  auto x = at::empty({T, W}, table.options().dtype(at::kFloat)), h = at::empty({T, W}, table.options());
+  if (T == 0 || W == 0) return {x, h};
+  c10::DeviceGuard g(table.device());
+  rn::SandwichArgs a{nullptr, table.data_ptr(), w.data_ptr(), wn.data_ptr(), nullptr, nullptr, ids.data_ptr<int64_t>(),
+                     nullptr, x.data_ptr<float>(), h.data_ptr(), (int)W, 1, (int)table.size(0), (float)eps};
+  const bool vec = W % 4 == 0 && rn::aligned(table.data_ptr(), 16) && rn::aligned(w.data_ptr(), 16) &&
+                   rn::aligned(wn.data_ptr(), 16);
+  SXE_DISPATCH_DT(dtype_of(table), D, rn::launch_sandwich<D>(a, T, vec));
+  SXE_LAUNCH_CHECK();
+  return {x, h};
+}
+
+// x fp32 [T, W]; y [rows, W] in the weights' dtype, rows = T or, with slots int32 [T, k], any; add fp32 [T, W] or
+// None; index int64 [R] or None -> [x' fp32 [R, W] (empty without need_x), h [R, W]]
+std::vector<at::Tensor> sandwich_norm(const at::Tensor& x, const at::Tensor& y, const at::Tensor& wp, const at::Tensor& wn,
+                                      const c10::optional<at::Tensor>& slots, const c10::optional<at::Tensor>& add,
+                                      const c10::optional<at::Tensor>& index, double eps, bool need_x) {
+  SXE_CHECK_CUDA(x);
+  SXE_CHECK(x.dim() == 2 && x.is_contiguous() && x.scalar_type() == at::kFloat, "sandwich_norm: x fp32 [T, W]");
+  const int64_t T = x.size(0), W = x.size(1);
+  for (const auto* p : {&wp, &wn})
+    SXE_CHECK(p->is_cuda() && p->is_contiguous() && p->numel() == W && p->scalar_type() == y.scalar_type(),
+              "sandwich_norm: norm weights [W] in y's dtype");
+  const bool has_s = slots.has_value() && slots->defined(), has_a = add.has_value() && add->defined(),
+             has_i = index.has_value() && index->defined();
+  SXE_CHECK(y.is_cuda() && y.dim() == 2 && y.is_contiguous() && y.size(1) == W && (has_s || y.size(0) == T),
+            "sandwich_norm: y [T, W]");
+  if (has_s)
+    SXE_CHECK(slots->is_cuda() && slots->scalar_type() == at::kInt && slots->is_contiguous() && slots->dim() == 2 &&
+                  slots->size(0) == T && slots->size(1) * T <= y.size(0), "sandwich_norm: slots int32 [T, k] of y's rows");
+  if (has_a)
+    SXE_CHECK(add->is_cuda() && add->scalar_type() == at::kFloat && add->is_contiguous() && add->sizes() == x.sizes(),
+              "sandwich_norm: add like x");
+  if (has_i)
+    SXE_CHECK(index->scalar_type() == at::kLong && index->is_contiguous() && index->is_cuda(), "sandwich_norm: index int64 [R]");
+  const int64_t R = has_i ? index->numel() : T;
+  auto xo = need_x ? at::empty({R, W}, x.options()) : at::empty({0}, x.options());
+  auto h = at::empty({R, W}, y.options());
+  if (R == 0 || W == 0) return {xo, h};
+  c10::DeviceGuard g(x.device());
+  rn::SandwichArgs a{x.data_ptr<float>(), y.data_ptr(), wp.data_ptr(), wn.data_ptr(), has_a ? add->data_ptr<float>() : nullptr,
+                     has_s ? slots->data_ptr<int>() : nullptr, nullptr, has_i ? index->data_ptr<int64_t>() : nullptr,
+                     need_x ? xo.data_ptr<float>() : nullptr, h.data_ptr(), (int)W, has_s ? (int)slots->size(1) : 1,
+                     (int)y.size(0), (float)eps};
+  bool vec = W % 4 == 0 && rn::aligned(a.x, 16) && rn::aligned(a.y, 16) && rn::aligned(a.wp, 16) && rn::aligned(a.wn, 16) &&
+             (!has_a || rn::aligned(a.add, 16));
+  SXE_DISPATCH_DT(dtype_of(y), D, rn::launch_sandwich<D>(a, R, vec));
+  SXE_LAUNCH_CHECK();
+  return {xo, h};
+}
+
+// x [T, N] contiguous, w [N], gate [T, N] (rows may be strided), one dtype -> rms(x) w sigmoid(gate)
+at::Tensor gated_rms_norm(const at::Tensor& x, const at::Tensor& w, const at::Tensor& gate, double eps) {
+  SXE_CHECK_CUDA(x);
+  SXE_CHECK(x.dim() == 2 && x.is_contiguous(), "gated_rms_norm: x [T, N]");
+  const int64_t T = x.size(0), W = x.size(1);
+  SXE_CHECK(w.is_cuda() && w.is_contiguous() && w.numel() == W && w.scalar_type() == x.scalar_type(), "gated_rms_norm: w [N]");
+  SXE_CHECK(gate.is_cuda() && gate.dim() == 2 && gate.size(0) == T && gate.size(1) == W && gate.stride(1) == 1 &&
+                gate.scalar_type() == x.scalar_type(), "gated_rms_norm: gate [T, N]");
+  auto out = at::empty_like(x);
+  if (T == 0 || W == 0) return out;
+  c10::DeviceGuard g(x.device());
+  const bool vec = W % 4 == 0 && gate.stride(0) % 4 == 0 && rn::aligned(x.data_ptr(), 16) && rn::aligned(w.data_ptr(), 16) &&
+                   rn::aligned(gate.data_ptr(), x.element_size() * 4);
+  SXE_DISPATCH_DT(dtype_of(x), D, {
+    using S = dt_traits<D>::storage;
+    auto go = [&](auto kern) {
+      hipLaunchKernelGGL(kern, dim3(T), dim3(rn::kThreads), 0, cur_stream(), static_cast<const S*>(x.data_ptr()),
+                         static_cast<const S*>(w.data_ptr()), static_cast<const S*>(gate.data_ptr()), gate.stride(0), (int)W,
+                         (float)eps, static_cast<S*>(out.data_ptr()));
+    };
+    switch (rn::row_chunks(W, vec)) {
+      case 1: go(rn::gated_rms_norm_kernel<D, 1>); break;
+      case 2: go(rn::gated_rms_norm_kernel<D, 2>); break;
+      case 4: go(rn::gated_rms_norm_kernel<D, 4>); break;
+      case 8: go(rn::gated_rms_norm_kernel<D, 8>); break;
+      case 16: go(rn::gated_rms_norm_kernel<D, 16>); break;
+      default: go(rn::gated_rms_norm_kernel<D, 0>); break;
+    }
+  });
+  SXE_LAUNCH_CHECK();
+  return out;
+}
 
 // table [V, W], ids int64 [T] -> [x fp32 [T, W], 16-bit copy (x itself for an fp32 table)]
 std::vector<at::Tensor> embed_scale(const at::Tensor& table, const at::Tensor& ids, double scale) {
@@ -276,8 +544,7 @@ std::vector<at::Tensor> residual_rms_norm(const at::Tensor& x, const c10::option
   c10::DeviceGuard g(x.device());
   const bool vec = W % 4 == 0 && rn::aligned(x.data_ptr(), 16) && rn::aligned(w.data_ptr(), 16) &&
                    (!has_y || rn::aligned(y->data_ptr(), 16));
-  const int64_t chunks = (W + 1023) / 1024;
-  const int C = !vec || chunks > 16 ? 0 : chunks <= 1 ? 1 : chunks <= 2 ? 2 : chunks <= 4 ? 4 : chunks <= 8 ? 8 : 16;
+  const int C = rn::row_chunks(W, vec);
   SXE_DISPATCH_DT(dt, D, {
     using S = dt_traits<D>::storage;
     auto go = [&](auto kern) {
@@ -342,11 +609,18 @@ TORCH_LIBRARY_FRAGMENT(sxe, m) {
   m.def("embed_scale(Tensor table, Tensor ids, float scale) -> Tensor[]");
   m.def("residual_rms_norm(Tensor x, Tensor? y, Tensor w, Tensor? index, float alpha, float eps, float offset, "
         "bool need_x) -> Tensor[]");
+  m.def("embed_norm(Tensor table, Tensor ids, Tensor w, Tensor wn, float eps) -> Tensor[]");
+  m.def("sandwich_norm(Tensor x, Tensor y, Tensor wp, Tensor wn, Tensor? slots, Tensor? add, Tensor? index, float eps, "
+        "bool need_x) -> Tensor[]");
+  m.def("gated_rms_norm(Tensor x, Tensor w, Tensor gate, float eps) -> Tensor");
   m.def("qkv_norm_append(Tensor proj, Tensor qw, Tensor kw, Tensor(a!) kc, Tensor(b!) vc, Tensor slots, int nq, int nkv, "
         "int dk, int dv, float eps) -> Tensor");
 }
 TORCH_LIBRARY_IMPL(sxe, CUDA, m) {
   m.impl("embed_scale", &sxe::embed_scale);
   m.impl("residual_rms_norm", &sxe::residual_rms_norm);
+  m.impl("embed_norm", &sxe::embed_norm);
+  m.impl("sandwich_norm", &sxe::sandwich_norm);
+  m.impl("gated_rms_norm", &sxe::gated_rms_norm);
   m.impl("qkv_norm_append", &sxe::qkv_norm_append);
 }

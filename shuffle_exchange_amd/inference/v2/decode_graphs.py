@@ -10,12 +10,12 @@ while the HBM time of the step is ~2 ms. The reference captures CUDA graphs only
   first use and sharing one memory pool;
 * all per-step metadata (token ids, positions, cache slots, block tables, lengths) lives in static
   device buffers refreshed by one pinned H2D copy per dtype before ``replay()``;
-* padding sequences point at a reserved scratch KV block (q_len = kv_len = 1), so every row the
-  graph computes is well defined and no real cache slot is touched;
+* padding sequences point at a reserved scratch KV block and state slot (q_len = kv_len = 1), so every
+  row the graph computes is well defined and no real cache slot is touched;
 * the paged-attention grid is fixed per graph by the KV bucket (splits of >= 256 keys, workgroups
   past a sequence's length exit at once).
 
-MoE models (data-dependent expert counts) and sliding windows narrower than the KV bucket run
+MoE models whose expert counts go through the host and sliding windows narrower than the KV bucket run
 eagerly.
 """
 import torch
@@ -38,12 +38,12 @@ class _StaticBatch:
         self.max_blocks = max_blocks
         self.max_kv_len = kv_bucket
         self.d64 = torch.zeros(4 * S, dtype=torch.int64, device=device)
-        self.d32 = torch.zeros(3 * S + S * max_blocks, dtype=torch.int32, device=device)
+        self.d32 = torch.zeros(4 * S + S * max_blocks, dtype=torch.int32, device=device)
         self.h64 = torch.zeros(4 * S, dtype=torch.int64, pin_memory=True)
-        self.h32 = torch.zeros(3 * S + S * max_blocks, dtype=torch.int32, pin_memory=True)
+        self.h32 = torch.zeros(4 * S + S * max_blocks, dtype=torch.int32, pin_memory=True)
         self.input_ids, self.positions, self.slots, self.last_idx = self.d64.view(4, S).unbind(0)
-        self.q_start, self.q_len, self.kv_len = self.d32[:3 * S].view(3, S).unbind(0)
-        self.block_table = self.d32[3 * S:].view(S, max_blocks)
+        self.q_start, self.q_len, self.kv_len, self.state_slots = self.d32[:4 * S].view(4, S).unbind(0)
+        self.block_table = self.d32[4 * S:].view(S, max_blocks)
         # host views read by the attention dispatch: no pure prefill, every row one query token
         self.host_seen = [1] * S
         self.host_q_len = [1] * S
@@ -59,6 +59,12 @@ class DecodeGraphRunner:
         self.max_context = max_context
         self.bs = kv_cache.block_size
         self.scratch_block = int(kv_cache.reserve(1)[0])
+        self.scratch_state = -1
+        if kv_cache.states is not None:
+            self.scratch_state = kv_cache.states.reserve()
+            for t in kv_cache.states.layers:
+                if t is not None:
+                    t[self.scratch_state].zero_()
         self._graphs = {}
         self._pool = None
         self.replays = 0
@@ -102,8 +108,8 @@ class DecodeGraphRunner:
         S, mb, bs = sb.num_seqs, sb.max_blocks, self.bs
         h64, h32 = sb.h64.view(4, S), sb.h32
         ids, pos, slots, last = h64.unbind(0)
-        qs, ql, kl = h32[:3 * S].view(3, S).unbind(0)
-        bt = h32[3 * S:].view(S, mb)
+        qs, ql, kl, ss = h32[:4 * S].view(4, S).unbind(0)
+        bt = h32[4 * S:].view(S, mb)
         scratch_slot = self.scratch_block * bs
         ids.zero_()
         pos.zero_()
@@ -112,13 +118,14 @@ class DecodeGraphRunner:
         qs.copy_(torch.arange(S, dtype=torch.int32))
         ql.fill_(1)
         kl.fill_(1)
+        ss.fill_(self.scratch_state)
         bt.fill_(self.scratch_block)
         for i, (s, t) in enumerate(zip(seqs, tokens)):
             p = s.seen_tokens
             ids[i] = int(t.reshape(-1)[0])
             pos[i] = p
             slots[i] = s.blocks[p // bs] * bs + p % bs
-            kl[i] = p + 1
+            kl[i], ss[i] = p + 1, s.state_slot
             nb = len(s.blocks)
             bt[i, :nb] = torch.tensor(s.blocks, dtype=torch.int32)
         sb.d64.copy_(sb.h64, non_blocking=True)
@@ -133,7 +140,12 @@ class DecodeGraphRunner:
         side = torch.cuda.Stream()
         side.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(side), torch.no_grad():
-            self.model.forward(sb, self.kv)  # warm-up: lazy inits, hipBLASLt heuristics; same KV writes as replay
+            # warm-up: lazy inits, hipBLASLt heuristics. KV writes land where the replay writes again; a
+            # recurrent state must advance once only, so this pass works on the scratch slot
+            slots = sb.state_slots.clone()
+            sb.state_slots.fill_(self.scratch_state)
+            self.model.forward(sb, self.kv)
+            sb.state_slots.copy_(slots)
         torch.cuda.current_stream().wait_stream(side)
         graph = torch.cuda.CUDAGraph()
         with torch.cuda.graph(graph, pool=self._pool), torch.no_grad():

@@ -19,7 +19,7 @@ from typing import Optional
 
 import torch
 
-from .ragged.ragged import BlockedKVCache, DSStateManager, RaggedBatch
+from .ragged.ragged import BlockedKVCache, DSStateManager, RaggedBatch, RecurrentStates
 
 
 class SchedulingResult(Enum):
@@ -59,6 +59,7 @@ class RaggedInferenceEngineConfig:
     state_manager: StateManagerConfig = field(default_factory=StateManagerConfig)
     kv_block_size: int = 64
     num_kv_blocks: Optional[int] = None
+    num_state_slots: Optional[int] = None  # recurrent layers: sequences that can hold a state (default: from memory)
     tensor_parallel: dict = field(default_factory=lambda: {"tp_size": 1})
     decode_graphs: bool = True  # replay pure-decode steps from captured HIP graphs (decode_graphs.py)
     weight_quant: Optional[str] = None  # "fp8" (W8A16) | "fp6" / "wf6af16" (FP6-LLM) | "fp4": weight-only decode GEMMs
@@ -101,9 +102,11 @@ class InferenceEngineV2:
         sm = self._config.state_manager
         dev = self._model.device
         bs = self._config.kv_block_size
+        states = self._make_states(dev, sm)
         nblocks = self._config.num_kv_blocks or self._size_cache(dev, bs)
         self._kv = BlockedKVCache(self._model.num_layers, nblocks, bs, dtype=self._model.dtype, device=dev,
                                   **self._cache_geometry())
+        self._kv.states = states
         max_blocks_seq = math.ceil(sm.max_context / bs)
         self._state = DSStateManager(self._kv, sm.max_tracked_sequences, max_blocks_seq)
         self._decode_graphs = None
@@ -114,19 +117,30 @@ class InferenceEngineV2:
             return {"layer_shapes": m.kv_shapes}
         return {"n_kv_heads": m.nkv, "head_dim": m.head_dim}
 
-    def _size_cache(self, dev, bs):
-        m = self._model
+    def _make_states(self, dev, sm):
+        """State slots of recurrent layers (None for a model without any): one per sequence that may be
+        tracked and one for padded graph rows, within a quarter of the memory budget."""
+        shapes = getattr(self._model, "state_shapes", None)
+        if shapes is None or all(s is None for s in shapes):
+            return None
+        per_slot = RecurrentStates.bytes_per_slot(shapes)
+        n = self._config.num_state_slots or max(1, min(sm.max_tracked_sequences, self._memory_budget(dev) // 4 // per_slot))
+        return RecurrentStates(shapes, int(n) + 1, device=dev)
+
+    def _memory_budget(self, dev):
         mc = self._config.state_manager.memory_config
         if dev.type != "cuda":
-            budget = 64 * 2**20
-        else:
-            free, _ = torch.cuda.mem_get_info(dev)
-            if mc.fraction is not None:
-                budget = int(free * mc.fraction)
-            elif mc.mode == "allocate":
-                budget = mc.size
-            else:
-                budget = max(0, free - mc.size)
+            return 64 * 2**20
+        free, _ = torch.cuda.mem_get_info(dev)
+        if mc.fraction is not None:
+            return int(free * mc.fraction)
+        if mc.mode == "allocate":
+            return mc.size
+        return max(0, free - mc.size)
+
+    def _size_cache(self, dev, bs):
+        m = self._model
+        budget = self._memory_budget(dev)
         return BlockedKVCache.blocks_for_budget(budget, m.num_layers, bs, dtype=m.dtype, **self._cache_geometry())
 
     # ------------------------------------------------------------------------------------ API
@@ -174,12 +188,14 @@ class InferenceEngineV2:
         return logits
 
     def _decode_runner(self):
-        """HIP-graph decode runner (decode_graphs.py), created on first use: GPU, dense models."""
+        """HIP-graph decode runner (decode_graphs.py), created on first use: GPU; dense models and those whose
+        expert routing stays on the device (``device_routing``)."""
         if self._decode_graphs is None:
             m = self._model
-            dense = not getattr(m, "is_moe", False) and not any(
-                "router" in L for L in getattr(m, "w", {}).get("layers", []))
+            dense = getattr(m, "device_routing", False) or (not getattr(m, "is_moe", False) and not any(
+                "router" in L for L in getattr(m, "w", {}).get("layers", [])))
             ok = (self._config.decode_graphs and m.device.type == "cuda" and dense and self._kv.free_blocks > 1
+                  and (self._kv.states is None or self._kv.states.free_slots > 0)
                   and self._tp == 1)  # collectives stay outside graph capture
             if ok:
                 from .decode_graphs import DecodeGraphRunner
@@ -206,6 +222,8 @@ class InferenceEngineV2:
         sm = self._config.state_manager
         new_seqs = sum(1 for u in uids if self._state.get_sequence(u) is None)
         if self._state.n_tracked_sequences + new_seqs > sm.max_tracked_sequences:
+            return SchedulingResult.EngineSequenceLimitExceeded
+        if self._kv.states is not None and new_seqs > self._kv.states.free_slots:
             return SchedulingResult.EngineSequenceLimitExceeded
         if len(uids) > sm.max_ragged_sequence_count:
             return SchedulingResult.BatchSequenceLimitExceeded

@@ -2,19 +2,29 @@
 per layer), served from the paged cache like the other families.
 
 Where ``hf_decoder.py`` describes a whole model with one set of sizes, here a ``LayeredSpec`` holds one
-``LayerSpec`` per layer: head counts, key and value sizes, window and feed-forward width may differ
-from layer to layer, and the KV cache takes its geometry per layer from ``kv_shapes``. The residual
-stream is 32-bit. Mechanisms are ops with parameters (ops/mix_attention.py, ops/residual_norm.py), and
-an architecture is one entry of ``ARCHITECTURES``: a function from its config to the spec plus a function
-from its checkpoint tensors to the packed layout:
-  * q | k | v | output gate -> ONE projection weight [nq dk + nkv (dk + dv) + nq dv, width];
+``LayerSpec`` per layer: mixer kind, head counts, key and value sizes, window and feed-forward may differ
+from layer to layer, and the cache takes its geometry per layer from ``kv_shapes`` (paged rows) and
+``state_shapes`` (recurrent state of a sequence). The residual stream is 32-bit. Mechanisms are ops with
+parameters (ops/mix_attention.py, ops/latent_attention.py, ops/linear_attention.py, ops/moe.py,
+ops/residual_norm.py), and an architecture is one entry of ``ARCHITECTURES``: a function from its config to
+the spec plus a function from its checkpoint tensors to the packed layout:
+  * projections of one input -> ONE weight (q | k | v | output gate; query latent | latent | key part);
   * gate | up -> one [2 ff, width] weight, ff zero-padded to a multiple of 16 (exact: the padding
-    contributes silu(0) * 0);
-  * per-head attention numbers as fp32 (ops/mix_attention.MixParams).
+    contributes silu(0) * 0); experts stacked [E, ff, width] / [E, width, ff];
+  * per-head attention numbers as fp32.
 
-Tobinex: x = embed * scale; per layer x <- norm1(alpha x + attention(x)), x <- norm2(alpha x + ff(x)), RMS
-norms with weights stored around zero, q / k norms over the whole projection, no rotation, distance
-bias, window with kept first tokens, softmax sink, talking heads, output gate, SwiGLU, tied LM head.
+Two residual forms (``LayeredSpec.residual``):
+  * "after": x <- norm(alpha x + sublayer(x));
+  * "sandwich": x <- x + norm_b(sublayer(norm_a(x))).
+``loop`` runs a range of layers several times with the same weights; every pass is a layer run of its own
+with its own cache or state, so ``num_layers`` counts runs.
+
+Tobinex: x = embed * scale; "after" with RMS norms stored around zero; q / k norms over the whole
+projection, no rotation, distance bias, window with kept first tokens, softmax sink, talking heads, output
+gate, SwiGLU, tied LM head.
+Bipotar: normed embedding; "sandwich" with plain RMS norms; linear attention with a decayed state or windowed
+latent attention; SwiGLU or routed experts with squared relu; a loop that adds the embedding output ahead of
+every pass but the first; separate scaled LM head.
 """
 import json
 import os
@@ -24,9 +34,13 @@ from typing import List, Optional
 import torch
 
 from ....ops.activation import gated_act
+from ....ops.latent_attention import latent_append, latent_attention, latent_row, rotation_table
 from ....ops.linear import fused_addnorm_linear, fused_gatesum_linear, fused_swiglu_linear, linear
+from ....ops.linear_attention import decay_attention, decay_table
 from ....ops.mix_attention import MixParams, cache_row, mix_attention, mix_attention_parts
-from ....ops.residual_norm import embed_scale, qkv_norm_append, residual_rms_norm
+from ....ops.moe import expert_mlp, route_topk
+from ....ops.residual_norm import (embed_norm, embed_scale, gated_rms_norm, qkv_norm_append, residual_rms_norm,
+                                   sandwich_norm)
 
 FF_MULTIPLE = 16
 
@@ -43,10 +57,52 @@ class AttentionSpec:
 
 
 @dataclass
+class LatentSpec:
+    """Keys and values from a cached latent (ops/latent_attention.py)."""
+    heads: int
+    dim: int                       # unrotated query / key size of a head
+    rot_dim: int                   # rotated query size of a head; one rotated key part for all heads
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot_base: float
+    window: Optional[int] = None
+
+
+@dataclass
+class LinearSpec:
+    """Linear attention with a decayed state (ops/linear_attention.py)."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: List[float] = field(default_factory=list)
+
+
+MIXERS = {c.__name__: c for c in (AttentionSpec, LatentSpec, LinearSpec)}
+
+
+@dataclass
+class MoESpec:
+    experts: int
+    top: int
+    ff: int
+    act: str = "relu2"
+
+
+@dataclass
 class LayerSpec:
-    mixer: AttentionSpec
-    ff: int = 0                    # 0: no feed-forward
+    mixer: object                  # one of MIXERS
+    ff: int = 0                    # 0: no dense feed-forward
     act: str = "silu"
+    moe: Optional[MoESpec] = None
+
+
+@dataclass
+class LoopSpec:
+    start: int
+    stop: int
+    times: int
 
 
 @dataclass
@@ -55,15 +111,56 @@ class LayeredSpec:
     vocab_size: int
     width: int
     eps: float
-    alpha: float                   # residual factor of the norm-after-sum layers
+    alpha: float = 1.0             # residual factor of the norm-after-sum layers
     embed_scale: float = 1.0
     norm_offset: float = 1.0       # 1: norm weights stored around zero; 0: plain
     layers: List[LayerSpec] = field(default_factory=list)
+    residual: str = "after"        # "after" | "sandwich"
+    loop: Optional[LoopSpec] = None
+    logit_scale: float = 1.0
+
+    def runs(self):
+        """[(layer index, whether the embedding output is added to x ahead of it)] in the order they run."""
+        n = len(self.layers)
+        if self.loop is None:
+            return [(i, False) for i in range(n)]
+        a, b = self.loop.start, self.loop.stop
+        out = [(i, False) for i in range(a)]
+        for t in range(self.loop.times):
+            out += [(i, t > 0 and i == a) for i in range(a, b)]
+        return out + [(i, False) for i in range(b, n)]
+
+    def to_dict(self):
+        from dataclasses import asdict
+        d = asdict(self)
+        for x, L in zip(d["layers"], self.layers):
+            x["mixer_kind"] = type(L.mixer).__name__
+        return d
 
     @classmethod
     def from_dict(cls, d):
-        layers = [LayerSpec(**{**x, "mixer": AttentionSpec(**x["mixer"])}) for x in d["layers"]]
-        return cls(**{**d, "layers": layers})
+        layers = []
+        for x in d["layers"]:
+            x = dict(x)
+            kind, moe = MIXERS[x.pop("mixer_kind", "AttentionSpec")], x.get("moe")
+            layers.append(LayerSpec(**{**x, "mixer": kind(**x["mixer"]), "moe": MoESpec(**moe) if moe else None}))
+        return cls(**{**d, "layers": layers, "loop": LoopSpec(**d["loop"]) if d.get("loop") else None})
+
+
+def checkpoint_tensor(sd, name, *shape):
+    if name not in sd:
+        raise KeyError(f"missing checkpoint tensor {name}")
+    if tuple(sd[name].shape) != shape:
+        raise ValueError(f"{name}: shape {tuple(sd[name].shape)}, the configuration says {shape}")
+    return sd[name]
+
+
+def pack_dense_ff(get, p, ff, width):
+    """SwiGLU weights: gate | up in one, ff zero-padded."""
+    pad = -ff % FF_MULTIPLE
+    rows = (lambda w: torch.nn.functional.pad(w, (0, 0, 0, pad)))
+    return {"gu": torch.cat([rows(get(p + "gate", ff, width)), rows(get(p + "up", ff, width))]),
+            "down": torch.nn.functional.pad(get(p + "down", width, ff), (0, pad))}
 
 
 # ------------------------------------------------------------------------------------- Tobinex
@@ -87,11 +184,7 @@ def _tobinex_spec(c):
 
 def _tobinex_weights(spec, sd):
     def get(name, *shape):
-        if name not in sd:
-            raise KeyError(f"missing checkpoint tensor {name}")
-        if tuple(sd[name].shape) != shape:
-            raise ValueError(f"{name}: shape {tuple(sd[name].shape)}, the configuration says {shape}")
-        return sd[name]
+        return checkpoint_tensor(sd, name, *shape)
     H = spec.width
     W = {"embed": get("embed", spec.vocab_size, H), "final": get("final.norm", H), "layers": []}
     for i, L in enumerate(spec.layers):
@@ -104,17 +197,87 @@ def _tobinex_weights(spec, sd):
              "r1": get(p + "r1", nq).float(), "r2": get(p + "r2", nq).float(), "sink": get(p + "sink", nq).float(),
              "talk": get(p + "talk", nq, nq).float()}
         if L.ff:
-            p, pad = f"l{i}.mlp.", -L.ff % FF_MULTIPLE
-            rows = (lambda w: torch.nn.functional.pad(w, (0, 0, 0, pad)))
             d["norm2"] = get(f"l{i}.norm2", H)
-            d["gu"] = torch.cat([rows(get(p + "gate", L.ff, H)), rows(get(p + "up", L.ff, H))])
-            d["down"] = torch.nn.functional.pad(get(p + "down", H, L.ff), (0, pad))
+            d.update(pack_dense_ff(get, f"l{i}.mlp.", L.ff, H))
+        W["layers"].append(d)
+    return W
+
+
+# ------------------------------------------------------------------------------------- Bipotar
+def _bipotar_mixer(i, kind, m):
+    if kind == "lightning":
+        if len(m["decay"]) != m["heads"]:
+            raise ValueError(f"layer {i}: {len(m['decay'])} decays for {m['heads']} heads")
+        return LinearSpec(int(m["heads"]), int(m["dim"]), int(m["vdim"]), [float(d) for d in m["decay"]])
+    if kind == "latent_attention":
+        if m["rot"]["dims"] != m["rot_dim"] or m["rot_dim"] % 2:
+            raise ValueError(f"layer {i}: rotation over {m['rot']['dims']} of {m['rot_dim']} rotated dimensions")
+        size = (m.get("mask") or {}).get("size")
+        return LatentSpec(int(m["heads"]), int(m["dim"]), int(m["rot_dim"]), int(m["vdim"]), int(m["q_rank"]),
+                          int(m["kv_rank"]), float(m["scale"]), float(m["rot"]["base"]), None if size is None else int(size))
+    raise NotImplementedError(f"layer {i}: mixer type {kind!r}")
+
+
+def _bipotar_spec(c):
+    layers = []
+    for i, L in enumerate(c["layers"]):
+        f = L.get("mlp") or {"kind": "dense", "ff": 0}
+        layer = LayerSpec(_bipotar_mixer(i, L["type"], L["mixer"]))
+        if f["kind"] == "dense":
+            layer.ff = int(f["ff"])
+        elif f["kind"] == "moe":
+            layer.moe = MoESpec(int(f["router"]["experts"]), int(f["router"]["top"]), int(f["expert"]["ff"]))
+            if not 0 < layer.moe.top <= layer.moe.experts:
+                raise ValueError(f"layer {i}: {layer.moe.top} of {layer.moe.experts} experts")
+        else:
+            raise NotImplementedError(f"layer {i}: feed-forward kind {f['kind']!r}")
+        layers.append(layer)
+    loop = c.get("loop")
+    if loop is not None:
+        loop = LoopSpec(int(loop["start"]), int(loop["stop"]), int(loop["times"]))
+        if not 0 <= loop.start <= loop.stop <= len(layers):
+            raise ValueError(f"loop over layers {loop.start} .. {loop.stop - 1} of {len(layers)}")
+    return LayeredSpec(c["architecture"], int(c["vocab"]), int(c["width"]), float(c["norm"]["eps"]), norm_offset=0.0,
+                       layers=layers, residual="sandwich", loop=loop, logit_scale=float(c["logit_scale"]))
+
+
+def _bipotar_weights(spec, sd):
+    def get(name, *shape):
+        return checkpoint_tensor(sd, name, *shape)
+    D, V = spec.width, spec.vocab_size
+    W = {"embed": get("embed", V, D), "embed_norm": get("embed.norm", D), "final": get("final.norm", D),
+         "head": get("head", V, D), "layers": []}
+    for i, L in enumerate(spec.layers):
+        a, p = L.mixer, f"l{i}.mix."
+        d = {"norm1": get(f"l{i}.norm1", D), "norm1b": get(f"l{i}.norm1b", D)}
+        if isinstance(a, LinearSpec):
+            kd, vd = a.heads * a.dim, a.heads * a.vdim
+            d["qkvg"] = torch.cat([get(p + "q", kd, D), get(p + "k", kd, D), get(p + "v", vd, D), get(p + "g", vd, D)])
+            d["o_norm"], d["o"], d["decay"] = get(p + "norm", vd), get(p + "o", D, vd), decay_table(a.decay)
+        else:
+            H, R = a.heads, a.kv_rank
+            uk, uv = get(p + "uk", H * a.dim, R), get(p + "uv", H * a.vdim, R)
+            d["dqkv"] = torch.cat([get(p + "dq", a.q_rank, D), get(p + "dkv", R + a.rot_dim, D)])
+            d["q_norm"], d["kv_norm"] = get(p + "dq.norm", a.q_rank), get(p + "dkv.norm", R)
+            d["uq"], d["o"] = get(p + "uq", H * (a.dim + a.rot_dim), a.q_rank), get(p + "o", D, H * a.vdim)
+            d["uk"], d["uv"] = uk.view(H, a.dim, R), uv.view(H, a.vdim, R).transpose(1, 2)
+            d["ukv"] = torch.cat([uk, uv])
+        if L.ff or L.moe:
+            p = f"l{i}.mlp."
+            d["norm2"], d["norm2b"] = get(f"l{i}.norm2", D), get(f"l{i}.norm2b", D)
+            if L.ff:
+                d.update(pack_dense_ff(get, p, L.ff, D))
+            else:
+                E, F = L.moe.experts, L.moe.ff
+                d["router"] = get(p + "router", E, D)
+                d["e_up"] = torch.stack([get(f"{p}e{e}.up", F, D) for e in range(E)])
+                d["e_down"] = torch.stack([get(f"{p}e{e}.down", D, F) for e in range(E)])
         W["layers"].append(d)
     return W
 
 
 # architecture name in config.json -> (config dict -> LayeredSpec, (spec, state dict) -> packed weights)
-ARCHITECTURES = {"Tobinex": (_tobinex_spec, _tobinex_weights)}
+ARCHITECTURES = {"Tobinex": (_tobinex_spec, _tobinex_weights), "Bipotar": (_bipotar_spec, _bipotar_weights)}
 
 
 def is_layered_config(cfg):
@@ -126,8 +289,9 @@ class RaggedLayeredDecoder:
     """Engine-facing model (InferenceEngineV2 protocol: num_layers / kv_shapes / dtype / device /
     vocab_size / forward(batch, kv_cache) -> fp32 logits of ``batch.last_idx``)."""
 
-    FP32_KEYS = ("r1", "r2", "sink", "talk")   # never rounded to the compute dtype
-    QUANT_KEYS = ("qkvg", "o", "gu", "down")
+    FP32_KEYS = ("r1", "r2", "sink", "talk", "decay")   # never rounded to the compute dtype
+    QUANT_KEYS = ("qkvg", "dqkv", "uq", "o", "gu", "down")
+    device_routing = True   # expert counts never go through the host: decode steps can be captured
 
     def __init__(self, spec: LayeredSpec, weights, dtype=torch.bfloat16, device=None, weight_quant=None):
         if dtype not in (torch.bfloat16, torch.float32):
@@ -151,16 +315,28 @@ class RaggedLayeredDecoder:
     def _finish(self):
         s = self.spec
         self.tp, self.tp_rank = 1, 0
-        self.num_layers, self.vocab_size = len(s.layers), s.vocab_size
-        self.kv_shapes = []
-        for L in s.layers:  # one row length for k and v of a layer: the matrix-core kernels take one
-            a = L.mixer
-            dk, dv = cache_row(a.dim, self._dtype), cache_row(a.vdim, self._dtype)
-            if dk != a.dim or dv != a.vdim or self._dtype == torch.bfloat16:
-                dk = dv = max(dk, dv)
-            self.kv_shapes.append((a.kv_heads, dk, dv))
-        self._mix = [MixParams(L["r1"], L["r2"], L["sink"], L["talk"]) for L in self.w["layers"]]
+        self.runs = s.runs()
+        self.num_layers, self.vocab_size = len(self.runs), s.vocab_size
+        self.kv_shapes = [self._kv_shape(s.layers[i].mixer) for i, _ in self.runs]
+        self.state_shapes = [self._state_shape(s.layers[i].mixer) for i, _ in self.runs]
+        self._mix = [MixParams(L["r1"], L["r2"], L["sink"], L["talk"]) if "r1" in L else None for L in self.w["layers"]]
         self.model = self
+
+    def _kv_shape(self, a):
+        """(kv heads, k row, v row) of a layer's paged cache."""
+        if isinstance(a, LinearSpec):
+            return (0, 0, 0)
+        if isinstance(a, LatentSpec):
+            return (1, sum(latent_row(a.kv_rank, a.rot_dim, self._dtype)), 0)
+        # one row length for k and v of a layer: the matrix-core kernels take one
+        dk, dv = cache_row(a.dim, self._dtype), cache_row(a.vdim, self._dtype)
+        if dk != a.dim or dv != a.vdim or self._dtype == torch.bfloat16:
+            dk = dv = max(dk, dv)
+        return (a.kv_heads, dk, dv)
+
+    @staticmethod
+    def _state_shape(a):
+        return (a.heads, a.dim, a.vdim) if isinstance(a, LinearSpec) else None
 
     @classmethod
     def restore(cls, spec, w, dtype, device, weight_quant=None):
@@ -233,6 +409,8 @@ class RaggedLayeredDecoder:
 
     @torch.no_grad()
     def forward(self, batch, kv_cache):
+        if self.spec.residual == "sandwich":
+            return self._forward_sandwich(batch, kv_cache)
         s, W = self.spec, self.w
         x, xb = embed_scale(W["embed"], batch.input_ids, s.embed_scale)
         pending = None  # the last sublayer's (output, norm weight), not yet added to x
@@ -250,13 +428,70 @@ class RaggedLayeredDecoder:
         _, h = residual_rms_norm(x, None, W["final"], 1.0, s.eps, s.norm_offset, index=batch.last_idx, need_x=False)
         return linear(h, W["embed"]).float()
 
+    # ------------------------------------------------------------------------- norm on both sides
+    def _linear_mixer(self, h, L, a, run, batch, kv_cache):
+        """Decayed linear attention; ``h`` the normed input [T, width]."""
+        proj = linear(h, L["qkvg"])
+        o = decay_attention(proj, kv_cache.layer_state(run), L["decay"], batch, a.heads, a.dim, a.vdim)
+        return linear(gated_rms_norm(o, L["o_norm"], proj[:, a.heads * (2 * a.dim + a.vdim):], self.spec.eps), L["o"])
+
+    def _latent_mixer(self, h, L, a, run, batch, kv_cache):
+        cache = kv_cache.layer_kv(run)[0]
+        rot = self._rotation(batch, a)
+        cq = latent_append(linear(h, L["dqkv"]), L["q_norm"], L["kv_norm"], cache, batch.slots, rot, a.q_rank, a.kv_rank,
+                           a.rot_dim, self.spec.eps)
+        o = latent_attention(linear(cq, L["uq"]), L["uk"], L["uv"], L["ukv"], cache, batch, rot, a.heads, a.dim, a.rot_dim,
+                             a.vdim, a.kv_rank, a.scale, a.window)
+        return linear(o, L["o"])
+
+    def _rotation(self, batch, a):
+        """The step's rotation table, shared by the layers with the same rotation."""
+        key = (a.rot_dim, a.rot_base)
+        if key not in self._rot:
+            self._rot[key] = rotation_table(batch.positions, *key)
+        return self._rot[key]
+
+    def _feed_forward(self, h, L, spec):
+        """-> (output rows, slots): slots None for one row a token (ops/residual_norm.sandwich_norm)."""
+        if spec.moe is None:
+            return linear(gated_act(linear(h, L["gu"]), spec.act), L["down"]), None
+        expert, weight = route_topk(h, L["router"], spec.moe.top)
+        return expert_mlp(h, expert, weight, L["e_up"], L["e_down"], spec.moe.act)
+
+    def _forward_sandwich(self, batch, kv_cache):
+        s, W = self.spec, self.w
+        self._rot = {}
+        steps = []  # (run, layer, is mixer, embedding output added first)
+        for r, (i, again) in enumerate(self.runs):
+            steps.append((r, i, True, again))
+            if "norm2" in W["layers"][i]:
+                steps.append((r, i, False, False))
+
+        def pre(n):  # weight of the norm in front of step n; after the last one the model's final norm
+            return W["final"] if n == len(steps) else W["layers"][steps[n][1]]["norm1" if steps[n][2] else "norm2"]
+        x, h = embed_norm(W["embed"], batch.input_ids, W["embed_norm"], s.eps, pre(0))
+        x0 = x
+        for n, (r, i, mixer, _) in enumerate(steps):
+            L, spec, slots = W["layers"][i], s.layers[i], None
+            if not mixer:
+                y, slots = self._feed_forward(h, L, spec)
+            elif isinstance(spec.mixer, LinearSpec):
+                y = self._linear_mixer(h, L, spec.mixer, r, batch, kv_cache)
+            else:
+                y = self._latent_mixer(h, L, spec.mixer, r, batch, kv_cache)
+            last = n + 1 == len(steps)
+            add = x0 if not last and steps[n + 1][3] else None
+            x, h = sandwich_norm(x, y, L["norm1b" if mixer else "norm2b"], pre(n + 1), s.eps, slots, add,
+                                 batch.last_idx if last else None, need_x=not last)
+        return linear(h, W["head"]).float() * s.logit_scale
+
 
 def load_layered_decoder(path, dtype=torch.bfloat16, device=None, weight_quant=None, tp_size=1):
     """A checkpoint directory (config.json + *.safetensors) -> RaggedLayeredDecoder."""
     from .hf_decoder import _load_state_dict
     if tp_size > 1:
-        raise NotImplementedError("layered decoders run on one GPU: talking heads couple all heads of a token, "
-                                  "so heads cannot be split over tensor-parallel ranks")
+        raise NotImplementedError("layered decoders run on one GPU: talking heads and norms over all heads couple the heads "
+                                  "of a token, so heads cannot be split over tensor-parallel ranks")
     with open(os.path.join(path, "config.json")) as f:
         cfg = json.load(f)
     make_spec, make_weights = ARCHITECTURES[cfg["architecture"]]

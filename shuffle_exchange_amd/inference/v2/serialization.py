@@ -112,8 +112,8 @@ def serialize_engine(engine, save_path):
         named = {k: v for k, v in m.w.items() if k != "layers"}
         for i, L in enumerate(m.w["layers"]):
             named.update({f"layers.{i}.{k}": v for k, v in L.items()})
-        desc = dict(common, implementation=type(m).__name__, spec=_jsonable(dataclasses.asdict(m.spec)),
-                    n_layers=len(m.w["layers"]))
+        spec = m.spec.to_dict() if hasattr(m.spec, "to_dict") else dataclasses.asdict(m.spec)
+        desc = dict(common, implementation=type(m).__name__, spec=_jsonable(spec), n_layers=len(m.w["layers"]))
         rank_meta = {"nq": m.nq, "nkv": m.nkv} if isinstance(m, RaggedDecoder) else {}
     elif isinstance(m, RaggedLlama):
         named = dict(m.model.state_dict())

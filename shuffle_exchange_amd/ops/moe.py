@@ -252,3 +252,40 @@ class IntWeight:
         if bias is not None:
             y = y + bias.to(y.dtype)
         return y.view(*x.shape[:-1], self.shape[0]).to(x.dtype)
+
+
+# ------------------------------------------------------- routed experts without a gate (device routing)
+EXPERT_ACTS = {"none": 0, "relu2": 1, "silu": 2}
+
+
+def route_topk(h, router, top):
+    """Logits h . router in fp32 (router [E, D] as stored), the ``top`` largest, weights = softmax over those
+    alone: (expert int32 [T, top], weight fp32 [T, top])."""
+    if _hip(h):
+        return tuple(torch.ops.sxe.route_topk(h, router, int(top)))
+    z = F.linear(h.float(), router.float())
+    val, idx = z.topk(top, dim=-1)
+    return idx.to(torch.int32), torch.softmax(val, -1)
+
+
+def expert_mlp(h, expert, weight, up, down, act="relu2"):
+    """Two-layer experts up [E, F, D], down [E, D, F] on the rows ``route_topk`` chose. Returns (y, slots): y
+    [T * top, D] holds weight * down(act(up h)) of every (token, choice) and y[slots[t, j]] belongs to token t. No
+    host synchronisation. Few rows per expert: the weights are streamed once (skinny kernels, rows stay
+    in token order); more: rows sorted by expert for the grouped kernels, which gather them on the fly."""
+    T, k = expert.shape
+    E = up.shape[0]
+    if _hip(h):
+        if T * k <= SKINNY_ROWS * E or not grouped_gemm_ok(h, up) or down.shape[1] % 128:
+            lists = torch.ops.sxe.moe_lists(expert, E)
+        else:
+            lists = torch.ops.sxe.moe_lists(expert, E)
+        return torch.ops.sxe.expert_mlp(h, expert, weight, up, down, *lists, EXPERT_ACTS[act])
+    y = torch.zeros(T * k, down.shape[1], dtype=h.dtype, device=h.device)
+    flat = expert.reshape(-1)
+    for e in flat.unique().tolist():
+        r = (flat == e).nonzero()[:, 0]
+        a = F.linear(h.index_select(0, r // k).float(), up[e].float())
+        a = {"relu2": lambda z: torch.relu(z) ** 2, "silu": F.silu, "none": lambda z: z}[act](a).to(h.dtype)
+        y[r] = (F.linear(a.float(), down[e].float()) * weight.reshape(-1, 1)[r]).to(h.dtype)
+    return y, torch.arange(T * k, dtype=torch.int32, device=h.device).view(T, k)

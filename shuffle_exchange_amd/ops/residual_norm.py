@@ -49,3 +49,41 @@ def qkv_norm_append(proj, q_norm, k_norm, kc, vc, slots, nq, nkv, dk, dv, eps):
     kc[s // bs, :, s % bs] = rows(k, nkv, dk, kc.shape[3])[ok]
     vc[s // bs, :, s % bs] = rows(v, nkv, dv, vc.shape[3])[ok]
     return rows(q, nq, dk, kc.shape[3])
+
+
+def _rms(x, weight, eps):
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * weight.float()
+
+
+def embed_norm(table, ids, weight, eps, next_weight):
+    """x = rms(table[ids]) * weight -> (x fp32, rms(x) * next_weight in the table's dtype)."""
+    if native.use_hip(table):
+        return tuple(torch.ops.sxe.embed_norm(table, ids, weight, next_weight, float(eps)))
+    x = _rms(table.index_select(0, ids).float(), weight, eps)
+    return x, _rms(x, next_weight, eps).to(table.dtype)
+
+
+def sandwich_norm(x, y, post_weight, next_weight, eps, slots=None, add=None, index=None, need_x=True):
+    """The sum of a sublayer that has a norm on both sides and the norm in front of the next one, plain
+    weights: x' = x + rms(y) * post_weight [+ add] -> (x' fp32, rms(x') * next_weight in y's dtype).
+
+    ``slots`` int32 [T, k]: y's row of token t is the sum of y[slots[t, j]] (expert outputs, one row per
+    (token, expert)). ``index`` picks rows; ``need_x`` False: x' itself is not used."""
+    if native.use_hip(x):
+        return tuple(torch.ops.sxe.sandwich_norm(x, y, post_weight, next_weight, slots, add, index, float(eps), bool(need_x)))
+    y = y.float()
+    if slots is not None:
+        y = y.index_select(0, slots.reshape(-1).long()).view(*slots.shape, -1).sum(1)
+    o = x + _rms(y, post_weight, eps)
+    if add is not None:
+        o = o + add
+    if index is not None:
+        o = o.index_select(0, index)
+    return o, _rms(o, next_weight, eps).to(next_weight.dtype)
+
+
+def gated_rms_norm(x, weight, gate, eps):
+    """rms(x) * weight * sigmoid(gate) over whole rows, plain weight; ``gate`` may be a column slice."""
+    if native.use_hip(x):
+        return torch.ops.sxe.gated_rms_norm(x, weight, gate, float(eps))
+    return (_rms(x.float(), weight, eps) * torch.sigmoid(gate.float())).to(x.dtype)
