@@ -17,6 +17,9 @@
 // the product) on the way into LDS, so the conversion is paid once per 128-row output tile, and
 // the MFMA loop is the bf16 one.
 //
+// Optional row gather (`rows`: sorted row -> row of X), so expert-sorted copies of the tokens are never
+// written, and an activation in the epilogue (squared relu; before the row scale) for experts without a gate.
+//
 // Geometry: 128 x 128 output tile, 4 waves (2 x 2, 64 x 64 each as 2 x 2 v_mfma_f32_32x32x16_bf16
 // accumulators), K in blocks of 128: both operands are K-contiguous (X rows; W[e] as [N, K], the
 // nn.Linear layout), staged through registers into XOR-swizzled LDS tiles (sxe_mfma.h RowStager)
@@ -32,6 +35,41 @@ namespace gg {
 using namespace mf;
 
 constexpr int BM = 128, BN = 128, BK = 128, NTHR = 256;
+enum : int { ACT_NONE = 0, ACT_RELU2 = 1 };
+
+__device__ __forceinline__ void act_acc(f32x16& c, int act) {
+  if (act == ACT_RELU2)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const float x = fmaxf(c[i], 0.f);
+      c[i] = x * x;
+    }
+}
+
+// RowStager<BM, BK, NTHR> over rows picked by an index
+struct GatherStager {
+  static constexpr int CPR = BK / 8, N = BM * CPR / NTHR;
+  u32x4 r[N];
+  const unsigned short* p[N];
+  __device__ __forceinline__ void rows(const unsigned short* base, int64_t ld, const int* idx, int lo, int hi, int X) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int c = threadIdx.x + i * NTHR, row = lo + c / CPR;
+      p[i] = row < hi ? base + (int64_t)(idx != nullptr ? min(max(idx[row], 0), X - 1) : row) * ld + c % CPR * 8 : nullptr;
+    }
+  }
+  __device__ __forceinline__ void load(int k) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) r[i] = p[i] != nullptr ? *reinterpret_cast<const u32x4*>(p[i] + k) : u32x4{0u, 0u, 0u, 0u};
+  }
+  __device__ __forceinline__ void store(char* lds) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int c = threadIdx.x + i * NTHR;
+      *reinterpret_cast<u32x4*>(lds + soff(c / CPR, c % CPR)) = r[i];
+    }
+  }
+};
 constexpr int TILE_BYTES = BM * ROWB;  // 32 KiB per operand tile
 
 // K block of ROWS weight rows stored as int8 (BITS 8) or packed int4 (BITS 4), widened to bf16
@@ -86,7 +124,8 @@ __global__ void __launch_bounds__(NTHR, 2) grouped_gemm_kernel(const unsigned sh
                                                                const unsigned short* __restrict__ W,
                                                                const int* __restrict__ offs, int E,
                                                                const ScaleT* __restrict__ scale,
-                                                               unsigned short* __restrict__ Y, int R, int N, int K) {
+                                                               unsigned short* __restrict__ Y, int R, int N, int K,
+                                                               const int* __restrict__ rows, int XR, int act) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   char* lA = smem;
   char* lB = smem + TILE_BYTES;
@@ -114,9 +153,10 @@ __global__ void __launch_bounds__(NTHR, 2) grouped_gemm_kernel(const unsigned sh
 #pragma unroll
     for (int j = 0; j < 2; ++j) acc[i][j] = zero16();
 
-  RowStager<BM, BK, NTHR> sa;
+  GatherStager sa;
   RowStager<BN, BK, NTHR> sb;
-  sa.load(X, K, lo, hi);  // rows lo .. lo+127 of X (zeros past hi), columns 0 .. 127
+  sa.rows(X, K, rows, lo, hi, XR);
+  sa.load(0);  // rows lo .. lo+127 (zeros past hi), columns 0 .. 127
   sb.load(We, K, n0, N);
   const int nk = K / BK;
   for (int kb = 0; kb < nk; ++kb) {
@@ -125,7 +165,7 @@ __global__ void __launch_bounds__(NTHR, 2) grouped_gemm_kernel(const unsigned sh
     sb.store(lB);
     __syncthreads();
     if (kb + 1 < nk) {  // next block's global loads overlap this block's MFMAs
-      sa.load(X + (kb + 1) * BK, K, lo, hi);
+      sa.load((kb + 1) * BK);
       sb.load(We + (kb + 1) * BK, K, n0, N);
     }
 #pragma unroll
@@ -149,6 +189,8 @@ __global__ void __launch_bounds__(NTHR, 2) grouped_gemm_kernel(const unsigned sh
     const int m = lo + wm * 64 + i * 32 + l32;  // lane's token row (transposed accumulators)
     if (m >= hi) continue;
     const float sm = scale ? (float)scale[m] : 1.f;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) act_acc(acc[i][j], act);
 #pragma unroll
     for (int j = 0; j < 2; ++j) store_acc_t(acc[i][j], Y + (int64_t)m * N + n0 + wn * 64 + j * 32 + 4 * h, sm);
   }
@@ -184,7 +226,8 @@ __global__ void __launch_bounds__(128 * WN, 1) grouped_gemm_dp_kernel(const unsi
                                                                 const unsigned short* __restrict__ W,
                                                                 const int* __restrict__ offs, int E,
                                                                 const ScaleT* __restrict__ scale,
-                                                                unsigned short* __restrict__ Y, int R, int N, int K) {
+                                                                unsigned short* __restrict__ Y, int R, int N, int K,
+                                                                const int* __restrict__ rows, int XR, int act) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
   int idx = blockIdx.x, e = 0, lo = 0, hi = 0;
   for (; e < E; ++e) {
@@ -204,12 +247,17 @@ __global__ void __launch_bounds__(128 * WN, 1) grouped_gemm_dp_kernel(const unsi
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int wm = w / WN, wn = w % WN, h = lane >> 5, l32 = lane & 31;
 
+  const unsigned short* xp[PI];  // the lane's source rows of X
+#pragma unroll
+  for (int j = 0; j < PI; ++j) {
+    const int row = 8 * (w * PI + j) + (lane >> 3), gr = min(lo + row, hi - 1);
+    xp[j] = X + (int64_t)(rows != nullptr ? min(max(rows[gr], 0), XR - 1) : gr) * K + 8 * ((lane & 7) ^ sw(row));
+  }
+
   auto issue = [&](char* buf, int kb) {
 #pragma unroll
     for (int j = 0; j < PI; ++j) {  // A: 32 instructions of 8 rows x 128 B
-      const int g = w * PI + j, row = 8 * g + (lane >> 3), slot = lane & 7;
-      const int gr = min(lo + row, hi - 1);
-      glds16(X + (int64_t)gr * K + (int64_t)kb * BKD + 8 * (slot ^ sw(row)), buf + 8 * g * 128);
+      glds16(xp[j] + (int64_t)kb * BKD, buf + 8 * (w * PI + j) * 128);
     }
 #pragma unroll
     for (int j = 0; j < PI; ++j) {  // B: the expert's weight rows n0 .. n0 + 255
@@ -258,6 +306,8 @@ __global__ void __launch_bounds__(128 * WN, 1) grouped_gemm_dp_kernel(const unsi
     const int m = lo + wm * 128 + i * 32 + l32;
     if (m >= hi) continue;
     const float sm = scale ? (float)scale[m] : 1.f;
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) act_acc(acc[i][j], act);
 #pragma unroll
     for (int j = 0; j < NJ; ++j)
       store_acc_t(acc[i][j], Y + (int64_t)m * N + n0 + wn * (BN / WN) + j * 32 + 4 * h, sm);
@@ -344,12 +394,21 @@ __global__ void __launch_bounds__(NTHR, 2) grouped_gemm_q_kernel(const unsigned 
 
 }  // namespace gg
 
-// y[R, N] = row_scale * x[R, K] @ w[e]^T per expert segment offsets[e] .. offsets[e+1]
-at::Tensor grouped_gemm(at::Tensor x, at::Tensor w, at::Tensor offsets, c10::optional<at::Tensor> row_scale) {
+// y[R, N] = row_scale * act(x[rows] @ w[e]^T) per expert segment offsets[e] .. offsets[e+1]; rows int32 [R] or
+// None (x has R rows)
+at::Tensor grouped_gemm_rows(at::Tensor x, at::Tensor w, at::Tensor offsets, c10::optional<at::Tensor> row_scale,
+                             c10::optional<at::Tensor> rows, int64_t act) {
   SXE_CHECK_CUDA(x);
   SXE_CHECK(x.dim() == 2 && x.is_contiguous() && x.scalar_type() == at::kBFloat16, "grouped_gemm: x [R, K] bf16");
   SXE_CHECK(w.dim() == 3 && w.is_contiguous() && w.scalar_type() == at::kBFloat16, "grouped_gemm: w [E, N, K] bf16");
-  const int64_t R = x.size(0), K = x.size(1), E = w.size(0), N = w.size(1);
+  const bool hr = rows.has_value() && rows->defined();
+  if (hr)
+    SXE_CHECK(rows->is_cuda() && rows->is_contiguous() && rows->scalar_type() == at::kInt && rows->dim() == 1 && x.size(0) > 0,
+              "grouped_gemm: rows int32 [R]");
+  SXE_CHECK(act == gg::ACT_NONE || act == gg::ACT_RELU2, "grouped_gemm: activation ", act);
+  const int64_t R = hr ? rows->numel() : x.size(0), K = x.size(1), E = w.size(0), N = w.size(1);
+  const int* ri = hr ? rows->data_ptr<int>() : nullptr;
+  const int XR = (int)x.size(0), ac = (int)act;
   SXE_CHECK(w.size(2) == K, "grouped_gemm: K mismatch");
   SXE_CHECK(K % gg::BK == 0 && N % gg::BN == 0, "grouped_gemm: K and N must be multiples of 128");
   SXE_CHECK(offsets.is_cuda() && offsets.scalar_type() == at::kInt && offsets.is_contiguous() &&
@@ -386,22 +445,22 @@ at::Tensor grouped_gemm(at::Tensor x, at::Tensor w, at::Tensor offsets, c10::opt
       if (wn == 2) {
         go(gg::dp::grouped_gemm_dp_kernel<__bf16, 2>, 256);
         hipLaunchKernelGGL((gg::dp::grouped_gemm_dp_kernel<__bf16, 2>), grid_dp, dim3(256), lds_dp, cur_stream(), X, Wp,
-                           off, (int)E, rs, Yp, (int)R, (int)N, (int)K);
+                           off, (int)E, rs, Yp, (int)R, (int)N, (int)K, ri, XR, ac);
       } else {
         go(gg::dp::grouped_gemm_dp_kernel<__bf16, 4>, 512);
         hipLaunchKernelGGL((gg::dp::grouped_gemm_dp_kernel<__bf16, 4>), grid_dp, dim3(512), lds_dp, cur_stream(), X, Wp,
-                           off, (int)E, rs, Yp, (int)R, (int)N, (int)K);
+                           off, (int)E, rs, Yp, (int)R, (int)N, (int)K, ri, XR, ac);
       }
     } else {
       const float* rs = hs ? row_scale->data_ptr<float>() : nullptr;
       if (wn == 2) {
         go(gg::dp::grouped_gemm_dp_kernel<float, 2>, 256);
         hipLaunchKernelGGL((gg::dp::grouped_gemm_dp_kernel<float, 2>), grid_dp, dim3(256), lds_dp, cur_stream(), X, Wp,
-                           off, (int)E, rs, Yp, (int)R, (int)N, (int)K);
+                           off, (int)E, rs, Yp, (int)R, (int)N, (int)K, ri, XR, ac);
       } else {
         go(gg::dp::grouped_gemm_dp_kernel<float, 4>, 512);
         hipLaunchKernelGGL((gg::dp::grouped_gemm_dp_kernel<float, 4>), grid_dp, dim3(512), lds_dp, cur_stream(), X, Wp,
-                           off, (int)E, rs, Yp, (int)R, (int)N, (int)K);
+                           off, (int)E, rs, Yp, (int)R, (int)N, (int)K, ri, XR, ac);
       }
     }
     SXE_LAUNCH_CHECK();
@@ -417,7 +476,7 @@ at::Tensor grouped_gemm(at::Tensor x, at::Tensor w, at::Tensor offsets, c10::opt
     }();
     (void)a;
     hipLaunchKernelGGL(gg::grouped_gemm_kernel<__bf16>, grid, dim3(gg::NTHR), lds, cur_stream(), X, Wp, off, (int)E,
-                       reinterpret_cast<const __bf16*>(row_scale->data_ptr()), Yp, (int)R, (int)N, (int)K);
+                       reinterpret_cast<const __bf16*>(row_scale->data_ptr()), Yp, (int)R, (int)N, (int)K, ri, XR, ac);
   } else {
     static bool a = [&] {
       SXE_HIP_CHECK(hipFuncSetAttribute((const void*)gg::grouped_gemm_kernel<float>,
@@ -426,10 +485,14 @@ at::Tensor grouped_gemm(at::Tensor x, at::Tensor w, at::Tensor offsets, c10::opt
     }();
     (void)a;
     hipLaunchKernelGGL(gg::grouped_gemm_kernel<float>, grid, dim3(gg::NTHR), lds, cur_stream(), X, Wp, off, (int)E,
-                       hs ? row_scale->data_ptr<float>() : nullptr, Yp, (int)R, (int)N, (int)K);
+                       hs ? row_scale->data_ptr<float>() : nullptr, Yp, (int)R, (int)N, (int)K, ri, XR, ac);
   }
   SXE_LAUNCH_CHECK();
   return y;
+}
+
+at::Tensor grouped_gemm(at::Tensor x, at::Tensor w, at::Tensor offsets, c10::optional<at::Tensor> row_scale) {
+  return grouped_gemm_rows(x, w, offsets, row_scale, c10::nullopt, gg::ACT_NONE);
 }
 
 // Mixed-precision experts: wq int8 [E, N, K] or packed int4 [E, N, K / 2] (uint8 storage), ws fp32
@@ -485,9 +548,11 @@ at::Tensor grouped_gemm_q(at::Tensor x, at::Tensor wq, at::Tensor ws, int64_t bi
 
 TORCH_LIBRARY_FRAGMENT(sxe, m) {
   m.def("grouped_gemm(Tensor x, Tensor w, Tensor offsets, Tensor? row_scale=None) -> Tensor");
+  m.def("grouped_gemm_rows(Tensor x, Tensor w, Tensor offsets, Tensor? row_scale, Tensor? rows, int act) -> Tensor");
   m.def("grouped_gemm_q(Tensor x, Tensor wq, Tensor ws, int bits, Tensor offsets, Tensor? row_scale=None) -> Tensor");
 }
 TORCH_LIBRARY_IMPL(sxe, CUDA, m) {
   m.impl("grouped_gemm", &sxe::grouped_gemm);
+  m.impl("grouped_gemm_rows", &sxe::grouped_gemm_rows);
   m.impl("grouped_gemm_q", &sxe::grouped_gemm_q);
 }

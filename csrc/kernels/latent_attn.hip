@@ -1,0 +1,876 @@
+// Attention over a paged low-rank latent (gfx950). A token's cache row [latent c (R) | rotated key part (rp)]
+// serves all heads; per head the unrotated key is W_uk c, the value W_uv c. ops/latent_attention.py has the
+// equations of the two ways to evaluate it.
+//
+//  * rotation_table: cos / sin of p base^(-2 i / dims) per token, once per step for all layers;
+//  * latent_append: norms of the query latent and of c, rotation of the key part, cache write;
+//  * generic form (fp32, any size): one workgroup per (token, head);
+//  * token form (decode, short continuations; bf16): latent_absorb forms W_uk^T q per head,
+//    latent_token runs one workgroup per (token, 32 heads, key split) with 64-key tiles of the cache in LDS,
+//    read by rows for the scores and transposed for the weighted sum of latents -- each cache byte crosses
+//    HBM once for all heads -- and latent_expand merges the splits and applies W_uv;
+//  * tile form (prompts; bf16): keys and values of the window are expanded by a library product, then one
+//    workgroup per (128 queries, head) in the flash manner. The rotated key part is read from the gathered
+//    cache rows, queries are rotated on the way into LDS.
+// Only visible keys are enumerated (window: i sees 0 <= i - j < window). Scores, softmax and sums are fp32.
+#include "sxe_common.h"
+#include "sxe_mfma.h"
+#include <torch/library.h>
+
+namespace sxe {
+namespace lt {
+using namespace mf;
+
+constexpr int kThreads = 256;
+
+__global__ __launch_bounds__(kThreads) void rotation_table_kernel(const int64_t* __restrict pos, int T, int half, double lbase,
+                                                                  float* __restrict out) {
+  const int i = blockIdx.x * kThreads + threadIdx.x;
+  if (i >= T * half) return;
+  const int t = i / half, d = i - t * half;
+  const double a = (double)pos[t] * exp2(-lbase * (double)d / (double)half);
+  double s, c;
+  sincos(a, &s, &c);
+  out[2 * i] = (float)c;
+  out[2 * i + 1] = (float)s;
+}
+
+// ---------------------------------------------------------------------------------------------- append
+struct AppendArgs {
+  const void* proj;  // [T, ld]: query latent | latent | key part
+  int64_t ld;
+  const void *qw, *kw;
+  const float* rot;  // [T, rot_dim / 2, 2]
+  const int64_t* slots;
+  void *cq, *cache;  // [T, q_rank]; [blocks * bs, row]
+  int q_rank, rank, R, rot_dim, row;
+  int64_t nslots;
+  float eps;
+};
+
+template <DT T, int V>
+__device__ __forceinline__ void ldv(const typename dt_traits<T>::storage* p, float (&v)[V]) {
+  if constexpr (V == 8) load8<T>(p, v);
+  else v[0] = to_f32<T>(*p);
+}
+template <DT T, int V>
+__device__ __forceinline__ void stv(typename dt_traits<T>::storage* p, const float (&v)[V]) {
+  if constexpr (V == 8) store8<T>(p, v);
+  else *p = from_f32<T>(v[0]);
+}
+
+template <DT T, int V>
+__global__ __launch_bounds__(kThreads) void latent_append_kernel(AppendArgs a) {
+  using S = typename dt_traits<T>::storage;
+  __shared__ float red[2][kThreads / 64];
+  const int64_t t = blockIdx.x;
+  const S* row = static_cast<const S*>(a.proj) + t * a.ld;
+  const int n = a.q_rank + a.rank;
+  float sq = 0.f, sk = 0.f, v[V], w[V];
+  for (int c = threadIdx.x * V; c < n; c += kThreads * V) {
+    ldv<T, V>(row + c, v);
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < V; ++i) s += v[i] * v[i];
+    if (c < a.q_rank) sq += s;
+    else sk += s;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((threadIdx.x & 63) == 0) {
+    red[0][threadIdx.x >> 6] = sq;
+    red[1][threadIdx.x >> 6] = sk;
+  }
+  __syncthreads();
+  sq = red[0][0] + red[0][1] + red[0][2] + red[0][3];
+  sk = red[1][0] + red[1][1] + red[1][2] + red[1][3];
+  const float rq = 1.f / sqrtf(sq / (float)a.q_rank + a.eps), rk = 1.f / sqrtf(sk / (float)a.rank + a.eps);
+  const int64_t slot = a.slots[t];
+  const bool keep = slot >= 0 && slot < a.nslots;
+  S* dst = static_cast<S*>(a.cache) + (keep ? slot : 0) * a.row;
+  for (int c = threadIdx.x * V; c < n; c += kThreads * V) {
+    ldv<T, V>(row + c, v);
+    const bool q = c < a.q_rank;
+    ldv<T, V>(q ? static_cast<const S*>(a.qw) + c : static_cast<const S*>(a.kw) + c - a.q_rank, w);
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] = v[i] * (q ? rq : rk) * w[i];
+    if (q) stv<T, V>(static_cast<S*>(a.cq) + t * a.q_rank + c, v);
+    else if (keep) stv<T, V>(dst + c - a.q_rank, v);
+  }
+  const int half = a.rot_dim / 2;
+  if (keep)
+    for (int i = threadIdx.x; i < half; i += kThreads) {
+      const float x = to_f32<T>(row[n + i]), y = to_f32<T>(row[n + half + i]);
+      const float c = a.rot[(t * half + i) * 2], s = a.rot[(t * half + i) * 2 + 1];
+      dst[a.R + i] = from_f32<T>(x * c - y * s);
+      dst[a.R + half + i] = from_f32<T>(y * c + x * s);
+    }
+}
+
+// --------------------------------------------------------------------------------------- generic form
+struct Args {
+  const void* q;  // [T, H * (dim + rot_dim)]
+  const float* rot;
+  const int* rows;  // [n, 2]: sequence, row of q
+  const int *table, *q_start, *q_len, *kv_len;  // table [S, max blocks]
+  const void* cache;
+  int64_t nblocks;
+  int maxb, bs, H, dim, rot_dim, rank, R, row, vdim, window;
+  float scale;
+};
+
+// visible keys [lo, hi) of query row t of sequence s
+__device__ __forceinline__ void key_range(const Args& a, int s, int t, int& lo, int& hi) {
+  const int pos = a.kv_len[s] - a.q_len[s] + (t - a.q_start[s]);
+  hi = min(pos + 1, a.maxb * a.bs);
+  lo = a.window > 0 ? max(0, pos + 1 - a.window) : 0;
+}
+__device__ __forceinline__ int64_t cache_at(const Args& a, int s, int j) {
+  const int b = j / a.bs;
+  int64_t blk = a.table[(int64_t)s * a.maxb + b];
+  if (blk < 0 || blk >= a.nblocks) blk = 0;
+  return (blk * a.bs + (j - b * a.bs)) * a.row;
+}
+
+// grid (n, H); uk [H, dim, rank], uv [H, rank, vdim]
+template <DT T>
+__global__ __launch_bounds__(kThreads) void latent_generic_kernel(Args a, const typename dt_traits<T>::storage* __restrict uk,
+                                                                  const typename dt_traits<T>::storage* __restrict uv,
+                                                                  typename dt_traits<T>::storage* __restrict out) {
+  using S = typename dt_traits<T>::storage;
+  extern __shared__ float sm[];
+  __shared__ float red[2][kThreads / 64];
+  float* qa = sm;                // [rank + rot_dim]
+  float* ol = qa + a.rank + a.rot_dim;  // [rank]
+  float* p = ol + a.rank;        // [kThreads]
+  const int s = a.rows[2 * blockIdx.x], t = a.rows[2 * blockIdx.x + 1], h = blockIdx.y, half = a.rot_dim / 2;
+  const S* q = static_cast<const S*>(a.q) + ((int64_t)t * a.H + h) * (a.dim + a.rot_dim);
+  for (int r = threadIdx.x; r < a.rank; r += kThreads) {
+    float x = 0.f;
+    for (int d = 0; d < a.dim; ++d) x += to_f32<T>(q[d]) * to_f32<T>(uk[((int64_t)h * a.dim + d) * a.rank + r]);
+    qa[r] = x * a.scale;
+    ol[r] = 0.f;
+  }
+  for (int i = threadIdx.x; i < half; i += kThreads) {
+    const float x = to_f32<T>(q[a.dim + i]), y = to_f32<T>(q[a.dim + half + i]);
+    const float c = a.rot[((int64_t)t * half + i) * 2], sn = a.rot[((int64_t)t * half + i) * 2 + 1];
+    qa[a.rank + i] = (x * c - y * sn) * a.scale;
+    qa[a.rank + half + i] = (y * c + x * sn) * a.scale;
+  }
+  __syncthreads();
+  int lo, hi;
+  key_range(a, s, t, lo, hi);
+  const S* cache = static_cast<const S*>(a.cache);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  float M = -INFINITY, L = 0.f;
+  for (int j0 = lo; j0 < hi; j0 += kThreads) {
+    const int j = j0 + threadIdx.x;
+    float x = -INFINITY;
+    if (j < hi) {
+      const S* c = cache + cache_at(a, s, j);
+      x = 0.f;
+      for (int r = 0; r < a.rank; ++r) x += qa[r] * to_f32<T>(c[r]);
+      for (int r = 0; r < a.rot_dim; ++r) x += qa[a.rank + r] * to_f32<T>(c[a.R + r]);
+    }
+    float m = wave_max(x);
+    if (lane == 0) red[0][wave] = m;
+    __syncthreads();
+    m = fmaxf(fmaxf(red[0][0], red[0][1]), fmaxf(red[0][2], red[0][3]));
+    const float Mn = fmaxf(M, m), f = M == -INFINITY ? 0.f : expf(M - Mn), e = j < hi ? expf(x - Mn) : 0.f;
+    p[threadIdx.x] = e;
+    float l = wave_sum(e);
+    if (lane == 0) red[1][wave] = l;
+    __syncthreads();
+    L = L * f + red[1][0] + red[1][1] + red[1][2] + red[1][3];
+    M = Mn;
+    const int nj = min(kThreads, hi - j0);
+    for (int r = threadIdx.x; r < a.rank; r += kThreads) {
+      float o = ol[r] * f;
+      for (int i = 0; i < nj; ++i) o += p[i] * to_f32<T>(cache[cache_at(a, s, j0 + i) + r]);
+      ol[r] = o;
+    }
+    __syncthreads();
+  }
+  const float inv = L > 0.f ? 1.f / L : 0.f;
+  for (int v = threadIdx.x; v < a.vdim; v += kThreads) {
+    float o = 0.f;
+    for (int r = 0; r < a.rank; ++r) o += ol[r] * to_f32<T>(uv[((int64_t)h * a.rank + r) * a.vdim + v]);
+    out[((int64_t)t * a.H + h) * a.vdim + v] = from_f32<T>(o * inv);
+  }
+}
+
+// ----------------------------------------------------------------------- per-head products (token form)
+// y[t, n] = sum_k x[t, k] W[k, n] for one head, TT tokens, N columns in chunks of 8 * LN: thread (k group,
+// 8 columns), k groups summed through shuffles and LDS. x fp32 in LDS [TT][K]. VEC: 16-byte weight loads.
+template <int TT, int LN, bool VEC>
+__device__ __forceinline__ void head_product(const float* x, const unsigned short* __restrict W, int K, int N, int n0, float* part,
+                                             float (&acc)[TT][8]) {
+  constexpr int KG = kThreads / LN;
+  const int ln = threadIdx.x % LN, kg = threadIdx.x / LN, n = n0 + ln * 8;
+#pragma unroll
+  for (int t = 0; t < TT; ++t)
+#pragma unroll
+    for (int i = 0; i < 8; ++i) acc[t][i] = 0.f;
+  if (n < N) {
+#pragma unroll 4
+    for (int k = kg; k < K; k += KG) {
+      float w[8];
+      if constexpr (VEC) {
+        load8<DT::BF16>(W + (int64_t)k * N + n, w);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) w[i] = n + i < N ? bf16_to_f32(W[(int64_t)k * N + n + i]) : 0.f;
+      }
+#pragma unroll
+      for (int t = 0; t < TT; ++t) {
+        const float xv = x[t * K + k];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[t][i] += xv * w[i];
+      }
+    }
+  }
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+#pragma unroll
+  for (int t = 0; t < TT; ++t)
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+#pragma unroll
+      for (int o = LN; o < 64; o <<= 1) acc[t][i] += __shfl_xor(acc[t][i], o, 64);
+      if (lane < LN) part[((wave * TT + t) * LN + lane) * 8 + i] = acc[t][i];
+    }
+  __syncthreads();
+}
+
+// grid (H, ceil(rank / (8 LN)), ceil(n / TT)) -> qa [n, H, row] bf16: W_uk^T q | rotated q, zero-padded
+template <int TT, int LN, bool VEC>
+__global__ __launch_bounds__(kThreads) void latent_absorb_kernel(Args a, int n, const unsigned short* __restrict uk,
+                                                                 unsigned short* __restrict qa) {
+  extern __shared__ float sm[];
+  float* x = sm;                    // [TT][dim]
+  float* part = sm + TT * a.dim;    // [4][TT][LN * 8]
+  const int h = blockIdx.x, n0 = blockIdx.y * LN * 8, i0 = blockIdx.z * TT, half = a.rot_dim / 2;
+  const unsigned short* q = static_cast<const unsigned short*>(a.q);
+  for (int i = threadIdx.x; i < TT * a.dim; i += kThreads) {
+    const int t = i / a.dim, d = i - t * a.dim;
+    x[i] = i0 + t < n ? bf16_to_f32(q[((int64_t)a.rows[2 * (i0 + t) + 1] * a.H + h) * (a.dim + a.rot_dim) + d]) : 0.f;
+  }
+  __syncthreads();
+  float acc[TT][8];
+  head_product<TT, LN, VEC>(x, uk + (int64_t)h * a.dim * a.rank, a.dim, a.rank, n0, part, acc);
+  for (int i = threadIdx.x; i < TT * LN * 8; i += kThreads) {
+    const int t = i / (LN * 8), c = i - t * (LN * 8);
+    if (i0 + t < n && n0 + c < a.R) {
+      float v = 0.f;
+      if (n0 + c < a.rank)
+#pragma unroll
+        for (int w = 0; w < 4; ++w) v += part[(w * TT + t) * LN * 8 + c];
+      qa[((int64_t)(i0 + t) * a.H + h) * a.row + n0 + c] = f32_to_bf16(v);
+    }
+  }
+  if (blockIdx.y == 0) {  // the rotated part and both parts' padding
+    const int rp = a.row - a.R, pad0 = gridDim.y * LN * 8;
+    for (int i = threadIdx.x; i < TT * rp; i += kThreads) {
+      const int t = i / rp, d = i - t * rp;
+      if (i0 + t >= n) continue;
+      const int64_t row = a.rows[2 * (i0 + t) + 1];
+      float v = 0.f;
+      if (d < a.rot_dim) {
+        const unsigned short* qr = q + (row * a.H + h) * (a.dim + a.rot_dim) + a.dim;
+        const int j = d < half ? d : d - half;
+        const float u = bf16_to_f32(qr[j]), w = bf16_to_f32(qr[half + j]);
+        const float c = a.rot[(row * half + j) * 2], s = a.rot[(row * half + j) * 2 + 1];
+        v = d < half ? u * c - w * s : w * c + u * s;
+      }
+      qa[((int64_t)(i0 + t) * a.H + h) * a.row + a.R + d] = f32_to_bf16(v);
+    }
+    for (int i = threadIdx.x; i < TT * (a.R - min(pad0, a.R)); i += kThreads) {
+      const int w = a.R - pad0, t = i / w, d = i - t * w;
+      if (i0 + t < n) qa[((int64_t)(i0 + t) * a.H + h) * a.row + pad0 + d] = 0;
+    }
+  }
+}
+
+// grid (H, ceil(vdim / (8 LN)), ceil(n / TT)): out[row, h, :] = W_uv (merged splits)
+template <int TT, int LN, bool VEC>
+__global__ __launch_bounds__(kThreads) void latent_expand_kernel(Args a, int n, int splits, const float* __restrict po,
+                                                                 const float* __restrict pml, const unsigned short* __restrict uv,
+                                                                 unsigned short* __restrict out) {
+  extern __shared__ float sm[];
+  float* x = sm;                    // [TT][rank]
+  float* part = sm + TT * a.rank;   // [4][TT][LN * 8]
+  const int h = blockIdx.x, n0 = blockIdx.y * LN * 8, i0 = blockIdx.z * TT;
+  const int64_t sstride = (int64_t)n * a.H;
+  for (int t = 0; t < TT; ++t) {
+    if (i0 + t >= n) {
+      for (int r = threadIdx.x; r < a.rank; r += kThreads) x[t * a.rank + r] = 0.f;
+      continue;
+    }
+    const int64_t th = (int64_t)(i0 + t) * a.H + h;
+    float M = -INFINITY, L = 0.f;
+    for (int s = 0; s < splits; ++s) M = fmaxf(M, pml[(s * sstride + th) * 2]);
+    for (int s = 0; s < splits; ++s) {
+      const float m = pml[(s * sstride + th) * 2];
+      if (m != -INFINITY) L += exp2f(m - M) * pml[(s * sstride + th) * 2 + 1];
+    }
+    const float inv = L > 0.f ? 1.f / L : 0.f;
+    for (int r = threadIdx.x; r < a.rank; r += kThreads) {
+      float v = 0.f;
+#pragma unroll 4
+      for (int s = 0; s < splits; ++s) {
+        const float m = pml[(s * sstride + th) * 2];
+        if (m != -INFINITY) v += exp2f(m - M) * po[(s * sstride + th) * a.R + r];
+      }
+      x[t * a.rank + r] = v * inv;
+    }
+  }
+  __syncthreads();
+  float acc[TT][8];
+  head_product<TT, LN, VEC>(x, uv + (int64_t)h * a.rank * a.vdim, a.rank, a.vdim, n0, part, acc);
+  for (int i = threadIdx.x; i < TT * LN * 8; i += kThreads) {
+    const int t = i / (LN * 8), c = i - t * (LN * 8);
+    if (i0 + t < n && n0 + c < a.vdim) {
+      float v = 0.f;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) v += part[(w * TT + t) * LN * 8 + c];
+      out[((int64_t)a.rows[2 * (i0 + t) + 1] * a.H + h) * a.vdim + n0 + c] = f32_to_bf16(v);
+    }
+  }
+}
+
+// ------------------------------------------------------------------------------------------ token form
+constexpr int kKeys = 64;
+constexpr int kSRow = kKeys + 4;  // fp32 score row of a head
+
+__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+
+// PN: 256-byte panels (128 columns) of the latent part, R <= 128 PN. grid (n, ceil(H / 32), splits)
+template <int PN>
+__global__ __launch_bounds__(kThreads, 1) void latent_token_kernel(Args a, int n, const unsigned short* __restrict qa,
+                                                                   float* __restrict po, float* __restrict pml) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  constexpr int PANEL = kKeys * ROWB, NS = 4 * PN + 2, NC = 4 * PN + 2;
+  char* lrot = smem + PN * PANEL;
+  float* ls = reinterpret_cast<float*>(smem + (PN + 1) * PANEL);  // [32 heads][kSRow]
+  const int i = blockIdx.x, g = blockIdx.y, sp = blockIdx.z;
+  const int s = a.rows[2 * i], t = a.rows[2 * i + 1];
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l16 = lane & 15, q16 = lane >> 4, l32 = lane & 31, hh = lane >> 5;
+  const int nr = a.R / 32, nrot = (a.row - a.R) / 32;  // 32-column steps
+  int lo, hi;
+  key_range(a, s, t, lo, hi);
+  {  // this split's keys, whole tiles
+    const int tiles = (hi - lo + kKeys - 1) / kKeys, per = (tiles + gridDim.z - 1) / gridDim.z;
+    lo = min(hi, lo + sp * per * kKeys);
+    hi = min(hi, lo + per * kKeys);
+  }
+  // queries: B fragments of 16 heads each, head 32 g + 16 b + l16
+  bf16x8 qf[NS][2];
+#pragma unroll
+  for (int b = 0; b < 2; ++b) {
+    const int h = 32 * g + 16 * b + l16;
+    const unsigned short* qr = qa + ((int64_t)i * a.H + min(h, a.H - 1)) * a.row;
+#pragma unroll
+    for (int k = 0; k < NS; ++k) {
+      const int st = k < 4 * PN ? k : nr + k - 4 * PN;
+      const bool ok = h < a.H && (k < 4 * PN ? k < nr : k - 4 * PN < nrot);
+      u32x4 z = {0u, 0u, 0u, 0u};
+      if (ok) z = *reinterpret_cast<const u32x4*>(qr + st * 32 + q16 * 8);
+      qf[k][b] = __builtin_bit_cast(bf16x8, z);
+    }
+  }
+  f32x16 acc[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) acc[j] = zero16();
+  float M = -INFINITY, L = 0.f;
+  const float sc2 = a.scale * LOG2E;
+  const unsigned short* cache = static_cast<const unsigned short*>(a.cache);
+  const int srow = threadIdx.x >> 2, sch = threadIdx.x & 3;
+  u32x4 st[NC];
+  auto load = [&](int j0) {
+    const int j = min(j0 + srow, hi - 1);  // a row past the end repeats the last one (its score is masked)
+    const unsigned short* src = cache + cache_at(a, s, j) + sch * 8;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      if (c < 4 * PN ? c < nr : c - 4 * PN < nrot)
+        st[c] = *reinterpret_cast<const u32x4*>(src + (c < 4 * PN ? c : nr + c - 4 * PN) * 32);
+    }
+  };
+  if (lo < hi) load(lo);
+  for (int j0 = lo; j0 < hi; j0 += kKeys) {
+    __syncthreads();  // the previous tile is read
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      if (c < 4 * PN) {
+        if (c < nr) *reinterpret_cast<u32x4*>(smem + (c >> 2) * PANEL + soff(srow, (c & 3) * 4 + sch)) = st[c];
+      } else if (c - 4 * PN < nrot) {
+        *reinterpret_cast<u32x4*>(lrot + soff(srow, (c - 4 * PN) * 4 + sch)) = st[c];
+      }
+    }
+    __syncthreads();
+    if (j0 + kKeys < hi) load(j0 + kKeys);
+    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;  // keys 16 w + 4 q16 + i, heads l16 and 16 + l16
+#pragma unroll
+    for (int k = 0; k < NS; ++k) {
+      if (k < 4 * PN ? k < nr : k - 4 * PN < nrot) {
+        const bf16x8 kf = k < 4 * PN ? lds_row16(smem + (k >> 2) * PANEL, 16 * w + l16, (k & 3) * 4 + q16)
+                                     : lds_row16(lrot, 16 * w + l16, (k - 4 * PN) * 4 + q16);
+        s0 = mfma16(kf, qf[k][0], s0);
+        s1 = mfma16(kf, qf[k][1], s1);
+      }
+    }
+    const int kj = 16 * w + 4 * q16;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const bool ok = j0 + kj + e < hi;
+      s0[e] = ok ? s0[e] * sc2 : -INFINITY;
+      s1[e] = ok ? s1[e] * sc2 : -INFINITY;
+    }
+    *reinterpret_cast<f32x4*>(ls + l16 * kSRow + kj) = s0;
+    *reinterpret_cast<f32x4*>(ls + (16 + l16) * kSRow + kj) = s1;
+    __syncthreads();
+    // every wave forms all weights of the tile: lane = head l32, keys 16 x + 4 hh + (0..3, 8..11)
+    f32x4 p[8];
+    float m = -INFINITY;
+#pragma unroll
+    for (int x = 0; x < 8; ++x) {
+      p[x] = *reinterpret_cast<const f32x4*>(ls + l32 * kSRow + 8 * x + 4 * hh);
+      m = fmaxf(m, fmaxf(fmaxf(p[x][0], p[x][1]), fmaxf(p[x][2], p[x][3])));
+    }
+    m = fmaxf(m, xor32(m));
+    const float Mn = fmaxf(M, m), f = fast_exp2(M - Mn);  // a tile has a visible key: Mn is finite
+    float l = 0.f;
+#pragma unroll
+    for (int x = 0; x < 8; ++x)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        p[x][e] = fast_exp2(p[x][e] - Mn);
+        l += p[x][e];
+      }
+    L = L * f + l + xor32(l);
+    M = Mn;
+    if (w < PN) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) acc[j][e] *= f;
+#pragma unroll
+      for (int x = 0; x < 4; ++x) {
+        bf16x8 b;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          b[e] = (__bf16)p[2 * x][e];
+          b[4 + e] = (__bf16)p[2 * x + 1][e];
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (w * 128 + j * 32 < a.R) acc[j] = mfma(lds_trA(smem + w * PANEL, 16 * x, j, lane), b, acc[j]);
+      }
+    }
+  }
+  const int h = 32 * g + l32;
+  if (h < a.H) {
+    const int64_t th = ((int64_t)sp * n + i) * a.H + h;
+    if (w == 0 && hh == 0) {
+      pml[th * 2] = M;
+      pml[th * 2 + 1] = L;
+    }
+    if (w < PN && lo < hi) {
+      float* o = po + th * a.R + w * 128;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (w * 128 + j * 32 < a.R) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            *reinterpret_cast<f32x4*>(o + j * 32 + 8 * e + 4 * hh) =
+                f32x4{acc[j][4 * e], acc[j][4 * e + 1], acc[j][4 * e + 2], acc[j][4 * e + 3]};
+        }
+    }
+  }
+}
+
+// ------------------------------------------------------------------------------------------- tile form
+constexpr int kQ = 128;
+typedef float f32x2_t __attribute__((ext_vector_type(2)));
+
+struct TileArgs {
+  const unsigned short *q, *kv, *lat;  // [T, H (dim + rot)], [Nk, H (dim + vdim)], [Nk, row]
+  const float* rot;
+  const int *chunks, *first, *q_start, *q_len, *kv_len;
+  unsigned short* out;  // [T, H vdim]
+  int64_t ldkv;
+  int H, dim, rot_dim, vdim, R, row, window, Nk;
+  float scale;
+};
+
+// DN, VP: dim and vdim padded to 64 / 128; the rotated part is padded to 64. grid (chunks of kQ rows, H)
+template <int DN, int VP>
+__global__ __launch_bounds__(kThreads, 2) void latent_tile_kernel(TileArgs a) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  constexpr int KC = DN / 8, VC = VP / 8, RC = 8, NN = DN / 16, NR = 4, NV = VP / 32;
+  const int c = blockIdx.x, h = blockIdx.y;
+  const int s = a.chunks[3 * c], row0 = a.chunks[3 * c + 1], n = a.chunks[3 * c + 2];
+  const int pos0 = a.kv_len[s] - a.q_len[s] + (row0 - a.q_start[s]);
+  const int f0 = a.first[2 * s], fp = a.first[2 * s + 1];  // list row and position of the first listed key
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l32 = lane & 31, hh = lane >> 5;
+  const int half = a.rot_dim / 2, ldq = a.H * (a.dim + a.rot_dim);
+  // ---- queries -> LDS -> fragments; the rotated part by pairs
+  char* lqr = smem + kQ * ROWB;
+  const unsigned short* qb = a.q + (int64_t)row0 * ldq + h * (a.dim + a.rot_dim);
+  const bool qv = a.dim % 8 == 0 && a.rot_dim % 8 == 0;
+  for (int x = threadIdx.x; x < kQ * KC; x += kThreads) {
+    const int t = x / KC, ch = x % KC;
+    u32x4 z = {0u, 0u, 0u, 0u};
+    if (t < n && ch * 8 < a.dim && qv) z = *reinterpret_cast<const u32x4*>(qb + (int64_t)t * ldq + ch * 8);
+    *reinterpret_cast<u32x4*>(smem + soff(t, ch)) = z;
+  }
+  for (int x = threadIdx.x; x < kQ * 64; x += kThreads) {
+    const int t = x >> 6, d = x & 63;
+    float v = 0.f;
+    if (t < n && d < a.rot_dim) {
+      const int j = d < half ? d : d - half;
+      const unsigned short* qr = qb + (int64_t)t * ldq + a.dim;
+      const float u = bf16_to_f32(qr[j]), y = bf16_to_f32(qr[half + j]);
+      const f32x2_t cs = *reinterpret_cast<const f32x2_t*>(a.rot + ((int64_t)(row0 + t) * half + j) * 2);
+      v = d < half ? u * cs[0] - y * cs[1] : y * cs[0] + u * cs[1];
+    }
+    *reinterpret_cast<unsigned short*>(lqr + soff(t, d >> 3) + (d & 7) * 2) = f32_to_bf16(v);
+  }
+  __syncthreads();
+  bf16x8 qn[NN], qr[NR];
+#pragma unroll
+  for (int k = 0; k < NN; ++k) qn[k] = lds_row16(smem, w * 32 + l32, 2 * k + hh);
+#pragma unroll
+  for (int k = 0; k < NR; ++k) qr[k] = lds_row16(lqr, w * 32 + l32, 2 * k + hh);
+  const int pw = pos0 + w * 32, pq = pw + l32;  // the wave's first position, the lane's
+  const int plast = pos0 + n - 1;
+  const int lo = max(fp, a.window > 0 ? pos0 + 1 - a.window : 0);
+  char *lk = smem, *lr = smem + kKeys * ROWB, *lv = smem + 2 * kKeys * ROWB;
+  constexpr int NK = kKeys * KC / kThreads, NRL = kKeys * RC / kThreads, NVL = kKeys * VC / kThreads;
+  u32x4 rk[NK], rr[NRL], rv[NVL];
+  const unsigned short *kb = a.kv + h * a.dim, *vb = a.kv + a.H * a.dim + h * a.vdim, *rb = a.lat + a.R;
+  auto at = [&](int j) { return (int64_t)min(max(f0 + j - fp, 0), a.Nk - 1); };
+  auto load = [&](int j0) {
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int x = threadIdx.x + i * kThreads, j = j0 + x / KC, ch = x % KC;
+      rk[i] = u32x4{0u, 0u, 0u, 0u};
+      if (j <= plast && ch * 8 < a.dim) rk[i] = *reinterpret_cast<const u32x4*>(kb + at(j) * a.ldkv + ch * 8);
+    }
+#pragma unroll
+    for (int i = 0; i < NRL; ++i) {
+      const int x = threadIdx.x + i * kThreads, j = j0 + x / RC, ch = x % RC;
+      rr[i] = u32x4{0u, 0u, 0u, 0u};
+      if (j <= plast && ch * 8 < a.rot_dim) rr[i] = *reinterpret_cast<const u32x4*>(rb + at(j) * a.row + ch * 8);
+    }
+#pragma unroll
+    for (int i = 0; i < NVL; ++i) {
+      const int x = threadIdx.x + i * kThreads, j = j0 + x / VC, ch = x % VC;
+      rv[i] = u32x4{0u, 0u, 0u, 0u};
+      if (j <= plast && ch * 8 < a.vdim) rv[i] = *reinterpret_cast<const u32x4*>(vb + at(j) * a.ldkv + ch * 8);
+    }
+  };
+  f32x16 acc[NV];
+#pragma unroll
+  for (int j = 0; j < NV; ++j) acc[j] = zero16();
+  float M = -INFINITY, L = 0.f;
+  const float sc2 = a.scale * LOG2E;
+  load(lo);
+  for (int j0 = lo; j0 <= plast; j0 += kKeys) {
+    __syncthreads();  // queries, or the previous tile, are read
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int x = threadIdx.x + i * kThreads;
+      *reinterpret_cast<u32x4*>(lk + soff(x / KC, x % KC)) = rk[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NRL; ++i) {
+      const int x = threadIdx.x + i * kThreads;
+      *reinterpret_cast<u32x4*>(lr + soff(x / RC, x % RC)) = rr[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NVL; ++i) {
+      const int x = threadIdx.x + i * kThreads;
+      *reinterpret_cast<u32x4*>(lv + soff(x / VC, x % VC)) = rv[i];
+    }
+    __syncthreads();
+    if (j0 + kKeys <= plast) load(j0 + kKeys);
+    // wave-uniform: all keys later than the wave's queries, or all in front of their windows
+    if (j0 > pw + 31 || (a.window > 0 && j0 + kKeys - 1 <= pw - a.window)) continue;
+    f32x16 sc[2];
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt) {
+      sc[kt] = zero16();
+#pragma unroll
+      for (int k = 0; k < NN; ++k) sc[kt] = mfma(lds_row16(lk, kt * 32 + l32, 2 * k + hh), qn[k], sc[kt]);
+#pragma unroll
+      for (int k = 0; k < NR; ++k)
+        if (k * 16 < a.rot_dim) sc[kt] = mfma(lds_row16(lr, kt * 32 + l32, 2 * k + hh), qr[k], sc[kt]);
+    }
+    const bool whole = j0 + kKeys - 1 <= pw && (a.window <= 0 || pw + 31 - j0 < a.window);
+    float m = -INFINITY;
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        float x = sc[kt][i] * sc2;
+        if (!whole) {
+          const int dist = pq - (j0 + kt * 32 + acc_row(i, hh));
+          if (dist < 0 || (a.window > 0 && dist >= a.window)) x = -INFINITY;
+        }
+        sc[kt][i] = x;
+        m = fmaxf(m, x);
+      }
+    m = fmaxf(m, xor32(m));
+    const float Mn = fmaxf(M, m), Ms = Mn == -INFINITY ? 0.f : Mn;  // no visible key yet: weights 0
+    const float f = fast_exp2(M - Ms);
+    float l = 0.f;
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        sc[kt][i] = fast_exp2(sc[kt][i] - Ms);
+        l += sc[kt][i];
+      }
+    L = L * f + l + xor32(l);
+    M = Mn;
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) acc[j][i] *= f;
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+      for (int x = 0; x < 2; ++x) {
+        const bf16x8 p = acc_to_b(sc[kt], x);
+#pragma unroll
+        for (int j = 0; j < NV; ++j) acc[j] = mfma(lds_trA(lv, kt * 32 + 16 * x, j, lane), p, acc[j]);
+      }
+  }
+  const int t = w * 32 + l32;
+  if (t < n) {
+    const float inv = L > 0.f ? 1.f / L : 0.f;
+    unsigned short* o = a.out + ((int64_t)(row0 + t) * a.H + h) * a.vdim;
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+#pragma unroll
+      for (int g = 0; g < 4; ++g) {
+        const int v = j * 32 + 8 * g + 4 * hh;
+        if (v < a.vdim) {
+          u16x4 r;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) r[e] = f32_to_bf16(acc[j][4 * g + e] * inv);
+          *reinterpret_cast<u16x4*>(o + v) = r;
+        }
+      }
+  }
+}
+
+inline bool aligned(const void* p, size_t n) { return reinterpret_cast<uintptr_t>(p) % n == 0; }
+
+// The fields of Args every form uses; q may be [T, H (dim + rot)] or None
+void check_batch(const at::Tensor& rows, const at::Tensor& table, const at::Tensor& q_start, const at::Tensor& q_len,
+                 const at::Tensor& kv_len, const at::Tensor& cache) {
+  const int64_t S = q_start.numel();
+  SXE_CHECK(rows.is_cuda() && rows.scalar_type() == at::kInt && rows.is_contiguous() && rows.dim() == 2 && rows.size(1) == 2,
+            "latent_attention: rows int32 [n, 2]");
+  SXE_CHECK(table.is_cuda() && table.scalar_type() == at::kInt && table.is_contiguous() && table.dim() == 2 && table.size(0) == S,
+            "latent_attention: block table int32 [S, blocks]");
+  for (const auto* t : {&q_start, &q_len, &kv_len})
+    SXE_CHECK(t->is_cuda() && t->is_contiguous() && t->scalar_type() == at::kInt && t->numel() == S, "latent_attention: int32 [S]");
+  SXE_CHECK(cache.is_cuda() && cache.dim() == 4 && cache.size(1) == 1 && cache.is_contiguous(),
+            "latent_attention: cache [blocks, 1, bs, row] contiguous");
+}
+
+}  // namespace lt
+
+at::Tensor rotation_table(const at::Tensor& positions, int64_t dims, double base) {
+  SXE_CHECK_CUDA(positions);
+  SXE_CHECK(positions.scalar_type() == at::kLong && positions.is_contiguous() && dims > 0 && dims % 2 == 0 && base > 0,
+            "rotation_table: positions int64, even dims");
+  const int64_t T = positions.numel(), half = dims / 2;
+  auto out = at::empty({T, half, 2}, positions.options().dtype(at::kFloat));
+  if (T == 0) return out;
+  SXE_CHECK(T * half < (1ll << 31), "rotation_table: too large");
+  c10::DeviceGuard g(positions.device());
+  hipLaunchKernelGGL(lt::rotation_table_kernel, dim3((T * half + lt::kThreads - 1) / lt::kThreads), dim3(lt::kThreads), 0,
+                     cur_stream(), positions.data_ptr<int64_t>(), (int)T, (int)half, std::log2(base), out.data_ptr<float>());
+  SXE_LAUNCH_CHECK();
+  return out;
+}
+
+at::Tensor latent_append(const at::Tensor& proj, const at::Tensor& qw, const at::Tensor& kw, at::Tensor cache,
+                         const at::Tensor& slots, const at::Tensor& rot, int64_t q_rank, int64_t rank, int64_t R, int64_t rot_dim,
+                         double eps) {
+  SXE_CHECK_CUDA(proj);
+  const int64_t T = proj.size(0);
+  SXE_CHECK(proj.dim() == 2 && proj.stride(1) == 1 && proj.size(1) >= q_rank + rank + rot_dim, "latent_append: proj");
+  SXE_CHECK(qw.is_contiguous() && qw.numel() == q_rank && kw.is_contiguous() && kw.numel() == rank && qw.is_cuda() && kw.is_cuda() &&
+                qw.scalar_type() == proj.scalar_type() && kw.scalar_type() == proj.scalar_type(), "latent_append: norm weights");
+  SXE_CHECK(cache.is_cuda() && cache.dim() == 4 && cache.size(1) == 1 && cache.is_contiguous() &&
+                cache.scalar_type() == proj.scalar_type() && R >= rank && cache.size(3) >= R + rot_dim,
+            "latent_append: cache [blocks, 1, bs, row]");
+  SXE_CHECK(slots.is_cuda() && slots.scalar_type() == at::kLong && slots.is_contiguous() && slots.numel() == T, "latent_append: slots");
+  SXE_CHECK(rot.is_cuda() && rot.scalar_type() == at::kFloat && rot.is_contiguous() && rot.numel() == T * rot_dim && rot_dim % 2 == 0,
+            "latent_append: rotation table");
+  auto cq = at::empty({T, q_rank}, proj.options());
+  if (T == 0) return cq;
+  c10::DeviceGuard g(proj.device());
+  lt::AppendArgs a{proj.data_ptr(), proj.stride(0), qw.data_ptr(), kw.data_ptr(), rot.data_ptr<float>(), slots.data_ptr<int64_t>(),
+                   cq.data_ptr(), cache.data_ptr(), (int)q_rank, (int)rank, (int)R, (int)rot_dim, (int)cache.size(3),
+                   cache.size(0) * cache.size(2), (float)eps};
+  const bool vec = q_rank % 8 == 0 && rank % 8 == 0 && proj.stride(0) % 8 == 0 && cache.size(3) % 8 == 0 &&
+                   lt::aligned(a.proj, 16) && lt::aligned(a.qw, 16) && lt::aligned(a.kw, 16) && lt::aligned(a.cq, 16) &&
+                   lt::aligned(a.cache, 16);
+  SXE_DISPATCH_DT(dtype_of(proj), D, {
+    if (vec) hipLaunchKernelGGL((lt::latent_append_kernel<D, 8>), dim3(T), dim3(lt::kThreads), 0, cur_stream(), a);
+    else hipLaunchKernelGGL((lt::latent_append_kernel<D, 1>), dim3(T), dim3(lt::kThreads), 0, cur_stream(), a);
+  });
+  SXE_LAUNCH_CHECK();
+  return cq;
+}
+
+// q [T, H (dim + rot)], uk [H, dim, rank], uv [H, rank, vdim], out [T, H vdim]; rows of `rows` are written
+void latent_attention_generic(const at::Tensor& q, const at::Tensor& uk, const at::Tensor& uv, const at::Tensor& cache,
+                              const at::Tensor& rot, const at::Tensor& rows, const at::Tensor& table, const at::Tensor& q_start,
+                              const at::Tensor& q_len, const at::Tensor& kv_len, at::Tensor out, int64_t rot_dim, int64_t R,
+                              double scale, int64_t window) {
+  SXE_CHECK_CUDA(q);
+  lt::check_batch(rows, table, q_start, q_len, kv_len, cache);
+  const int64_t n = rows.size(0), H = uk.size(0), dim = uk.size(1), rank = uk.size(2), vdim = uv.size(2);
+  SXE_CHECK(q.is_contiguous() && q.dim() == 2 && q.size(1) == H * (dim + rot_dim) && uk.is_contiguous() && uv.is_contiguous() &&
+                uv.size(0) == H && uv.size(1) == rank && out.is_contiguous() && out.size(0) == q.size(0) && out.size(1) == H * vdim &&
+                cache.size(3) >= R + rot_dim && R >= rank,
+            "latent_attention: shapes");
+  SXE_CHECK(rot.is_contiguous() && rot.scalar_type() == at::kFloat && rot.numel() == q.size(0) * rot_dim, "latent_attention: rotation");
+  for (const auto* t : {&uk, &uv, &cache, (const at::Tensor*)&out})
+    SXE_CHECK(t->is_cuda() && t->scalar_type() == q.scalar_type(), "latent_attention: one dtype");
+  if (n == 0) return;
+  c10::DeviceGuard g(q.device());
+  lt::Args a{q.data_ptr(), rot.data_ptr<float>(), rows.data_ptr<int>(), table.data_ptr<int>(), q_start.data_ptr<int>(),
+             q_len.data_ptr<int>(), kv_len.data_ptr<int>(), cache.data_ptr(), cache.size(0), (int)table.size(1), (int)cache.size(2),
+             (int)H, (int)dim, (int)rot_dim, (int)rank, (int)R, (int)cache.size(3), (int)vdim, (int)window, (float)scale};
+  const size_t lds = sizeof(float) * (2 * rank + rot_dim + lt::kThreads);
+  SXE_CHECK(lds <= 150 * 1024 && H <= 65535, "latent_attention: latent of ", rank, " does not fit a workgroup");
+  SXE_DISPATCH_DT(dtype_of(q), D, {
+    using S = dt_traits<D>::storage;
+    SXE_HIP_CHECK(hipFuncSetAttribute((const void*)lt::latent_generic_kernel<D>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    hipLaunchKernelGGL((lt::latent_generic_kernel<D>), dim3(n, H), dim3(lt::kThreads), lds, cur_stream(), a,
+                       static_cast<const S*>(uk.data_ptr()), static_cast<const S*>(uv.data_ptr()), static_cast<S*>(out.data_ptr()));
+  });
+  SXE_LAUNCH_CHECK();
+}
+
+// The token form's three launches; out [T, H vdim], bf16, R <= 512
+void latent_attention_token(const at::Tensor& q, const at::Tensor& uk, const at::Tensor& uv, const at::Tensor& cache,
+                            const at::Tensor& rot, const at::Tensor& rows, const at::Tensor& table, const at::Tensor& q_start,
+                            const at::Tensor& q_len, const at::Tensor& kv_len, at::Tensor out, int64_t splits, int64_t rot_dim,
+                            int64_t R, double scale, int64_t window) {
+  SXE_CHECK_CUDA(q);
+  lt::check_batch(rows, table, q_start, q_len, kv_len, cache);
+  const int64_t n = rows.size(0), H = uk.size(0), dim = uk.size(1), rank = uk.size(2), vdim = uv.size(2), row = cache.size(3);
+  SXE_CHECK(q.is_contiguous() && q.dim() == 2 && q.size(1) == H * (dim + rot_dim) && uk.is_contiguous() && uv.is_contiguous() &&
+                uv.size(0) == H && uv.size(1) == rank && out.is_contiguous() && out.size(0) == q.size(0) && out.size(1) == H * vdim &&
+                R >= rank && R % 32 == 0 && R <= 512 && row % 32 == 0 && row - R >= rot_dim && row - R <= 64 && scale > 0,
+            "latent_attention: shapes");
+  SXE_CHECK(rot.is_contiguous() && rot.scalar_type() == at::kFloat && rot.numel() == q.size(0) * rot_dim, "latent_attention: rotation");
+  for (const auto* t : {&q, &uk, &uv, &cache, (const at::Tensor*)&out})
+    SXE_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16, "latent_attention: token form takes bf16");
+  SXE_CHECK(lt::aligned(cache.data_ptr(), 16) && splits >= 1 && splits <= 65535 && H <= 65535, "latent_attention: splits");
+  if (n == 0) return;
+  c10::DeviceGuard g(q.device());
+  lt::Args a{q.data_ptr(), rot.data_ptr<float>(), rows.data_ptr<int>(), table.data_ptr<int>(), q_start.data_ptr<int>(),
+             q_len.data_ptr<int>(), kv_len.data_ptr<int>(), cache.data_ptr(), cache.size(0), (int)table.size(1), (int)cache.size(2),
+             (int)H, (int)dim, (int)rot_dim, (int)rank, (int)R, (int)row, (int)vdim, (int)window, (float)scale};
+  auto qa = at::empty({n, H, row}, q.options());
+  auto po = at::empty({splits, n, H, R}, q.options().dtype(at::kFloat)), pml = at::empty({splits, n, H, 2}, po.options());
+  auto u16 = [](const at::Tensor& t) { return static_cast<unsigned short*>(t.data_ptr()); };
+  auto heads = [&](auto kern, int64_t K, int64_t N, int TT, int LN, auto... more) {
+    const size_t lds = sizeof(float) * (TT * K + 4 * TT * LN * 8);
+    SXE_CHECK(lds <= 150 * 1024 && (n + TT - 1) / TT <= 65535, "latent_attention: sizes");
+    SXE_HIP_CHECK(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    hipLaunchKernelGGL(kern, dim3(H, (N + LN * 8 - 1) / (LN * 8), (n + TT - 1) / TT), dim3(lt::kThreads), lds, cur_stream(), a, (int)n,
+                       more...);
+  };
+  const bool vk = rank % 8 == 0 && lt::aligned(uk.data_ptr(), 16), vv = vdim % 8 == 0 && lt::aligned(uv.data_ptr(), 16);
+  if (!vk) heads(lt::latent_absorb_kernel<4, 16, false>, dim, rank, 4, 16, u16(uk), u16(qa));
+  else if (n == 1) heads(lt::latent_absorb_kernel<1, 16, true>, dim, rank, 1, 16, u16(uk), u16(qa));
+  else if (n <= 4) heads(lt::latent_absorb_kernel<4, 16, true>, dim, rank, 4, 16, u16(uk), u16(qa));
+  else heads(lt::latent_absorb_kernel<8, 16, true>, dim, rank, 8, 16, u16(uk), u16(qa));
+  auto token = [&](auto kern, int PN) {
+    const size_t lds = (PN + 1) * lt::kKeys * mf::ROWB + 32 * lt::kSRow * sizeof(float);
+    SXE_HIP_CHECK(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    hipLaunchKernelGGL(kern, dim3(n, (H + 31) / 32, splits), dim3(lt::kThreads), lds, cur_stream(), a, (int)n,
+                       (const unsigned short*)u16(qa), po.data_ptr<float>(), pml.data_ptr<float>());
+  };
+  if (R <= 128) token(lt::latent_token_kernel<1>, 1);
+  else if (R <= 256) token(lt::latent_token_kernel<2>, 2);
+  else token(lt::latent_token_kernel<4>, 4);
+  const float *ppo = po.data_ptr<float>(), *pm = pml.data_ptr<float>();
+  const int sp = (int)splits;
+  if (!vv) heads(lt::latent_expand_kernel<4, 16, false>, rank, vdim, 4, 16, sp, ppo, pm, u16(uv), u16(out));
+  else if (n == 1) heads(lt::latent_expand_kernel<1, 4, true>, rank, vdim, 1, 4, sp, ppo, pm, u16(uv), u16(out));
+  else if (n <= 4) heads(lt::latent_expand_kernel<4, 4, true>, rank, vdim, 4, 4, sp, ppo, pm, u16(uv), u16(out));
+  else heads(lt::latent_expand_kernel<8, 16, true>, rank, vdim, 8, 16, sp, ppo, pm, u16(uv), u16(out));
+  SXE_LAUNCH_CHECK();
+}
+
+// kv [Nk, H (dim + vdim)]: all heads' keys, then all heads' values; lat [Nk, row]: the cache rows they come from
+void latent_attention_tile(const at::Tensor& q, const at::Tensor& kv, const at::Tensor& lat, const at::Tensor& rot,
+                           const at::Tensor& chunks, const at::Tensor& first, const at::Tensor& q_start, const at::Tensor& q_len,
+                           const at::Tensor& kv_len, at::Tensor out, int64_t H, int64_t dim, int64_t rot_dim, int64_t vdim, int64_t R,
+                           double scale, int64_t window) {
+  SXE_CHECK_CUDA(q);
+  const int64_t S = q_start.numel(), nc = chunks.size(0), Nk = kv.size(0);
+  for (const auto* t : {&q, &kv, &lat, (const at::Tensor*)&out})
+    SXE_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16 && t->is_contiguous() && t->dim() == 2 && lt::aligned(t->data_ptr(), 16),
+              "latent_attention: tile form takes bf16 rows");
+  SXE_CHECK(dim <= 128 && vdim <= 128 && rot_dim <= 64 && dim % 8 == 0 && vdim % 8 == 0 && rot_dim % 8 == 0 &&
+                q.size(1) == H * (dim + rot_dim) && kv.size(1) == H * (dim + vdim) && lat.size(0) == Nk && lat.size(1) >= R + rot_dim &&
+                R % 8 == 0 && lat.size(1) % 8 == 0 && out.size(0) == q.size(0) && out.size(1) == H * vdim,
+            "latent_attention: tile form shapes");
+  SXE_CHECK(chunks.is_cuda() && chunks.scalar_type() == at::kInt && chunks.is_contiguous() && chunks.dim() == 2 && chunks.size(1) == 3 &&
+                first.is_cuda() && first.scalar_type() == at::kInt && first.is_contiguous() && first.numel() == 2 * S,
+            "latent_attention: tables");
+  for (const auto* t : {&q_start, &q_len, &kv_len})
+    SXE_CHECK(t->is_cuda() && t->is_contiguous() && t->scalar_type() == at::kInt && t->numel() == S, "latent_attention: int32 [S]");
+  SXE_CHECK(rot.is_contiguous() && rot.scalar_type() == at::kFloat && rot.numel() == q.size(0) * rot_dim, "latent_attention: rotation");
+  if (nc == 0 || Nk == 0) return;
+  SXE_CHECK(H <= 65535, "latent_attention: heads");
+  c10::DeviceGuard g(q.device());
+  auto u16 = [](const at::Tensor& t) { return static_cast<unsigned short*>(t.data_ptr()); };
+  lt::TileArgs a{u16(q), u16(kv), u16(lat), rot.data_ptr<float>(), chunks.data_ptr<int>(), first.data_ptr<int>(), q_start.data_ptr<int>(),
+                 q_len.data_ptr<int>(), kv_len.data_ptr<int>(), u16(out), kv.stride(0), (int)H, (int)dim, (int)rot_dim, (int)vdim, (int)R,
+                 (int)lat.size(1), (int)window, (int)Nk, (float)scale};
+  auto go = [&](auto kern) {
+    const size_t lds = 2 * lt::kQ * mf::ROWB;  // the key tile (3 panels of 64 rows) fits in the queries' space
+    SXE_HIP_CHECK(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    hipLaunchKernelGGL(kern, dim3(nc, H), dim3(lt::kThreads), lds, cur_stream(), a);
+  };
+  if (dim <= 64 && vdim <= 64) go(lt::latent_tile_kernel<64, 64>);
+  else if (dim <= 64) go(lt::latent_tile_kernel<64, 128>);
+  else if (vdim <= 64) go(lt::latent_tile_kernel<128, 64>);
+  else go(lt::latent_tile_kernel<128, 128>);
+  SXE_LAUNCH_CHECK();
+}
+
+}  // namespace sxe
+
+TORCH_LIBRARY_FRAGMENT(sxe, m) {
+  m.def("rotation_table(Tensor positions, int dims, float base) -> Tensor");
+  m.def("latent_append(Tensor proj, Tensor qw, Tensor kw, Tensor(a!) cache, Tensor slots, Tensor rot, int q_rank, int rank, int R, "
+        "int rot_dim, float eps) -> Tensor");
+  m.def("latent_attention_generic(Tensor q, Tensor uk, Tensor uv, Tensor cache, Tensor rot, Tensor rows, Tensor table, "
+        "Tensor q_start, Tensor q_len, Tensor kv_len, Tensor(a!) out, int rot_dim, int R, float scale, int window) -> ()");
+  m.def("latent_attention_token(Tensor q, Tensor uk, Tensor uv, Tensor cache, Tensor rot, Tensor rows, Tensor table, "
+        "Tensor q_start, Tensor q_len, Tensor kv_len, Tensor(a!) out, int splits, int rot_dim, int R, float scale, int window) -> ()");
+  m.def("latent_attention_tile(Tensor q, Tensor kv, Tensor lat, Tensor rot, Tensor chunks, Tensor first, Tensor q_start, "
+        "Tensor q_len, Tensor kv_len, Tensor(a!) out, int H, int dim, int rot_dim, int vdim, int R, float scale, int window) -> ()");
+}
+TORCH_LIBRARY_IMPL(sxe, CUDA, m) {
+  m.impl("rotation_table", &sxe::rotation_table);
+  m.impl("latent_append", &sxe::latent_append);
+  m.impl("latent_attention_generic", &sxe::latent_attention_generic);
+  m.impl("latent_attention_token", &sxe::latent_attention_token);
+  m.impl("latent_attention_tile", &sxe::latent_attention_tile);
+}

@@ -257,7 +257,7 @@ __global__ __launch_bounds__(kThreads) void gated_rms_norm_kernel(const typename
       const f32x4 g = load4<T>(gr + c), q = load4<T>(w + c);
       f32x4 h;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) h[j] = v[i][j] * rs * q[j] / (1.f + __expf(-g[j]));
+      for (int j = 0; j < 4; ++j) h[j] = v[i][j] * rs * q[j] / (1.f + expf(-g[j]));
       store4<T>(out + t * W + c, h);
     }
   } else {
@@ -268,7 +268,7 @@ __global__ __launch_bounds__(kThreads) void gated_rms_norm_kernel(const typename
     ss = block_sum<kThreads / 64>(ss, red);
     const float rs = 1.f / sqrtf(ss / (float)W + eps);
     for (int c = threadIdx.x; c < W; c += kThreads)
-      out[t * W + c] = from_f32<T>(to_f32<T>(xr[c]) * rs * to_f32<T>(w[c]) / (1.f + __expf(-to_f32<T>(gr[c]))));
+      out[t * W + c] = from_f32<T>(to_f32<T>(xr[c]) * rs * to_f32<T>(w[c]) / (1.f + expf(-to_f32<T>(gr[c]))));
   }
 }
 

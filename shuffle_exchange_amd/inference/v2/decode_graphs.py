@@ -49,7 +49,11 @@ class _StaticBatch:
         self.host_q_len = [1] * S
         self.host_q_start = list(range(S))
         self.host_kv_len = [kv_bucket] * S
+        self.rows = torch.arange(S, dtype=torch.int32, device=device)[:, None].repeat(1, 2)
         self.copied = None  # event: last H2D copy out of the pinned buffers
+
+    def token_rows(self, below=None):
+        return self.rows
 
 
 class DecodeGraphRunner:

@@ -25,8 +25,8 @@ def main(argv=None):
     a = ap.parse_args(argv)
     from . import RaggedInferenceEngineConfig, build_hf_engine
     if torch.cuda.is_available():
-        from ...ops import native
-        native.ensure_serving_library()
+        from .model_implementations.layered_decoder import ensure_library
+        ensure_library(a.model)
     eng = build_hf_engine(a.model, RaggedInferenceEngineConfig(num_kv_blocks=a.kv_blocks), dtype=getattr(torch, a.dtype),
                           weight_quant=a.weight_quant)
     prompts = [[int(x) for x in p.split(",") if x.strip()] for p in a.prompt]

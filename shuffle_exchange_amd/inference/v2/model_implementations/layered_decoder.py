@@ -280,6 +280,22 @@ def _bipotar_weights(spec, sd):
 ARCHITECTURES = {"Tobinex": (_tobinex_spec, _tobinex_weights), "Bipotar": (_bipotar_spec, _bipotar_weights)}
 
 
+# csrc/kernels sources a checkout with nothing built compiles to serve an architecture
+SERVING_UNITS = {"Tobinex": ("act", "mix_attn", "residual_norm", "skinny_gemm"),
+                 "Bipotar": ("act", "experts", "grouped_gemm", "latent_attn", "linear_attn", "residual_norm", "skinny_gemm")}
+
+
+def ensure_library(path):
+    """The HIP library that serving the checkpoint in ``path`` needs, compiled if nothing is built."""
+    from ....ops import native
+    with open(os.path.join(path, "config.json")) as f:
+        arch = json.load(f).get("architecture")
+    if arch in SERVING_UNITS:
+        native.ensure_serving_library(arch.lower(), SERVING_UNITS[arch])
+    else:
+        native.ensure_serving_library()
+
+
 def is_layered_config(cfg):
     return cfg.get("architecture") in ARCHITECTURES
 

@@ -297,6 +297,16 @@ class RaggedBatch:
             self._tables[key] = (slots, self._upload(first, 2))
         return self._tables[key]
 
+    def token_rows(self, below=None):
+        """int32 [n, 2] on the device: (sequence, row) of every new token of the sequences with fewer than
+        ``below`` new tokens (None: all)."""
+        key = ("tokens", below)
+        if key not in self._tables:
+            rows = [(i, q + j) for i, (q, n) in enumerate(zip(self.host_q_start, self.host_q_len))
+                    if below is None or n < below for j in range(n)]
+            self._tables[key] = self._upload(rows, 2)
+        return self._tables[key]
+
     def _upload(self, rows, n):
         t = torch.tensor(rows, dtype=torch.int32).reshape(-1, n)
         return t.pin_memory().to(self.slots.device, non_blocking=True) if self.slots.is_cuda else t

@@ -72,8 +72,8 @@ def main(argv=None):
         print("trace_run needs a GPU", file=sys.stderr)
         return 2
     torch.set_float32_matmul_precision("highest")
-    from ...ops import native
-    native.ensure_serving_library()
+    from .model_implementations.layered_decoder import ensure_library
+    ensure_library(a.model)
     engine = engine_for_trace(a.model, getattr(torch, a.dtype), a.max_tokens)
     replay(engine, sys.stdin, a.out)
     return 0

@@ -13,7 +13,6 @@ latent (decode: the cache row is read once for all heads).
 import torch
 
 from . import native
-from .paged_attention import choose_splits
 
 TILE_MIN = 32  # sequences with at least this many new tokens take the expanded form
 PAD = 32       # bf16 cache rows: both parts padded to a multiple of this
@@ -73,43 +72,43 @@ def latent_attention(q, uk, uv, ukv, cache, batch, rot, heads, dim, rot_dim, vdi
     if not native.use_hip(q):
         return latent_attention_reference(q, uk, uv, cache, batch, rot, heads, dim, rot_dim, vdim, rank, scale, window)
     R, _ = latent_row(rank, rot_dim, q.dtype)
-    keys = int(batch.max_kv_len) if not window else min(int(batch.max_kv_len), int(window))
     if form == "auto":
         tile = ukv is not None and tile_ok(q, dim, rot_dim, vdim) and max(batch.host_q_len) >= TILE_MIN
-        rest = min(batch.host_q_len) < TILE_MIN
-        token = "token" if token_ok(q, R, rot_dim, scale) else "generic"
+        least = TILE_MIN if tile and min(batch.host_q_len) < TILE_MIN else 1
+        token = token_ok(q, R, rot_dim, scale)
     else:
-        tile, rest, token = form == "tile", form != "tile", form
+        tile, least, token = form == "tile", 1, form == "token"
     out = torch.empty(q.shape[0], heads * vdim, dtype=q.dtype, device=q.device)
+    w = int(window or 0)
+    lens = (batch.q_start, batch.q_len, batch.kv_len)
     if tile:
-        least = 1 if not rest else TILE_MIN
         slots, first = batch.key_rows(window, least)
-        lat = torch.ops.sxe.gather_latent(cache, slots)
+        lat = cache.view(-1, cache.shape[3]).index_select(0, slots)
         kv = torch.nn.functional.linear(lat[:, :rank], ukv)
-        table = batch.chunks(TILE_TOKENS, least)
-        torch.ops.sxe.latent_attention_tile(q, kv, lat, rot, table, first, batch.q_start, batch.q_len, batch.kv_len, out,
-                                            int(heads), int(dim), int(rot_dim), int(vdim), int(R), float(scale), int(window or 0))
-        if not rest:
+        torch.ops.sxe.latent_attention_tile(q, kv, lat, rot, batch.chunks(TILE_TOKENS, least), first, *lens, out, int(heads), int(dim),
+                                            int(rot_dim), int(vdim), int(R), float(scale), w)
+        if least == 1:
             return out
-    limit = TILE_MIN if tile else 0  # sequences at or above it are done
-    if token == "generic":
-        torch.ops.sxe.latent_attention_generic(q, uk, uv, cache, rot, batch.block_table, batch.q_start, batch.q_len,
-                                               batch.kv_len, out, limit, int(rot_dim), int(R), float(scale), int(window or 0))
-        return out
-    splits = choose_splits(q.shape[0], -(-heads // 32), keys)
-    qa = torch.ops.sxe.latent_absorb(q, uk, rot, int(rot_dim), int(R), int(cache.shape[3]))
-    part, ml = torch.ops.sxe.latent_attention_token(qa, cache, batch.block_table, batch.q_start, batch.q_len, batch.kv_len,
-                                                    limit, keys, int(splits), int(R), float(scale), int(window or 0))
-    torch.ops.sxe.latent_expand(part, ml, uv, batch.q_start, batch.q_len, limit, out)
+    rows = batch.token_rows(TILE_MIN if tile else None)  # tokens of the other sequences
+    if token:
+        keys = int(batch.max_kv_len) if not w else min(int(batch.max_kv_len), w)
+        wgs = max(1, rows.shape[0] * -(-heads // TOKEN_HEADS))
+        splits = max(1, min(-(-keys // TOKEN_KEYS), TOKEN_WGS // wgs))
+        torch.ops.sxe.latent_attention_token(q, uk, uv, cache, rot, rows, batch.block_table, *lens, out, splits, int(rot_dim),
+                                             int(R), float(scale), w)
+    else:
+        torch.ops.sxe.latent_attention_generic(q, uk, uv, cache, rot, rows, batch.block_table, *lens, out, int(rot_dim), int(R),
+                                               float(scale), w)
     return out
 
 
+TOKEN_HEADS, TOKEN_KEYS, TOKEN_WGS = 32, 64, 256  # token form: heads and keys of a tile; workgroups to aim for with key splits
 TILE_TOKENS = 128  # query tokens of a workgroup of the expanded form
 
 
 def tile_ok(q, dim, rot_dim, vdim):
     return (q.dtype == torch.bfloat16 and dim <= 128 and rot_dim <= 64 and vdim <= 128 and dim % 8 == 0 and rot_dim % 8 == 0
-            and vdim % 8 == 0)
+            and vdim % 8 == 0 and q.data_ptr() % 16 == 0)
 
 
 def token_ok(q, R, rot_dim, scale):

@@ -34,7 +34,7 @@ def decay_attention(proj, state, decay, batch, heads, dim, vdim, act="silu", for
                                                       batch.state_slots, int(heads), int(dim), int(vdim), act == "silu")
         table = batch.chunks(CHUNK)
         return torch.ops.sxe.decay_attention_chunk(proj, state, decay, batch.q_start, batch.q_len, batch.kv_len,
-                                                   batch.state_slots, table, int(heads), int(dim), int(vdim), act == "silu")
+                                                   batch.state_slots, table, CHUNK, int(heads), int(dim), int(vdim), act == "silu")
     return decay_attention_reference(proj, state, decay, batch, heads, dim, vdim, act)
 
 

@@ -268,24 +268,31 @@ def route_topk(h, router, top):
     return idx.to(torch.int32), torch.softmax(val, -1)
 
 
+SKINNY_ROWS = 16  # mean rows per expert up to which the skinny expert kernels are used
+
+
 def expert_mlp(h, expert, weight, up, down, act="relu2"):
     """Two-layer experts up [E, F, D], down [E, D, F] on the rows ``route_topk`` chose. Returns (y, slots): y
-    [T * top, D] holds weight * down(act(up h)) of every (token, choice) and y[slots[t, j]] belongs to token t. No
-    host synchronisation. Few rows per expert: the weights are streamed once (skinny kernels, rows stay
-    in token order); more: rows sorted by expert for the grouped kernels, which gather them on the fly."""
+    [T * top, D] holds weight * down(act(up h)) of every (token, choice), y[slots[t, j]] belongs to token t. No
+    host synchronisation. Rows are sorted by expert and gathered inside the first product; few rows per
+    expert stream the weights through the skinny kernels, more take the grouped ones (csrc/kernels/experts.hip,
+    grouped_gemm.hip)."""
     T, k = expert.shape
     E = up.shape[0]
     if _hip(h):
-        if T * k <= SKINNY_ROWS * E or not grouped_gemm_ok(h, up) or down.shape[1] % 128:
-            lists = torch.ops.sxe.moe_lists(expert, E)
-        else:
-            lists = torch.ops.sxe.moe_lists(expert, E)
-        return torch.ops.sxe.expert_mlp(h, expert, weight, up, down, *lists, EXPERT_ACTS[act])
+        rows, ws, slots, offs, active = torch.ops.sxe.moe_lists(expert, weight, E)
+        R = T * k
+        if (R > SKINNY_ROWS * E and act in ("relu2", "none") and grouped_gemm_ok(h, up) and up.shape[1] % 128 == 0
+                and down.shape[1] % 128 == 0):
+            a = torch.ops.sxe.grouped_gemm_rows(h, up, offs, None, rows, EXPERT_ACTS[act])
+            return torch.ops.sxe.grouped_gemm_rows(a, down, offs, ws, None, 0), slots
+        a = torch.ops.sxe.expert_gemm(h, up, offs, active, rows, None, R, EXPERT_ACTS[act])
+        return torch.ops.sxe.expert_gemm(a, down, offs, active, None, ws, R, 0), slots
     y = torch.zeros(T * k, down.shape[1], dtype=h.dtype, device=h.device)
     flat = expert.reshape(-1)
+    f = {"relu2": lambda z: torch.relu(z) ** 2, "silu": F.silu, "none": lambda z: z}[act]
     for e in flat.unique().tolist():
         r = (flat == e).nonzero()[:, 0]
-        a = F.linear(h.index_select(0, r // k).float(), up[e].float())
-        a = {"relu2": lambda z: torch.relu(z) ** 2, "silu": F.silu, "none": lambda z: z}[act](a).to(h.dtype)
+        a = f(F.linear(h.index_select(0, r // k).float(), up[e].float())).to(h.dtype)
         y[r] = (F.linear(a.float(), down[e].float()) * weight.reshape(-1, 1)[r]).to(h.dtype)
     return y, torch.arange(T * k, dtype=torch.int32, device=h.device).view(T, k)

@@ -68,13 +68,10 @@ def require_cpu():
     return torch.ops.sxe_cpu
 
 
-SERVING_UNITS = ("act", "mix_attn", "residual_norm", "skinny_gemm")
-
-
-def ensure_serving_library():
-    """For command-line serving: use the full HIP library when it is built, else compile the kernels of the
-    layered decoders (SERVING_UNITS) into a library of their own, once per checkout (the build is
-    incremental: it is brought up to date when a source changed)."""
+def ensure_serving_library(name=None, units=None):
+    """For command-line serving: use the full HIP library when it is built, else compile ``units`` (sources of
+    csrc/kernels; None: all of them) into a library of their own called after ``name``, once per checkout
+    (the build is incremental: it is brought up to date when a source changed)."""
     global HIP_LIB
     if _state["hip"] is not None or os.path.exists(HIP_LIB):
         return
@@ -84,9 +81,9 @@ def ensure_serving_library():
     spec = importlib.util.spec_from_file_location("sxe_build", os.path.join(root, "csrc", "build.py"))
     b = importlib.util.module_from_spec(spec)
     spec.loader.exec_module(b)
-    out = os.path.join(_HERE, "_sxe_hip_serving.so")
+    out = HIP_LIB if units is None else os.path.join(_HERE, f"_sxe_hip_{name}.so")
     print("compiling the serving kernels", file=sys.stderr, flush=True)
-    b.build(only="hip", units=SERVING_UNITS, hip_out=out, verbose=False)
+    b.build(only="hip", units=units, hip_out=out, verbose=False)
     HIP_LIB = out
 
 
