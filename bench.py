@@ -28,7 +28,7 @@ architecture (no network access for checkpoints/datasets).
                       (auto_ac_policy: none when the activations fit -- from 2 GPUs --, else the
                       MLP-only policy that keeps the attention outputs, else full layers)
 ``--serve`` measures serving instead (one GPU, random weights): prefill and decode tokens/s of the layered
-decoder and of Llama at equal layer sizes.
+decoders, of Llama and of Mixtral at equal layer sizes (``--serve-models`` picks some of them).
 
 Every JSON line carries the full ZeRO/SP/EP configuration, the measured per-step communication
 volume per collective (``comm_measured``: calls and bytes per rank per step, from the comm facade's
@@ -239,14 +239,16 @@ def main():
                     help="offload configs: Twin-Flow offload_optimizer.ratio (share of the optimizer on the "
                          "host; default 1.0 = the whole optimizer, the reference's ZeRO-Infinity setting)")
     ap.add_argument("--serve", nargs="?", const="all", default=None, metavar="SIZE[,SIZE]",
-                    help="instead of training: prefill / decode throughput of the Tobinex decoder beside Llama at "
-                         "equal layer sizes (shuffle_exchange_amd/inference/v2/serve_bench.py), one JSON line each")
+                    help="instead of training: prefill / decode throughput of the Tobinex and Bipotar decoders beside Llama and "
+                         "Mixtral at equal layer sizes (shuffle_exchange_amd/inference/v2/serve_bench.py), one JSON line each")
+    ap.add_argument("--serve-models", default=None, metavar="MODEL[,MODEL]", help="models of --serve (default: all)")
     ap.add_argument("--device", default="cuda", choices=["cuda", "cpu"],
                     help="cpu = plumbing dry-run over gloo (tests only; invalid for the metric)")
     args = ap.parse_args()
     if args.serve is not None:
         from shuffle_exchange_amd.inference.v2 import serve_bench
-        serve_bench.run(sizes=None if args.serve == "all" else args.serve.split(","))
+        serve_bench.run(sizes=None if args.serve == "all" else args.serve.split(","),
+                        models=args.serve_models.split(",") if args.serve_models else None)
         return
     c = CONFIGS[args.config]
     on_gpu = args.device == "cuda"

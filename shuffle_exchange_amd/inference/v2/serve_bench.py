@@ -1,10 +1,13 @@
-"""Serving throughput of a layered decoder (layered_decoder.py) beside the Llama model at equal size:
-prefill and decode tokens/s through ``InferenceEngineV2.put`` with random weights of real-model layer
-sizes (``bench.py --serve``).
+"""Serving throughput of the layered decoders (layered_decoder.py) beside the Llama and Mixtral models at
+equal size: prefill and decode tokens/s through ``InferenceEngineV2.put`` with random weights of
+real-model layer sizes (``bench.py --serve``).
 
-The Llama model has the same width, heads, head size, feed-forward width, layer count and vocabulary; the
-layered design adds its output gate projection, the window (prompts longer than it attend to fewer keys)
-and the head mix. One JSON line per (size, model, workload).
+Every model has the same width, heads, head size, layer count and vocabulary. Tobinex and Llama share the
+dense feed-forward width; Tobinex adds its output gate projection, the window (prompts longer than it
+attend to fewer keys) and the head mix. Bipotar runs four layers twice -- latent attention + dense, twice
+linear attention + experts, latent attention + experts -- and shares Llama's feed-forward width in the dense
+layer, Mixtral's experts in the others (without the gate projection). One JSON line per (size, model,
+workload).
 """
 import json
 import time
@@ -15,6 +18,10 @@ import torch
 SIZES = {"8b": (4096, 32, 8, 128, 14336, 8, 32000, 1024, 16),
          "3b": (3072, 24, 8, 128, 8192, 8, 32000, 1024, 16),
          "1b": (2048, 16, 4, 128, 8192, 8, 32000, 512, 4)}
+# Bipotar: latent ranks of queries and keys, rotated size, window, experts, chosen, expert ff
+LATENT_MOE = {"8b": (1536, 512, 64, 1024, 32, 4, 1792),
+              "3b": (1024, 512, 64, 1024, 32, 4, 1536),
+              "1b": (768, 256, 64, 512, 16, 2, 1024)}
 PREFILL = ((1, 2048), (4, 2048), (1, 8192))      # (sequences, tokens each)
 DECODE = ((1, 2048), (4, 2048), (32, 2048), (128, 2048))  # (sequences, context)
 
@@ -47,7 +54,53 @@ def llama_model(size, device):
         return LlamaForCausalLM(cfg).to(torch.bfloat16).eval()
 
 
-MODELS = {"tobinex": tobinex_model, "llama": llama_model}
+def bipotar_model(size, device):
+    from ...ops.linear_attention import decay_table
+    from .model_implementations.layered_decoder import (LatentSpec, LayeredSpec, LayerSpec, LinearSpec, LoopSpec, MoESpec,
+                                                        RaggedLayeredDecoder)
+    D, H, _, d, ff, n, V, _, _ = SIZES[size]
+    qr, kr, rot, win, E, top, eff = LATENT_MOE[size]
+    latent = LatentSpec(H, d, rot, d, qr, kr, (d + rot) ** -0.5, 10000.0, win)
+    light = LinearSpec(H, d, d, [1 - 2.0 ** -(1 + 9 * h / (H - 1)) for h in range(H)])
+    moe = MoESpec(E, top, eff)
+    spec = LayeredSpec("Bipotar", V, D, 1e-5, norm_offset=0.0, residual="sandwich", loop=LoopSpec(0, 4, n // 4), layers=[
+        LayerSpec(latent, ff), LayerSpec(light, moe=moe), LayerSpec(light, moe=moe), LayerSpec(latent, moe=moe)])
+    bf = dict(dtype=torch.bfloat16, device=device)
+
+    def w(*shape):
+        return torch.randn(*shape, **bf) * shape[-1] ** -0.5
+
+    def one(k):
+        return torch.ones(k, **bf)
+    W = {"embed": w(V, D), "embed_norm": one(D), "final": one(D), "head": w(V, D), "layers": []}
+    for L in spec.layers:
+        x = {k: one(D) for k in ("norm1", "norm1b", "norm2", "norm2b")}
+        if L.mixer is light:
+            x.update(qkvg=w(4 * H * d, D), o_norm=one(H * d), o=w(D, H * d), decay=decay_table(light.decay, device))
+        else:
+            uk, uv = w(H * d, kr), w(H * d, kr)
+            x.update(dqkv=w(qr + kr + rot, D), q_norm=one(qr), kv_norm=one(kr), uq=w(H * (d + rot), qr), uk=uk.view(H, d, kr),
+                     uv=uv.view(H, d, kr).transpose(1, 2), ukv=torch.cat([uk, uv]), o=w(D, H * d))
+        if L.moe:
+            x.update(router=w(E, D), e_up=w(E, eff, D), e_down=w(E, D, eff))
+        else:
+            x.update(gu=w(2 * ff, D), down=w(D, ff))
+        W["layers"].append(x)
+    return RaggedLayeredDecoder(spec, W, torch.bfloat16, device)
+
+
+def mixtral_model(size, device):
+    from ...models import MixtralForCausalLM, mixtral_config
+    D, H, G, d, _, n, V, _, _ = SIZES[size]
+    _, _, _, _, E, top, eff = LATENT_MOE[size]
+    cfg = mixtral_config("mixtral-tiny", hidden_size=D, intermediate_size=eff, num_attention_heads=H, num_key_value_heads=G,
+                         num_hidden_layers=n, vocab_size=V, max_position_embeddings=16384, num_local_experts=E,
+                         num_experts_per_tok=top)
+    with torch.device(device):
+        return MixtralForCausalLM(cfg).to(torch.bfloat16).eval()
+
+
+MODELS = {"tobinex": tobinex_model, "bipotar": bipotar_model, "llama": llama_model, "mixtral": mixtral_model}
 
 
 def run(sizes=None, models=None, steps=16, warmup=4, emit=lambda row: print(json.dumps(row), flush=True), prefill=PREFILL,
