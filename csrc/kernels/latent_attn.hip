@@ -10,12 +10,15 @@
 //    read by rows for the scores and transposed for the weighted sum of latents -- each cache byte crosses
 //    HBM once for all heads -- and latent_expand merges the splits and applies W_uv;
 //  * tile form (prompts; bf16): keys and values of the window are expanded by a library product, then one
-//    workgroup per (128 queries, head) in the flash manner. The rotated key part is read from the gathered
-//    cache rows, queries are rotated on the way into LDS.
+//    workgroup per (256 queries, head) in the flash manner (8 waves of 32 queries, 64-key tiles loaded straight
+//    to a double-buffered LDS ring). The rotated key part is read from the gathered cache rows, queries are
+//    rotated on the way into their registers.
 // Only visible keys are enumerated (window: i sees 0 <= i - j < window). Scores, softmax and sums are fp32.
 #include "sxe_common.h"
 #include "sxe_mfma.h"
+#include "sxe_tile.h"
 #include <torch/library.h>
+#include <type_traits>
 
 namespace sxe {
 namespace lt {
@@ -298,30 +301,39 @@ __global__ __launch_bounds__(kThreads) void latent_expand_kernel(Args a, int n, 
   extern __shared__ float sm[];
   float* x = sm;                    // [TT][rank]
   float* part = sm + TT * a.rank;   // [4][TT][LN * 8]
+  float* wts = part + 4 * TT * LN * 8;  // [TT][splits]
   const int h = blockIdx.x, n0 = blockIdx.y * LN * 8, i0 = blockIdx.z * TT;
   const int64_t sstride = (int64_t)n * a.H;
-  for (int t = 0; t < TT; ++t) {
-    if (i0 + t >= n) {
-      for (int r = threadIdx.x; r < a.rank; r += kThreads) x[t * a.rank + r] = 0.f;
-      continue;
-    }
-    const int64_t th = (int64_t)(i0 + t) * a.H + h;
+  // weights of the splits: 2^(M_s - M) / sum, one wave per token
+  const int lane = threadIdx.x & 63;
+  for (int t = threadIdx.x >> 6; t < TT; t += 4) {
+    if (i0 + t >= n) continue;
+    const float* ml = pml + ((int64_t)(i0 + t) * a.H + h) * 2;
     float M = -INFINITY, L = 0.f;
-    for (int s = 0; s < splits; ++s) M = fmaxf(M, pml[(s * sstride + th) * 2]);
-    for (int s = 0; s < splits; ++s) {
-      const float m = pml[(s * sstride + th) * 2];
-      if (m != -INFINITY) L += exp2f(m - M) * pml[(s * sstride + th) * 2 + 1];
+    for (int s = lane; s < splits; s += 64) M = fmaxf(M, ml[s * sstride * 2]);
+    M = wave_max(M);
+    for (int s = lane; s < splits; s += 64) {
+      const float m = ml[s * sstride * 2], f = m == -INFINITY ? 0.f : exp2f(m - M);
+      wts[t * splits + s] = f;
+      if (f > 0.f) L += f * ml[s * sstride * 2 + 1];
     }
+    L = wave_sum(L);
     const float inv = L > 0.f ? 1.f / L : 0.f;
-    for (int r = threadIdx.x; r < a.rank; r += kThreads) {
-      float v = 0.f;
-#pragma unroll 4
+    for (int s = lane; s < splits; s += 64) wts[t * splits + s] *= inv;  // the lane's own entries
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < TT * a.rank; i += kThreads) {
+    const int t = i / a.rank, r = i - t * a.rank;
+    float v = 0.f;
+    if (i0 + t < n) {
+      const float* p = po + ((int64_t)(i0 + t) * a.H + h) * a.R + r;
+#pragma unroll 8
       for (int s = 0; s < splits; ++s) {
-        const float m = pml[(s * sstride + th) * 2];
-        if (m != -INFINITY) v += exp2f(m - M) * po[(s * sstride + th) * a.R + r];
+        const float f = wts[t * splits + s], o = p[s * sstride * a.R];
+        v += f > 0.f ? f * o : 0.f;  // a split without keys has not written its part
       }
-      x[t * a.rank + r] = v * inv;
     }
+    x[i] = v;
   }
   __syncthreads();
   float acc[TT][8];
@@ -490,8 +502,7 @@ __global__ __launch_bounds__(kThreads, 1) void latent_token_kernel(Args a, int n
 }
 
 // ------------------------------------------------------------------------------------------- tile form
-constexpr int kQ = 128;
-typedef float f32x2_t __attribute__((ext_vector_type(2)));
+constexpr int kQ = 256, kTileWaves = 8;
 
 struct TileArgs {
   const unsigned short *q, *kv, *lat;  // [T, H (dim + rot)], [Nk, H (dim + vdim)], [Nk, row]
@@ -503,156 +514,176 @@ struct TileArgs {
   float scale;
 };
 
-// DN, VP: dim and vdim padded to 64 / 128; the rotated part is padded to 64. grid (chunks of kQ rows, H)
-template <int DN, int VP>
-__global__ __launch_bounds__(kThreads, 2) void latent_tile_kernel(TileArgs a) {
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  constexpr int KC = DN / 8, VC = VP / 8, RC = 8, NN = DN / 16, NR = 4, NV = VP / 32;
-  const int c = blockIdx.x, h = blockIdx.y;
-  const int s = a.chunks[3 * c], row0 = a.chunks[3 * c + 1], n = a.chunks[3 * c + 2];
-  const int pos0 = a.kv_len[s] - a.q_len[s] + (row0 - a.q_start[s]);
-  const int f0 = a.first[2 * s], fp = a.first[2 * s + 1];  // list row and position of the first listed key
-  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l32 = lane & 31, hh = lane >> 5;
-  const int half = a.rot_dim / 2, ldq = a.H * (a.dim + a.rot_dim);
-  // ---- queries -> LDS -> fragments; the rotated part by pairs
-  char* lqr = smem + kQ * ROWB;
-  const unsigned short* qb = a.q + (int64_t)row0 * ldq + h * (a.dim + a.rot_dim);
-  const bool qv = a.dim % 8 == 0 && a.rot_dim % 8 == 0;
-  for (int x = threadIdx.x; x < kQ * KC; x += kThreads) {
-    const int t = x / KC, ch = x % KC;
-    u32x4 z = {0u, 0u, 0u, 0u};
-    if (t < n && ch * 8 < a.dim && qv) z = *reinterpret_cast<const u32x4*>(qb + (int64_t)t * ldq + ch * 8);
-    *reinterpret_cast<u32x4*>(smem + soff(t, ch)) = z;
+// One 64-key tile of a wave's online softmax: S^T = K Q^T (a lane holds one query's scores), the weights are the
+// B operand of O^T += V^T P^T as they are. MASK: some key of the tile is hidden from some query of the wave.
+template <bool MASK, int DN, int VP>
+__device__ __forceinline__ void latent_tile_step(const tl::LaneOffs<DN>& ok, const tl::LaneOffs<64>& orr, const tl::LaneOffs<VP>& ov,
+                                                 const char* lk, const bf16x8 (&qn)[DN / 16], const bf16x8 (&qr)[4],
+                                                 f32x16 (&acc)[VP / 32], float& M, float& L, float c, int j0, int pw, int lane,
+                                                 int win) {
+  const char *lr = lk + kKeys * 2 * DN, *lv = lr + kKeys * 128;
+  const int l32 = lane & 31, hh = lane >> 5;
+  // halves of the tile hidden from the whole wave: in front of every window, behind every query
+  const bool skip0 = MASK && pw - (j0 + 31) >= win, skip1 = MASK && j0 + 32 > pw + 31;
+  f32x16 s[2];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    s[j] = zero16();
+    if (j == 0 ? skip0 : skip1) continue;
+#pragma unroll
+    for (int k = 0; k < DN / 16; ++k) s[j] = mfma(tl::row_at(lk + 32 * j * 2 * DN, ok.row[k]), qn[k], s[j]);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) s[j] = mfma(tl::row_at(lr + 32 * j * 128, orr.row[k]), qr[k], s[j]);
   }
-  for (int x = threadIdx.x; x < kQ * 64; x += kThreads) {
-    const int t = x >> 6, d = x & 63;
-    float v = 0.f;
-    if (t < n && d < a.rot_dim) {
+  float mx = -INFINITY;
+  int dd = pw + l32 - j0 - 4 * hh;  // distance to the lane's first key row
+  if (MASK) asm volatile("" : "+v"(dd));
+#pragma unroll
+  for (int j = 0; j < 2; ++j)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      if (MASK) s[j][i] = (unsigned)(dd - 32 * j - acc_row(i, 0)) < (unsigned)win ? s[j][i] : -INFINITY;
+      mx = fmaxf(mx, s[j][i]);
+    }
+  mx = fmaxf(mx, xor32(mx)) * c;
+  // the reference maximum moves only when a tile exceeds it by 2^8; the sums are rescaled only then
+  const bool grow = mx > M + 8.f;
+  const float Mn = grow ? mx : M, ref = Mn == -INFINITY ? 0.f : Mn, alpha = fast_exp2(M - ref);
+  float ps = 0.f;
+#pragma unroll
+  for (int j = 0; j < 2; ++j)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const float p = fast_exp2(__builtin_fmaf(s[j][i], c, -ref));
+      s[j][i] = p;
+      ps += p;
+    }
+  L = L * alpha + ps;
+  M = Mn;
+  if (__any(grow)) {
+#pragma unroll
+    for (int t = 0; t < VP / 32; ++t)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) acc[t][i] *= alpha;
+  }
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    if (j == 0 ? skip0 : skip1) continue;
+#pragma unroll
+    for (int x = 0; x < 2; ++x) {
+      const bf16x8 p = acc_to_b(s[j], x);
+#pragma unroll
+      for (int t = 0; t < VP / 32; ++t) acc[t] = mfma(tl::tr_at(lv + (32 * j + 16 * x) * 2 * VP, ov.tr[t]), p, acc[t]);
+    }
+  }
+}
+
+// 8 rotated query components d0 .. d0 + 7 (zeros beyond rot_dim); qr: the head's rotated part, cs its table row
+__device__ __forceinline__ bf16x8 rotated8(const unsigned short* qr, const float* cs, int d0, int rot_dim) {
+  const int half = rot_dim / 2;
+  bf16x8 r;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) r[e] = (__bf16)0.f;
+  if (d0 >= rot_dim) return r;
+  if (half % 8 == 0) {
+    const bool lo = d0 < half;
+    const int j0 = lo ? d0 : d0 - half;
+    float u[8], y[8], t[16];
+    load8<DT::BF16>(qr + j0, u);
+    load8<DT::BF16>(qr + half + j0, y);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) *reinterpret_cast<f32x4*>(t + 4 * e) = *reinterpret_cast<const f32x4*>(cs + 2 * j0 + 4 * e);
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+      r[e] = (__bf16)(lo ? u[e] * t[2 * e] - y[e] * t[2 * e + 1] : y[e] * t[2 * e] + u[e] * t[2 * e + 1]);
+    return r;
+  }
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const int d = d0 + e;
+    if (d < rot_dim) {
       const int j = d < half ? d : d - half;
-      const unsigned short* qr = qb + (int64_t)t * ldq + a.dim;
-      const float u = bf16_to_f32(qr[j]), y = bf16_to_f32(qr[half + j]);
-      const f32x2_t cs = *reinterpret_cast<const f32x2_t*>(a.rot + ((int64_t)(row0 + t) * half + j) * 2);
-      v = d < half ? u * cs[0] - y * cs[1] : y * cs[0] + u * cs[1];
+      const float u = bf16_to_f32(qr[j]), y = bf16_to_f32(qr[half + j]), co = cs[2 * j], si = cs[2 * j + 1];
+      r[e] = (__bf16)(d < half ? u * co - y * si : y * co + u * si);
     }
-    *reinterpret_cast<unsigned short*>(lqr + soff(t, d >> 3) + (d & 7) * 2) = f32_to_bf16(v);
   }
-  __syncthreads();
-  bf16x8 qn[NN], qr[NR];
-#pragma unroll
-  for (int k = 0; k < NN; ++k) qn[k] = lds_row16(smem, w * 32 + l32, 2 * k + hh);
-#pragma unroll
-  for (int k = 0; k < NR; ++k) qr[k] = lds_row16(lqr, w * 32 + l32, 2 * k + hh);
-  const int pw = pos0 + w * 32, pq = pw + l32;  // the wave's first position, the lane's
-  const int plast = pos0 + n - 1;
-  const int lo = max(fp, a.window > 0 ? pos0 + 1 - a.window : 0);
-  char *lk = smem, *lr = smem + kKeys * ROWB, *lv = smem + 2 * kKeys * ROWB;
-  constexpr int NK = kKeys * KC / kThreads, NRL = kKeys * RC / kThreads, NVL = kKeys * VC / kThreads;
-  u32x4 rk[NK], rr[NRL], rv[NVL];
+  return r;
+}
+
+// DN, VP: dim and vdim padded to 64 / 128; the rotated part is padded to 64. grid (H, chunks of kQ rows): a head's
+// chunks share an XCD when the heads are a multiple of its count
+template <int DN, int VP>
+__global__ __launch_bounds__(64 * kTileWaves, 1) void latent_tile_kernel(TileArgs a) {
+  char* smem = tl::lds;
+  constexpr int KB = kKeys * 2 * DN, RB = kKeys * 128, SLOT = KB + RB + kKeys * 2 * VP;
+  const int c = gridDim.y - 1 - blockIdx.y, h = blockIdx.x;  // late chunks see more keys: first
+  const int s = a.chunks[3 * c], row0 = a.chunks[3 * c + 1], n = a.chunks[3 * c + 2];
+  const int pos0 = a.kv_len[s] - a.q_len[s] + (row0 - a.q_start[s]), plast = pos0 + n - 1;
+  const int f0 = a.first[2 * s], fp = a.first[2 * s + 1];  // list row and position of the first listed key
+  const int win = a.window > 0 ? a.window : 0x7fffffff;
+  const int lo = max(fp, a.window > 0 ? pos0 + 1 - a.window : 0), ntiles = (plast - lo) / kKeys + 1;
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l32 = lane & 31, hh = lane >> 5;
   const unsigned short *kb = a.kv + h * a.dim, *vb = a.kv + a.H * a.dim + h * a.vdim, *rb = a.lat + a.R;
-  auto at = [&](int j) { return (int64_t)min(max(f0 + j - fp, 0), a.Nk - 1); };
-  auto load = [&](int j0) {
-#pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int x = threadIdx.x + i * kThreads, j = j0 + x / KC, ch = x % KC;
-      rk[i] = u32x4{0u, 0u, 0u, 0u};
-      if (j <= plast && ch * 8 < a.dim) rk[i] = *reinterpret_cast<const u32x4*>(kb + at(j) * a.ldkv + ch * 8);
-    }
-#pragma unroll
-    for (int i = 0; i < NRL; ++i) {
-      const int x = threadIdx.x + i * kThreads, j = j0 + x / RC, ch = x % RC;
-      rr[i] = u32x4{0u, 0u, 0u, 0u};
-      if (j <= plast && ch * 8 < a.rot_dim) rr[i] = *reinterpret_cast<const u32x4*>(rb + at(j) * a.row + ch * 8);
-    }
-#pragma unroll
-    for (int i = 0; i < NVL; ++i) {
-      const int x = threadIdx.x + i * kThreads, j = j0 + x / VC, ch = x % VC;
-      rv[i] = u32x4{0u, 0u, 0u, 0u};
-      if (j <= plast && ch * 8 < a.vdim) rv[i] = *reinterpret_cast<const u32x4*>(vb + at(j) * a.ldkv + ch * 8);
-    }
+  auto issue = [&](int t, char* slot) {
+    const int j0 = lo + t * kKeys;
+    auto at = [&](int r) { return (int64_t)min(max(f0 + min(j0 + r, plast) - fp, 0), a.Nk - 1); };
+    tl::load_tile<kKeys, DN, kTileWaves>(slot, a.dim / 8, [&](int r) { return kb + at(r) * a.ldkv; });
+    tl::load_tile<kKeys, 64, kTileWaves>(slot + KB, a.rot_dim / 8, [&](int r) { return rb + at(r) * a.row; });
+    tl::load_tile<kKeys, VP, kTileWaves>(slot + KB + RB, a.vdim / 8, [&](int r) { return vb + at(r) * a.ldkv; });
   };
-  f32x16 acc[NV];
+  issue(0, smem);
+  bf16x8 qn[DN / 16], qr[4];
+  {
+    const int64_t t = row0 + min(w * 32 + l32, n - 1);
+    const unsigned short* q = a.q + (t * a.H + h) * (a.dim + a.rot_dim);
 #pragma unroll
-  for (int j = 0; j < NV; ++j) acc[j] = zero16();
+    for (int k = 0; k < DN / 16; ++k) {
+      u32x4 z = {0u, 0u, 0u, 0u};
+      if (16 * k + 8 * hh < a.dim) z = *reinterpret_cast<const u32x4*>(q + 16 * k + 8 * hh);
+      qn[k] = __builtin_bit_cast(bf16x8, z);
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k) qr[k] = rotated8(q + a.dim, a.rot + t * a.rot_dim, 16 * k + 8 * hh, a.rot_dim);
+  }
+  const int pw = pos0 + w * 32;  // the wave's first position
+  tl::LaneOffs<DN> ok;
+  tl::LaneOffs<64> orr;
+  tl::LaneOffs<VP> ov;
+  ok.init(lane);
+  orr.init(lane);
+  ov.init(lane);
+  f32x16 acc[VP / 32];
+#pragma unroll
+  for (int j = 0; j < VP / 32; ++j) acc[j] = zero16();
   float M = -INFINITY, L = 0.f;
-  const float sc2 = a.scale * LOG2E;
-  load(lo);
-  for (int j0 = lo; j0 <= plast; j0 += kKeys) {
-    __syncthreads();  // queries, or the previous tile, are read
-#pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int x = threadIdx.x + i * kThreads;
-      *reinterpret_cast<u32x4*>(lk + soff(x / KC, x % KC)) = rk[i];
+  const float sc = a.scale * LOG2E;
+  tl::wait_loads();
+  __syncthreads();
+  auto step = [&](int t, auto slot) {
+    constexpr int CUR = decltype(slot)::value;
+    if (t + 1 < ntiles) issue(t + 1, smem + (CUR ^ 1) * SLOT);
+    const int j0 = lo + t * kKeys;
+    const char* lk = smem + CUR * SLOT;
+    if (w * 32 < n && j0 <= pw + 31 && pw - (j0 + kKeys - 1) < win) {
+      if (j0 + kKeys - 1 <= pw && pw + 31 - j0 < win)
+        latent_tile_step<false, DN, VP>(ok, orr, ov, lk, qn, qr, acc, M, L, sc, j0, pw, lane, win);
+      else
+        latent_tile_step<true, DN, VP>(ok, orr, ov, lk, qn, qr, acc, M, L, sc, j0, pw, lane, win);
     }
-#pragma unroll
-    for (int i = 0; i < NRL; ++i) {
-      const int x = threadIdx.x + i * kThreads;
-      *reinterpret_cast<u32x4*>(lr + soff(x / RC, x % RC)) = rr[i];
-    }
-#pragma unroll
-    for (int i = 0; i < NVL; ++i) {
-      const int x = threadIdx.x + i * kThreads;
-      *reinterpret_cast<u32x4*>(lv + soff(x / VC, x % VC)) = rv[i];
-    }
+    tl::wait_loads();
     __syncthreads();
-    if (j0 + kKeys <= plast) load(j0 + kKeys);
-    // wave-uniform: all keys later than the wave's queries, or all in front of their windows
-    if (j0 > pw + 31 || (a.window > 0 && j0 + kKeys - 1 <= pw - a.window)) continue;
-    f32x16 sc[2];
-#pragma unroll
-    for (int kt = 0; kt < 2; ++kt) {
-      sc[kt] = zero16();
-#pragma unroll
-      for (int k = 0; k < NN; ++k) sc[kt] = mfma(lds_row16(lk, kt * 32 + l32, 2 * k + hh), qn[k], sc[kt]);
-#pragma unroll
-      for (int k = 0; k < NR; ++k)
-        if (k * 16 < a.rot_dim) sc[kt] = mfma(lds_row16(lr, kt * 32 + l32, 2 * k + hh), qr[k], sc[kt]);
-    }
-    const bool whole = j0 + kKeys - 1 <= pw && (a.window <= 0 || pw + 31 - j0 < a.window);
-    float m = -INFINITY;
-#pragma unroll
-    for (int kt = 0; kt < 2; ++kt)
-#pragma unroll
-      for (int i = 0; i < 16; ++i) {
-        float x = sc[kt][i] * sc2;
-        if (!whole) {
-          const int dist = pq - (j0 + kt * 32 + acc_row(i, hh));
-          if (dist < 0 || (a.window > 0 && dist >= a.window)) x = -INFINITY;
-        }
-        sc[kt][i] = x;
-        m = fmaxf(m, x);
-      }
-    m = fmaxf(m, xor32(m));
-    const float Mn = fmaxf(M, m), Ms = Mn == -INFINITY ? 0.f : Mn;  // no visible key yet: weights 0
-    const float f = fast_exp2(M - Ms);
-    float l = 0.f;
-#pragma unroll
-    for (int kt = 0; kt < 2; ++kt)
-#pragma unroll
-      for (int i = 0; i < 16; ++i) {
-        sc[kt][i] = fast_exp2(sc[kt][i] - Ms);
-        l += sc[kt][i];
-      }
-    L = L * f + l + xor32(l);
-    M = Mn;
-#pragma unroll
-    for (int j = 0; j < NV; ++j)
-#pragma unroll
-      for (int i = 0; i < 16; ++i) acc[j][i] *= f;
-#pragma unroll
-    for (int kt = 0; kt < 2; ++kt)
-#pragma unroll
-      for (int x = 0; x < 2; ++x) {
-        const bf16x8 p = acc_to_b(sc[kt], x);
-#pragma unroll
-        for (int j = 0; j < NV; ++j) acc[j] = mfma(lds_trA(lv, kt * 32 + 16 * x, j, lane), p, acc[j]);
-      }
+  };
+  for (int t = 0; t < ntiles; t += 2) {
+    step(t, std::integral_constant<int, 0>{});
+    if (t + 1 < ntiles) step(t + 1, std::integral_constant<int, 1>{});
   }
   const int t = w * 32 + l32;
+  L += xor32(L);
   if (t < n) {
     const float inv = L > 0.f ? 1.f / L : 0.f;
     unsigned short* o = a.out + ((int64_t)(row0 + t) * a.H + h) * a.vdim;
 #pragma unroll
-    for (int j = 0; j < NV; ++j)
+    for (int j = 0; j < VP / 32; ++j)
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
         const int v = j * 32 + 8 * g + 4 * hh;
@@ -776,7 +807,7 @@ void latent_attention_token(const at::Tensor& q, const at::Tensor& uk, const at:
   SXE_CHECK(rot.is_contiguous() && rot.scalar_type() == at::kFloat && rot.numel() == q.size(0) * rot_dim, "latent_attention: rotation");
   for (const auto* t : {&q, &uk, &uv, &cache, (const at::Tensor*)&out})
     SXE_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16, "latent_attention: token form takes bf16");
-  SXE_CHECK(lt::aligned(cache.data_ptr(), 16) && splits >= 1 && splits <= 65535 && H <= 65535, "latent_attention: splits");
+  SXE_CHECK(lt::aligned(cache.data_ptr(), 16) && splits >= 1 && splits <= 256 && H <= 65535, "latent_attention: splits");
   if (n == 0) return;
   c10::DeviceGuard g(q.device());
   lt::Args a{q.data_ptr(), rot.data_ptr<float>(), rows.data_ptr<int>(), table.data_ptr<int>(), q_start.data_ptr<int>(),
@@ -786,7 +817,7 @@ void latent_attention_token(const at::Tensor& q, const at::Tensor& uk, const at:
   auto po = at::empty({splits, n, H, R}, q.options().dtype(at::kFloat)), pml = at::empty({splits, n, H, 2}, po.options());
   auto u16 = [](const at::Tensor& t) { return static_cast<unsigned short*>(t.data_ptr()); };
   auto heads = [&](auto kern, int64_t K, int64_t N, int TT, int LN, auto... more) {
-    const size_t lds = sizeof(float) * (TT * K + 4 * TT * LN * 8);
+    const size_t lds = sizeof(float) * (TT * (K + splits) + 4 * TT * LN * 8);
     SXE_CHECK(lds <= 150 * 1024 && (n + TT - 1) / TT <= 65535, "latent_attention: sizes");
     SXE_HIP_CHECK(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
     hipLaunchKernelGGL(kern, dim3(H, (N + LN * 8 - 1) / (LN * 8), (n + TT - 1) / TT), dim3(lt::kThreads), lds, cur_stream(), a, (int)n,
@@ -836,21 +867,21 @@ void latent_attention_tile(const at::Tensor& q, const at::Tensor& kv, const at::
     SXE_CHECK(t->is_cuda() && t->is_contiguous() && t->scalar_type() == at::kInt && t->numel() == S, "latent_attention: int32 [S]");
   SXE_CHECK(rot.is_contiguous() && rot.scalar_type() == at::kFloat && rot.numel() == q.size(0) * rot_dim, "latent_attention: rotation");
   if (nc == 0 || Nk == 0) return;
-  SXE_CHECK(H <= 65535, "latent_attention: heads");
+  SXE_CHECK(nc <= 65535, "latent_attention: chunks");
   c10::DeviceGuard g(q.device());
   auto u16 = [](const at::Tensor& t) { return static_cast<unsigned short*>(t.data_ptr()); };
   lt::TileArgs a{u16(q), u16(kv), u16(lat), rot.data_ptr<float>(), chunks.data_ptr<int>(), first.data_ptr<int>(), q_start.data_ptr<int>(),
                  q_len.data_ptr<int>(), kv_len.data_ptr<int>(), u16(out), kv.stride(0), (int)H, (int)dim, (int)rot_dim, (int)vdim, (int)R,
                  (int)lat.size(1), (int)window, (int)Nk, (float)scale};
-  auto go = [&](auto kern) {
-    const size_t lds = 2 * lt::kQ * mf::ROWB;  // the key tile (3 panels of 64 rows) fits in the queries' space
+  auto go = [&](auto kern, int DN, int VP) {
+    const size_t lds = 2 * lt::kKeys * (2 * DN + 128 + 2 * VP);
     SXE_HIP_CHECK(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-    hipLaunchKernelGGL(kern, dim3(nc, H), dim3(lt::kThreads), lds, cur_stream(), a);
+    hipLaunchKernelGGL(kern, dim3(H, nc), dim3(64 * lt::kTileWaves), lds, cur_stream(), a);
   };
-  if (dim <= 64 && vdim <= 64) go(lt::latent_tile_kernel<64, 64>);
-  else if (dim <= 64) go(lt::latent_tile_kernel<64, 128>);
-  else if (vdim <= 64) go(lt::latent_tile_kernel<128, 64>);
-  else go(lt::latent_tile_kernel<128, 128>);
+  if (dim <= 64 && vdim <= 64) go(lt::latent_tile_kernel<64, 64>, 64, 64);
+  else if (dim <= 64) go(lt::latent_tile_kernel<64, 128>, 64, 128);
+  else if (vdim <= 64) go(lt::latent_tile_kernel<128, 64>, 128, 64);
+  else go(lt::latent_tile_kernel<128, 128>, 128, 128);
   SXE_LAUNCH_CHECK();
 }
 

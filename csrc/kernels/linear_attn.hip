@@ -10,12 +10,15 @@
 //      2. state_scan: element by element through a sequence's chunks, S_in(c+1) = decay^n S_in(c) + D(c); the
 //         incoming state replaces D, the last one goes to the sequence's slot;
 //      3. chunk_out: o_i = decay^(i+1) S_in^T q_i + sum_(j<=i) decay^(i-j) (q_i . k_j) v_j.
+//    1. also leaves the activated keys and values in the projection, so 3. takes its tiles straight to LDS.
 //    Everything with a decay or a state in it keeps ~2^-17: the decayed keys of 1. and the state of 3. enter
 //    the matrix products as two bf16 numbers (head and remainder); the in-chunk weight of 3. is rounded once,
 //    as the operand of the value product, like the other attention kernels' weights.
 #include "sxe_common.h"
 #include "sxe_mfma.h"
+#include "sxe_tile.h"
 #include <torch/library.h>
+#include <type_traits>
 
 namespace sxe {
 namespace la {
@@ -147,42 +150,35 @@ __global__ __launch_bounds__(kThreads) void step_kernel(Args a) {
 }
 
 // ----------------------------------------------------------------------------------------- chunk form
-constexpr int kTile = 64;  // tokens staged together
-constexpr int kQTile = 128;
+constexpr int kTile = 64;    // tokens staged together
+constexpr int kChunk = 256;  // tokens of a chunk
+constexpr int kOutWaves = kChunk / 32;
 
 // weight decay^n, n >= 0
 __device__ __forceinline__ float decay_pow(float lg, int n) { return fast_exp2(lg * (float)n); }
 
-// 8 activated values of a token's head row (zeros outside)
-__device__ __forceinline__ bf16x8 act8(const unsigned short* p, bool ok, bool act) {
-  bf16x8 r;
-  if (!ok) {
+__device__ __forceinline__ bf16x8 load8b(const unsigned short* p, bool ok) {
+  u32x4 z = {0u, 0u, 0u, 0u};
+  if (ok) z = *reinterpret_cast<const u32x4*>(p);
+  return __builtin_bit_cast(bf16x8, z);
+}
+__device__ __forceinline__ bf16x8 silu8(bf16x8 r) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) r[i] = (__bf16)0.f;
-    return r;
-  }
-  r = *reinterpret_cast<const bf16x8*>(p);
-  if (act) {
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const float x = (float)r[i];
-      r[i] = (__bf16)(x * __builtin_amdgcn_rcpf(1.f + fast_exp2(-LOG2E * x)));
-    }
+  for (int i = 0; i < 8; ++i) {
+    const float x = (float)r[i];
+    r[i] = (__bf16)(x * __builtin_amdgcn_rcpf(1.f + fast_exp2(-LOG2E * x)));
   }
   return r;
 }
 
-__device__ __forceinline__ bf16x8 raw8(const unsigned short* p, bool ok) { return act8(p, ok, false); }
-
-// DP, VP: dim and vdim padded to 64 / 128. grid (chunks, H); d_out [chunks, H, dim, vdim] fp32
+// DP, VP: dim and vdim padded to 64 / 128. grid (H, chunks); d_out [chunks, H, dim, vdim] fp32
 template <int DP, int VP>
 __global__ __launch_bounds__(kThreads, 2) void chunk_state_kernel(Args a, const int* __restrict chunks, float* __restrict d_out) {
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  char *lh = smem, *ll = smem + kTile * ROWB, *lv = smem + 2 * kTile * ROWB;
-  const int c = blockIdx.x, h = blockIdx.y;
+  char *lh = tl::lds, *ll = lh + kTile * 2 * DP, *lv = ll + kTile * 2 * DP;
+  const int c = blockIdx.y, h = blockIdx.x;
   const int row0 = chunks[3 * c + 1], n = chunks[3 * c + 2];
-  const unsigned short* kb = static_cast<const unsigned short*>(a.proj) + (int64_t)row0 * a.ld + (a.H + h) * a.dim;
-  const unsigned short* vb = static_cast<const unsigned short*>(a.proj) + (int64_t)row0 * a.ld + 2 * a.H * a.dim + h * a.vdim;
+  unsigned short* kb = static_cast<unsigned short*>(const_cast<void*>(a.proj)) + (int64_t)row0 * a.ld + (a.H + h) * a.dim;
+  unsigned short* vb = static_cast<unsigned short*>(const_cast<void*>(a.proj)) + (int64_t)row0 * a.ld + 2 * a.H * a.dim + h * a.vdim;
   const float lg = a.decay[a.H + h];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l32 = lane & 31, hh = lane >> 5;
   constexpr int DT_ = DP / 32, NV = VP / 32 * DT_ / 4;  // wave: one 32-row tile of dim, NV column tiles
@@ -191,27 +187,36 @@ __global__ __launch_bounds__(kThreads, 2) void chunk_state_kernel(Args a, const 
 #pragma unroll
   for (int j = 0; j < NV; ++j) acc[j] = zero16();
   constexpr int KC = DP / 8, VC = VP / 8, NK = kTile * KC / kThreads, NVL = kTile * VC / kThreads;
+  int ok[2], ov[NV][2];  // the lane's transposed-read offsets
+  {
+    tl::LaneOffs<DP> k;
+    tl::LaneOffs<VP> v;
+    k.init(lane);
+    v.init(lane);
+#pragma unroll
+    for (int e = 0; e < 2; ++e) {
+#pragma unroll
+      for (int t = 0; t < DT_; ++t)
+        if (t == dt) ok[e] = k.tr[t][e];
+#pragma unroll
+      for (int t = 0; t < VP / 32; ++t)
+#pragma unroll
+        for (int j = 0; j < NV; ++j)
+          if (t == vt0 + j) ov[j][e] = v.tr[t][e];
+    }
+  }
   bf16x8 rk[NK], rv[NVL];
   auto load = [&](int t0) {
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
       const int x = threadIdx.x + i * kThreads, t = t0 + x / KC, ch = x % KC;
-      rk[i] = raw8(kb + (int64_t)t * a.ld + ch * 8, t < n && ch * 8 < a.dim);
+      rk[i] = load8b(kb + (int64_t)t * a.ld + ch * 8, t < n && ch * 8 < a.dim);
     }
 #pragma unroll
     for (int i = 0; i < NVL; ++i) {
       const int x = threadIdx.x + i * kThreads, t = t0 + x / VC, ch = x % VC;
-      rv[i] = raw8(vb + (int64_t)t * a.ld + ch * 8, t < n && ch * 8 < a.vdim);
+      rv[i] = load8b(vb + (int64_t)t * a.ld + ch * 8, t < n && ch * 8 < a.vdim);
     }
-  };
-  auto silu8 = [&](bf16x8 r) {
-    if (!a.act) return r;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const float x = (float)r[i];
-      r[i] = (__bf16)(x * __builtin_amdgcn_rcpf(1.f + fast_exp2(-LOG2E * x)));
-    }
-    return r;
   };
   load(0);
   for (int t0 = 0; t0 < n; t0 += kTile) {
@@ -219,7 +224,11 @@ __global__ __launch_bounds__(kThreads, 2) void chunk_state_kernel(Args a, const 
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
       const int x = threadIdx.x + i * kThreads, t = x / KC, ch = x % KC;
-      const bf16x8 k8 = silu8(rk[i]);
+      bf16x8 k8 = rk[i];
+      if (a.act) {
+        k8 = silu8(k8);
+        if (t0 + t < n && ch * 8 < a.dim) *reinterpret_cast<bf16x8*>(kb + (int64_t)(t0 + t) * a.ld + ch * 8) = k8;
+      }
       const float f = t0 + t < n ? decay_pow(lg, n - 1 - t0 - t) : 0.f;
       bf16x8 hi, lo;
 #pragma unroll
@@ -228,22 +237,27 @@ __global__ __launch_bounds__(kThreads, 2) void chunk_state_kernel(Args a, const 
         hi[e] = (__bf16)y;
         lo[e] = (__bf16)(y - (float)hi[e]);
       }
-      *reinterpret_cast<bf16x8*>(lh + soff(t, ch)) = hi;
-      *reinterpret_cast<bf16x8*>(ll + soff(t, ch)) = lo;
+      *reinterpret_cast<bf16x8*>(lh + tl::off<DP>(t, ch)) = hi;
+      *reinterpret_cast<bf16x8*>(ll + tl::off<DP>(t, ch)) = lo;
     }
 #pragma unroll
     for (int i = 0; i < NVL; ++i) {
-      const int x = threadIdx.x + i * kThreads;
-      *reinterpret_cast<bf16x8*>(lv + soff(x / VC, x % VC)) = silu8(rv[i]);
+      const int x = threadIdx.x + i * kThreads, t = x / VC, ch = x % VC;
+      bf16x8 v8 = rv[i];
+      if (a.act) {
+        v8 = silu8(v8);
+        if (t0 + t < n && ch * 8 < a.vdim) *reinterpret_cast<bf16x8*>(vb + (int64_t)(t0 + t) * a.ld + ch * 8) = v8;
+      }
+      *reinterpret_cast<bf16x8*>(lv + tl::off<VP>(t, ch)) = v8;
     }
     __syncthreads();
     if (t0 + kTile < n) load(t0 + kTile);
 #pragma unroll
     for (int s = 0; s < kTile / 16; ++s) {
-      const bf16x8 ah = lds_trA(lh, 16 * s, dt, lane), al = lds_trA(ll, 16 * s, dt, lane);
+      const bf16x8 ah = tl::tr_at(lh + 16 * s * 2 * DP, ok), al = tl::tr_at(ll + 16 * s * 2 * DP, ok);
 #pragma unroll
       for (int j = 0; j < NV; ++j) {
-        const bf16x8 b = lds_trA(lv, 16 * s, vt0 + j, lane);
+        const bf16x8 b = tl::tr_at(lv + 16 * s * 2 * VP, ov[j]);
         acc[j] = mfma(ah, b, acc[j]);
         acc[j] = mfma(al, b, acc[j]);
       }
@@ -273,67 +287,74 @@ __global__ __launch_bounds__(kThreads) void state_scan_kernel(Args a, const int*
   f32x4 x = {0.f, 0.f, 0.f, 0.f};
   if (a.kv_len[s] != n) x = *reinterpret_cast<const f32x4*>(st);
   const float lg = a.decay[a.H + h];
-  for (; c < nchunks && chunks[3 * c] == s; ++c) {
-    float* p = buf + ((int64_t)c * a.H + h) * N + e;
-    const f32x4 d = *reinterpret_cast<const f32x4*>(p);
-    unsigned u[4];
+  int last = c;
+  while (last < nchunks && chunks[3 * last] == s) ++last;
+  constexpr int U = 4;  // chunks in flight
+  const int64_t step = (int64_t)a.H * N;
+  float* p = buf + ((int64_t)c * a.H + h) * N + e;
+  for (; c < last; c += U, p += U * step) {
+    f32x4 d[U];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const unsigned short hi = f32_to_bf16(x[j]), lo = f32_to_bf16(x[j] - bf16_to_f32(hi));
-      u[j] = ((unsigned)hi << 16) | lo;
+    for (int i = 0; i < U; ++i)
+      if (c + i < last) d[i] = *reinterpret_cast<const f32x4*>(p + i * step);
+#pragma unroll
+    for (int i = 0; i < U; ++i) {
+      if (c + i >= last) break;
+      unsigned u[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const unsigned short hi = f32_to_bf16(x[j]), lo = f32_to_bf16(x[j] - bf16_to_f32(hi));
+        u[j] = ((unsigned)hi << 16) | lo;
+      }
+      *reinterpret_cast<u32x4*>(p + i * step) = u32x4{u[0], u[1], u[2], u[3]};
+      const float f = decay_pow(lg, chunks[3 * (c + i) + 2]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) x[j] = f * x[j] + d[i][j];
     }
-    *reinterpret_cast<u32x4*>(p) = u32x4{u[0], u[1], u[2], u[3]};
-    const float f = decay_pow(lg, chunks[3 * c + 2]);
-#pragma unroll
-    for (int j = 0; j < 4; ++j) x[j] = f * x[j] + d[j];
   }
   *reinterpret_cast<f32x4*>(st) = x;
 }
 
-// grid (chunks * (chunk size / kQTile), H)
+// grid (H, chunks): 8 waves of 32 queries each. k and v of proj hold activated values already.
 template <int DP, int VP>
-__global__ __launch_bounds__(kThreads, 2) void chunk_out_kernel(Args a, const int* __restrict chunks, int qtiles,
-                                                                const float* __restrict buf) {
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  const int c = blockIdx.x / qtiles, q0 = (blockIdx.x % qtiles) * kQTile, h = blockIdx.y;
-  const int sq = chunks[3 * c], row0 = chunks[3 * c + 1], n = chunks[3 * c + 2];
-  if (q0 >= n) return;
+__global__ __launch_bounds__(64 * kOutWaves, 1) void chunk_out_kernel(Args a, const int* __restrict chunks,
+                                                                      const float* __restrict buf) {
+  constexpr int SLOT = kTile * (2 * DP + 2 * VP), NS = DP / 16, NV = VP / 32, VC = VP / 8;
+  char *slot0 = tl::lds, *ls = tl::lds + SLOT;  // the second slot takes the state's place
+  const int c = blockIdx.y, h = blockIdx.x;
+  const int sq = chunks[3 * c], row0 = chunks[3 * c + 1], n = chunks[3 * c + 2], ntiles = (n + kTile - 1) / kTile;
   const bool empty = a.kv_len[sq] == a.q_len[sq] && row0 == a.q_start[sq];  // nothing comes in
   const unsigned short* base = static_cast<const unsigned short*>(a.proj) + (int64_t)row0 * a.ld;
   const unsigned short *qb = base + h * a.dim, *kb = base + (a.H + h) * a.dim, *vb = base + 2 * a.H * a.dim + h * a.vdim;
   const float lg = a.decay[a.H + h];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l32 = lane & 31, hh = lane >> 5;
-  constexpr int KC = DP / 8, VC = VP / 8, NS = DP / 16, NV = VP / 32;
-
-  // ---- queries: staged once, kept as fragments (in the key product's order and in the transposed reads')
-  for (int x = threadIdx.x; x < kQTile * KC; x += kThreads) {
-    const int t = x / KC, ch = x % KC;
-    *reinterpret_cast<bf16x8*>(smem + soff(t, ch)) = act8(qb + (int64_t)(q0 + t) * a.ld + ch * 8, q0 + t < n && ch * 8 < a.dim, a.act);
-  }
-  __syncthreads();
-  const int iq = q0 + w * 32 + l32;  // the lane's query
+  const int q0 = (w < kOutWaves / 2 ? w : kOutWaves + kOutWaves / 2 - 1 - w) * 32;  // a SIMD's two waves: one early, one late
+  const int iq = q0 + l32;
+  auto issue = [&](int t, char* slot) {
+    auto row = [&](int r) { return (int64_t)min(t * kTile + r, n - 1) * a.ld; };
+    tl::load_tile<kTile, DP, kOutWaves>(slot, a.dim / 8, [&](int r) { return kb + row(r); });
+    tl::load_tile<kTile, VP, kOutWaves>(slot + kTile * 2 * DP, a.vdim / 8, [&](int r) { return vb + row(r); });
+  };
+  issue(0, slot0);
   bf16x8 qf[NS];
 #pragma unroll
-  for (int s = 0; s < NS; ++s) qf[s] = lds_row16(smem, w * 32 + l32, 2 * s + hh);
+  for (int s = 0; s < NS; ++s) {
+    qf[s] = load8b(qb + (int64_t)min(iq, n - 1) * a.ld + 16 * s + 8 * hh, 16 * s + 8 * hh < a.dim);
+    if (a.act) qf[s] = silu8(qf[s]);
+  }
+  tl::LaneOffs<DP> ok;
+  tl::LaneOffs<VP> ov;
+  ok.init(lane);
+  ov.init(lane);
   f32x16 acc[NV];
 #pragma unroll
   for (int j = 0; j < NV; ++j) acc[j] = zero16();
 
   // ---- decay^(i+1) S_in^T q_i
   if (!empty) {
-    typedef unsigned long long u64;
-    bf16x8 qp[NS];
-#pragma unroll
-    for (int s = 0; s < NS; ++s) {
-      union { u64 u[2]; bf16x8 b; } t;
-      t.u[0] = *reinterpret_cast<const u64*>(smem + soff(w * 32 + l32, 2 * s) + 8 * hh);
-      t.u[1] = *reinterpret_cast<const u64*>(smem + soff(w * 32 + l32, 2 * s + 1) + 8 * hh);
-      qp[s] = t.b;
-    }
-    __syncthreads();
-    char *lh = smem, *ll = smem + DP * ROWB;
+    char *lh = ls, *ll = ls + DP * 2 * VP;
     const unsigned* sp = reinterpret_cast<const unsigned*>(buf) + ((int64_t)c * a.H + h) * a.dim * a.vdim;
-    for (int x = threadIdx.x; x < DP * VC; x += kThreads) {
+    for (int x = threadIdx.x; x < DP * VC; x += 64 * kOutWaves) {
       const int d = x / VC, ch = x % VC;
       u32x4 u0 = {0u, 0u, 0u, 0u}, u1 = {0u, 0u, 0u, 0u};
       if (d < a.dim && ch * 8 < a.vdim) {
@@ -349,84 +370,72 @@ __global__ __launch_bounds__(kThreads, 2) void chunk_out_kernel(Args a, const in
       lo[1] = (u0[2] & 0xffffu) | (u0[3] << 16);
       lo[2] = (u1[0] & 0xffffu) | (u1[1] << 16);
       lo[3] = (u1[2] & 0xffffu) | (u1[3] << 16);
-      *reinterpret_cast<u32x4*>(lh + soff(d, ch)) = hi;
-      *reinterpret_cast<u32x4*>(ll + soff(d, ch)) = lo;
+      *reinterpret_cast<u32x4*>(lh + tl::off<VP>(d, ch)) = hi;
+      *reinterpret_cast<u32x4*>(ll + tl::off<VP>(d, ch)) = lo;
     }
     __syncthreads();
 #pragma unroll
-    for (int s = 0; s < NS; ++s)
+    for (int s = 0; s < NS; ++s) {
+      // the query fragment in the transposed reads' k order: lanes of the two halves exchange 8 bytes
+      const u32x4 u = __builtin_bit_cast(u32x4, qf[s]);
+      const auto x = __builtin_amdgcn_permlane32_swap(u[0], u[2], false, false);
+      const auto y = __builtin_amdgcn_permlane32_swap(u[1], u[3], false, false);
+      const bf16x8 q = __builtin_bit_cast(bf16x8, u32x4{x[0], y[0], x[1], y[1]});
 #pragma unroll
       for (int j = 0; j < NV; ++j) {
-        acc[j] = mfma(lds_trA(lh, 16 * s, j, lane), qp[s], acc[j]);
-        acc[j] = mfma(lds_trA(ll, 16 * s, j, lane), qp[s], acc[j]);
+        acc[j] = mfma(tl::tr_at(lh + 16 * s * 2 * VP, ov.tr[j]), q, acc[j]);
+        acc[j] = mfma(tl::tr_at(ll + 16 * s * 2 * VP, ov.tr[j]), q, acc[j]);
       }
+    }
     const float f = decay_pow(lg, iq + 1);
 #pragma unroll
     for (int j = 0; j < NV; ++j)
 #pragma unroll
       for (int i = 0; i < 16; ++i) acc[j][i] *= f;
   }
+  float fk[16];  // decay from a key of a 32-key block to the block's last key
+#pragma unroll
+  for (int i = 0; i < 16; ++i) fk[i] = decay_pow(lg, 31 - acc_row(i, hh));
+  tl::wait_loads();
+  __syncthreads();
 
-  // ---- keys of the chunk up to the tile's last query
-  char *lk = smem, *lv = smem + kTile * ROWB;
-  const int kend = min(n, q0 + kQTile);
-  constexpr int NK = kTile * KC / kThreads, NVL = kTile * VC / kThreads;
-  bf16x8 rk[NK], rv[NVL];
-  auto load = [&](int t0) {
+  // ---- the chunk's keys up to the query
+  auto step = [&](int t, auto slot) {
+    constexpr int CUR = decltype(slot)::value;
+    const char* lk = CUR ? ls : slot0;
+    const char* lv = lk + kTile * 2 * DP;
+    if (t + 1 < ntiles) issue(t + 1, CUR ? slot0 : ls);
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int x = threadIdx.x + i * kThreads, t = t0 + x / KC, ch = x % KC;
-      rk[i] = raw8(kb + (int64_t)t * a.ld + ch * 8, t < kend && ch * 8 < a.dim);
-    }
-#pragma unroll
-    for (int i = 0; i < NVL; ++i) {
-      const int x = threadIdx.x + i * kThreads, t = t0 + x / VC, ch = x % VC;
-      rv[i] = raw8(vb + (int64_t)t * a.ld + ch * 8, t < kend && ch * 8 < a.vdim);
-    }
-  };
-  auto silu8 = [&](bf16x8 r) {
-    if (!a.act) return r;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const float x = (float)r[i];
-      r[i] = (__bf16)(x * __builtin_amdgcn_rcpf(1.f + fast_exp2(-LOG2E * x)));
-    }
-    return r;
-  };
-  load(0);
-  for (int t0 = 0; t0 < kend; t0 += kTile) {
-    __syncthreads();  // the previous tile (or the state) is read
-#pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int x = threadIdx.x + i * kThreads;
-      *reinterpret_cast<bf16x8*>(lk + soff(x / KC, x % KC)) = silu8(rk[i]);
-    }
-#pragma unroll
-    for (int i = 0; i < NVL; ++i) {
-      const int x = threadIdx.x + i * kThreads;
-      *reinterpret_cast<bf16x8*>(lv + soff(x / VC, x % VC)) = silu8(rv[i]);
-    }
-    __syncthreads();
-    if (t0 + kTile < kend) load(t0 + kTile);
-#pragma unroll
-    for (int kt = 0; kt < kTile / 32; ++kt) {
-      const int j0 = t0 + kt * 32;
-      if (j0 > q0 + w * 32 + 31) continue;  // wave-uniform: every key of the tile is later than every query
+    for (int kt = 0; kt < 2; ++kt) {
+      const int j0 = t * kTile + kt * 32;
+      if (j0 > q0) continue;  // wave-uniform
       f32x16 sc = zero16();
 #pragma unroll
-      for (int s = 0; s < NS; ++s) sc = mfma(lds_row16(lk, kt * 32 + l32, 2 * s + hh), qf[s], sc);
+      for (int s = 0; s < NS; ++s) sc = mfma(tl::row_at(lk + kt * 32 * 2 * DP, ok.row[s]), qf[s], sc);
+      if (j0 < q0) {
+        const float f = decay_pow(lg, iq - j0 - 31);
 #pragma unroll
-      for (int i = 0; i < 16; ++i) {
-        const int dist = iq - j0 - acc_row(i, hh);
-        sc[i] = dist >= 0 ? sc[i] * decay_pow(lg, dist) : 0.f;
+        for (int i = 0; i < 16; ++i) sc[i] *= f * fk[i];
+      } else {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+          const int dist = l32 - acc_row(i, hh);
+          sc[i] = dist >= 0 ? sc[i] * decay_pow(lg, dist) : 0.f;
+        }
       }
 #pragma unroll
-      for (int s = 0; s < 2; ++s) {
-        const bf16x8 p = acc_to_b(sc, s);
+      for (int x = 0; x < 2; ++x) {
+        const bf16x8 p = acc_to_b(sc, x);
 #pragma unroll
-        for (int j = 0; j < NV; ++j) acc[j] = mfma(lds_trA(lv, kt * 32 + 16 * s, j, lane), p, acc[j]);
+        for (int j = 0; j < NV; ++j) acc[j] = mfma(tl::tr_at(lv + (kt * 32 + 16 * x) * 2 * VP, ov.tr[j]), p, acc[j]);
       }
     }
+    tl::wait_loads();
+    __syncthreads();
+  };
+  for (int t = 0; t < ntiles; t += 2) {
+    step(t, std::integral_constant<int, 0>{});
+    if (t + 1 < ntiles) step(t + 1, std::integral_constant<int, 1>{});
   }
   if (iq < n) {
     unsigned short* o = static_cast<unsigned short*>(a.out) + (int64_t)(row0 + iq) * a.H * a.vdim + h * a.vdim;
@@ -505,8 +514,9 @@ at::Tensor decay_attention_step(const at::Tensor& proj, at::Tensor state, const 
   return out;
 }
 
-// chunks int32 [n, 3]: (sequence, first row, rows <= size), a sequence's chunks in order and side by side
-at::Tensor decay_attention_chunk(const at::Tensor& proj, at::Tensor state, const at::Tensor& decay, const at::Tensor& q_start,
+// chunks int32 [n, 3]: (sequence, first row, rows <= kChunk), a sequence's chunks in order and side by side. With an
+// activation, the k and v columns of proj are replaced by their activated values.
+at::Tensor decay_attention_chunk(at::Tensor proj, at::Tensor state, const at::Tensor& decay, const at::Tensor& q_start,
                                  const at::Tensor& q_len, const at::Tensor& kv_len, const at::Tensor& slots,
                                  const at::Tensor& chunks, int64_t size, int64_t H, int64_t dim, int64_t vdim, bool act) {
   at::Tensor out;
@@ -516,27 +526,25 @@ at::Tensor decay_attention_chunk(const at::Tensor& proj, at::Tensor state, const
                 proj.stride(0) % 8 == 0 && reinterpret_cast<uintptr_t>(proj.data_ptr()) % 16 == 0,
             "decay_attention: chunk form takes bf16, sizes up to 128 in multiples of 8");
   SXE_CHECK(chunks.is_cuda() && chunks.scalar_type() == at::kInt && chunks.is_contiguous() && chunks.dim() == 2 &&
-                chunks.size(1) == 3 && size > 0, "decay_attention: chunks int32 [n, 3]");
+                chunks.size(1) == 3 && size == la::kChunk, "decay_attention: chunks int32 [n, 3] of up to ", la::kChunk, " rows");
   const int64_t S = q_start.numel(), nc = chunks.size(0);
   if (S == 0 || nc == 0) return out;
-  SXE_CHECK(H <= 65535 && nc < (1 << 24), "decay_attention: sizes");
+  SXE_CHECK(H <= 65535 && nc <= 65535, "decay_attention: sizes");
   auto buf = at::empty({nc, H, dim, vdim}, proj.options().dtype(at::kFloat));
-  const int qt = (int)((size + la::kQTile - 1) / la::kQTile);
-  auto go = [&](auto ks, auto ko, int DP) {
-    const size_t l1 = 3 * la::kTile * mf::ROWB;
-    const size_t l3 = std::max(2 * DP, la::kQTile) * mf::ROWB;
+  auto go = [&](auto ks, auto ko, int DP, int VP) {
+    const size_t l1 = la::kTile * (4 * DP + 2 * VP), slot = la::kTile * (2 * DP + 2 * VP);
+    const size_t l3 = slot + std::max<size_t>(slot, 4 * DP * VP);
     SXE_HIP_CHECK(hipFuncSetAttribute((const void*)ks, hipFuncAttributeMaxDynamicSharedMemorySize, (int)l1));
     SXE_HIP_CHECK(hipFuncSetAttribute((const void*)ko, hipFuncAttributeMaxDynamicSharedMemorySize, (int)l3));
-    hipLaunchKernelGGL(ks, dim3(nc, H), dim3(la::kThreads), l1, cur_stream(), a, chunks.data_ptr<int>(), buf.data_ptr<float>());
+    hipLaunchKernelGGL(ks, dim3(H, nc), dim3(la::kThreads), l1, cur_stream(), a, chunks.data_ptr<int>(), buf.data_ptr<float>());
     hipLaunchKernelGGL(la::state_scan_kernel, dim3(S, H, (dim * vdim + 4 * la::kThreads - 1) / (4 * la::kThreads)),
                        dim3(la::kThreads), 0, cur_stream(), a, chunks.data_ptr<int>(), (int)nc, buf.data_ptr<float>());
-    hipLaunchKernelGGL(ko, dim3(nc * qt, H), dim3(la::kThreads), l3, cur_stream(), a, chunks.data_ptr<int>(), qt,
-                       buf.data_ptr<float>());
+    hipLaunchKernelGGL(ko, dim3(H, nc), dim3(64 * la::kOutWaves), l3, cur_stream(), a, chunks.data_ptr<int>(), buf.data_ptr<float>());
   };
-  if (dim <= 64 && vdim <= 64) go(la::chunk_state_kernel<64, 64>, la::chunk_out_kernel<64, 64>, 64);
-  else if (dim <= 64) go(la::chunk_state_kernel<64, 128>, la::chunk_out_kernel<64, 128>, 64);
-  else if (vdim <= 64) go(la::chunk_state_kernel<128, 64>, la::chunk_out_kernel<128, 64>, 128);
-  else go(la::chunk_state_kernel<128, 128>, la::chunk_out_kernel<128, 128>, 128);
+  if (dim <= 64 && vdim <= 64) go(la::chunk_state_kernel<64, 64>, la::chunk_out_kernel<64, 64>, 64, 64);
+  else if (dim <= 64) go(la::chunk_state_kernel<64, 128>, la::chunk_out_kernel<64, 128>, 64, 128);
+  else if (vdim <= 64) go(la::chunk_state_kernel<128, 64>, la::chunk_out_kernel<128, 64>, 128, 64);
+  else go(la::chunk_state_kernel<128, 128>, la::chunk_out_kernel<128, 128>, 128, 128);
   SXE_LAUNCH_CHECK();
   return out;
 }
@@ -546,7 +554,7 @@ at::Tensor decay_attention_chunk(const at::Tensor& proj, at::Tensor state, const
 TORCH_LIBRARY_FRAGMENT(sxe, m) {
   m.def("decay_attention_step(Tensor proj, Tensor(a!) state, Tensor decay, Tensor q_start, Tensor q_len, Tensor kv_len, "
         "Tensor slots, int H, int dim, int vdim, bool act) -> Tensor");
-  m.def("decay_attention_chunk(Tensor proj, Tensor(a!) state, Tensor decay, Tensor q_start, Tensor q_len, Tensor kv_len, "
+  m.def("decay_attention_chunk(Tensor(b!) proj, Tensor(a!) state, Tensor decay, Tensor q_start, Tensor q_len, Tensor kv_len, "
         "Tensor slots, Tensor chunks, int size, int H, int dim, int vdim, bool act) -> Tensor");
 }
 TORCH_LIBRARY_IMPL(sxe, CUDA, m) {

@@ -103,7 +103,7 @@ def latent_attention(q, uk, uv, ukv, cache, batch, rot, heads, dim, rot_dim, vdi
 
 
 TOKEN_HEADS, TOKEN_KEYS, TOKEN_WGS = 32, 64, 256  # token form: heads and keys of a tile; workgroups to aim for with key splits
-TILE_TOKENS = 128  # query tokens of a workgroup of the expanded form
+TILE_TOKENS = 256  # query tokens of a workgroup of the expanded form
 
 
 def tile_ok(q, dim, rot_dim, vdim):

@@ -26,7 +26,8 @@ def decay_attention(proj, state, decay, batch, heads, dim, vdim, act="silu", for
     """``proj`` [T, q | k | v | ...] (head by head, before the activation ``act``: "silu" or None);
     ``state`` [slots, heads, dim, vdim] fp32, advanced in place at ``batch.state_slots``; ``decay`` from
     ``decay_table``. Returns o [T, heads * vdim]. ``form``: "step" one token after the other, "chunk" matrix
-    products over chunks of tokens (bf16), "auto" by shape."""
+    products over chunks of tokens (bf16), "auto" by shape. The chunk form leaves the activated k and v in
+    ``proj``."""
     if native.use_hip(proj):
         chunk = form == "chunk" or (form == "auto" and chunk_ok(proj, dim, vdim) and max(batch.host_q_len) > STEP_MAX)
         if not chunk:
