@@ -2,8 +2,10 @@
 //
 //  * route_logits: h . router^T in fp32. bf16 operands go through the matrix cores (products of two bf16
 //    numbers are exact in fp32 and the accumulation is fp32), anything else through a plain fp32 kernel.
+//    Few tokens: one wave per (expert, 8 tokens) in fp32; one to four: the norm that produces h is the kernel's
+//    prologue (sxe_sandwich.h).
 //  * route_top: the k largest logits of a token (lowest index first among equals) and the softmax over them.
-//  * moe_lists: (token, choice) assignments sorted by expert: row -> token, row -> weight, (token, choice) -> row,
+//  * lists: (token, choice) assignments sorted by expert: row -> token, row -> weight, (token, choice) -> row,
 //    expert offsets and the experts that have rows. A row's place inside its expert depends on the order of
 //    atomics, its result does not.
 //  * expert_gemm: y[r] = weight[r] * act(x[token(r)] . W[e]^T) for rows sorted by expert.
@@ -13,6 +15,7 @@
 //    Many rows per expert: grouped_gemm.hip.
 #include "sxe_common.h"
 #include "sxe_mfma.h"
+#include "sxe_sandwich.h"
 #include <torch/library.h>
 
 namespace sxe {
@@ -82,13 +85,70 @@ __global__ __launch_bounds__(256) void route_logits_generic_kernel(const typenam
   if (lane == 0) z[(int64_t)t * E + e] = s;
 }
 
+// few tokens, bf16, K % 8 == 0, 16-byte aligned rows: one wave per (expert, 8 tokens), grid (ceil(E / 4), ceil(T / 8))
+__global__ __launch_bounds__(256) void route_logits_few_kernel(const unsigned short* __restrict x, int64_t ldx,
+                                                               const unsigned short* __restrict w, int T, int E, int K,
+                                                               float* __restrict z) {
+  const int e = blockIdx.x * 4 + (threadIdx.x >> 6), t0 = blockIdx.y * 8, lane = threadIdx.x & 63;
+  if (e >= E) return;
+  float s[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+  for (int c = lane * 8; c < K; c += 512) {
+    float a[8];
+    load8<DT::BF16>(w + (int64_t)e * K + c, a);
+#pragma unroll
+    for (int t = 0; t < 8; ++t) {
+      float b[8];
+      load8<DT::BF16>(x + (int64_t)min(t0 + t, T - 1) * ldx + c, b);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s[t] += a[i] * b[i];
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < 8; ++t) {
+    const float v = wave_sum(s[t]);
+    if (lane == 0 && t0 + t < T) z[(int64_t)(t0 + t) * E + e] = v;
+  }
+}
+
+// decode: h is built by every workgroup (norms around the residual sum) and written, with the sum, by the first;
+// one wave per expert. grid (ceil(E / 8)); M <= 4 rows
+__global__ __launch_bounds__(512) void route_sandwich_kernel(sw::Args a, const unsigned short* __restrict w, int M, int E, int K,
+                                                             unsigned short* __restrict h, float* __restrict z) {
+  extern __shared__ __attribute__((aligned(16))) unsigned short act[];  // [M][K]
+  __shared__ float red[8][sw::kMaxM], rinv[sw::kMaxM];
+  const int e = blockIdx.x * 8 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const unsigned short* wr = w + (int64_t)min(e, E - 1) * K;
+  sw::build<512, 2, true>(a, M, K, blockIdx.x == 0, act, rinv, red);
+  if (blockIdx.x == 0)
+    for (int i = threadIdx.x * 8; i < M * K; i += 512 * 8) *reinterpret_cast<u16x8*>(h + i) = *reinterpret_cast<u16x8*>(act + i);
+  if (e >= E) return;
+  float s[sw::kMaxM] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int c = lane * 8; c < K; c += 512) {
+    float x[8];
+    load8<DT::BF16>(wr + c, x);
+#pragma unroll
+    for (int m = 0; m < sw::kMaxM; ++m) {
+      if (m >= M) break;
+      float b[8];
+      load8<DT::BF16>(act + m * K + c, b);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s[m] += x[i] * b[i];
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < sw::kMaxM; ++m) {
+    const float v = wave_sum(s[m]);
+    if (lane == 0 && m < M) z[(int64_t)m * E + e] = v;
+  }
+}
+
 constexpr int kMaxE = 1024;
 
-// one wave per token, 4 waves per workgroup
-__global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict z, int T, int E, int k, int* __restrict idx,
-                                                        float* __restrict wt) {
-  const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (t >= T) return;
+// the k largest of a token's logits and their softmax weights, by one wave
+__device__ __forceinline__ void route_top(const float* __restrict z, int t, int E, int k, int* idx, float* wt) {
+  const int lane = threadIdx.x & 63;
   constexpr int N = kMaxE / 64;
   float v[N];
 #pragma unroll
@@ -127,21 +187,38 @@ __global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict 
   for (int j = lane; j < k; j += 64) wt[(int64_t)t * k + j] /= sum;
 }
 
+// one wave per token, 4 waves per workgroup
+__global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict z, int T, int E, int k, int* __restrict idx,
+                                                        float* __restrict wt) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (t < T) route_top(z, t, E, k, idx, wt);
+}
+
 // ------------------------------------------------------------------------------------------------ lists
 constexpr int kListThreads = 1024;
 
-// R <= kListThreads: everything in one workgroup
-__global__ __launch_bounds__(kListThreads) void moe_lists_small_kernel(const int* __restrict expert, const float* __restrict wt, int R,
+// R <= kListThreads: everything in one workgroup; z (logits of R / k tokens) or null: choose the experts first
+__global__ __launch_bounds__(kListThreads) void moe_lists_small_kernel(const float* __restrict z, int* expert, float* wt, int R,
                                                                        int k, int E, int* __restrict token, float* __restrict ws,
                                                                        int* __restrict slots, int* __restrict offs,
                                                                        int* __restrict active) {
   __shared__ int cnt[kMaxE], off[kMaxE + 1];
+  __shared__ int se[kListThreads];
+  __shared__ float sw_[kListThreads];
   const int i = threadIdx.x;
   for (int e = i; e < E; e += kListThreads) cnt[e] = 0;
+  if (z != nullptr)
+    for (int t = i >> 6; t < R / k; t += kListThreads / 64) route_top(z, t, E, k, se, sw_);
   __syncthreads();
   int e = 0, rank = 0;
+  float w = 0.f;
   if (i < R) {
-    e = min(max(expert[i], 0), E - 1);
+    if (z != nullptr) {
+      expert[i] = se[i];
+      wt[i] = sw_[i];
+    }
+    e = z != nullptr ? se[i] : min(max(expert[i], 0), E - 1);
+    w = z != nullptr ? sw_[i] : wt[i];
     rank = atomicAdd(&cnt[e], 1);
   }
   __syncthreads();
@@ -173,7 +250,7 @@ __global__ __launch_bounds__(kListThreads) void moe_lists_small_kernel(const int
   if (i < R) {
     const int r = off[e] + rank;
     token[r] = i / k;
-    ws[r] = wt[i];
+    ws[r] = w;
     slots[i] = r;
   }
 }
@@ -369,76 +446,111 @@ inline bool aligned(const void* p, size_t n) { return reinterpret_cast<uintptr_t
 
 }  // namespace ex
 
-// h [T, K], router [E, K] -> [expert int32 [T, k], weight fp32 [T, k]]
-std::vector<at::Tensor> route_topk(const at::Tensor& h, const at::Tensor& router, int64_t k) {
-  SXE_CHECK_CUDA(h);
+namespace ex {
+
+void route_logits(const at::Tensor& h, const at::Tensor& router, at::Tensor& z) {
   SXE_CHECK(h.dim() == 2 && h.stride(1) == 1 && router.dim() == 2 && router.is_contiguous() && router.is_cuda() &&
-                router.size(1) == h.size(1) && router.scalar_type() == h.scalar_type(), "route_topk: h [T, K], router [E, K]");
+                router.size(1) == h.size(1) && router.scalar_type() == h.scalar_type(), "route: h [T, K], router [E, K]");
   const int64_t T = h.size(0), K = h.size(1), E = router.size(0);
-  SXE_CHECK(E <= ex::kMaxE && k > 0 && k <= E, "route_topk: up to ", ex::kMaxE, " experts, k of them");
-  auto f = h.options().dtype(at::kFloat);
-  auto z = at::empty({T, E}, f), wt = at::empty({T, k}, f), idx = at::empty({T, k}, h.options().dtype(at::kInt));
-  if (T == 0) return {idx, wt};
-  c10::DeviceGuard g(h.device());
-  if (h.scalar_type() == at::kBFloat16 && K % 16 == 0 && h.stride(0) % 8 == 0 && ex::aligned(h.data_ptr(), 16) &&
-      ex::aligned(router.data_ptr(), 16)) {
-    const dim3 grid((T + 31) / 32, (E + 31) / 32);
-    auto go = [&](auto kern, int nw) {
-      hipLaunchKernelGGL(kern, grid, dim3(64 * nw), 0, cur_stream(), static_cast<const unsigned short*>(h.data_ptr()), h.stride(0),
-                         static_cast<const unsigned short*>(router.data_ptr()), (int)T, (int)E, (int)K, z.data_ptr<float>());
-    };
-    if (T <= 1024 && K >= 1024) go(ex::route_logits_kernel<14>, 14);
-    else go(ex::route_logits_kernel<4>, 4);
+  SXE_CHECK(E > 0 && E <= kMaxE && T < (1ll << 31), "route: up to ", kMaxE, " experts");
+  const bool vec = h.scalar_type() == at::kBFloat16 && h.stride(0) % 8 == 0 && aligned(h.data_ptr(), 16) && aligned(router.data_ptr(), 16);
+  auto u16 = [](const at::Tensor& t) { return static_cast<const unsigned short*>(t.data_ptr()); };
+  if (vec && K % 8 == 0 && T <= 256) {
+    hipLaunchKernelGGL(route_logits_few_kernel, dim3((E + 3) / 4, (T + 7) / 8), dim3(256), 0, cur_stream(), u16(h), h.stride(0),
+                       u16(router), (int)T, (int)E, (int)K, z.data_ptr<float>());
+  } else if (vec && K % 16 == 0) {
+    hipLaunchKernelGGL(route_logits_kernel<4>, dim3((T + 31) / 32, (E + 31) / 32), dim3(256), 0, cur_stream(), u16(h), h.stride(0),
+                       u16(router), (int)T, (int)E, (int)K, z.data_ptr<float>());
   } else {
-    SXE_CHECK(T < (1ll << 31), "route_topk: rows");
     SXE_DISPATCH_DT(dtype_of(h), D, {
       using S = dt_traits<D>::storage;
-      hipLaunchKernelGGL((ex::route_logits_generic_kernel<D>), dim3(T, (E + 3) / 4), dim3(256), 0, cur_stream(),
+      hipLaunchKernelGGL((route_logits_generic_kernel<D>), dim3(T, (E + 3) / 4), dim3(256), 0, cur_stream(),
                          static_cast<const S*>(h.data_ptr()), h.stride(0), static_cast<const S*>(router.data_ptr()), (int)E, (int)K,
                          z.data_ptr<float>());
     });
   }
-  hipLaunchKernelGGL(ex::route_top_kernel, dim3((T + 3) / 4), dim3(256), 0, cur_stream(), z.data_ptr<float>(), (int)T, (int)E, (int)k,
-                     idx.data_ptr<int>(), wt.data_ptr<float>());
-  SXE_LAUNCH_CHECK();
-  return {idx, wt};
 }
 
-// expert int32 [T, k], weight fp32 [T, k] -> [token int32 [R], weight fp32 [R], slots int32 [T, k], offsets int32
-// [E + 1], active int32 [1 + E] (count, then the experts that have rows)]
-std::vector<at::Tensor> moe_lists(const at::Tensor& expert, const at::Tensor& weight, int64_t E) {
-  SXE_CHECK_CUDA(expert);
-  SXE_CHECK(expert.dim() == 2 && expert.is_contiguous() && expert.scalar_type() == at::kInt && weight.is_cuda() &&
-                weight.is_contiguous() && weight.scalar_type() == at::kFloat && weight.sizes() == expert.sizes(),
-            "moe_lists: expert int32 [T, k], weight fp32 [T, k]");
-  SXE_CHECK(E > 0 && E <= ex::kMaxE && expert.numel() < (1ll << 31), "moe_lists: sizes");
-  const int64_t R = expert.numel(), k = expert.size(1);
-  auto io = expert.options();
-  auto token = at::empty({R}, io), slots = at::empty_like(expert), offs = at::empty({E + 1}, io), active = at::empty({E + 1}, io);
-  auto ws = at::empty({R}, weight.options());
-  if (R == 0) return {token, ws, slots, offs, active};
-  c10::DeviceGuard g(expert.device());
-  const int* ep = expert.data_ptr<int>();
-  const float* wp = weight.data_ptr<float>();
-  if (R <= ex::kListThreads) {
-    hipLaunchKernelGGL(ex::moe_lists_small_kernel, dim3(1), dim3(ex::kListThreads), 0, cur_stream(), ep, wp, (int)R, (int)k, (int)E,
-                       token.data_ptr<int>(), ws.data_ptr<float>(), slots.data_ptr<int>(), offs.data_ptr<int>(),
-                       active.data_ptr<int>());
+// logits [T, E] -> [expert int32 [T, k], weight fp32 [T, k], token int32 [R], weight fp32 [R], slots int32 [T, k],
+// offsets int32 [E + 1], active int32 [1 + E] (count, then the experts that have rows)]
+std::vector<at::Tensor> choose(const at::Tensor& z, int64_t k) {
+  const int64_t T = z.size(0), E = z.size(1), R = T * k;
+  SXE_CHECK(k > 0 && k <= E && R < (1ll << 31), "route: top ", k, " of ", E);
+  auto io = z.options().dtype(at::kInt);
+  auto idx = at::empty({T, k}, io), token = at::empty({R}, io), slots = at::empty({T, k}, io), offs = at::empty({E + 1}, io),
+       active = at::empty({E + 1}, io);
+  auto wt = at::empty({T, k}, z.options()), ws = at::empty({R}, z.options());
+  if (R == 0) return {idx, wt, token, ws, slots, offs, active};
+  if (R <= kListThreads) {
+    hipLaunchKernelGGL(moe_lists_small_kernel, dim3(1), dim3(kListThreads), 0, cur_stream(), z.data_ptr<float>(), idx.data_ptr<int>(),
+                       wt.data_ptr<float>(), (int)R, (int)k, (int)E, token.data_ptr<int>(), ws.data_ptr<float>(),
+                       slots.data_ptr<int>(), offs.data_ptr<int>(), active.data_ptr<int>());
   } else {
+    hipLaunchKernelGGL(route_top_kernel, dim3((T + 3) / 4), dim3(256), 0, cur_stream(), z.data_ptr<float>(), (int)T, (int)E, (int)k,
+                       idx.data_ptr<int>(), wt.data_ptr<float>());
     auto counts = at::empty({E}, io);
     counts.zero_();
-    const dim3 grid((R + ex::kListThreads - 1) / ex::kListThreads);
-    hipLaunchKernelGGL(ex::moe_rank_kernel, grid, dim3(ex::kListThreads), 0, cur_stream(), ep, (int)R, (int)E, counts.data_ptr<int>(),
-                       slots.data_ptr<int>());
-    hipLaunchKernelGGL(ex::moe_place_kernel, grid, dim3(ex::kListThreads), 0, cur_stream(), ep, wp, (int)R, (int)k, (int)E,
-                       counts.data_ptr<int>(), token.data_ptr<int>(), ws.data_ptr<float>(), slots.data_ptr<int>(),
+    const dim3 grid((R + kListThreads - 1) / kListThreads);
+    hipLaunchKernelGGL(moe_rank_kernel, grid, dim3(kListThreads), 0, cur_stream(), idx.data_ptr<int>(), (int)R, (int)E,
+                       counts.data_ptr<int>(), slots.data_ptr<int>());
+    hipLaunchKernelGGL(moe_place_kernel, grid, dim3(kListThreads), 0, cur_stream(), idx.data_ptr<int>(), wt.data_ptr<float>(), (int)R,
+                       (int)k, (int)E, counts.data_ptr<int>(), token.data_ptr<int>(), ws.data_ptr<float>(), slots.data_ptr<int>(),
                        offs.data_ptr<int>(), active.data_ptr<int>());
   }
-  SXE_LAUNCH_CHECK();
-  return {token, ws, slots, offs, active};
+  return {idx, wt, token, ws, slots, offs, active};
 }
 
-// x [Tx, K], w [E, N, K]; rows sorted by expert (offs, active of moe_lists); token int32 [R] or None (x has R rows);
+}  // namespace ex
+
+// h [T, K], router [E, K] -> the chosen experts, their weights and the expert-sorted lists (ex::choose)
+std::vector<at::Tensor> route_topk(const at::Tensor& h, const at::Tensor& router, int64_t k) {
+  SXE_CHECK_CUDA(h);
+  c10::DeviceGuard g(h.device());
+  auto z = at::empty({h.size(0), router.size(0)}, h.options().dtype(at::kFloat));
+  if (h.size(0) > 0) ex::route_logits(h, router, z);
+  auto out = ex::choose(z, k);
+  SXE_LAUNCH_CHECK();
+  return out;
+}
+
+// Decode: v = x + rms(y) wp [+ add], h = rms(v) wn, then route_topk(h). Returns [v fp32 [M, K], h bf16 [M, K], route_topk's].
+std::vector<at::Tensor> route_sandwich(const at::Tensor& x, const at::Tensor& y, const at::Tensor& wp, const at::Tensor& wn,
+                                       const c10::optional<at::Tensor>& slots, const c10::optional<at::Tensor>& add, double eps,
+                                       const at::Tensor& router, int64_t k) {
+  SXE_CHECK_CUDA(x);
+  SXE_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2 && x.is_contiguous(), "route_sandwich: x fp32 [M, K]");
+  const int64_t M = x.size(0), K = x.size(1), E = router.size(0);
+  SXE_CHECK(M >= 1 && M <= sw::kMaxM && K % 8 == 0 && M * K <= 2 * 8 * 512, "route_sandwich: up to 4 rows, M K <= 8192");
+  const bool has_s = slots.has_value() && slots->defined(), has_a = add.has_value() && add->defined();
+  SXE_CHECK(y.is_cuda() && y.scalar_type() == at::kBFloat16 && y.dim() == 2 && y.is_contiguous() && y.size(1) == K &&
+                (has_s || y.size(0) == M), "route_sandwich: y bf16 [M, K]");
+  for (const auto* p : {&wp, &wn})
+    SXE_CHECK(p->is_cuda() && p->scalar_type() == at::kBFloat16 && p->is_contiguous() && p->numel() == K, "route_sandwich: norms");
+  SXE_CHECK(router.is_cuda() && router.scalar_type() == at::kBFloat16 && router.is_contiguous() && router.dim() == 2 &&
+                router.size(1) == K && E > 0 && E <= ex::kMaxE, "route_sandwich: router bf16 [E, K]");
+  if (has_s)
+    SXE_CHECK(slots->is_cuda() && slots->scalar_type() == at::kInt && slots->is_contiguous() && slots->dim() == 2 &&
+                  slots->size(0) == M && slots->numel() <= y.size(0), "route_sandwich: slots int32 [M, k]");
+  if (has_a)
+    SXE_CHECK(add->is_cuda() && add->scalar_type() == at::kFloat && add->is_contiguous() && add->sizes() == x.sizes(),
+              "route_sandwich: add like x");
+  for (const void* q : {(const void*)x.data_ptr(), (const void*)y.data_ptr(), (const void*)wp.data_ptr(), (const void*)wn.data_ptr(),
+                        (const void*)router.data_ptr(), has_a ? (const void*)add->data_ptr() : nullptr})
+    SXE_CHECK(ex::aligned(q, 16), "route_sandwich: 16-byte aligned operands");
+  c10::DeviceGuard g(x.device());
+  auto v = at::empty_like(x), h = at::empty({M, K}, y.options()), z = at::empty({M, E}, x.options());
+  auto u16 = [](const at::Tensor& t) { return static_cast<unsigned short*>(t.data_ptr()); };
+  sw::Args a{u16(y), u16(wp), u16(wn), x.data_ptr<float>(), has_a ? add->data_ptr<float>() : nullptr,
+             has_s ? slots->data_ptr<int>() : nullptr, has_s ? (int)slots->size(1) : 1, (float)eps, v.data_ptr<float>()};
+  hipLaunchKernelGGL(ex::route_sandwich_kernel, dim3((E + 7) / 8), dim3(512), M * K * 2, cur_stream(), a, (const unsigned short*)u16(router),
+                     (int)M, (int)E, (int)K, u16(h), z.data_ptr<float>());
+  std::vector<at::Tensor> out{v, h};
+  for (auto& t : ex::choose(z, k)) out.push_back(t);
+  SXE_LAUNCH_CHECK();
+  return out;
+}
+
+// x [Tx, K], w [E, N, K]; rows sorted by expert (offs, active of ex::choose); token int32 [R] or None (x has R rows);
 // ws fp32 [R] or None -> [R, N]
 at::Tensor expert_gemm(const at::Tensor& x, const at::Tensor& w, const at::Tensor& offs, const at::Tensor& active,
                        const c10::optional<at::Tensor>& token, const c10::optional<at::Tensor>& ws, int64_t R, int64_t act) {
@@ -484,11 +596,12 @@ at::Tensor expert_gemm(const at::Tensor& x, const at::Tensor& w, const at::Tenso
 
 TORCH_LIBRARY_FRAGMENT(sxe, m) {
   m.def("route_topk(Tensor h, Tensor router, int k) -> Tensor[]");
-  m.def("moe_lists(Tensor expert, Tensor weight, int E) -> Tensor[]");
+  m.def("route_sandwich(Tensor x, Tensor y, Tensor wp, Tensor wn, Tensor? slots, Tensor? add, float eps, Tensor router, int k) -> "
+        "Tensor[]");
   m.def("expert_gemm(Tensor x, Tensor w, Tensor offs, Tensor active, Tensor? token, Tensor? ws, int R, int act) -> Tensor");
 }
 TORCH_LIBRARY_IMPL(sxe, CUDA, m) {
   m.impl("route_topk", &sxe::route_topk);
-  m.impl("moe_lists", &sxe::moe_lists);
+  m.impl("route_sandwich", &sxe::route_sandwich);
   m.impl("expert_gemm", &sxe::expert_gemm);
 }

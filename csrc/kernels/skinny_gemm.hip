@@ -19,6 +19,7 @@
 //    flight, so the norm / gated-activation launches (4-5 us each at batch 1, latency-bound) are
 //    gone from the decode layer. Workgroup 0 also writes the new residual stream h = x + res.
 #include "sxe_common.h"
+#include "sxe_sandwich.h"
 #include <torch/library.h>
 
 namespace sxe {
@@ -55,7 +56,8 @@ __device__ __forceinline__ void load_x(Frag& f, const unsigned short* __restrict
   }
 }
 
-enum : int { PRO_NONE = 0, PRO_RMS = 1, PRO_SWIGLU = 2, PRO_MERGE = 3, PRO_ADDNORM = 4, PRO_GATESUM = 5 };
+enum : int { PRO_NONE = 0, PRO_RMS = 1, PRO_SWIGLU = 2, PRO_MERGE = 3, PRO_ADDNORM = 4, PRO_GATESUM = 5, PRO_SANDWICH = 6,
+              PRO_GATENORM = 7 };
 constexpr int kProMaxM = 4;
 
 struct ProArgs {
@@ -91,6 +93,9 @@ struct ProArgs {
   // GATESUM: input = sigmoid(gate) * sum over `splits` of po [splits, M, K] (fp32)
   const unsigned short* gate;
   int64_t gate_ld;
+  // SANDWICH: norms on both sides of the residual sum (sxe_sandwich.h)
+  sw::Args sand;
+  // GATENORM: input = rms(x) gw sigmoid(gate)
 };
 
 // output column of lane `col` in tile `tile` (identity unless the RoPE epilogue pairs columns)
@@ -232,7 +237,12 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
     build_gatesum<NT>(M, K, p, act);
     return;
   }
-  constexpr bool NORM = MODE == PRO_RMS || MODE == PRO_ADDNORM;
+  if constexpr (MODE == PRO_SANDWICH) {
+    __shared__ float sred[NT / 64][kProMaxM];
+    sw::build<NT, 2, false>(p.sand, M, K, blockIdx.x == 0, act, rinv, sred);
+    return;
+  }
+  constexpr bool NORM = MODE == PRO_RMS || MODE == PRO_ADDNORM || MODE == PRO_GATENORM;
   if constexpr (NORM) {
     klo = 0;
     khi = K;
@@ -258,12 +268,13 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
         b[u] = *reinterpret_cast<const u16x8*>(xr + K);
       } else {
         gw[u] = *reinterpret_cast<const u16x8*>(p.gw + (ok ? c : 0));
+        if constexpr (MODE == PRO_GATENORM) b[u] = *reinterpret_cast<const u16x8*>(p.gate + (ok ? m * p.gate_ld + c : 0));
         if constexpr (MODE == PRO_ADDNORM) {
           const float* rp = p.res32 + (int64_t)(ok ? m : 0) * K + (ok ? c : 0);
           r0[u] = *reinterpret_cast<const f32x4*>(rp);
           r1[u] = *reinterpret_cast<const f32x4*>(rp + 4);
           if (p.rw != nullptr) b[u] = *reinterpret_cast<const u16x8*>(p.rw + (ok ? c : 0));
-        } else if (p.res != nullptr) b[u] = *reinterpret_cast<const u16x8*>(p.res + (int64_t)(ok ? m : 0) * ldx + (ok ? c : 0));
+        } else if (MODE != PRO_GATENORM && p.res != nullptr) b[u] = *reinterpret_cast<const u16x8*>(p.res + (int64_t)(ok ? m : 0) * ldx + (ok ? c : 0));
       }
     }
 #pragma unroll
@@ -294,7 +305,7 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
             *reinterpret_cast<f32x4*>(p.hout32 + (int64_t)m * K + c) = f32x4{v[0], v[1], v[2], v[3]};
             *reinterpret_cast<f32x4*>(p.hout32 + (int64_t)m * K + c + 4) = f32x4{v[4], v[5], v[6], v[7]};
           }
-        } else if (p.res != nullptr) {
+        } else if (MODE != PRO_GATENORM && p.res != nullptr) {
 #pragma unroll
           for (int j = 0; j < 8; ++j) v[j] = bf16_to_f32(f32_to_bf16(v[j] + bf16_to_f32(b[u][j])));
           if (p.hout != nullptr && blockIdx.x == 0) store8<DT::BF16>(p.hout + (int64_t)m * K + c, v);
@@ -304,6 +315,7 @@ __device__ __forceinline__ void build_act(const unsigned short* __restrict x, in
         for (int j = 0; j < 8; ++j) {
           q += v[j] * v[j];
           o[j] = v[j] * (MODE == PRO_ADDNORM ? p.offset + bf16_to_f32(gw[u][j]) : bf16_to_f32(gw[u][j]));
+          if (MODE == PRO_GATENORM) o[j] /= 1.f + __expf(-bf16_to_f32(b[u][j]));
         }
 #pragma unroll
         for (int mm = 0; mm < kProMaxM; ++mm)
@@ -403,7 +415,8 @@ __global__ __launch_bounds__(NW * 64) void skinny_gemm_kernel(const unsigned sho
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int m = 4 * g + r;
-        const float sc = MODE == PRO_RMS || MODE == PRO_ADDNORM ? rinv[m < kProMaxM ? m : 0] : 1.f;
+        constexpr bool kScaled = MODE == PRO_RMS || MODE == PRO_ADDNORM || MODE == PRO_SANDWICH || MODE == PRO_GATENORM;
+        const float sc = kScaled ? rinv[m < kProMaxM ? m : 0] : 1.f;
         if (m < M) y[(int64_t)m * ldy + n] = f32_to_bf16(t[r] * sc + b);
       }
     }
@@ -861,10 +874,14 @@ static at::Tensor skinny_launch(int mode, const unsigned short* xp, int64_t ldx,
   const int ss_total = (K + sg::kSS - 1) / sg::kSS, tiles = (N + 15) / 16;
   int nw = 4, spw = 1;
   sg::plan(tiles, ss_total, nw, spw);
+  if (mode == sg::PRO_SANDWICH && (int64_t)M * K > 2 * 8 * 256) {  // the prologue keeps its rows in registers
+    nw = 8;
+    spw = (ss_total + nw - 1) / nw;
+  }
   pro.nt = sg::nt_loads();
-  static bool attr[2][2] = {};
+  static bool attr[8][2] = {};
   auto go = [&](auto kern, int ni) {
-    bool& done = attr[mode == sg::PRO_ADDNORM][ni];
+    bool& done = attr[mode][ni];
     if (!done) {
       SXE_HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, 144 * 1024));
       done = true;
@@ -876,6 +893,12 @@ static at::Tensor skinny_launch(int mode, const unsigned short* xp, int64_t ldx,
   if (mode == sg::PRO_ADDNORM) {
     if (nw == 4) go(sg::skinny_gemm_kernel<4, sg::PRO_ADDNORM, false>, 0);
     else go(sg::skinny_gemm_kernel<8, sg::PRO_ADDNORM, false>, 1);
+  } else if (mode == sg::PRO_SANDWICH) {
+    if (nw == 4) go(sg::skinny_gemm_kernel<4, sg::PRO_SANDWICH, false>, 0);
+    else go(sg::skinny_gemm_kernel<8, sg::PRO_SANDWICH, false>, 1);
+  } else if (mode == sg::PRO_GATENORM) {
+    if (nw == 4) go(sg::skinny_gemm_kernel<4, sg::PRO_GATENORM, false>, 0);
+    else go(sg::skinny_gemm_kernel<8, sg::PRO_GATENORM, false>, 1);
   } else {
     if (nw == 4) go(sg::skinny_gemm_kernel<4, sg::PRO_GATESUM, false>, 0);
     else go(sg::skinny_gemm_kernel<8, sg::PRO_GATESUM, false>, 1);
@@ -946,9 +969,63 @@ at::Tensor skinny_gemm_gatesum(const at::Tensor& part, const c10::optional<at::T
   return skinny_launch(sg::PRO_GATESUM, nullptr, K, M, w, pro);
 }
 
+// Decode, norms on both sides of the residual sum (PRO_SANDWICH): v = x + rms(y) wp [+ add], out = (rms(v) wn) . w^T.
+// x, add fp32 [M, K]; y bf16 [rows, K], with slots int32 [M, k] the sum of k rows. Returns [out [M, N], v].
+std::vector<at::Tensor> skinny_gemm_sandwich(const at::Tensor& x, const at::Tensor& y, const at::Tensor& wp, const at::Tensor& wn,
+                                             const c10::optional<at::Tensor>& slots, const c10::optional<at::Tensor>& add, double eps,
+                                             const at::Tensor& w) {
+  SXE_CHECK_CUDA(x);
+  SXE_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2 && x.is_contiguous(), "skinny_gemm_sandwich: x fp32 [M, K]");
+  const int M = x.size(0), K = x.size(1);
+  SXE_CHECK(w.dim() == 2 && w.size(1) == K && (int64_t)M * K <= 2 * 8 * 512, "skinny_gemm_sandwich: w [N, K], M K <= 8192");
+  const bool has_s = slots.has_value() && slots->defined(), has_a = add.has_value() && add->defined();
+  SXE_CHECK(y.is_cuda() && y.scalar_type() == at::kBFloat16 && y.dim() == 2 && y.is_contiguous() && y.size(1) == K &&
+                (has_s || y.size(0) == M), "skinny_gemm_sandwich: y bf16 [M, K]");
+  for (const auto* p : {&wp, &wn})
+    SXE_CHECK(p->is_cuda() && p->scalar_type() == at::kBFloat16 && p->is_contiguous() && p->numel() == K, "skinny_gemm_sandwich: norms");
+  if (has_s)
+    SXE_CHECK(slots->is_cuda() && slots->scalar_type() == at::kInt && slots->is_contiguous() && slots->dim() == 2 &&
+                  slots->size(0) == M && slots->numel() <= y.size(0), "skinny_gemm_sandwich: slots int32 [M, k]");
+  if (has_a)
+    SXE_CHECK(add->is_cuda() && add->scalar_type() == at::kFloat && add->is_contiguous() && add->sizes() == x.sizes(),
+              "skinny_gemm_sandwich: add like x");
+  for (const void* q : {(const void*)x.data_ptr(), (const void*)y.data_ptr(), (const void*)wp.data_ptr(), (const void*)wn.data_ptr(),
+                        has_a ? (const void*)add->data_ptr() : nullptr})
+    SXE_CHECK(reinterpret_cast<uintptr_t>(q) % 16 == 0, "skinny_gemm_sandwich: 16-byte aligned operands");
+  c10::DeviceGuard gd(x.device());
+  auto v = at::empty_like(x);
+  sg::ProArgs pro{};
+  auto u16 = [](const at::Tensor& t) { return reinterpret_cast<const unsigned short*>(t.data_ptr()); };
+  pro.sand = sw::Args{u16(y), u16(wp), u16(wn), x.data_ptr<float>(), has_a ? add->data_ptr<float>() : nullptr,
+                      has_s ? slots->data_ptr<int>() : nullptr, has_s ? (int)slots->size(1) : 1, (float)eps, v.data_ptr<float>()};
+  return {skinny_launch(sg::PRO_SANDWICH, nullptr, K, M, w, pro), v};
+}
+
+// Decode (PRO_GATENORM): (rms(x) gw sigmoid(gate)) . w^T; x bf16 [M, K], gate bf16 [M, K] (row stride free)
+at::Tensor skinny_gemm_gatenorm(const at::Tensor& x, const at::Tensor& gw, const at::Tensor& gate, double eps, const at::Tensor& w) {
+  SXE_CHECK_CUDA(x);
+  SXE_CHECK(x.scalar_type() == at::kBFloat16 && x.dim() == 2 && x.is_contiguous(), "skinny_gemm_gatenorm: x bf16 [M, K]");
+  const int M = x.size(0), K = x.size(1);
+  SXE_CHECK(w.dim() == 2 && w.size(1) == K && gw.is_cuda() && gw.scalar_type() == at::kBFloat16 && gw.is_contiguous() &&
+                gw.numel() == K, "skinny_gemm_gatenorm: gw [K], w [N, K]");
+  SXE_CHECK(gate.is_cuda() && gate.scalar_type() == at::kBFloat16 && gate.dim() == 2 && gate.size(0) == M && gate.size(1) == K &&
+                gate.stride(1) == 1 && gate.stride(0) % 8 == 0, "skinny_gemm_gatenorm: gate bf16 [M, K], 16-B rows");
+  for (const void* q : {(const void*)x.data_ptr(), (const void*)gw.data_ptr(), (const void*)gate.data_ptr()})
+    SXE_CHECK(reinterpret_cast<uintptr_t>(q) % 16 == 0, "skinny_gemm_gatenorm: 16-byte aligned operands");
+  c10::DeviceGuard gd(x.device());
+  sg::ProArgs pro{};
+  pro.gw = reinterpret_cast<const unsigned short*>(gw.data_ptr());
+  pro.eps = (float)eps;
+  pro.gate = reinterpret_cast<const unsigned short*>(gate.data_ptr());
+  pro.gate_ld = gate.stride(0);
+  return skinny_launch(sg::PRO_GATENORM, reinterpret_cast<const unsigned short*>(x.data_ptr()), x.stride(0), M, w, pro);
+}
+
 }  // namespace sxe
 
 TORCH_LIBRARY_FRAGMENT(sxe, m) {
+  m.def("skinny_gemm_sandwich(Tensor x, Tensor y, Tensor wp, Tensor wn, Tensor? slots, Tensor? add, float eps, Tensor w) -> Tensor[]");
+  m.def("skinny_gemm_gatenorm(Tensor x, Tensor gw, Tensor gate, float eps, Tensor w) -> Tensor");
   m.def("skinny_gemm(Tensor x, Tensor w, Tensor? bias) -> Tensor");
   m.def("skinny_gemm_fp8w(Tensor x, Tensor wq, Tensor wscale, Tensor? bias) -> Tensor");
   m.def("skinny_gemm_pro(Tensor x, Tensor? res, Tensor? gw, float eps, Tensor w, Tensor? wscale, Tensor? bias, "
@@ -961,6 +1038,8 @@ TORCH_LIBRARY_FRAGMENT(sxe, m) {
         "Tensor sin, Tensor pos, Tensor slots, Tensor(a!) cache, int nq, int nkv) -> Tensor[]");
 }
 TORCH_LIBRARY_IMPL(sxe, CUDA, m) {
+  m.impl("skinny_gemm_sandwich", &sxe::skinny_gemm_sandwich);
+  m.impl("skinny_gemm_gatenorm", &sxe::skinny_gemm_gatenorm);
   m.impl("skinny_gemm", &sxe::skinny_gemm);
   m.impl("skinny_gemm_fp8w", &sxe::skinny_gemm_fp8w);
   m.impl("skinny_gemm_pro", &sxe::skinny_gemm_pro);

@@ -35,10 +35,11 @@ import torch
 
 from ....ops.activation import gated_act
 from ....ops.latent_attention import latent_append, latent_attention, latent_row, rotation_table
-from ....ops.linear import fused_addnorm_linear, fused_gatesum_linear, fused_swiglu_linear, linear
+from ....ops.linear import (fused_addnorm_linear, fused_gatenorm_linear, fused_gatesum_linear, fused_sandwich_linear,
+                            fused_swiglu_linear, linear)
 from ....ops.linear_attention import decay_attention, decay_table
 from ....ops.mix_attention import MixParams, cache_row, mix_attention, mix_attention_parts
-from ....ops.moe import expert_mlp, route_topk
+from ....ops.moe import expert_mlp, fused_sandwich_route, route_topk
 from ....ops.residual_norm import (embed_norm, embed_scale, gated_rms_norm, qkv_norm_append, residual_rms_norm,
                                    sandwich_norm)
 
@@ -445,17 +446,38 @@ class RaggedLayeredDecoder:
         return linear(h, W["embed"]).float()
 
     # ------------------------------------------------------------------------- norm on both sides
-    def _linear_mixer(self, h, L, a, run, batch, kv_cache):
-        """Decayed linear attention; ``h`` the normed input [T, width]."""
-        proj = linear(h, L["qkvg"])
-        o = decay_attention(proj, kv_cache.layer_state(run), L["decay"], batch, a.heads, a.dim, a.vdim)
-        return linear(gated_rms_norm(o, L["o_norm"], proj[:, a.heads * (2 * a.dim + a.vdim):], self.spec.eps), L["o"])
+    # The sum and the norms between two sublayers stay pending until the next sublayer's first product asks for
+    # its input: at decode that product builds it in its own launch.
+    def _normed(self, st, pre, index=None, last=False):
+        """The next sublayer's input rms(x) * pre, the pending sum taken into x first."""
+        if st.pending is not None:
+            y, post, slots, add = st.pending
+            st.x, st.h = sandwich_norm(st.x, y, post, pre, self.spec.eps, slots, add, index, need_x=not last)
+            st.pending = None
+        return st.h
 
-    def _latent_mixer(self, h, L, a, run, batch, kv_cache):
+    def _project(self, st, pre, weight):
+        if st.pending is not None and self._fusable(st.x.shape[0]):
+            y, post, slots, add = st.pending
+            r = fused_sandwich_linear(st.x, y, post, pre, self.spec.eps, slots, add, weight)
+            if r is not None:
+                st.x, st.pending = r[1], None
+                return r[0]
+        return linear(self._normed(st, pre), weight)
+
+    def _linear_mixer(self, st, L, a, run, batch, kv_cache):
+        """Decayed linear attention."""
+        proj = self._project(st, L["norm1"], L["qkvg"])
+        o = decay_attention(proj, kv_cache.layer_state(run), L["decay"], batch, a.heads, a.dim, a.vdim)
+        gate = proj[:, a.heads * (2 * a.dim + a.vdim):]
+        y = fused_gatenorm_linear(o, L["o_norm"], gate, self.spec.eps, L["o"]) if self._fusable(o.shape[0]) else None
+        return linear(gated_rms_norm(o, L["o_norm"], gate, self.spec.eps), L["o"]) if y is None else y
+
+    def _latent_mixer(self, st, L, a, run, batch, kv_cache):
+        proj = self._project(st, L["norm1"], L["dqkv"])
         cache = kv_cache.layer_kv(run)[0]
         rot = self._rotation(batch, a)
-        cq = latent_append(linear(h, L["dqkv"]), L["q_norm"], L["kv_norm"], cache, batch.slots, rot, a.q_rank, a.kv_rank,
-                           a.rot_dim, self.spec.eps)
+        cq = latent_append(proj, L["q_norm"], L["kv_norm"], cache, batch.slots, rot, a.q_rank, a.kv_rank, a.rot_dim, self.spec.eps)
         o = latent_attention(linear(cq, L["uq"]), L["uk"], L["uv"], L["ukv"], cache, batch, rot, a.heads, a.dim, a.rot_dim,
                              a.vdim, a.kv_rank, a.scale, a.window)
         return linear(o, L["o"])
@@ -467,39 +489,48 @@ class RaggedLayeredDecoder:
             self._rot[key] = rotation_table(batch.positions, *key)
         return self._rot[key]
 
-    def _feed_forward(self, h, L, spec):
+    def _feed_forward(self, st, L, spec):
         """-> (output rows, slots): slots None for one row a token (ops/residual_norm.sandwich_norm)."""
         if spec.moe is None:
-            return linear(gated_act(linear(h, L["gu"]), spec.act), L["down"]), None
-        expert, weight = route_topk(h, L["router"], spec.moe.top)
-        return expert_mlp(h, expert, weight, L["e_up"], L["e_down"], spec.moe.act)
+            gu = self._project(st, L["norm2"], L["gu"])
+            y = fused_swiglu_linear(gu, L["down"]) if self._fusable(gu.shape[0]) and spec.act == "silu" else None
+            return (linear(gated_act(gu, spec.act), L["down"]) if y is None else y), None
+        r = None
+        if st.pending is not None and self._fusable(st.x.shape[0]):
+            y, post, slots, add = st.pending
+            r = fused_sandwich_route(st.x, y, post, L["norm2"], self.spec.eps, slots, add, L["router"], spec.moe.top)
+        if r is not None:
+            (st.x, h, routing), st.pending = r, None
+        else:
+            h = self._normed(st, L["norm2"])
+            routing = route_topk(h, L["router"], spec.moe.top)
+        return expert_mlp(h, routing, L["e_up"], L["e_down"], spec.moe.act)
 
     def _forward_sandwich(self, batch, kv_cache):
         s, W = self.spec, self.w
         self._rot = {}
-        steps = []  # (run, layer, is mixer, embedding output added first)
+        x0, h = embed_norm(W["embed"], batch.input_ids, W["embed_norm"], s.eps, W["layers"][self.runs[0][0]]["norm1"])
+        st = _Stream(x0, h)
         for r, (i, again) in enumerate(self.runs):
-            steps.append((r, i, True, again))
-            if "norm2" in W["layers"][i]:
-                steps.append((r, i, False, False))
-
-        def pre(n):  # weight of the norm in front of step n; after the last one the model's final norm
-            return W["final"] if n == len(steps) else W["layers"][steps[n][1]]["norm1" if steps[n][2] else "norm2"]
-        x, h = embed_norm(W["embed"], batch.input_ids, W["embed_norm"], s.eps, pre(0))
-        x0 = x
-        for n, (r, i, mixer, _) in enumerate(steps):
-            L, spec, slots = W["layers"][i], s.layers[i], None
-            if not mixer:
-                y, slots = self._feed_forward(h, L, spec)
-            elif isinstance(spec.mixer, LinearSpec):
-                y = self._linear_mixer(h, L, spec.mixer, r, batch, kv_cache)
-            else:
-                y = self._latent_mixer(h, L, spec.mixer, r, batch, kv_cache)
-            last = n + 1 == len(steps)
-            add = x0 if not last and steps[n + 1][3] else None
-            x, h = sandwich_norm(x, y, L["norm1b" if mixer else "norm2b"], pre(n + 1), s.eps, slots, add,
-                                 batch.last_idx if last else None, need_x=not last)
+            L, spec = W["layers"][i], s.layers[i]
+            if again:
+                st.pending = st.pending[:3] + (x0,)
+            mixer = self._linear_mixer if isinstance(spec.mixer, LinearSpec) else self._latent_mixer
+            st.pending = (mixer(st, L, spec.mixer, r, batch, kv_cache), L["norm1b"], None, None)
+            if "norm2" in L:
+                y, slots = self._feed_forward(st, L, spec)
+                st.pending = (y, L["norm2b"], slots, None)
+        h = self._normed(st, W["final"], batch.last_idx, last=True)
         return linear(h, W["head"]).float() * s.logit_scale
+
+
+@dataclass
+class _Stream:
+    """The 32-bit residual stream between sublayers: x, and either the normed input ``h`` of the next sublayer or
+    the last one's ``pending`` (output, its norm weight, slots, rows to add) that x does not hold yet."""
+    x: torch.Tensor
+    h: Optional[torch.Tensor] = None
+    pending: Optional[tuple] = None
 
 
 def load_layered_decoder(path, dtype=torch.bfloat16, device=None, weight_quant=None, tp_size=1):

@@ -161,6 +161,34 @@ def fused_gatesum_linear(part, gate, weight):
     return torch.ops.sxe.skinny_gemm_gatesum(part, gate, wk[0])
 
 
+def sandwich_fusable(x, y, *weights):
+    """Whether the decode kernels with the sandwich-norm prologue (csrc/include/sxe_sandwich.h) take these rows:
+    up to 4, M K <= 8192."""
+    M, K = x.shape
+    return (0 < M <= 4 and K % 8 == 0 and M * K <= 8192 and x.is_contiguous() and y.is_contiguous()
+            and all(t.dtype == torch.bfloat16 and t.is_contiguous() and t.data_ptr() % 16 == 0 for t in (y, *weights)))
+
+
+def fused_sandwich_linear(x, y, post_weight, next_weight, eps, slots, add, weight):
+    """Decode (<= 4 rows): ``sandwich_norm`` (ops/residual_norm.py) and the projection that reads its result in
+    ONE launch (skinny_gemm.hip PRO_SANDWICH): (linear(h, weight), x'). None when not covered."""
+    wk = _pro_weight(weight)
+    if wk is None or wk[1] is not None or not sandwich_fusable(x, y, post_weight, next_weight) or x.shape[1] != wk[0].shape[1]:
+        return None
+    return torch.ops.sxe.skinny_gemm_sandwich(x, y, post_weight, next_weight, slots, add, float(eps), wk[0])
+
+
+def fused_gatenorm_linear(x, norm_weight, gate, eps, weight):
+    """Decode (<= 4 rows): ``linear(gated_rms_norm(x, norm_weight, gate), weight)`` in ONE launch (skinny_gemm.hip
+    PRO_GATENORM). None when not covered."""
+    wk = _pro_weight(weight)
+    if (wk is None or wk[1] is not None or not _pro_ok(x) or not x.is_contiguous() or x.shape[1] != wk[0].shape[1]
+            or x.shape[1] % 8 or gate.stride(0) % 8 or gate.data_ptr() % 16 or norm_weight.data_ptr() % 16
+            or x.numel() * 2 > 144 * 1024):
+        return None
+    return torch.ops.sxe.skinny_gemm_gatenorm(x, norm_weight, gate, float(eps), wk[0])
+
+
 # Hand-written weight-gradient GEMM (csrc/kernels/gemm_wgrad.hip: k-major operands read through LDS
 # with ds_read_b64_tr_b16, fp32 accumulate in the epilogue): no transposed copies of dY / X at all.
 # Measured on MI355X at 8192 tokens (tools/wgrad_exp.py, profiles/wgrad_kernel.log): 28672x4096

@@ -13,6 +13,8 @@ Parity: reference inference/v2/kernels/ragged_ops/top_k_gating (:15), moe_scatte
 moe_gather (:21); training dispatch/combine of runtime moe/sharded_moe.py:587-678. CPU tensors
 (gloo plumbing tests) take the equivalent PyTorch ops.
 """
+from typing import NamedTuple
+
 import torch
 import torch.nn.functional as F
 
@@ -256,43 +258,57 @@ class IntWeight:
 
 # ------------------------------------------------------- routed experts without a gate (device routing)
 EXPERT_ACTS = {"none": 0, "relu2": 1, "silu": 2}
+SKINNY_ROWS = 16  # mean rows per expert up to which the skinny expert kernels are used
+
+
+class Routing(NamedTuple):
+    expert: torch.Tensor   # int32 [T, top]
+    weight: torch.Tensor   # fp32 [T, top]
+    lists: tuple = ()      # GPU: the assignments sorted by expert (csrc/kernels/experts.hip)
 
 
 def route_topk(h, router, top):
     """Logits h . router in fp32 (router [E, D] as stored), the ``top`` largest, weights = softmax over those
-    alone: (expert int32 [T, top], weight fp32 [T, top])."""
+    alone."""
     if _hip(h):
-        return tuple(torch.ops.sxe.route_topk(h, router, int(top)))
+        idx, wt, *lists = torch.ops.sxe.route_topk(h, router, int(top))
+        return Routing(idx, wt, tuple(lists))
     z = F.linear(h.float(), router.float())
     val, idx = z.topk(top, dim=-1)
-    return idx.to(torch.int32), torch.softmax(val, -1)
+    return Routing(idx.to(torch.int32), torch.softmax(val, -1))
 
 
-SKINNY_ROWS = 16  # mean rows per expert up to which the skinny expert kernels are used
+def fused_sandwich_route(x, y, post_weight, next_weight, eps, slots, add, router, top):
+    """Decode (<= 4 rows): ``sandwich_norm`` (ops/residual_norm.py) and ``route_topk`` of its result in two
+    launches: (x', h, Routing). None when not covered."""
+    from .linear import sandwich_fusable
+    if not sandwich_fusable(x, y, post_weight, next_weight, router):
+        return None
+    v, h, idx, wt, *lists = torch.ops.sxe.route_sandwich(x, y, post_weight, next_weight, slots, add, float(eps), router, int(top))
+    return v, h, Routing(idx, wt, tuple(lists))
 
 
-def expert_mlp(h, expert, weight, up, down, act="relu2"):
+def expert_mlp(h, routing, up, down, act="relu2"):
     """Two-layer experts up [E, F, D], down [E, D, F] on the rows ``route_topk`` chose. Returns (y, slots): y
     [T * top, D] holds weight * down(act(up h)) of every (token, choice), y[slots[t, j]] belongs to token t. No
     host synchronisation. Rows are sorted by expert and gathered inside the first product; few rows per
     expert stream the weights through the skinny kernels, more take the grouped ones (csrc/kernels/experts.hip,
     grouped_gemm.hip)."""
-    T, k = expert.shape
-    E = up.shape[0]
+    T, k = routing.expert.shape
+    E, R = up.shape[0], T * k
     if _hip(h):
-        rows, ws, slots, offs, active = torch.ops.sxe.moe_lists(expert, weight, E)
-        R = T * k
+        rows, ws, slots, offs, active = routing.lists
         if (R > SKINNY_ROWS * E and act in ("relu2", "none") and grouped_gemm_ok(h, up) and up.shape[1] % 128 == 0
                 and down.shape[1] % 128 == 0):
             a = torch.ops.sxe.grouped_gemm_rows(h, up, offs, None, rows, EXPERT_ACTS[act])
             return torch.ops.sxe.grouped_gemm_rows(a, down, offs, ws, None, 0), slots
         a = torch.ops.sxe.expert_gemm(h, up, offs, active, rows, None, R, EXPERT_ACTS[act])
         return torch.ops.sxe.expert_gemm(a, down, offs, active, None, ws, R, 0), slots
-    y = torch.zeros(T * k, down.shape[1], dtype=h.dtype, device=h.device)
-    flat = expert.reshape(-1)
+    y = torch.zeros(R, down.shape[1], dtype=h.dtype, device=h.device)
+    flat = routing.expert.reshape(-1)
     f = {"relu2": lambda z: torch.relu(z) ** 2, "silu": F.silu, "none": lambda z: z}[act]
     for e in flat.unique().tolist():
         r = (flat == e).nonzero()[:, 0]
         a = f(F.linear(h.index_select(0, r // k).float(), up[e].float())).to(h.dtype)
-        y[r] = (F.linear(a.float(), down[e].float()) * weight.reshape(-1, 1)[r]).to(h.dtype)
-    return y, torch.arange(T * k, dtype=torch.int32, device=h.device).view(T, k)
+        y[r] = (F.linear(a.float(), down[e].float()) * routing.weight.reshape(-1, 1)[r]).to(h.dtype)
+    return y, torch.arange(R, dtype=torch.int32, device=h.device).view(T, k)

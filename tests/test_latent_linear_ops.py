@@ -236,12 +236,13 @@ def test_routed_experts(T, E, k, D, F, device, dtype):
     ref = O.moe_ff(h.double(), {n: t.double() for n, t in w.items()}, "", {"router": {"experts": E, "top": k}})
     up, down = (torch.stack([w[f"e{e}.{n}"] for e in range(E)]).to(device) for n in ("up", "down"))
     hd = h.to(device)
-    idx, wt = ME.route_topk(hd, w["router"].to(device), k)
+    routing = ME.route_topk(hd, w["router"].to(device), k)
+    idx, wt = routing[:2]
     z = h.double() @ w["router"].double().T
     val, ri = z.topk(k, dim=-1)
     torch.testing.assert_close(wt.double().cpu(), torch.softmax(val, -1), rtol=2e-5, atol=1e-6)
     assert torch.equal(idx.cpu().long(), ri)  # the fp32 order of random logits
-    y, slots = ME.expert_mlp(hd, idx, wt, up, down)
+    y, slots = ME.expert_mlp(hd, routing, up, down)
     assert sorted(slots.cpu().reshape(-1).tolist()) == list(range(T * k))
     got = y.cpu().double()[slots.cpu().long().reshape(-1)].view(T, k, D).sum(1)
     close(got, ref, 2e-2 if dtype == torch.bfloat16 else 2e-5)
@@ -251,7 +252,7 @@ def test_routed_experts(T, E, k, D, F, device, dtype):
 def test_route_topk_prefers_the_lower_index_and_survives_nan():
     h = torch.zeros(3, 32, dtype=torch.bfloat16, device="cuda")
     h[2] = float("nan")
-    idx, wt = ME.route_topk(h, torch.randn(12, 32, device="cuda").to(torch.bfloat16), 4)
+    idx, wt = ME.route_topk(h, torch.randn(12, 32, device="cuda").to(torch.bfloat16), 4)[:2]
     assert idx[:2].tolist() == [[0, 1, 2, 3]] * 2 and bool((wt[:2] == 0.25).all())
     assert bool(((idx >= 0) & (idx < 12)).all())
 
@@ -294,3 +295,36 @@ def test_embed_and_gated_norm(W, device, dtype):
     close(gh, O.rms_norm(ref, wn.double(), 1e-3), tol)
     go = RN.gated_rms_norm(x.to(device), w.to(device), gate.to(device)[:, 8:8 + W], 1e-3)
     close(go, O.rms_norm(x.double(), w.double(), 1e-3) * torch.sigmoid(gate.double()[:, 8:8 + W]), tol)
+
+
+# ------------------------------------------------------------------------------- fused decode launches
+@gpu
+@pytest.mark.parametrize("M,K,N", [(1, 4096, 96), (2, 4096, 48), (4, 2048, 4096), (3, 72, 24), (1, 8192, 32), (2, 256, 28672)])
+def test_fused_sandwich_launches(M, K, N):
+    from shuffle_exchange_amd.ops import linear as LI
+    g = torch.Generator().manual_seed(K)
+    k, eps, E = 3, 1e-4, 11
+    x, add = torch.randn(M, K, generator=g) * 3, torch.randn(M, K, generator=g)
+    y, wp, wn, w, router = (torch.randn(*s, generator=g).to(torch.bfloat16) for s in ((M * k, K), (K,), (K,), (N, K), (E, K)))
+    slots = torch.randperm(M * k, generator=g).view(M, k).to(torch.int32)
+    xd, yd, wpd, wnd, wd, rd, ad, sd = (t.cuda() for t in (x, y, wp, wn, w, router, add, slots))
+    for use_slots in (False, True):
+        for use_add in (False, True):
+            yy = y.double()[slots.long()].sum(1) if use_slots else y.double()[:M]
+            v = x.double() + O.rms_norm(yy, wp.double(), eps) + (add.double() if use_add else 0)
+            h = O.rms_norm(v, wn.double(), eps)
+            args = (xd, yd if use_slots else yd[:M], wpd, wnd, eps, sd if use_slots else None, ad if use_add else None)
+            out, gx = LI.fused_sandwich_linear(*args, wd)
+            close(gx, v, 1e-5)
+            close(out, h @ w.double().T, 2e-2)
+            gx, gh, routing = ME.fused_sandwich_route(*args, rd, 4)
+            close(gx, v, 1e-5)
+            close(gh, h, 1e-2)
+            val, idx = (gh.double().cpu() @ router.double().T).topk(4, dim=-1)
+            assert torch.equal(routing.expert.cpu().long(), idx)
+            torch.testing.assert_close(routing.weight.double().cpu(), torch.softmax(val, -1), rtol=1e-4, atol=1e-6)
+    assert LI.fused_sandwich_linear(torch.zeros(2, 8192, device="cuda"), torch.zeros(2, 8192, device="cuda").bfloat16(),
+                                    wpd.new_ones(8192), wpd.new_ones(8192), eps, None, None, wpd.new_ones(8, 8192)) is None
+    gate = torch.randn(M, K + 16, generator=g).to(torch.bfloat16)
+    out = LI.fused_gatenorm_linear(yd[:M], wpd, gate.cuda()[:, 16:], eps, wd)
+    close(out, (O.rms_norm(y.double()[:M], wp.double(), eps) * torch.sigmoid(gate.double()[:, 16:])) @ w.double().T, 2e-2)
