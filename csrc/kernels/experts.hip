@@ -2,8 +2,7 @@
 //
 //  * route_logits: h . router^T in fp32. bf16 operands go through the matrix cores (products of two bf16
 //    numbers are exact in fp32 and the accumulation is fp32), anything else through a plain fp32 kernel.
-//    Few tokens: one wave per (expert, 8 tokens) in fp32; one to four: the norm that produces h is the kernel's
-//    prologue (sxe_sandwich.h).
+//    One to four tokens: the norm that produces h is the kernel's prologue (sxe_sandwich.h).
 //  * route_top: the k largest logits of a token (lowest index first among equals) and the softmax over them.
 //  * lists: (token, choice) assignments sorted by expert: row -> token, row -> weight, (token, choice) -> row,
 //    expert offsets and the experts that have rows. A row's place inside its expert depends on the order of
@@ -85,29 +84,41 @@ __global__ __launch_bounds__(256) void route_logits_generic_kernel(const typenam
   if (lane == 0) z[(int64_t)t * E + e] = s;
 }
 
-// few tokens, bf16, K % 8 == 0, 16-byte aligned rows: one wave per (expert, 8 tokens), grid (ceil(E / 4), ceil(T / 8))
-__global__ __launch_bounds__(256) void route_logits_few_kernel(const unsigned short* __restrict x, int64_t ldx,
-                                                               const unsigned short* __restrict w, int T, int E, int K,
-                                                               float* __restrict z) {
-  const int e = blockIdx.x * 4 + (threadIdx.x >> 6), t0 = blockIdx.y * 8, lane = threadIdx.x & 63;
-  if (e >= E) return;
-  float s[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int c = lane * 8; c < K; c += 512) {
-    float a[8];
-    load8<DT::BF16>(w + (int64_t)e * K + c, a);
+// few tokens, bf16, K % 8 == 0, 16-byte aligned rows: 16 tokens x 16 experts per workgroup, 16 waves share K in
+// super-steps of 256 whose loads are all in flight together. grid (ceil(E / 16), ceil(T / 16))
+__global__ __launch_bounds__(1024) void route_logits_few_kernel(const unsigned short* __restrict x, int64_t ldx,
+                                                                const unsigned short* __restrict w, int T, int E, int K,
+                                                                float* __restrict z) {
+  __shared__ float part[16][16][17];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, g = lane >> 4;
+  const int e0 = blockIdx.x * 16, t0 = blockIdx.y * 16;
+  const unsigned short* xr = x + (int64_t)min(t0 + l16, T - 1) * ldx + 8 * g;
+  const unsigned short* wr = w + (int64_t)min(e0 + l16, E - 1) * K + 8 * g;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = wave * 256; k0 < K; k0 += 16 * 256) {
+    u32x4 a[8], b[8];
 #pragma unroll
-    for (int t = 0; t < 8; ++t) {
-      float b[8];
-      load8<DT::BF16>(x + (int64_t)min(t0 + t, T - 1) * ldx + c, b);
-#pragma unroll
-      for (int i = 0; i < 8; ++i) s[t] += a[i] * b[i];
+    for (int u = 0; u < 8; ++u) {
+      const int k = k0 + u * 32;
+      a[u] = b[u] = u32x4{0u, 0u, 0u, 0u};
+      if (k + 8 * g < K) {
+        a[u] = *reinterpret_cast<const u32x4*>(xr + k);
+        b[u] = *reinterpret_cast<const u32x4*>(wr + k);
+      }
     }
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a[u]), __builtin_bit_cast(bf16x8, b[u]), acc, 0, 0, 0);
   }
 #pragma unroll
-  for (int t = 0; t < 8; ++t) {
-    const float v = wave_sum(s[t]);
-    if (lane == 0 && t0 + t < T) z[(int64_t)(t0 + t) * E + e] = v;
+  for (int i = 0; i < 4; ++i) part[wave][4 * g + i][l16] = acc[i];
+  __syncthreads();
+  const int t = threadIdx.x >> 4, e = threadIdx.x & 15;
+  if (threadIdx.x < 256 && t0 + t < T && e0 + e < E) {
+    float s = 0.f;
+#pragma unroll
+    for (int q = 0; q < 16; ++q) s += part[q][t][e];
+    z[(int64_t)(t0 + t) * E + e0 + e] = s;
   }
 }
 
@@ -119,24 +130,32 @@ __global__ __launch_bounds__(512) void route_sandwich_kernel(sw::Args a, const u
   __shared__ float red[8][sw::kMaxM], rinv[sw::kMaxM];
   const int e = blockIdx.x * 8 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   const unsigned short* wr = w + (int64_t)min(e, E - 1) * K;
+  constexpr int U = 8;  // router chunks in flight across the prologue
+  u16x8 wv[U];
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int c = u * 512 + lane * 8;
+    wv[u] = *reinterpret_cast<const u16x8*>(wr + (c < K ? c : 0));
+  }
   sw::build<512, 2, true>(a, M, K, blockIdx.x == 0, act, rinv, red);
   if (blockIdx.x == 0)
     for (int i = threadIdx.x * 8; i < M * K; i += 512 * 8) *reinterpret_cast<u16x8*>(h + i) = *reinterpret_cast<u16x8*>(act + i);
   if (e >= E) return;
   float s[sw::kMaxM] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int c = lane * 8; c < K; c += 512) {
-    float x[8];
-    load8<DT::BF16>(wr + c, x);
+  auto add = [&](const u16x8& wc, int c) {
 #pragma unroll
     for (int m = 0; m < sw::kMaxM; ++m) {
       if (m >= M) break;
       float b[8];
       load8<DT::BF16>(act + m * K + c, b);
 #pragma unroll
-      for (int i = 0; i < 8; ++i) s[m] += x[i] * b[i];
+      for (int i = 0; i < 8; ++i) s[m] += bf16_to_f32(wc[i]) * b[i];
     }
-  }
+  };
+#pragma unroll
+  for (int u = 0; u < U; ++u)
+    if (u * 512 + lane * 8 < K) add(wv[u], u * 512 + lane * 8);
+  for (int c = U * 512 + lane * 8; c < K; c += 512) add(*reinterpret_cast<const u16x8*>(wr + c), c);
 #pragma unroll
   for (int m = 0; m < sw::kMaxM; ++m) {
     const float v = wave_sum(s[m]);
@@ -456,7 +475,7 @@ void route_logits(const at::Tensor& h, const at::Tensor& router, at::Tensor& z) 
   const bool vec = h.scalar_type() == at::kBFloat16 && h.stride(0) % 8 == 0 && aligned(h.data_ptr(), 16) && aligned(router.data_ptr(), 16);
   auto u16 = [](const at::Tensor& t) { return static_cast<const unsigned short*>(t.data_ptr()); };
   if (vec && K % 8 == 0 && T <= 256) {
-    hipLaunchKernelGGL(route_logits_few_kernel, dim3((E + 3) / 4, (T + 7) / 8), dim3(256), 0, cur_stream(), u16(h), h.stride(0),
+    hipLaunchKernelGGL(route_logits_few_kernel, dim3((E + 15) / 16, (T + 15) / 16), dim3(1024), 0, cur_stream(), u16(h), h.stride(0),
                        u16(router), (int)T, (int)E, (int)K, z.data_ptr<float>());
   } else if (vec && K % 16 == 0) {
     hipLaunchKernelGGL(route_logits_kernel<4>, dim3((T + 31) / 32, (E + 31) / 32), dim3(256), 0, cur_stream(), u16(h), h.stride(0),

@@ -6,9 +6,10 @@
 //  * latent_append: norms of the query latent and of c, rotation of the key part, cache write;
 //  * generic form (fp32, any size): one workgroup per (token, head);
 //  * token form (decode, short continuations; bf16): latent_absorb forms W_uk^T q per head,
-//    latent_token runs one workgroup per (token, 32 heads, key split) with 64-key tiles of the cache in LDS,
+//    latent_token runs one workgroup per (token, 32 heads, key split) with 32-key tiles of the cache in LDS,
 //    read by rows for the scores and transposed for the weighted sum of latents -- each cache byte crosses
-//    HBM once for all heads -- and latent_expand merges the splits and applies W_uv;
+//    HBM once for all heads --, latent_merge adds the splits and latent_expand applies W_uv (one token: the merge
+//    is its prologue);
 //  * tile form (prompts; bf16): keys and values of the window are expanded by a library product, then one
 //    workgroup per (256 queries, head) in the flash manner (8 waves of 32 queries, 64-key tiles loaded straight
 //    to a double-buffered LDS ring). The rotated key part is read from the gathered cache rows, queries are
@@ -135,7 +136,7 @@ __device__ __forceinline__ int64_t cache_at(const Args& a, int s, int j) {
   return (blk * a.bs + (j - b * a.bs)) * a.row;
 }
 
-// grid (n, H); uk [H, dim, rank], uv [H, rank, vdim]
+// grid (n, H); uk [H, rank, dim], uv [H, vdim, rank]
 template <DT T>
 __global__ __launch_bounds__(kThreads) void latent_generic_kernel(Args a, const typename dt_traits<T>::storage* __restrict uk,
                                                                   const typename dt_traits<T>::storage* __restrict uv,
@@ -150,7 +151,7 @@ __global__ __launch_bounds__(kThreads) void latent_generic_kernel(Args a, const 
   const S* q = static_cast<const S*>(a.q) + ((int64_t)t * a.H + h) * (a.dim + a.rot_dim);
   for (int r = threadIdx.x; r < a.rank; r += kThreads) {
     float x = 0.f;
-    for (int d = 0; d < a.dim; ++d) x += to_f32<T>(q[d]) * to_f32<T>(uk[((int64_t)h * a.dim + d) * a.rank + r]);
+    for (int d = 0; d < a.dim; ++d) x += to_f32<T>(q[d]) * to_f32<T>(uk[((int64_t)h * a.rank + r) * a.dim + d]);
     qa[r] = x * a.scale;
     ol[r] = 0.f;
   }
@@ -197,255 +198,222 @@ __global__ __launch_bounds__(kThreads) void latent_generic_kernel(Args a, const 
   const float inv = L > 0.f ? 1.f / L : 0.f;
   for (int v = threadIdx.x; v < a.vdim; v += kThreads) {
     float o = 0.f;
-    for (int r = 0; r < a.rank; ++r) o += ol[r] * to_f32<T>(uv[((int64_t)h * a.rank + r) * a.vdim + v]);
+    for (int r = 0; r < a.rank; ++r) o += ol[r] * to_f32<T>(uv[((int64_t)h * a.vdim + v) * a.rank + r]);
     out[((int64_t)t * a.H + h) * a.vdim + v] = from_f32<T>(o * inv);
   }
 }
 
 // ----------------------------------------------------------------------- per-head products (token form)
-// y[t, n] = sum_k x[t, k] W[k, n] for one head, TT tokens, N columns in chunks of 8 * LN: thread (k group,
-// 8 columns), k groups summed through shuffles and LDS. x fp32 in LDS [TT][K]. VEC: 16-byte weight loads.
-template <int TT, int LN, bool VEC>
-__device__ __forceinline__ void head_product(const float* x, const unsigned short* __restrict W, int K, int N, int n0, float* part,
-                                             float (&acc)[TT][8]) {
-  constexpr int KG = kThreads / LN;
-  const int ln = threadIdx.x % LN, kg = threadIdx.x / LN, n = n0 + ln * 8;
-#pragma unroll
-  for (int t = 0; t < TT; ++t)
-#pragma unroll
-    for (int i = 0; i < 8; ++i) acc[t][i] = 0.f;
-  if (n < N) {
-#pragma unroll 4
-    for (int k = kg; k < K; k += KG) {
-      float w[8];
-      if constexpr (VEC) {
-        load8<DT::BF16>(W + (int64_t)k * N + n, w);
-      } else {
-#pragma unroll
-        for (int i = 0; i < 8; ++i) w[i] = n + i < N ? bf16_to_f32(W[(int64_t)k * N + n + i]) : 0.f;
-      }
-#pragma unroll
-      for (int t = 0; t < TT; ++t) {
-        const float xv = x[t * K + k];
-#pragma unroll
-        for (int i = 0; i < 8; ++i) acc[t][i] += xv * w[i];
-      }
-    }
-  }
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-#pragma unroll
-  for (int t = 0; t < TT; ++t)
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-#pragma unroll
-      for (int o = LN; o < 64; o <<= 1) acc[t][i] += __shfl_xor(acc[t][i], o, 64);
-      if (lane < LN) part[((wave * TT + t) * LN + lane) * 8 + i] = acc[t][i];
-    }
-  __syncthreads();
-}
-
-// grid (H, ceil(rank / (8 LN)), ceil(n / TT)) -> qa [n, H, row] bf16: W_uk^T q | rotated q, zero-padded
-template <int TT, int LN, bool VEC>
-__global__ __launch_bounds__(kThreads) void latent_absorb_kernel(Args a, int n, const unsigned short* __restrict uk,
-                                                                 unsigned short* __restrict qa) {
-  extern __shared__ float sm[];
-  float* x = sm;                    // [TT][dim]
-  float* part = sm + TT * a.dim;    // [4][TT][LN * 8]
-  const int h = blockIdx.x, n0 = blockIdx.y * LN * 8, i0 = blockIdx.z * TT, half = a.rot_dim / 2;
-  const unsigned short* q = static_cast<const unsigned short*>(a.q);
-  for (int i = threadIdx.x; i < TT * a.dim; i += kThreads) {
-    const int t = i / a.dim, d = i - t * a.dim;
-    x[i] = i0 + t < n ? bf16_to_f32(q[((int64_t)a.rows[2 * (i0 + t) + 1] * a.H + h) * (a.dim + a.rot_dim) + d]) : 0.f;
-  }
-  __syncthreads();
-  float acc[TT][8];
-  head_product<TT, LN, VEC>(x, uk + (int64_t)h * a.dim * a.rank, a.dim, a.rank, n0, part, acc);
-  for (int i = threadIdx.x; i < TT * LN * 8; i += kThreads) {
-    const int t = i / (LN * 8), c = i - t * (LN * 8);
-    if (i0 + t < n && n0 + c < a.R) {
-      float v = 0.f;
-      if (n0 + c < a.rank)
-#pragma unroll
-        for (int w = 0; w < 4; ++w) v += part[(w * TT + t) * LN * 8 + c];
-      qa[((int64_t)(i0 + t) * a.H + h) * a.row + n0 + c] = f32_to_bf16(v);
-    }
-  }
-  if (blockIdx.y == 0) {  // the rotated part and both parts' padding
-    const int rp = a.row - a.R, pad0 = gridDim.y * LN * 8;
-    for (int i = threadIdx.x; i < TT * rp; i += kThreads) {
-      const int t = i / rp, d = i - t * rp;
-      if (i0 + t >= n) continue;
-      const int64_t row = a.rows[2 * (i0 + t) + 1];
-      float v = 0.f;
-      if (d < a.rot_dim) {
-        const unsigned short* qr = q + (row * a.H + h) * (a.dim + a.rot_dim) + a.dim;
-        const int j = d < half ? d : d - half;
-        const float u = bf16_to_f32(qr[j]), w = bf16_to_f32(qr[half + j]);
-        const float c = a.rot[(row * half + j) * 2], s = a.rot[(row * half + j) * 2 + 1];
-        v = d < half ? u * c - w * s : w * c + u * s;
-      }
-      qa[((int64_t)(i0 + t) * a.H + h) * a.row + a.R + d] = f32_to_bf16(v);
-    }
-    for (int i = threadIdx.x; i < TT * (a.R - min(pad0, a.R)); i += kThreads) {
-      const int w = a.R - pad0, t = i / w, d = i - t * w;
-      if (i0 + t < n) qa[((int64_t)(i0 + t) * a.H + h) * a.row + pad0 + d] = 0;
-    }
-  }
-}
-
-// grid (H, ceil(vdim / (8 LN)), ceil(n / TT)): out[row, h, :] = W_uv (merged splits)
-template <int TT, int LN, bool VEC>
-__global__ __launch_bounds__(kThreads) void latent_expand_kernel(Args a, int n, int splits, const float* __restrict po,
-                                                                 const float* __restrict pml, const unsigned short* __restrict uv,
-                                                                 unsigned short* __restrict out) {
-  extern __shared__ float sm[];
-  float* x = sm;                    // [TT][rank]
-  float* part = sm + TT * a.rank;   // [4][TT][LN * 8]
-  float* wts = part + 4 * TT * LN * 8;  // [TT][splits]
-  const int h = blockIdx.x, n0 = blockIdx.y * LN * 8, i0 = blockIdx.z * TT;
-  const int64_t sstride = (int64_t)n * a.H;
-  // weights of the splits: 2^(M_s - M) / sum, one wave per token
-  const int lane = threadIdx.x & 63;
-  for (int t = threadIdx.x >> 6; t < TT; t += 4) {
-    if (i0 + t >= n) continue;
-    const float* ml = pml + ((int64_t)(i0 + t) * a.H + h) * 2;
-    float M = -INFINITY, L = 0.f;
-    for (int s = lane; s < splits; s += 64) M = fmaxf(M, ml[s * sstride * 2]);
-    M = wave_max(M);
-    for (int s = lane; s < splits; s += 64) {
-      const float m = ml[s * sstride * 2], f = m == -INFINITY ? 0.f : exp2f(m - M);
-      wts[t * splits + s] = f;
-      if (f > 0.f) L += f * ml[s * sstride * 2 + 1];
-    }
-    L = wave_sum(L);
-    const float inv = L > 0.f ? 1.f / L : 0.f;
-    for (int s = lane; s < splits; s += 64) wts[t * splits + s] *= inv;  // the lane's own entries
-  }
-  __syncthreads();
-  for (int i = threadIdx.x; i < TT * a.rank; i += kThreads) {
-    const int t = i / a.rank, r = i - t * a.rank;
-    float v = 0.f;
-    if (i0 + t < n) {
-      const float* p = po + ((int64_t)(i0 + t) * a.H + h) * a.R + r;
-#pragma unroll 8
-      for (int s = 0; s < splits; ++s) {
-        const float f = wts[t * splits + s], o = p[s * sstride * a.R];
-        v += f > 0.f ? f * o : 0.f;  // a split without keys has not written its part
-      }
-    }
-    x[i] = v;
-  }
-  __syncthreads();
-  float acc[TT][8];
-  head_product<TT, LN, VEC>(x, uv + (int64_t)h * a.rank * a.vdim, a.rank, a.vdim, n0, part, acc);
-  for (int i = threadIdx.x; i < TT * LN * 8; i += kThreads) {
-    const int t = i / (LN * 8), c = i - t * (LN * 8);
-    if (i0 + t < n && n0 + c < a.vdim) {
-      float v = 0.f;
-#pragma unroll
-      for (int w = 0; w < 4; ++w) v += part[(w * TT + t) * LN * 8 + c];
-      out[((int64_t)a.rows[2 * (i0 + t) + 1] * a.H + h) * a.vdim + n0 + c] = f32_to_bf16(v);
-    }
-  }
-}
-
-// ------------------------------------------------------------------------------------------ token form
-constexpr int kKeys = 64;
-constexpr int kSRow = kKeys + 4;  // fp32 score row of a head
-
 __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
 }
 
-// PN: 256-byte panels (128 columns) of the latent part, R <= 128 PN. grid (n, ceil(H / 32), splits)
+// y = x W^T for 16 rows x and 16 rows of W (both K contiguous, K % 8 == 0): the workgroup's 4 waves split K;
+// thread i gets element (row i / 16, column i % 16). xrow / wrow: the lane's row (l16), always readable.
+__device__ __forceinline__ float head_product(const unsigned short* xrow, const unsigned short* wrow, int K, float (*part)[16][17]) {
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l16 = lane & 15, g = lane >> 4;
+  constexpr int U = 4;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = w * 32; k0 < K; k0 += U * 128) {
+    u32x4 a[U], b[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = k0 + u * 128 + 8 * g;
+      a[u] = b[u] = u32x4{0u, 0u, 0u, 0u};
+      if (k < K) {
+        a[u] = *reinterpret_cast<const u32x4*>(xrow + k);
+        b[u] = *reinterpret_cast<const u32x4*>(wrow + k);
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) acc = mfma16(__builtin_bit_cast(bf16x8, a[u]), __builtin_bit_cast(bf16x8, b[u]), acc);
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) part[w][4 * g + i][l16] = acc[i];
+  __syncthreads();
+  const int r = threadIdx.x >> 4, c = threadIdx.x & 15;
+  return part[0][r][c] + part[1][r][c] + part[2][r][c] + part[3][r][c];
+}
+
+// grid (R / 16 + 1, H, ceil(n / 16)) -> qa [n, H, row] bf16: W_uk^T q | rotated q, zero-padded; uk [H, rank, dim]
+__global__ __launch_bounds__(kThreads) void latent_absorb_kernel(Args a, int n, const unsigned short* __restrict uk,
+                                                                 unsigned short* __restrict qa) {
+  __shared__ float part[4][16][17];
+  const int c0 = blockIdx.x * 16, h = blockIdx.y, i0 = blockIdx.z * 16, half = a.rot_dim / 2, l16 = threadIdx.x & 15;
+  const unsigned short* q = static_cast<const unsigned short*>(a.q);
+  if (c0 < a.R) {
+    const int64_t row = a.rows[2 * min(i0 + l16, n - 1) + 1];
+    const unsigned short* wr = uk + ((int64_t)h * a.rank + min(c0 + l16, a.rank - 1)) * a.dim;
+    const float v = head_product(q + (row * a.H + h) * (a.dim + a.rot_dim), wr, a.dim, part);
+    const int i = i0 + (threadIdx.x >> 4), c = c0 + l16;
+    if (i < n) qa[((int64_t)i * a.H + h) * a.row + c] = c < a.rank ? f32_to_bf16(v) : 0;
+    return;
+  }
+  const int rp = a.row - a.R;
+  for (int x = threadIdx.x; x < 16 * rp; x += kThreads) {
+    const int i = i0 + x / rp, d = x % rp;
+    if (i >= n) continue;
+    const int64_t row = a.rows[2 * i + 1];
+    float v = 0.f;
+    if (d < a.rot_dim) {
+      const unsigned short* qr = q + (row * a.H + h) * (a.dim + a.rot_dim) + a.dim;
+      const int j = d < half ? d : d - half;
+      const float u = bf16_to_f32(qr[j]), y = bf16_to_f32(qr[half + j]);
+      const float co = a.rot[(row * half + j) * 2], si = a.rot[(row * half + j) * 2 + 1];
+      v = d < half ? u * co - y * si : y * co + u * si;
+    }
+    qa[((int64_t)i * a.H + h) * a.row + a.R + d] = f32_to_bf16(v);
+  }
+}
+
+// weights of a (token, head)'s splits, 2^(M_s - M) / sum, by one wave; ml: its (max, sum) of split 0
+__device__ __forceinline__ void split_weights(const float* ml, int64_t stride, int splits, float* wts) {
+  const int lane = threadIdx.x & 63;
+  float M = -INFINITY, L = 0.f;
+  for (int s = lane; s < splits; s += 64) M = fmaxf(M, ml[s * stride]);
+  M = wave_max(M);
+  for (int s = lane; s < splits; s += 64) {
+    const float m = ml[s * stride], f = m == -INFINITY ? 0.f : exp2f(m - M);
+    wts[s] = f;
+    if (f > 0.f) L += f * ml[s * stride + 1];
+  }
+  L = wave_sum(L);
+  const float inv = L > 0.f ? 1.f / L : 0.f;
+  for (int s = lane; s < splits; s += 64) wts[s] *= inv;  // the lane's own entries
+}
+
+// 4 merged components: a split without keys has not written its part
+__device__ __forceinline__ f32x4 merged4(const float* p, int64_t stride, int splits, const float* wts) {
+  f32x4 v = {0.f, 0.f, 0.f, 0.f};
+  constexpr int U = 8;
+  for (int s0 = 0; s0 < splits; s0 += U) {
+    f32x4 t[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) t[u] = *reinterpret_cast<const f32x4*>(p + min(s0 + u, splits - 1) * stride);
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const float f = s0 + u < splits ? wts[min(s0 + u, splits - 1)] : 0.f;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] += f > 0.f ? f * t[u][e] : 0.f;
+    }
+  }
+  return v;
+}
+
+constexpr int kMaxSplits = 256;
+
+// grid (H, n): ol [n, H, R] bf16
+__global__ __launch_bounds__(128) void latent_merge_kernel(Args a, int n, int splits, const float* __restrict po,
+                                                           const float* __restrict pml, unsigned short* __restrict ol) {
+  __shared__ float wts[kMaxSplits];
+  const int64_t th = (int64_t)blockIdx.y * a.H + blockIdx.x, ss = (int64_t)n * a.H;
+  if (threadIdx.x < 64) split_weights(pml + th * 2, ss * 2, splits, wts);
+  __syncthreads();
+  for (int c = threadIdx.x * 4; c < a.R; c += 512) {
+    const f32x4 v = merged4(po + th * a.R + c, ss * a.R, splits, wts);
+    *reinterpret_cast<u16x4*>(ol + th * a.R + c) = u16x4{f32_to_bf16(v[0]), f32_to_bf16(v[1]), f32_to_bf16(v[2]), f32_to_bf16(v[3])};
+  }
+}
+
+// grid (ceil(vdim / 16), H, ceil(n / 16)): out[row, h, :] = W_uv ol; uv [H, vdim, rank]. MERGE: n == 1, the merged
+// latent is formed here.
+template <bool MERGE>
+__global__ __launch_bounds__(kThreads) void latent_expand_kernel(Args a, int n, int splits, const float* __restrict po,
+                                                                 const float* __restrict pml, const unsigned short* __restrict ol,
+                                                                 const unsigned short* __restrict uv, unsigned short* __restrict out) {
+  __shared__ float part[4][16][17], wts[MERGE ? kMaxSplits : 1];
+  __shared__ __attribute__((aligned(16))) unsigned short x[MERGE ? 512 : 8];
+  const int c0 = blockIdx.x * 16, h = blockIdx.y, i0 = blockIdx.z * 16, l16 = threadIdx.x & 15;
+  const unsigned short* xr = x;
+  if constexpr (MERGE) {
+    if (threadIdx.x < 64) split_weights(pml + h * 2, (int64_t)a.H * 2, splits, wts);
+    __syncthreads();
+    if (threadIdx.x * 4 < a.R) {
+      const int c = threadIdx.x * 4;
+      const f32x4 v = merged4(po + (int64_t)h * a.R + c, (int64_t)a.H * a.R, splits, wts);
+      *reinterpret_cast<u16x4*>(x + c) = u16x4{f32_to_bf16(v[0]), f32_to_bf16(v[1]), f32_to_bf16(v[2]), f32_to_bf16(v[3])};
+    }
+    __syncthreads();
+  } else {
+    xr = ol + ((int64_t)min(i0 + l16, n - 1) * a.H + h) * a.R;
+  }
+  const float v = head_product(xr, uv + ((int64_t)h * a.vdim + min(c0 + l16, a.vdim - 1)) * a.rank, a.rank, part);
+  const int i = i0 + (threadIdx.x >> 4), c = c0 + l16;
+  if (i < n && c < a.vdim) out[((int64_t)a.rows[2 * i + 1] * a.H + h) * a.vdim + c] = f32_to_bf16(v);
+}
+
+// ------------------------------------------------------------------------------------------ token form
+constexpr int kKeys = 64;       // keys of a tile of the tile form
+constexpr int kTok = 32;        // ... of the token form
+constexpr int kSRow = kTok + 4;  // fp32 score row of a head
+
+// PN 256-byte panels hold the latent (R = 128 PN), one more the rotated part (64 columns). grid (n, ceil(H / 32),
+// splits). Waves: scores of (16 keys, 16 heads) each; then PN 32-column tiles of the latent sum each, all heads.
 template <int PN>
-__global__ __launch_bounds__(kThreads, 1) void latent_token_kernel(Args a, int n, const unsigned short* __restrict qa,
+__global__ __launch_bounds__(kThreads, 2) void latent_token_kernel(Args a, int n, const unsigned short* __restrict qa,
                                                                    float* __restrict po, float* __restrict pml) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  constexpr int PANEL = kKeys * ROWB, NS = 4 * PN + 2, NC = 4 * PN + 2;
-  char* lrot = smem + PN * PANEL;
+  constexpr int PANEL = kTok * ROWB, NS = 4 * PN + 2, NC = 2 * PN + 1, ROW = 128 * PN + 64;
   float* ls = reinterpret_cast<float*>(smem + (PN + 1) * PANEL);  // [32 heads][kSRow]
   const int i = blockIdx.x, g = blockIdx.y, sp = blockIdx.z;
   const int s = a.rows[2 * i], t = a.rows[2 * i + 1];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l16 = lane & 15, q16 = lane >> 4, l32 = lane & 31, hh = lane >> 5;
-  const int nr = a.R / 32, nrot = (a.row - a.R) / 32;  // 32-column steps
   int lo, hi;
   key_range(a, s, t, lo, hi);
   {  // this split's keys, whole tiles
-    const int tiles = (hi - lo + kKeys - 1) / kKeys, per = (tiles + gridDim.z - 1) / gridDim.z;
-    lo = min(hi, lo + sp * per * kKeys);
-    hi = min(hi, lo + per * kKeys);
+    const int tiles = (hi - lo + kTok - 1) / kTok, per = (tiles + gridDim.z - 1) / gridDim.z;
+    lo = min(hi, lo + sp * per * kTok);
+    hi = min(hi, lo + per * kTok);
   }
-  // queries: B fragments of 16 heads each, head 32 g + 16 b + l16
-  bf16x8 qf[NS][2];
+  const unsigned short* cache = static_cast<const unsigned short*>(a.cache);
+  const int srow = threadIdx.x >> 3, sch = threadIdx.x & 7;
+  auto at = [&](int j0) { return cache_at(a, s, max(min(j0 + srow, hi - 1), 0)); };  // past the end: the last row (masked)
+  u32x4 st[NC];
+  auto load = [&](int64_t off) {
 #pragma unroll
-  for (int b = 0; b < 2; ++b) {
-    const int h = 32 * g + 16 * b + l16;
-    const unsigned short* qr = qa + ((int64_t)i * a.H + min(h, a.H - 1)) * a.row;
+    for (int c = 0; c < NC; ++c) st[c] = *reinterpret_cast<const u32x4*>(cache + off + c * 64 + sch * 8);
+  };
+  int64_t next = 0;
+  bf16x8 qf[NS];  // B fragments of 16 heads
+  if (lo < hi) {
+    const int64_t first = at(lo);
+    next = at(lo + kTok);
+    const int h = 32 * g + 16 * (w >> 1) + l16;
+    const unsigned short* qr = qa + ((int64_t)i * a.H + min(h, a.H - 1)) * ROW + q16 * 8;
+    load(first);
 #pragma unroll
-    for (int k = 0; k < NS; ++k) {
-      const int st = k < 4 * PN ? k : nr + k - 4 * PN;
-      const bool ok = h < a.H && (k < 4 * PN ? k < nr : k - 4 * PN < nrot);
-      u32x4 z = {0u, 0u, 0u, 0u};
-      if (ok) z = *reinterpret_cast<const u32x4*>(qr + st * 32 + q16 * 8);
-      qf[k][b] = __builtin_bit_cast(bf16x8, z);
-    }
+    for (int k = 0; k < NS; ++k) qf[k] = *reinterpret_cast<const bf16x8*>(qr + k * 32);
   }
-  f32x16 acc[4];
+  f32x16 acc[PN];
 #pragma unroll
-  for (int j = 0; j < 4; ++j) acc[j] = zero16();
+  for (int j = 0; j < PN; ++j) acc[j] = zero16();
   float M = -INFINITY, L = 0.f;
   const float sc2 = a.scale * LOG2E;
-  const unsigned short* cache = static_cast<const unsigned short*>(a.cache);
-  const int srow = threadIdx.x >> 2, sch = threadIdx.x & 3;
-  u32x4 st[NC];
-  auto load = [&](int j0) {
-    const int j = min(j0 + srow, hi - 1);  // a row past the end repeats the last one (its score is masked)
-    const unsigned short* src = cache + cache_at(a, s, j) + sch * 8;
-#pragma unroll
-    for (int c = 0; c < NC; ++c) {
-      if (c < 4 * PN ? c < nr : c - 4 * PN < nrot)
-        st[c] = *reinterpret_cast<const u32x4*>(src + (c < 4 * PN ? c : nr + c - 4 * PN) * 32);
-    }
-  };
-  if (lo < hi) load(lo);
-  for (int j0 = lo; j0 < hi; j0 += kKeys) {
+  for (int j0 = lo; j0 < hi; j0 += kTok) {
     __syncthreads();  // the previous tile is read
 #pragma unroll
-    for (int c = 0; c < NC; ++c) {
-      if (c < 4 * PN) {
-        if (c < nr) *reinterpret_cast<u32x4*>(smem + (c >> 2) * PANEL + soff(srow, (c & 3) * 4 + sch)) = st[c];
-      } else if (c - 4 * PN < nrot) {
-        *reinterpret_cast<u32x4*>(lrot + soff(srow, (c - 4 * PN) * 4 + sch)) = st[c];
-      }
-    }
+    for (int c = 0; c < NC; ++c) *reinterpret_cast<u32x4*>(smem + (c >> 1) * PANEL + soff(srow, (c & 1) * 8 + sch)) = st[c];
     __syncthreads();
-    if (j0 + kKeys < hi) load(j0 + kKeys);
-    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;  // keys 16 w + 4 q16 + i, heads l16 and 16 + l16
-#pragma unroll
-    for (int k = 0; k < NS; ++k) {
-      if (k < 4 * PN ? k < nr : k - 4 * PN < nrot) {
-        const bf16x8 kf = k < 4 * PN ? lds_row16(smem + (k >> 2) * PANEL, 16 * w + l16, (k & 3) * 4 + q16)
-                                     : lds_row16(lrot, 16 * w + l16, (k - 4 * PN) * 4 + q16);
-        s0 = mfma16(kf, qf[k][0], s0);
-        s1 = mfma16(kf, qf[k][1], s1);
-      }
+    if (j0 + kTok < hi) {
+      load(next);
+      next = at(j0 + 2 * kTok);
     }
-    const int kj = 16 * w + 4 * q16;
+    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;  // keys 16 (w & 1) + 4 q16 + e, head 16 (w >> 1) + l16
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const bool ok = j0 + kj + e < hi;
-      s0[e] = ok ? s0[e] * sc2 : -INFINITY;
-      s1[e] = ok ? s1[e] * sc2 : -INFINITY;
+    for (int k = 0; k < NS; k += 2) {
+      s0 = mfma16(lds_row16(smem + (k >> 2) * PANEL, 16 * (w & 1) + l16, (k & 3) * 4 + q16), qf[k], s0);
+      s1 = mfma16(lds_row16(smem + (k >> 2) * PANEL, 16 * (w & 1) + l16, ((k + 1) & 3) * 4 + q16), qf[k + 1], s1);
     }
-    *reinterpret_cast<f32x4*>(ls + l16 * kSRow + kj) = s0;
-    *reinterpret_cast<f32x4*>(ls + (16 + l16) * kSRow + kj) = s1;
+    const int kj = 16 * (w & 1) + 4 * q16;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) s0[e] = j0 + kj + e < hi ? (s0[e] + s1[e]) * sc2 : -INFINITY;
+    *reinterpret_cast<f32x4*>(ls + (16 * (w >> 1) + l16) * kSRow + kj) = s0;
     __syncthreads();
-    // every wave forms all weights of the tile: lane = head l32, keys 16 x + 4 hh + (0..3, 8..11)
-    f32x4 p[8];
+    // every wave forms all weights of the tile: lane = head l32, keys 8 x + 4 hh + e
+    f32x4 p[4];
     float m = -INFINITY;
 #pragma unroll
-    for (int x = 0; x < 8; ++x) {
+    for (int x = 0; x < 4; ++x) {
       p[x] = *reinterpret_cast<const f32x4*>(ls + l32 * kSRow + 8 * x + 4 * hh);
       m = fmaxf(m, fmaxf(fmaxf(p[x][0], p[x][1]), fmaxf(p[x][2], p[x][3])));
     }
@@ -453,7 +421,7 @@ __global__ __launch_bounds__(kThreads, 1) void latent_token_kernel(Args a, int n
     const float Mn = fmaxf(M, m), f = fast_exp2(M - Mn);  // a tile has a visible key: Mn is finite
     float l = 0.f;
 #pragma unroll
-    for (int x = 0; x < 8; ++x)
+    for (int x = 0; x < 4; ++x)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         p[x][e] = fast_exp2(p[x][e] - Mn);
@@ -461,22 +429,22 @@ __global__ __launch_bounds__(kThreads, 1) void latent_token_kernel(Args a, int n
       }
     L = L * f + l + xor32(l);
     M = Mn;
-    if (w < PN) {
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
+    for (int j = 0; j < PN; ++j)
 #pragma unroll
-        for (int e = 0; e < 16; ++e) acc[j][e] *= f;
+      for (int e = 0; e < 16; ++e) acc[j][e] *= f;
 #pragma unroll
-      for (int x = 0; x < 4; ++x) {
-        bf16x8 b;
+    for (int x = 0; x < 2; ++x) {
+      bf16x8 b;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          b[e] = (__bf16)p[2 * x][e];
-          b[4 + e] = (__bf16)p[2 * x + 1][e];
-        }
+      for (int e = 0; e < 4; ++e) {
+        b[e] = (__bf16)p[2 * x][e];
+        b[4 + e] = (__bf16)p[2 * x + 1][e];
+      }
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-          if (w * 128 + j * 32 < a.R) acc[j] = mfma(lds_trA(smem + w * PANEL, 16 * x, j, lane), b, acc[j]);
+      for (int j = 0; j < PN; ++j) {
+        const int ct = w * PN + j;
+        acc[j] = mfma(lds_trA(smem + (ct >> 2) * PANEL, 16 * x, ct & 3, lane), b, acc[j]);
       }
     }
   }
@@ -487,16 +455,13 @@ __global__ __launch_bounds__(kThreads, 1) void latent_token_kernel(Args a, int n
       pml[th * 2] = M;
       pml[th * 2 + 1] = L;
     }
-    if (w < PN && lo < hi) {
-      float* o = po + th * a.R + w * 128;
+    if (lo < hi) {
+      float* o = po + th * a.R + w * PN * 32 + 4 * hh;
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (w * 128 + j * 32 < a.R) {
+      for (int j = 0; j < PN; ++j)
 #pragma unroll
-          for (int e = 0; e < 4; ++e)
-            *reinterpret_cast<f32x4*>(o + j * 32 + 8 * e + 4 * hh) =
-                f32x4{acc[j][4 * e], acc[j][4 * e + 1], acc[j][4 * e + 2], acc[j][4 * e + 3]};
-        }
+        for (int e = 0; e < 4; ++e)
+          *reinterpret_cast<f32x4*>(o + j * 32 + 8 * e) = f32x4{acc[j][4 * e], acc[j][4 * e + 1], acc[j][4 * e + 2], acc[j][4 * e + 3]};
     }
   }
 }
@@ -761,16 +726,16 @@ at::Tensor latent_append(const at::Tensor& proj, const at::Tensor& qw, const at:
   return cq;
 }
 
-// q [T, H (dim + rot)], uk [H, dim, rank], uv [H, rank, vdim], out [T, H vdim]; rows of `rows` are written
+// q [T, H (dim + rot)], uk [H, rank, dim], uv [H, vdim, rank], out [T, H vdim]; rows of `rows` are written
 void latent_attention_generic(const at::Tensor& q, const at::Tensor& uk, const at::Tensor& uv, const at::Tensor& cache,
                               const at::Tensor& rot, const at::Tensor& rows, const at::Tensor& table, const at::Tensor& q_start,
                               const at::Tensor& q_len, const at::Tensor& kv_len, at::Tensor out, int64_t rot_dim, int64_t R,
                               double scale, int64_t window) {
   SXE_CHECK_CUDA(q);
   lt::check_batch(rows, table, q_start, q_len, kv_len, cache);
-  const int64_t n = rows.size(0), H = uk.size(0), dim = uk.size(1), rank = uk.size(2), vdim = uv.size(2);
+  const int64_t n = rows.size(0), H = uk.size(0), rank = uk.size(1), dim = uk.size(2), vdim = uv.size(1);
   SXE_CHECK(q.is_contiguous() && q.dim() == 2 && q.size(1) == H * (dim + rot_dim) && uk.is_contiguous() && uv.is_contiguous() &&
-                uv.size(0) == H && uv.size(1) == rank && out.is_contiguous() && out.size(0) == q.size(0) && out.size(1) == H * vdim &&
+                uv.size(0) == H && uv.size(2) == rank && out.is_contiguous() && out.size(0) == q.size(0) && out.size(1) == H * vdim &&
                 cache.size(3) >= R + rot_dim && R >= rank,
             "latent_attention: shapes");
   SXE_CHECK(rot.is_contiguous() && rot.scalar_type() == at::kFloat && rot.numel() == q.size(0) * rot_dim, "latent_attention: rotation");
@@ -792,57 +757,57 @@ void latent_attention_generic(const at::Tensor& q, const at::Tensor& uk, const a
   SXE_LAUNCH_CHECK();
 }
 
-// The token form's three launches; out [T, H vdim], bf16, R <= 512
+// The token form's launches; out [T, H vdim], bf16; cache rows of R = 128 i <= 512 latent and 64 rotated columns
 void latent_attention_token(const at::Tensor& q, const at::Tensor& uk, const at::Tensor& uv, const at::Tensor& cache,
                             const at::Tensor& rot, const at::Tensor& rows, const at::Tensor& table, const at::Tensor& q_start,
                             const at::Tensor& q_len, const at::Tensor& kv_len, at::Tensor out, int64_t splits, int64_t rot_dim,
                             int64_t R, double scale, int64_t window) {
   SXE_CHECK_CUDA(q);
   lt::check_batch(rows, table, q_start, q_len, kv_len, cache);
-  const int64_t n = rows.size(0), H = uk.size(0), dim = uk.size(1), rank = uk.size(2), vdim = uv.size(2), row = cache.size(3);
+  const int64_t n = rows.size(0), H = uk.size(0), rank = uk.size(1), dim = uk.size(2), vdim = uv.size(1), row = cache.size(3);
   SXE_CHECK(q.is_contiguous() && q.dim() == 2 && q.size(1) == H * (dim + rot_dim) && uk.is_contiguous() && uv.is_contiguous() &&
-                uv.size(0) == H && uv.size(1) == rank && out.is_contiguous() && out.size(0) == q.size(0) && out.size(1) == H * vdim &&
-                R >= rank && R % 32 == 0 && R <= 512 && row % 32 == 0 && row - R >= rot_dim && row - R <= 64 && scale > 0,
+                uv.size(0) == H && uv.size(2) == rank && out.is_contiguous() && out.size(0) == q.size(0) && out.size(1) == H * vdim &&
+                R >= rank && R % 128 == 0 && R <= 512 && row == R + 64 && rot_dim <= 64 && scale > 0 && dim % 8 == 0 && rank % 8 == 0 &&
+                rot_dim % 2 == 0 && (dim + rot_dim) % 8 == 0,
             "latent_attention: shapes");
   SXE_CHECK(rot.is_contiguous() && rot.scalar_type() == at::kFloat && rot.numel() == q.size(0) * rot_dim, "latent_attention: rotation");
   for (const auto* t : {&q, &uk, &uv, &cache, (const at::Tensor*)&out})
     SXE_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16, "latent_attention: token form takes bf16");
-  SXE_CHECK(lt::aligned(cache.data_ptr(), 16) && splits >= 1 && splits <= 256 && H <= 65535, "latent_attention: splits");
+  SXE_CHECK(lt::aligned(cache.data_ptr(), 16) && splits >= 1 && splits <= lt::kMaxSplits && H <= 65535 && n <= 65535, "latent_attention: splits");
   if (n == 0) return;
   c10::DeviceGuard g(q.device());
   lt::Args a{q.data_ptr(), rot.data_ptr<float>(), rows.data_ptr<int>(), table.data_ptr<int>(), q_start.data_ptr<int>(),
              q_len.data_ptr<int>(), kv_len.data_ptr<int>(), cache.data_ptr(), cache.size(0), (int)table.size(1), (int)cache.size(2),
              (int)H, (int)dim, (int)rot_dim, (int)rank, (int)R, (int)row, (int)vdim, (int)window, (float)scale};
-  auto qa = at::empty({n, H, row}, q.options());
-  auto po = at::empty({splits, n, H, R}, q.options().dtype(at::kFloat)), pml = at::empty({splits, n, H, 2}, po.options());
+  SXE_CHECK((n + 15) / 16 <= 65535 && lt::aligned(q.data_ptr(), 16) && lt::aligned(uk.data_ptr(), 16) && lt::aligned(uv.data_ptr(), 16),
+            "latent_attention: 16-byte aligned operands");
+  auto f32 = q.options().dtype(at::kFloat);
+  auto qa = at::empty({n, H, row}, q.options()), po = at::empty({splits, n, H, R}, f32), pml = at::empty({splits, n, H, 2}, f32);
   auto u16 = [](const at::Tensor& t) { return static_cast<unsigned short*>(t.data_ptr()); };
-  auto heads = [&](auto kern, int64_t K, int64_t N, int TT, int LN, auto... more) {
-    const size_t lds = sizeof(float) * (TT * (K + splits) + 4 * TT * LN * 8);
-    SXE_CHECK(lds <= 150 * 1024 && (n + TT - 1) / TT <= 65535, "latent_attention: sizes");
-    SXE_HIP_CHECK(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-    hipLaunchKernelGGL(kern, dim3(H, (N + LN * 8 - 1) / (LN * 8), (n + TT - 1) / TT), dim3(lt::kThreads), lds, cur_stream(), a, (int)n,
-                       more...);
-  };
-  const bool vk = rank % 8 == 0 && lt::aligned(uk.data_ptr(), 16), vv = vdim % 8 == 0 && lt::aligned(uv.data_ptr(), 16);
-  if (!vk) heads(lt::latent_absorb_kernel<4, 16, false>, dim, rank, 4, 16, u16(uk), u16(qa));
-  else if (n == 1) heads(lt::latent_absorb_kernel<1, 16, true>, dim, rank, 1, 16, u16(uk), u16(qa));
-  else if (n <= 4) heads(lt::latent_absorb_kernel<4, 16, true>, dim, rank, 4, 16, u16(uk), u16(qa));
-  else heads(lt::latent_absorb_kernel<8, 16, true>, dim, rank, 8, 16, u16(uk), u16(qa));
+  const unsigned nz = (unsigned)((n + 15) / 16);
+  hipLaunchKernelGGL(lt::latent_absorb_kernel, dim3(R / 16 + 1, H, nz), dim3(lt::kThreads), 0, cur_stream(), a, (int)n,
+                     (const unsigned short*)u16(uk), u16(qa));
   auto token = [&](auto kern, int PN) {
-    const size_t lds = (PN + 1) * lt::kKeys * mf::ROWB + 32 * lt::kSRow * sizeof(float);
+    const size_t lds = (PN + 1) * lt::kTok * mf::ROWB + 32 * lt::kSRow * sizeof(float);
     SXE_HIP_CHECK(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
     hipLaunchKernelGGL(kern, dim3(n, (H + 31) / 32, splits), dim3(lt::kThreads), lds, cur_stream(), a, (int)n,
                        (const unsigned short*)u16(qa), po.data_ptr<float>(), pml.data_ptr<float>());
   };
-  if (R <= 128) token(lt::latent_token_kernel<1>, 1);
-  else if (R <= 256) token(lt::latent_token_kernel<2>, 2);
+  if (R == 128) token(lt::latent_token_kernel<1>, 1);
+  else if (R == 256) token(lt::latent_token_kernel<2>, 2);
+  else if (R == 384) token(lt::latent_token_kernel<3>, 3);
   else token(lt::latent_token_kernel<4>, 4);
   const float *ppo = po.data_ptr<float>(), *pm = pml.data_ptr<float>();
-  const int sp = (int)splits;
-  if (!vv) heads(lt::latent_expand_kernel<4, 16, false>, rank, vdim, 4, 16, sp, ppo, pm, u16(uv), u16(out));
-  else if (n == 1) heads(lt::latent_expand_kernel<1, 4, true>, rank, vdim, 1, 4, sp, ppo, pm, u16(uv), u16(out));
-  else if (n <= 4) heads(lt::latent_expand_kernel<4, 4, true>, rank, vdim, 4, 4, sp, ppo, pm, u16(uv), u16(out));
-  else heads(lt::latent_expand_kernel<8, 16, true>, rank, vdim, 8, 16, sp, ppo, pm, u16(uv), u16(out));
+  const dim3 eg((vdim + 15) / 16, H, nz);
+  if (n == 1) {
+    hipLaunchKernelGGL(lt::latent_expand_kernel<true>, eg, dim3(lt::kThreads), 0, cur_stream(), a, (int)n, (int)splits, ppo, pm,
+                       (const unsigned short*)nullptr, (const unsigned short*)u16(uv), u16(out));
+  } else {
+    auto ol = at::empty({n, H, R}, q.options());
+    hipLaunchKernelGGL(lt::latent_merge_kernel, dim3(H, n), dim3(128), 0, cur_stream(), a, (int)n, (int)splits, ppo, pm, u16(ol));
+    hipLaunchKernelGGL(lt::latent_expand_kernel<false>, eg, dim3(lt::kThreads), 0, cur_stream(), a, (int)n, (int)splits, ppo, pm,
+                       (const unsigned short*)u16(ol), (const unsigned short*)u16(uv), u16(out));
+  }
   SXE_LAUNCH_CHECK();
 }
 

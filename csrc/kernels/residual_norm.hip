@@ -157,16 +157,38 @@ __global__ __launch_bounds__(kThreads) void sandwich_norm_kernel(SandwichArgs a)
   S* hr = static_cast<S*>(a.h) + o * W;
   float ss = 0.f;
   if constexpr (C > 0) {
-    f32x4 v[C];
+    // everything the row needs is in flight before the first reduction
+    f32x4 v[C], x0[C], g[C];
 #pragma unroll
-    for (int i = 0; i < C; ++i) v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int k = a.slots != nullptr ? a.k : 1;
-    for (int j = 0; j < k; ++j) {
-      const S* yr = yb + (a.slots != nullptr ? (int64_t)a.slots[r * a.k + j] : y0) * W;
+    for (int i = 0; i < C; ++i) {
+      const int c = min((i * kThreads + (int)threadIdx.x) * 4, W - 4);
+      v[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+      x0[i] = xr != nullptr ? *reinterpret_cast<const f32x4*>(xr + c) : v[i];
+      g[i] = load4<T>(wp + c);
+    }
+    if (a.slots == nullptr) {
 #pragma unroll
       for (int i = 0; i < C; ++i) {
         const int c = (i * kThreads + threadIdx.x) * 4;
-        if (c < W && ok) v[i] += load4<T>(yr + c);
+        if (c < W && ok) v[i] = load4<T>(yb + y0 * W + c);
+      }
+    } else {
+      constexpr int J = 4;  // rows in flight
+      for (int j0 = 0; j0 < a.k; j0 += J) {
+        const S* yr[J];
+#pragma unroll
+        for (int j = 0; j < J; ++j) yr[j] = yb + (int64_t)a.slots[r * a.k + min(j0 + j, a.k - 1)] * W;
+#pragma unroll
+        for (int i = 0; i < C; ++i) {
+          const int c = (i * kThreads + threadIdx.x) * 4;
+          if (c >= W) continue;
+          f32x4 t[J];
+#pragma unroll
+          for (int j = 0; j < J; ++j) t[j] = load4<T>(yr[j] + c);
+#pragma unroll
+          for (int j = 0; j < J; ++j)
+            if (j0 + j < a.k) v[i] += t[j];
+        }
       }
     }
 #pragma unroll
@@ -178,10 +200,8 @@ __global__ __launch_bounds__(kThreads) void sandwich_norm_kernel(SandwichArgs a)
     for (int i = 0; i < C; ++i) {
       const int c = (i * kThreads + threadIdx.x) * 4;
       if (c >= W) continue;
-      const f32x4 g = load4<T>(wp + c);
 #pragma unroll
-      for (int j = 0; j < 4; ++j) v[i][j] = v[i][j] * rp * g[j];
-      if (xr != nullptr) v[i] += *reinterpret_cast<const f32x4*>(xr + c);
+      for (int j = 0; j < 4; ++j) v[i][j] = v[i][j] * rp * g[i][j] + x0[i][j];
       if (ar != nullptr) v[i] += *reinterpret_cast<const f32x4*>(ar + c);
       if (a.xo != nullptr) *reinterpret_cast<f32x4*>(a.xo + o * W + c) = v[i];
       ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];

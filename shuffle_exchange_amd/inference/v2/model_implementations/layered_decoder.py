@@ -261,7 +261,7 @@ def _bipotar_weights(spec, sd):
             d["dqkv"] = torch.cat([get(p + "dq", a.q_rank, D), get(p + "dkv", R + a.rot_dim, D)])
             d["q_norm"], d["kv_norm"] = get(p + "dq.norm", a.q_rank), get(p + "dkv.norm", R)
             d["uq"], d["o"] = get(p + "uq", H * (a.dim + a.rot_dim), a.q_rank), get(p + "o", D, H * a.vdim)
-            d["uk"], d["uv"] = uk.view(H, a.dim, R), uv.view(H, a.vdim, R).transpose(1, 2)
+            d["uk"], d["uv"] = uk.view(H, a.dim, R).transpose(1, 2), uv.view(H, a.vdim, R)
             d["ukv"] = torch.cat([uk, uv])
         if L.ff or L.moe:
             p = f"l{i}.mlp."

@@ -79,8 +79,8 @@ def bipotar_model(size, device):
             x.update(qkvg=w(4 * H * d, D), o_norm=one(H * d), o=w(D, H * d), decay=decay_table(light.decay, device))
         else:
             uk, uv = w(H * d, kr), w(H * d, kr)
-            x.update(dqkv=w(qr + kr + rot, D), q_norm=one(qr), kv_norm=one(kr), uq=w(H * (d + rot), qr), uk=uk.view(H, d, kr),
-                     uv=uv.view(H, d, kr).transpose(1, 2), ukv=torch.cat([uk, uv]), o=w(D, H * d))
+            x.update(dqkv=w(qr + kr + rot, D), q_norm=one(qr), kv_norm=one(kr), uq=w(H * (d + rot), qr), uk=uk.view(H, d, kr).transpose(1, 2),
+                     uv=uv.view(H, d, kr), ukv=torch.cat([uk, uv]), o=w(D, H * d))
         if L.moe:
             x.update(router=w(E, D), e_up=w(E, eff, D), e_down=w(E, D, eff))
         else:

@@ -14,14 +14,14 @@ import torch
 
 from . import native
 
-TILE_MIN = 32  # sequences with at least this many new tokens take the expanded form
-PAD = 32       # bf16 cache rows: both parts padded to a multiple of this
+TILE_MIN = 32          # sequences with at least this many new tokens take the expanded form
+PAD_RANK, PAD_ROT = 128, 64  # bf16 cache rows: the parts' lengths are padded to multiples of these
 
 
 def latent_row(rank, rot, dtype):
     """(latent length, rotated length) of a cache row; bf16 rows are zero-padded for the matrix cores."""
     if dtype == torch.bfloat16:
-        return -(-rank // PAD) * PAD, -(-rot // PAD) * PAD
+        return -(-rank // PAD_RANK) * PAD_RANK, -(-rot // PAD_ROT) * PAD_ROT
     return rank, rot
 
 
@@ -64,8 +64,8 @@ def latent_append(proj, q_norm, kv_norm, cache, slots, rot, q_rank, rank, rot_di
 
 def latent_attention(q, uk, uv, ukv, cache, batch, rot, heads, dim, rot_dim, vdim, rank, scale, window=None, form="auto"):
     """``q`` [T, heads * (dim + rot_dim)] (per head [unrotated | to be rotated]) against the paged latent
-    ``cache``; ``uk`` [heads, dim, rank], ``uv`` [heads, rank, vdim], ``ukv`` [heads * (dim + vdim), rank] the same
-    weights stacked key rows first (None: the expanded form is not used). Returns [T, heads * vdim].
+    ``cache``; ``uk`` [heads, rank, dim] and ``uv`` [heads, vdim, rank] (the product's inner dimension last), ``ukv``
+    [heads * (dim + vdim), rank] the same weights stacked key rows first (None: the expanded form is not used). Returns [T, heads * vdim].
 
     ``form``: "token" one token's heads against the latents, "tile" keys and values expanded for tiles of
     tokens, "generic" any size and dtype, "auto" by shape (sequences of a batch may take different forms)."""
@@ -75,7 +75,7 @@ def latent_attention(q, uk, uv, ukv, cache, batch, rot, heads, dim, rot_dim, vdi
     if form == "auto":
         tile = ukv is not None and tile_ok(q, dim, rot_dim, vdim) and max(batch.host_q_len) >= TILE_MIN
         least = TILE_MIN if tile and min(batch.host_q_len) < TILE_MIN else 1
-        token = token_ok(q, R, rot_dim, scale)
+        token = token_ok(q, dim, rot_dim, rank, R, scale)
     else:
         tile, least, token = form == "tile", 1, form == "token"
     out = torch.empty(q.shape[0], heads * vdim, dtype=q.dtype, device=q.device)
@@ -111,8 +111,9 @@ def tile_ok(q, dim, rot_dim, vdim):
             and vdim % 8 == 0 and q.data_ptr() % 16 == 0)
 
 
-def token_ok(q, R, rot_dim, scale):
-    return q.dtype == torch.bfloat16 and R <= 512 and rot_dim <= 64 and scale > 0
+def token_ok(q, dim, rot_dim, rank, R, scale):
+    return (q.dtype == torch.bfloat16 and R <= 512 and rot_dim <= 64 and scale > 0 and dim % 8 == 0 and rank % 8 == 0
+            and rot_dim % 8 == 0 and q.data_ptr() % 16 == 0)
 
 
 def latent_attention_reference(q, uk, uv, cache, batch, rot, heads, dim, rot_dim, vdim, rank, scale, window=None):
@@ -128,7 +129,7 @@ def latent_attention_reference(q, uk, uv, cache, batch, rot, heads, dim, rot_dim
             continue
         rows = cache[batch.block_table[s, :(kl + bs - 1) // bs].long(), 0].reshape(-1, cache.shape[3])[:kl].float()
         c, kr = rows[:, :rank], rows[:, R:R + rot_dim]
-        k, v = torch.matmul(c, uk.float().transpose(1, 2)), torch.matmul(c, uv.float())
+        k, v = torch.matmul(c, uk.float()), torch.matmul(c, uv.float().transpose(1, 2))
         sc = torch.matmul(qn[a:a + n].transpose(0, 1), k.transpose(1, 2))
         sc = (sc + torch.matmul(qr[a:a + n].transpose(0, 1), kr.t())) * scale
         dist = torch.arange(kl - n, kl, device=q.device)[:, None] - torch.arange(kl, device=q.device)[None, :]

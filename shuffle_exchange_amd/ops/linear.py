@@ -161,6 +161,10 @@ def fused_gatesum_linear(part, gate, weight):
     return torch.ops.sxe.skinny_gemm_gatesum(part, gate, wk[0])
 
 
+# wider products run more workgroups than fit at once, each building the input again
+SANDWICH_MAX_N = int(os.environ.get("SXE_SANDWICH_MAX_N", 8192))
+
+
 def sandwich_fusable(x, y, *weights):
     """Whether the decode kernels with the sandwich-norm prologue (csrc/include/sxe_sandwich.h) take these rows:
     up to 4, M K <= 8192."""
@@ -173,7 +177,8 @@ def fused_sandwich_linear(x, y, post_weight, next_weight, eps, slots, add, weigh
     """Decode (<= 4 rows): ``sandwich_norm`` (ops/residual_norm.py) and the projection that reads its result in
     ONE launch (skinny_gemm.hip PRO_SANDWICH): (linear(h, weight), x'). None when not covered."""
     wk = _pro_weight(weight)
-    if wk is None or wk[1] is not None or not sandwich_fusable(x, y, post_weight, next_weight) or x.shape[1] != wk[0].shape[1]:
+    if (wk is None or wk[1] is not None or wk[0].shape[0] > SANDWICH_MAX_N or x.shape[1] != wk[0].shape[1]
+            or not sandwich_fusable(x, y, post_weight, next_weight)):
         return None
     return torch.ops.sxe.skinny_gemm_sandwich(x, y, post_weight, next_weight, slots, add, float(eps), wk[0])
 
