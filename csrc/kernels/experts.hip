@@ -500,13 +500,15 @@ std::vector<at::Tensor> choose(const at::Tensor& z, int64_t k) {
        active = at::empty({E + 1}, io);
   auto wt = at::empty({T, k}, z.options()), ws = at::empty({R}, z.options());
   if (R == 0) return {idx, wt, token, ws, slots, offs, active};
-  if (R <= kListThreads) {
-    hipLaunchKernelGGL(moe_lists_small_kernel, dim3(1), dim3(kListThreads), 0, cur_stream(), z.data_ptr<float>(), idx.data_ptr<int>(),
-                       wt.data_ptr<float>(), (int)R, (int)k, (int)E, token.data_ptr<int>(), ws.data_ptr<float>(),
-                       slots.data_ptr<int>(), offs.data_ptr<int>(), active.data_ptr<int>());
-  } else {
+  const bool small = R <= kListThreads, one = small && T <= 16;  // one: a wave per token chooses in the same workgroup
+  if (!one)
     hipLaunchKernelGGL(route_top_kernel, dim3((T + 3) / 4), dim3(256), 0, cur_stream(), z.data_ptr<float>(), (int)T, (int)E, (int)k,
                        idx.data_ptr<int>(), wt.data_ptr<float>());
+  if (small) {
+    hipLaunchKernelGGL(moe_lists_small_kernel, dim3(1), dim3(kListThreads), 0, cur_stream(), one ? z.data_ptr<float>() : nullptr,
+                       idx.data_ptr<int>(), wt.data_ptr<float>(), (int)R, (int)k, (int)E, token.data_ptr<int>(), ws.data_ptr<float>(),
+                       slots.data_ptr<int>(), offs.data_ptr<int>(), active.data_ptr<int>());
+  } else {
     auto counts = at::empty({E}, io);
     counts.zero_();
     const dim3 grid((R + kListThreads - 1) / kListThreads);

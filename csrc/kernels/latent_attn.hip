@@ -6,7 +6,7 @@
 //  * latent_append: norms of the query latent and of c, rotation of the key part, cache write;
 //  * generic form (fp32, any size): one workgroup per (token, head);
 //  * token form (decode, short continuations; bf16): latent_absorb forms W_uk^T q per head,
-//    latent_token runs one workgroup per (token, 32 heads, key split) with 32-key tiles of the cache in LDS,
+//    latent_token runs one workgroup per (token, 32 heads, key split) with 64-key tiles of the cache in LDS,
 //    read by rows for the scores and transposed for the weighted sum of latents -- each cache byte crosses
 //    HBM once for all heads --, latent_merge adds the splits and latent_expand applies W_uv (one token: the merge
 //    is its prologue);
@@ -344,20 +344,32 @@ __global__ __launch_bounds__(kThreads) void latent_expand_kernel(Args a, int n, 
 
 // ------------------------------------------------------------------------------------------ token form
 constexpr int kKeys = 64;       // keys of a tile of the tile form
-constexpr int kTok = 32;        // ... of the token form
+constexpr int kTok = 64, kTokWaves = 8;  // ... of the token form
 constexpr int kSRow = kTok + 4;  // fp32 score row of a head
 
-// PN 256-byte panels hold the latent (R = 128 PN), one more the rotated part (64 columns). grid (n, ceil(H / 32),
-// splits). Waves: scores of (16 keys, 16 heads) each; then PN 32-column tiles of the latent sum each, all heads.
+constexpr int kTabMax = 1024;   // most block-table entries of a split (kept in LDS)
+
+// barrier without waiting for the loads in flight
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+// PN 256-byte panels hold the latent (R = 128 PN), a 128-byte one the rotated part. grid (n, ceil(H / 32), splits).
+// Tiles arrive by direct-to-LDS loads, one ahead. 8 waves: scores of (16 keys, 16 heads) each; then the 32-column
+// tiles w, w + 8, .. of the latent sum, all heads.
 template <int PN>
-__global__ __launch_bounds__(kThreads, 2) void latent_token_kernel(Args a, int n, const unsigned short* __restrict qa,
-                                                                   float* __restrict po, float* __restrict pml) {
-  extern __shared__ __attribute__((aligned(16))) char smem[];
-  constexpr int PANEL = kTok * ROWB, NS = 4 * PN + 2, NC = 2 * PN + 1, ROW = 128 * PN + 64;
-  float* ls = reinterpret_cast<float*>(smem + (PN + 1) * PANEL);  // [32 heads][kSRow]
+__global__ __launch_bounds__(64 * kTokWaves, 1) void latent_token_kernel(Args a, int n, const unsigned short* __restrict qa,
+                                                                         float* __restrict po, float* __restrict pml) {
+  char* smem = tl::lds;
+  constexpr int PANEL = kTok * 256, SLOT = PN * PANEL + kTok * 128, NS = 4 * PN + 2, ROW = 128 * PN + 64;
+  constexpr int CT = 4 * PN, NT = (CT + kTokWaves - 1) / kTokWaves;
+  float* ls = reinterpret_cast<float*>(smem + 2 * SLOT);          // [32 heads][kSRow]
+  int* tab = reinterpret_cast<int*>(smem + 2 * SLOT + 32 * kSRow * 4);  // [kTabMax]
   const int i = blockIdx.x, g = blockIdx.y, sp = blockIdx.z;
   const int s = a.rows[2 * i], t = a.rows[2 * i + 1];
-  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, l16 = lane & 15, q16 = lane >> 4, l32 = lane & 31, hh = lane >> 5;
+  const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int l16 = lane & 15, q16 = lane >> 4, l32 = lane & 31, hh = lane >> 5;
   int lo, hi;
   key_range(a, s, t, lo, hi);
   {  // this split's keys, whole tiles
@@ -365,76 +377,121 @@ __global__ __launch_bounds__(kThreads, 2) void latent_token_kernel(Args a, int n
     lo = min(hi, lo + sp * per * kTok);
     hi = min(hi, lo + per * kTok);
   }
+  const int ntiles = (hi - lo + kTok - 1) / kTok, b0 = lo / a.bs;
   const unsigned short* cache = static_cast<const unsigned short*>(a.cache);
-  const int srow = threadIdx.x >> 3, sch = threadIdx.x & 7;
-  auto at = [&](int j0) { return cache_at(a, s, max(min(j0 + srow, hi - 1), 0)); };  // past the end: the last row (masked)
-  u32x4 st[NC];
-  auto load = [&](int64_t off) {
-#pragma unroll
-    for (int c = 0; c < NC; ++c) st[c] = *reinterpret_cast<const u32x4*>(cache + off + c * 64 + sch * 8);
+  const int* row = a.table + (int64_t)s * a.maxb + b0;
+  auto at = [&](int j, auto entry) {  // cache row of key j; past the end: the last one (masked)
+    j = min(j, hi - 1);
+    const int b = j / a.bs;
+    int64_t blk = entry(min(b - b0, kTabMax - 1));
+    if (blk < 0 || blk >= a.nblocks) blk = 0;
+    return cache + (blk * a.bs + (j - b * a.bs)) * ROW;
   };
-  int64_t next = 0;
+  const int r0 = 4 * w + (lane >> 4), r2 = 8 * w + (lane >> 3);  // rows this lane loads: r0, r0 + 32 (one swizzle); r2
+  const int c0 = ((lane & 15) ^ tl::swz<128>(r0)) * 8, c2 = ((lane & 7) ^ tl::swz<64>(r2)) * 8;
+  auto issue = [&](int j0, char* slot, auto entry) {
+    const unsigned short *p0 = at(j0 + r0, entry), *p1 = at(j0 + 32 + r0, entry), *p2 = at(j0 + r2, entry);
+#pragma unroll
+    for (int p = 0; p < PN; ++p) {
+      tl::glds16(p0 + p * 128 + c0, slot + p * PANEL + w * 1024);
+      tl::glds16(p1 + p * 128 + c0, slot + p * PANEL + (w + 8) * 1024);
+    }
+    tl::glds16(p2 + PN * 128 + c2, slot + PN * PANEL + w * 1024);
+  };
+  // the first tile takes its blocks from memory; the table is in LDS for the others
+  if (ntiles > 0) issue(lo, smem, [&](int x) { return row[x]; });
+  if (ntiles > 1)
+    for (int x = threadIdx.x; x < min((hi - 1) / a.bs - b0 + 1, kTabMax); x += 64 * kTokWaves) tab[x] = row[x];
   bf16x8 qf[NS];  // B fragments of 16 heads
-  if (lo < hi) {
-    const int64_t first = at(lo);
-    next = at(lo + kTok);
-    const int h = 32 * g + 16 * (w >> 1) + l16;
+  {
+    const int h = 32 * g + 16 * (w >> 2) + l16;
     const unsigned short* qr = qa + ((int64_t)i * a.H + min(h, a.H - 1)) * ROW + q16 * 8;
-    load(first);
 #pragma unroll
     for (int k = 0; k < NS; ++k) qf[k] = *reinterpret_cast<const bf16x8*>(qr + k * 32);
   }
-  f32x16 acc[PN];
+  // LDS read offsets: score rows (chunks q16 + 4 i of a panel: the swizzle's low bits move with i), value columns
+  const int kr = 16 * (w & 3) + l16;
+  int ko[4], kp[2];
 #pragma unroll
-  for (int j = 0; j < PN; ++j) acc[j] = zero16();
+  for (int k = 0; k < 4; ++k) ko[k] = tl::off<128>(kr, 4 * k + q16);
+#pragma unroll
+  for (int k = 0; k < 2; ++k) kp[k] = tl::off<64>(kr, 4 * k + q16);
+  int vo[NT][2];
+  {
+    tl::LaneOffs<128> o;
+    o.init(lane);
+#pragma unroll
+    for (int j = 0; j < NT; ++j)
+#pragma unroll
+      for (int x = 0; x < 4; ++x)
+        if (((w + kTokWaves * j) & 3) == x) {
+          vo[j][0] = o.tr[x][0] + ((w + kTokWaves * j) >> 2) * PANEL;
+          vo[j][1] = o.tr[x][1] + ((w + kTokWaves * j) >> 2) * PANEL;
+        }
+  }
+  f32x16 acc[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) acc[j] = zero16();
   float M = -INFINITY, L = 0.f;
   const float sc2 = a.scale * LOG2E;
-  for (int j0 = lo; j0 < hi; j0 += kTok) {
-    __syncthreads();  // the previous tile is read
+  // one copy of the loop body: few tiles run per workgroup, so instructions fetched twice would cost more than
+  // the slot's address arithmetic
+#pragma unroll 1
+  for (int tile = 0; tile < ntiles; ++tile) {
+    const int j0 = lo + tile * kTok, cur = tile & 1;
+    const char *lk = smem + cur * SLOT, *lr = lk + PN * PANEL;
+    tl::wait_loads();
+    lds_barrier();  // the tile has landed for every wave, and every wave is done with the one before
+    if (tile + 1 < ntiles) issue(j0 + kTok, smem + (cur ^ 1) * SLOT, [&](int x) { return tab[x]; });
+    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;  // keys 16 (w & 3) + 4 q16 + e, head 16 (w >> 2) + l16
+    bf16x8 kf[NS];
 #pragma unroll
-    for (int c = 0; c < NC; ++c) *reinterpret_cast<u32x4*>(smem + (c >> 1) * PANEL + soff(srow, (c & 1) * 8 + sch)) = st[c];
-    __syncthreads();
-    if (j0 + kTok < hi) {
-      load(next);
-      next = at(j0 + 2 * kTok);
-    }
-    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;  // keys 16 (w & 1) + 4 q16 + e, head 16 (w >> 1) + l16
+    for (int k = 0; k < 4 * PN; ++k) kf[k] = tl::row_at(lk + (k >> 2) * PANEL, ko[k & 3]);
+#pragma unroll
+    for (int k = 0; k < 2; ++k) kf[4 * PN + k] = tl::row_at(lr, kp[k]);
 #pragma unroll
     for (int k = 0; k < NS; k += 2) {
-      s0 = mfma16(lds_row16(smem + (k >> 2) * PANEL, 16 * (w & 1) + l16, (k & 3) * 4 + q16), qf[k], s0);
-      s1 = mfma16(lds_row16(smem + (k >> 2) * PANEL, 16 * (w & 1) + l16, ((k + 1) & 3) * 4 + q16), qf[k + 1], s1);
+      s0 = mfma16(kf[k], qf[k], s0);
+      s1 = mfma16(kf[k + 1], qf[k + 1], s1);
     }
-    const int kj = 16 * (w & 1) + 4 * q16;
+    const int kj = 16 * (w & 3) + 4 * q16;
 #pragma unroll
     for (int e = 0; e < 4; ++e) s0[e] = j0 + kj + e < hi ? (s0[e] + s1[e]) * sc2 : -INFINITY;
-    *reinterpret_cast<f32x4*>(ls + (16 * (w >> 1) + l16) * kSRow + kj) = s0;
-    __syncthreads();
+    *reinterpret_cast<f32x4*>(ls + (16 * (w >> 2) + l16) * kSRow + kj) = s0;
+    lds_barrier();
     // every wave forms all weights of the tile: lane = head l32, keys 8 x + 4 hh + e
-    f32x4 p[4];
+    f32x4 p[8];
     float m = -INFINITY;
 #pragma unroll
-    for (int x = 0; x < 4; ++x) {
-      p[x] = *reinterpret_cast<const f32x4*>(ls + l32 * kSRow + 8 * x + 4 * hh);
-      m = fmaxf(m, fmaxf(fmaxf(p[x][0], p[x][1]), fmaxf(p[x][2], p[x][3])));
-    }
+    for (int x = 0; x < 8; ++x) p[x] = *reinterpret_cast<const f32x4*>(ls + l32 * kSRow + 8 * x + 4 * hh);
+    bf16x8 vf[4][NT];
+#pragma unroll
+    for (int x = 0; x < 4; ++x)
+#pragma unroll
+      for (int j = 0; j < NT; ++j)
+        if (CT % kTokWaves == 0 || w + kTokWaves * j < CT) vf[x][j] = tl::tr_at(lk + 16 * x * 256, vo[j]);
+#pragma unroll
+    for (int x = 0; x < 8; ++x) m = fmaxf(m, fmaxf(fmaxf(p[x][0], p[x][1]), fmaxf(p[x][2], p[x][3])));
     m = fmaxf(m, xor32(m));
     const float Mn = fmaxf(M, m), f = fast_exp2(M - Mn);  // a tile has a visible key: Mn is finite
     float l = 0.f;
 #pragma unroll
-    for (int x = 0; x < 4; ++x)
+    for (int x = 0; x < 8; ++x)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         p[x][e] = fast_exp2(p[x][e] - Mn);
         l += p[x][e];
       }
     L = L * f + l + xor32(l);
+    if (__any(Mn > M)) {
+#pragma unroll
+      for (int j = 0; j < NT; ++j)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) acc[j][e] *= f;
+    }
     M = Mn;
 #pragma unroll
-    for (int j = 0; j < PN; ++j)
-#pragma unroll
-      for (int e = 0; e < 16; ++e) acc[j][e] *= f;
-#pragma unroll
-    for (int x = 0; x < 2; ++x) {
+    for (int x = 0; x < 4; ++x) {
       bf16x8 b;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
@@ -442,10 +499,8 @@ __global__ __launch_bounds__(kThreads, 2) void latent_token_kernel(Args a, int n
         b[4 + e] = (__bf16)p[2 * x + 1][e];
       }
 #pragma unroll
-      for (int j = 0; j < PN; ++j) {
-        const int ct = w * PN + j;
-        acc[j] = mfma(lds_trA(smem + (ct >> 2) * PANEL, 16 * x, ct & 3, lane), b, acc[j]);
-      }
+      for (int j = 0; j < NT; ++j)
+        if (CT % kTokWaves == 0 || w + kTokWaves * j < CT) acc[j] = mfma(vf[x][j], b, acc[j]);
     }
   }
   const int h = 32 * g + l32;
@@ -455,13 +510,16 @@ __global__ __launch_bounds__(kThreads, 2) void latent_token_kernel(Args a, int n
       pml[th * 2] = M;
       pml[th * 2 + 1] = L;
     }
-    if (lo < hi) {
-      float* o = po + th * a.R + w * PN * 32 + 4 * hh;
+    if (ntiles > 0) {
 #pragma unroll
-      for (int j = 0; j < PN; ++j)
+      for (int j = 0; j < NT; ++j) {
+        const int ct = w + kTokWaves * j;
+        if (ct >= CT) break;
+        float* o = po + th * a.R + ct * 32 + 4 * hh;
 #pragma unroll
         for (int e = 0; e < 4; ++e)
-          *reinterpret_cast<f32x4*>(o + j * 32 + 8 * e) = f32x4{acc[j][4 * e], acc[j][4 * e + 1], acc[j][4 * e + 2], acc[j][4 * e + 3]};
+          *reinterpret_cast<f32x4*>(o + 8 * e) = f32x4{acc[j][4 * e], acc[j][4 * e + 1], acc[j][4 * e + 2], acc[j][4 * e + 3]};
+      }
     }
   }
 }
@@ -779,6 +837,12 @@ void latent_attention_token(const at::Tensor& q, const at::Tensor& uk, const at:
   lt::Args a{q.data_ptr(), rot.data_ptr<float>(), rows.data_ptr<int>(), table.data_ptr<int>(), q_start.data_ptr<int>(),
              q_len.data_ptr<int>(), kv_len.data_ptr<int>(), cache.data_ptr(), cache.size(0), (int)table.size(1), (int)cache.size(2),
              (int)H, (int)dim, (int)rot_dim, (int)rank, (int)R, (int)row, (int)vdim, (int)window, (float)scale};
+  {  // a split's block-table entries fit in LDS
+    const int64_t bs = cache.size(2), most = window > 0 ? std::min<int64_t>(window, table.size(1) * bs) : table.size(1) * bs;
+    const int64_t per = std::max<int64_t>(1, (lt::kTabMax - 2) * bs / lt::kTok - 1) * lt::kTok;
+    splits = std::max(splits, (most + per - 1) / per);
+    SXE_CHECK(splits <= lt::kMaxSplits, "latent_attention: ", most, " keys in blocks of ", bs, " are too many");
+  }
   SXE_CHECK((n + 15) / 16 <= 65535 && lt::aligned(q.data_ptr(), 16) && lt::aligned(uk.data_ptr(), 16) && lt::aligned(uv.data_ptr(), 16),
             "latent_attention: 16-byte aligned operands");
   auto f32 = q.options().dtype(at::kFloat);
@@ -788,9 +852,9 @@ void latent_attention_token(const at::Tensor& q, const at::Tensor& uk, const at:
   hipLaunchKernelGGL(lt::latent_absorb_kernel, dim3(R / 16 + 1, H, nz), dim3(lt::kThreads), 0, cur_stream(), a, (int)n,
                      (const unsigned short*)u16(uk), u16(qa));
   auto token = [&](auto kern, int PN) {
-    const size_t lds = (PN + 1) * lt::kTok * mf::ROWB + 32 * lt::kSRow * sizeof(float);
+    const size_t lds = 2 * lt::kTok * (PN * 256 + 128) + 32 * lt::kSRow * sizeof(float) + lt::kTabMax * sizeof(int);
     SXE_HIP_CHECK(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-    hipLaunchKernelGGL(kern, dim3(n, (H + 31) / 32, splits), dim3(lt::kThreads), lds, cur_stream(), a, (int)n,
+    hipLaunchKernelGGL(kern, dim3(n, (H + 31) / 32, splits), dim3(64 * lt::kTokWaves), lds, cur_stream(), a, (int)n,
                        (const unsigned short*)u16(qa), po.data_ptr<float>(), pml.data_ptr<float>());
   };
   if (R == 128) token(lt::latent_token_kernel<1>, 1);

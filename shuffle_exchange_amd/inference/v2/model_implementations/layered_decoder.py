@@ -207,9 +207,10 @@ def _tobinex_weights(spec, sd):
 # ------------------------------------------------------------------------------------- Bipotar
 def _bipotar_mixer(i, kind, m):
     if kind == "lightning":
-        if len(m["decay"]) != m["heads"]:
-            raise ValueError(f"layer {i}: {len(m['decay'])} decays for {m['heads']} heads")
-        return LinearSpec(int(m["heads"]), int(m["dim"]), int(m["vdim"]), [float(d) for d in m["decay"]])
+        decay = m["decay"] if isinstance(m["decay"], list) else [m["decay"]] * m["heads"]
+        if len(decay) != m["heads"]:
+            raise ValueError(f"layer {i}: {len(decay)} decays for {m['heads']} heads")
+        return LinearSpec(int(m["heads"]), int(m["dim"]), int(m["vdim"]), [float(d) for d in decay])
     if kind == "latent_attention":
         if m["rot"]["dims"] != m["rot_dim"] or m["rot_dim"] % 2:
             raise ValueError(f"layer {i}: rotation over {m['rot']['dims']} of {m['rot_dim']} rotated dimensions")
@@ -239,7 +240,7 @@ def _bipotar_spec(c):
         if not 0 <= loop.start <= loop.stop <= len(layers):
             raise ValueError(f"loop over layers {loop.start} .. {loop.stop - 1} of {len(layers)}")
     return LayeredSpec(c["architecture"], int(c["vocab"]), int(c["width"]), float(c["norm"]["eps"]), norm_offset=0.0,
-                       layers=layers, residual="sandwich", loop=loop, logit_scale=float(c["logit_scale"]))
+                       layers=layers, residual="sandwich", loop=loop, logit_scale=float(c.get("logit_scale", 1.0)))
 
 
 def _bipotar_weights(spec, sd):

@@ -55,6 +55,8 @@ CONFIGS = {
     # more heads than a tile, a long latent, windows beyond a key tile, a loop that runs once, layers behind the loop
     "wide": config(192, 80, [latent(34, 128, 32, 128, 96, 300, 130, dense(200)), light(2, 64, 24, moe(9, 3, 136)),
                              latent(2, 64, 64, 64, 64, 256, 64, moe(2, 2, 64))], (0, 1, 1)),
+    # rows in multiples of 64 throughout, for quantized projections
+    "aligned": config(128, 96, [latent(2, 48, 16, 64, 64, 64, 50, dense(192)), light(2, 64, 64, moe(4, 2, 64))], (0, 2, 2)),
     "single": config(64, 64, [latent(4, 16, 8, 16, 24, 32, 20, dense(48))], (0, 0, 1)),
     "state": config(64, 64, [light(4, 16, 16, dense(48), [0.2, 0.9, 0.99, 1.0])], (0, 1, 1)),
 }
@@ -278,6 +280,16 @@ def test_serialized_engine(tmp_path, device, dtype):
         return  # the rebuilt engine takes the process's device
     again = build_engine_from_ds_checkpoint(str(tmp_path / "saved"), RaggedInferenceEngineConfig(num_kv_blocks=8))
     torch.testing.assert_close(again.put([0], [toks]).cpu(), y)
+
+
+@pytest.mark.gpu
+def test_quantized_projections(tmp_path):
+    """Dense projections as fp8 weights (experts, latent and router weights stay as they are)."""
+    path, cfg, w = checkpoint(tmp_path, "aligned", 25, O.random_model)
+    eng = build_hf_engine(path, RaggedInferenceEngineConfig(num_kv_blocks=16), weight_quant="fp8")
+    toks = prompt(cfg, 60, 2)
+    got, ref = run(eng, 0, toks, [40, 1]).double(), O.forward(cfg, w, toks)
+    assert float((got - ref).pow(2).mean(-1).sqrt().median() / ref.std()) < 0.2
 
 
 @pytest.mark.parametrize("device,dtype", DEVICES)
