@@ -235,18 +235,38 @@ __device__ __forceinline__ float head_product(const unsigned short* xrow, const 
   return part[0][r][c] + part[1][r][c] + part[2][r][c] + part[3][r][c];
 }
 
-// grid (R / 16 + 1, H, ceil(n / 16)) -> qa [n, H, row] bf16: W_uk^T q | rotated q, zero-padded; uk [H, rank, dim]
+// grid (R / 64 + 1, H, ceil(n / 16)) -> qa [n, H, row] bf16: W_uk^T q | rotated q, zero-padded; uk [H, rank, dim].
+// A wave takes 16 columns and the whole (short) inner dimension.
 __global__ __launch_bounds__(kThreads) void latent_absorb_kernel(Args a, int n, const unsigned short* __restrict uk,
                                                                  unsigned short* __restrict qa) {
-  __shared__ float part[4][16][17];
-  const int c0 = blockIdx.x * 16, h = blockIdx.y, i0 = blockIdx.z * 16, half = a.rot_dim / 2, l16 = threadIdx.x & 15;
+  const int h = blockIdx.y, i0 = blockIdx.z * 16, half = a.rot_dim / 2, l16 = threadIdx.x & 15, g = (threadIdx.x & 63) >> 4;
   const unsigned short* q = static_cast<const unsigned short*>(a.q);
-  if (c0 < a.R) {
+  if ((int)blockIdx.x * 64 < a.R) {
+    const int c = blockIdx.x * 64 + (threadIdx.x >> 6) * 16 + l16;
     const int64_t row = a.rows[2 * min(i0 + l16, n - 1) + 1];
-    const unsigned short* wr = uk + ((int64_t)h * a.rank + min(c0 + l16, a.rank - 1)) * a.dim;
-    const float v = head_product(q + (row * a.H + h) * (a.dim + a.rot_dim), wr, a.dim, part);
-    const int i = i0 + (threadIdx.x >> 4), c = c0 + l16;
-    if (i < n) qa[((int64_t)i * a.H + h) * a.row + c] = c < a.rank ? f32_to_bf16(v) : 0;
+    const unsigned short* xr = q + (row * a.H + h) * (a.dim + a.rot_dim);
+    const unsigned short* wr = uk + ((int64_t)h * a.rank + min(c, a.rank - 1)) * a.dim;
+    constexpr int U = 4;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < a.dim; k0 += U * 32) {
+      u32x4 x[U], w[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int k = k0 + u * 32 + 8 * g;
+        x[u] = w[u] = u32x4{0u, 0u, 0u, 0u};
+        if (k < a.dim) {
+          x[u] = *reinterpret_cast<const u32x4*>(xr + k);
+          w[u] = *reinterpret_cast<const u32x4*>(wr + k);
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < U; ++u) acc = mfma16(__builtin_bit_cast(bf16x8, x[u]), __builtin_bit_cast(bf16x8, w[u]), acc);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = i0 + 4 * g + e;
+      if (i < n) qa[((int64_t)i * a.H + h) * a.row + c] = c < a.rank ? f32_to_bf16(acc[e]) : 0;
+    }
     return;
   }
   const int rp = a.row - a.R;
@@ -849,7 +869,7 @@ void latent_attention_token(const at::Tensor& q, const at::Tensor& uk, const at:
   auto qa = at::empty({n, H, row}, q.options()), po = at::empty({splits, n, H, R}, f32), pml = at::empty({splits, n, H, 2}, f32);
   auto u16 = [](const at::Tensor& t) { return static_cast<unsigned short*>(t.data_ptr()); };
   const unsigned nz = (unsigned)((n + 15) / 16);
-  hipLaunchKernelGGL(lt::latent_absorb_kernel, dim3(R / 16 + 1, H, nz), dim3(lt::kThreads), 0, cur_stream(), a, (int)n,
+  hipLaunchKernelGGL(lt::latent_absorb_kernel, dim3(R / 64 + 1, H, nz), dim3(lt::kThreads), 0, cur_stream(), a, (int)n,
                      (const unsigned short*)u16(uk), u16(qa));
   auto token = [&](auto kern, int PN) {
     const size_t lds = 2 * lt::kTok * (PN * 256 + 128) + 32 * lt::kSRow * sizeof(float) + lt::kTabMax * sizeof(int);

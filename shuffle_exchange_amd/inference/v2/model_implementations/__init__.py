@@ -6,7 +6,7 @@
   Mistral, Mixtral, Qwen2, Qwen2-MoE, Phi, Phi-3, Falcon, OPT -- converted once into the packed
   layout of the gfx950 kernels;
 * ``RaggedLayeredDecoder`` (layered_decoder.py): designs whose config lists every layer with sizes of its
-  own (Tobinex).
+  own (Tobinex, Bipotar).
 """
 from .hf_decoder import RaggedDecoder, load_hf_decoder, spec_from_hf_config  # noqa: F401
 from .layered_decoder import RaggedLayeredDecoder, load_layered_decoder  # noqa: F401

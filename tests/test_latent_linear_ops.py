@@ -159,7 +159,7 @@ def test_latent_attention_generic_form(window, device, dtype):
 
 
 @gpu
-@pytest.mark.parametrize("H,dim,rd,vdim,R", [(6, 64, 16, 64, 96), (34, 128, 64, 128, 512), (3, 24, 8, 12, 248), (16, 32, 32, 36, 320),
+@pytest.mark.parametrize("H,dim,rd,vdim,R", [(5, 48, 32, 40, 112), (34, 128, 64, 128, 512), (3, 24, 8, 12, 248), (16, 32, 32, 36, 320),
                                              (1, 8, 8, 5, 8), (2, 200, 48, 20, 136)])
 @pytest.mark.parametrize("window", [None, 1, 33, 64, 128])
 def test_latent_attention_token_form(window, H, dim, rd, vdim, R):
@@ -173,7 +173,7 @@ def test_latent_attention_token_form_large_batch_and_key_splits():
 
 
 @gpu
-@pytest.mark.parametrize("H,dim,rd,vdim", [(3, 64, 16, 64), (2, 128, 64, 128), (4, 40, 8, 72), (2, 96, 32, 24)])
+@pytest.mark.parametrize("H,dim,rd,vdim", [(3, 56, 48, 64), (2, 128, 64, 128), (4, 40, 8, 72), (2, 96, 32, 24)])
 @pytest.mark.parametrize("window", [None, 1, 50, 64, 130])
 def test_latent_attention_tile_form(window, H, dim, rd, vdim):
     latent_case([(0, 300), (77, 128), (500, 1), (0, 2), (130, 129)], H, dim, rd, vdim, 72, window, torch.bfloat16, "cuda", "tile")
@@ -181,7 +181,7 @@ def test_latent_attention_tile_form(window, H, dim, rd, vdim):
 
 @gpu
 def test_latent_attention_forms_mixed_in_a_batch():
-    latent_case([(0, 90), (300, 1), (40, 2), (64, 33), (9, 31)], 3, 64, 16, 64, 96, 50, torch.bfloat16, "cuda", None)
+    latent_case([(0, 90), (300, 1), (40, 2), (64, 33), (9, 31)], 3, 80, 48, 56, 104, 50, torch.bfloat16, "cuda", None)
 
 
 @gpu
