@@ -2,6 +2,7 @@
 torchrun's OMP_NUM_THREADS=1, CPU shares per rank / NUMA node, and the host-memory pre-flight."""
 import json
 import os
+import re
 import subprocess
 import sys
 
@@ -72,7 +73,7 @@ def test_torchrun_eight_ranks_each_get_their_share(tmp_path):
            "127.0.0.1", "--master-port", "29671", str(script)]
     r = subprocess.run(cmd, env=env, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True, timeout=300)
     assert r.returncode == 0, r.stdout[-3000:]
-    probes = [json.loads(l.split("PROBE ", 1)[1]) for l in r.stdout.splitlines() if "PROBE " in l]
+    probes = [json.loads(x) for x in re.findall(r"PROBE (\{[^{}]*\})", r.stdout)]  # ranks share one stdout: lines may run together
     assert len(probes) == 8
     cores = len(os.sched_getaffinity(0))
     for p in probes:
