@@ -895,10 +895,10 @@ void latent_attention_token(const at::Tensor& q, const at::Tensor& uk, const at:
   SXE_LAUNCH_CHECK();
 }
 
-// kv [Nk, H (dim + vdim)]: all heads' keys, then all heads' values; lat [Nk, row]: the cache rows they come from
+// chunks int32 [n, 3]: (sequence, first row, rows <= kQ); kv [Nk, H (dim + vdim)]: all heads' keys, then all heads' values; lat [Nk, row]: the cache rows they come from
 void latent_attention_tile(const at::Tensor& q, const at::Tensor& kv, const at::Tensor& lat, const at::Tensor& rot,
-                           const at::Tensor& chunks, const at::Tensor& first, const at::Tensor& q_start, const at::Tensor& q_len,
-                           const at::Tensor& kv_len, at::Tensor out, int64_t H, int64_t dim, int64_t rot_dim, int64_t vdim, int64_t R,
+                           const at::Tensor& chunks, int64_t size, const at::Tensor& first, const at::Tensor& q_start,
+                           const at::Tensor& q_len, const at::Tensor& kv_len, at::Tensor out, int64_t H, int64_t dim, int64_t rot_dim, int64_t vdim, int64_t R,
                            double scale, int64_t window) {
   SXE_CHECK_CUDA(q);
   const int64_t S = q_start.numel(), nc = chunks.size(0), Nk = kv.size(0);
@@ -910,7 +910,7 @@ void latent_attention_tile(const at::Tensor& q, const at::Tensor& kv, const at::
                 R % 8 == 0 && lat.size(1) % 8 == 0 && out.size(0) == q.size(0) && out.size(1) == H * vdim,
             "latent_attention: tile form shapes");
   SXE_CHECK(chunks.is_cuda() && chunks.scalar_type() == at::kInt && chunks.is_contiguous() && chunks.dim() == 2 && chunks.size(1) == 3 &&
-                first.is_cuda() && first.scalar_type() == at::kInt && first.is_contiguous() && first.numel() == 2 * S,
+                size == lt::kQ && first.is_cuda() && first.scalar_type() == at::kInt && first.is_contiguous() && first.numel() == 2 * S,
             "latent_attention: tables");
   for (const auto* t : {&q_start, &q_len, &kv_len})
     SXE_CHECK(t->is_cuda() && t->is_contiguous() && t->scalar_type() == at::kInt && t->numel() == S, "latent_attention: int32 [S]");
@@ -944,7 +944,7 @@ TORCH_LIBRARY_FRAGMENT(sxe, m) {
         "Tensor q_start, Tensor q_len, Tensor kv_len, Tensor(a!) out, int rot_dim, int R, float scale, int window) -> ()");
   m.def("latent_attention_token(Tensor q, Tensor uk, Tensor uv, Tensor cache, Tensor rot, Tensor rows, Tensor table, "
         "Tensor q_start, Tensor q_len, Tensor kv_len, Tensor(a!) out, int splits, int rot_dim, int R, float scale, int window) -> ()");
-  m.def("latent_attention_tile(Tensor q, Tensor kv, Tensor lat, Tensor rot, Tensor chunks, Tensor first, Tensor q_start, "
+  m.def("latent_attention_tile(Tensor q, Tensor kv, Tensor lat, Tensor rot, Tensor chunks, int size, Tensor first, Tensor q_start, "
         "Tensor q_len, Tensor kv_len, Tensor(a!) out, int H, int dim, int rot_dim, int vdim, int R, float scale, int window) -> ()");
 }
 TORCH_LIBRARY_IMPL(sxe, CUDA, m) {

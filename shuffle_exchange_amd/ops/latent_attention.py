@@ -85,8 +85,8 @@ def latent_attention(q, uk, uv, ukv, cache, batch, rot, heads, dim, rot_dim, vdi
         slots, first = batch.key_rows(window, least)
         lat = cache.view(-1, cache.shape[3]).index_select(0, slots)
         kv = torch.nn.functional.linear(lat[:, :rank], ukv)
-        torch.ops.sxe.latent_attention_tile(q, kv, lat, rot, batch.chunks(TILE_TOKENS, least), first, *lens, out, int(heads), int(dim),
-                                            int(rot_dim), int(vdim), int(R), float(scale), w)
+        torch.ops.sxe.latent_attention_tile(q, kv, lat, rot, batch.chunks(TILE_TOKENS, least), TILE_TOKENS, first, *lens, out,
+                                            int(heads), int(dim), int(rot_dim), int(vdim), int(R), float(scale), w)
         if least == 1:
             return out
     rows = batch.token_rows(TILE_MIN if tile else None)  # tokens of the other sequences
